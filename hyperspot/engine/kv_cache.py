@@ -294,6 +294,12 @@ class KVPages(NamedTuple):
     v: torch.Tensor
 
 
+class LatentKV(NamedTuple):
+    """Pages [NB, BS, width] of one row per token for all heads."""
+
+    kv: torch.Tensor
+
+
 class RecurrentState(NamedTuple):
     """Float state pool of one layer, indexed by the sequence's row in the
     BlockManager: S [slots, H, D, E], with a normalizer also n [slots, H, D]
@@ -307,12 +313,17 @@ class RecurrentState(NamedTuple):
 def allocate_caches(spec, config, num_blocks: int, num_slots: int,
                     dtype: torch.dtype, device) -> list:
     """Per-layer caches following the model's layout."""
-    from .layer_spec import PagedKV
+    from .layer_spec import LatentPages, SharedCache, StateSlots
     layout = spec.cache_layout(max(config.tp_size, 1))
     bs = config.block_size
     caches = []
     for c in layout:
-        if not isinstance(c, PagedKV):
+        if isinstance(c, SharedCache):
+            caches.append(caches[c.layer])
+        elif isinstance(c, LatentPages):
+            caches.append(LatentKV(torch.zeros(num_blocks, bs, c.width,
+                                               dtype=dtype, device=device)))
+        elif isinstance(c, StateSlots):
             z = lambda *shape: torch.zeros(num_slots, *shape,
                                            dtype=torch.float32, device=device)
             caches.append(
@@ -342,17 +353,17 @@ def compute_num_gpu_blocks(spec, config, device, safety_frac: float = None,
     frac = safety_frac if safety_frac is not None else config.gpu_memory_utilization
     if device == "cpu" or (hasattr(device, "type") and device.type == "cpu"):
         return 512
-    from .layer_spec import PagedKV
+    from .layer_spec import StateSlots
     free, total = torch.cuda.mem_get_info(device)
     budget = int(total * frac) - (total - free)
     elem_bytes = 1 if getattr(config, "kv_dtype", "bfloat16") == "fp8" \
         else 4 if config.dtype == "float32" else 2
     per_block = 0
     for c in spec.cache_layout(max(config.tp_size, 1)):
-        if isinstance(c, PagedKV):
-            per_block += config.block_size * c.bytes_per_token(elem_bytes)
-        else:
+        if isinstance(c, StateSlots):
             budget -= num_slots * c.bytes_per_slot()
+        else:
+            per_block += config.block_size * c.bytes_per_token(elem_bytes)
     if budget <= 0:
         raise RuntimeError(
             f"recurrent state for {num_slots} sequences does not fit in "

@@ -1,13 +1,16 @@
 """Per-layer descriptions for models whose layers are not all alike.
 
 A ``HybridSpec`` is a ``ModelSpec`` with an explicit list of layers, each one
-mixer (windowed differential attention, gated linear attention, matrix LSTM)
-and an optional feed-forward.  Every size and constant of a mixer is a field
-here; the layer classes in ``hyperspot.models.mixers`` read nothing else.
+mixer (windowed differential attention, windowed latent attention, gated
+linear attention, matrix LSTM, lightning attention) and an optional
+feed-forward (dense, or a mixture of experts).  Every size and constant of a
+layer part is a field here; the layer classes in ``hyperspot.models.mixers``
+read nothing else.
 
 ``cache_layout`` tells the cache manager what a layer keeps per sequence:
-pages that grow with the tokens (``PagedKV``) or a fixed-size recurrent state
-(``StateSlots``), both already divided over the tensor-parallel ranks.
+pages that grow with the tokens (``PagedKV``, ``LatentPages``), a fixed-size
+recurrent state (``StateSlots``), or nothing of its own (``SharedCache``), all
+already divided over the tensor-parallel ranks.
 """
 
 from __future__ import annotations
@@ -32,6 +35,27 @@ class PagedKV:
 
     def bytes_per_token(self, elem: int) -> int:
         return self.kv_heads * (self.k_dim + self.v_dim) * elem
+
+
+@dataclass(frozen=True)
+class LatentPages:
+    """Pages [NB, BS, width] of one row per token that all heads share (every
+    tensor-parallel rank keeps the whole row)."""
+
+    width: int
+
+    def bytes_per_token(self, elem: int) -> int:
+        return self.width * elem
+
+
+@dataclass(frozen=True)
+class SharedCache:
+    """The layer reads the cache of an earlier layer and keeps nothing."""
+
+    layer: int
+
+    def bytes_per_token(self, elem: int) -> int:
+        return 0
 
 
 @dataclass(frozen=True)
@@ -130,13 +154,97 @@ class MatrixLSTM:
             raise ValueError("mlstm: gate_cap must not be zero")
 
 
-Mixer = Union[DiffAttention, GatedLinear, MatrixLSTM]
+@dataclass(frozen=True)
+class LatentAttention:
+    """Sliding-window attention whose keys and values are expanded per head
+    from one latent per token; a rotated key part is shared by all heads.
+    With `kv_from` the latents are those of an earlier layer."""
+
+    heads: int
+    dim: int            # unrotated query/key size per head
+    rot_dim: int        # rotated query/key size
+    vdim: int
+    kv_rank: int
+    scale: float
+    window: int
+    rot_base: float
+    kv_from: Optional[int] = None
+
+    def cache(self, tp: int) -> Union[LatentPages, SharedCache]:
+        if self.kv_from is not None:
+            return SharedCache(self.kv_from)
+        return LatentPages(self.kv_rank + self.rot_dim)
+
+    def params(self, width: int) -> int:
+        n = (width * self.heads * (self.dim + self.rot_dim + self.vdim)
+             + self.kv_rank * self.heads * (self.dim + self.vdim))
+        if self.kv_from is None:
+            n += width * (self.kv_rank + self.rot_dim) + self.kv_rank
+        return n
+
+    def check(self) -> None:
+        if self.rot_dim % 2:
+            raise ValueError("latent attention: rotary size must be even")
+        if self.window < 1:
+            raise ValueError("latent attention: window must be at least 1")
+
+
+@dataclass(frozen=True)
+class Lightning:
+    """Linear attention with a constant decay per head, SiLU on queries, keys
+    and values, one norm over all heads together and a sigmoid gate."""
+
+    heads: int
+    dim: int
+    vdim: int
+    decay: Tuple[float, ...]
+
+    def cache(self, tp: int) -> StateSlots:
+        return StateSlots(self.heads // tp, self.dim, self.vdim)
+
+    def params(self, width: int) -> int:
+        d, e = self.heads * self.dim, self.heads * self.vdim
+        return width * (2 * d + 3 * e) + e
+
+    def check(self) -> None:
+        if len(self.decay) != self.heads:
+            raise ValueError("lightning: one decay per head")
+        if not all(0.0 <= x <= 1.0 for x in self.decay):
+            raise ValueError("lightning: decays must be within [0, 1]")
+
+
+Mixer = Union[DiffAttention, GatedLinear, MatrixLSTM, LatentAttention,
+              Lightning]
+
+
+@dataclass(frozen=True)
+class Experts:
+    """Mixture of gated-SiLU experts; `shared` is the size of an expert that
+    every token also passes, weighted by a sigmoid gate (None: there is
+    none)."""
+
+    experts: int
+    top: int
+    ff: int
+    shared: Optional[int] = None
+
+    def params(self, width: int) -> int:
+        n = width * self.experts * (1 + 3 * self.ff)
+        if self.shared is not None:
+            n += width * (1 + 3 * self.shared)
+        return n
+
+    def check(self) -> None:
+        if not 1 <= self.top <= self.experts:
+            raise ValueError("experts: top must be between 1 and the number "
+                             "of experts")
 
 
 @dataclass(frozen=True)
 class LayerSpec:
     mixer: Mixer
-    ff: Optional[int] = None      # feed-forward size; None: no feed-forward
+    # dense feed-forward size, experts, or None for no feed-forward
+    ff: Union[None, int, Experts] = None
 
 
 @dataclass
@@ -146,18 +254,27 @@ class HybridSpec(ModelSpec):
 
     architecture: str = ""
     layers: Tuple[LayerSpec, ...] = field(default_factory=tuple)
+    norm_params: int = 0          # parameters of one norm
+    norms: int = 2                # norms per sublayer
+    embed_scale: float = 1.0
+    # size of a token's own input to every layer (0: there is none)
+    side_dim: int = 0
 
     def param_count(self) -> int:
         h = self.hidden_size
         n = self.vocab_size * h * (1 if self.tie_embeddings else 2)
-        norm = 2 * h + 1
+        n += self.norm_params
         for layer in self.layers:
-            n += layer.mixer.params(h) + 2 * norm
+            n += layer.mixer.params(h) + self.norms * self.norm_params
             if layer.ff is not None:
-                n += 3 * h * layer.ff + 2 * norm
-        return n + norm
+                n += layer.ff.params(h) if isinstance(layer.ff, Experts) \
+                    else 3 * h * layer.ff
+                n += self.norms * self.norm_params
+            if self.side_dim:
+                n += (self.vocab_size + 2 * h) * self.side_dim + h
+        return n
 
-    def cache_layout(self, tp: int) -> List[Union[PagedKV, StateSlots]]:
+    def cache_layout(self, tp: int) -> list:
         return [layer.mixer.cache(tp) for layer in self.layers]
 
     @property
@@ -168,18 +285,42 @@ class HybridSpec(ModelSpec):
     def has_state(self) -> bool:
         return any(isinstance(c, StateSlots) for c in self.cache_layout(1))
 
+    @property
+    def latent_windows(self) -> List[int]:
+        """Distinct windows of the latent-attention layers."""
+        return sorted({layer.mixer.window for layer in self.layers
+                       if isinstance(layer.mixer, LatentAttention)})
+
 
 def hybrid_spec(name: str, architecture: str, width: int, vocab: int,
                 eps: float, layers, max_position: int = 1 << 20,
-                tie_embeddings: bool = True) -> HybridSpec:
-    """Build a checked HybridSpec.  The per-model fields of ModelSpec that
-    only make sense for uniform layers are zero."""
+                tie_embeddings: bool = True, **kw) -> HybridSpec:
+    """Build a checked HybridSpec; `kw` are its own fields.  The per-model
+    fields of ModelSpec that only make sense for uniform layers are zero."""
     layers = tuple(layers)
-    for layer in layers:
+    for i, layer in enumerate(layers):
         layer.mixer.check()
+        if isinstance(layer.ff, Experts):
+            layer.ff.check()
+        _check_shared_cache(layers, i)
     return HybridSpec(
         name=name, hidden_size=width, num_layers=len(layers), num_heads=0,
         num_kv_heads=0, head_dim=0, intermediate_size=0, vocab_size=vocab,
         rms_eps=eps, max_position=max_position,
         tie_embeddings=tie_embeddings, architecture=architecture,
-        layers=layers)
+        layers=layers, **kw)
+
+
+def _check_shared_cache(layers, i: int) -> None:
+    m = layers[i].mixer
+    j = getattr(m, "kv_from", None)
+    if j is None:
+        return
+    o = layers[j].mixer if 0 <= j < i else None
+    if not isinstance(o, LatentAttention) or o.kv_from is not None:
+        raise ValueError(f"layer {i}: kv_from must name an earlier "
+                         "latent-attention layer with latents of its own")
+    if (o.kv_rank, o.rot_dim, o.rot_base) != (m.kv_rank, m.rot_dim,
+                                              m.rot_base):
+        raise ValueError(f"layer {i}: latent sizes and rotation differ from "
+                         f"layer {j}'s")

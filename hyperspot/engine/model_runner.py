@@ -18,7 +18,8 @@ import torch
 
 from hyperspot import ops
 from hyperspot.models import build_model
-from hyperspot.models.llama import ForwardMeta, prefill_tiles
+from hyperspot.models.llama import (ABSORB_TOKENS, SPAN_TOKENS, ForwardMeta,
+                                    LatentSpan, prefill_tiles)
 
 from .config import EngineConfig
 from .kv_cache import (BlockManager, allocate_caches,
@@ -189,9 +190,13 @@ class ModelRunner:
             logits_indices=torch.tensor(logit_rows, dtype=torch.long, device=d),
         )
         if self.spec.is_hybrid:
-            self._add_hybrid_meta(
-                meta, [bm.row_of[r.request_id] for r in batch.requests],
-                [b - a for a, b in zip(starts, starts[1:])])
+            rows = [bm.row_of[r.request_id] for r in batch.requests]
+            lens = [b - a for a, b in zip(starts, starts[1:])]
+            self._add_hybrid_meta(meta, rows, lens)
+            if d.type == "cuda":
+                meta.latent = {w: self._latent_span(
+                    w, rows, [r.chunk_start for r in batch.requests], lens)
+                    for w in self.spec.latent_windows}
         input_ids = torch.tensor(ids, dtype=torch.long, device=d)
         return input_ids, meta
 
@@ -206,6 +211,37 @@ class ModelRunner:
         meta.state_slots = dev[:n]
         meta.tile_start = dev[n:2 * n + 1]
         meta.tiles = dev[2 * n + 1:].view(-1, 2)
+
+    def _latent_span(self, window: int, rows: List[int], begin: List[int],
+                     lens: List[int]) -> LatentSpan:
+        """Work lists of latent attention (see LatentSpan) for portions that
+        begin at these positions."""
+        import numpy as np
+        bm = self.block_manager
+        slots, start, first, short, n, row0 = [], [], [], [], 0, 0
+        for row, b, m in zip(rows, begin, lens):
+            start.append(n)
+            first.append(max(0, b - window + 1))
+            if m <= ABSORB_TOKENS:
+                short += range(row0, row0 + m)
+            else:
+                p = np.arange(first[-1], b + m)
+                s = bm.tables_np[row, p // bm.block_size].astype(np.int64) \
+                    * bm.block_size + p % bm.block_size
+                pad = -len(p) % 8
+                slots += [s, np.full(pad, -1)] if pad else [s]
+                n += len(p) + pad
+            row0 += m
+        tiles = [[i, a] for i, m in enumerate(lens) if m > ABSORB_TOKENS
+                 for a in range(0, m, SPAN_TOKENS)]
+        flat = start + first + [x for t in tiles for x in t] + short
+        dev = torch.tensor(flat, dtype=torch.int32, device=self.device)
+        k, t = len(rows), 2 * len(tiles)
+        return LatentSpan(
+            torch.from_numpy(np.concatenate(slots) if slots
+                             else np.empty(0, np.int64)).to(self.device),
+            dev[:k], dev[k:2 * k], dev[2 * k:2 * k + t].view(-1, 2),
+            dev[2 * k + t:] if short else None)
 
     def _decode_inputs(self, batch: ScheduledBatch):
         """Vectorized decode-step prep: numpy state + pinned staging (the
@@ -356,6 +392,13 @@ class ModelRunner:
                 1, self.max_blocks_per_seq, dtype=torch.int32, device=d)
             meta.block_tables = io["block_tables"]
             meta.row_seq = torch.zeros(T, dtype=torch.int32, device=d)
+            # a whole prompt: its tokens are the kv rows, one to one
+            zero = torch.zeros(1, dtype=torch.int32, device=d)
+            tiles = torch.tensor(prefill_tiles([T], SPAN_TOKENS)[0],
+                                 dtype=torch.int32, device=d)
+            meta.latent = {w: LatentSpan(io["slot_mapping"], zero, zero,
+                                         tiles, None)
+                           for w in self.spec.latent_windows}
         # the graph reads every tensor of meta at each replay: keep them all
         io["meta"] = meta
         for _ in range(2):

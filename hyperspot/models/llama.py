@@ -15,7 +15,7 @@ Model set and serving contract per the reference's spec-only llm-gateway
 from __future__ import annotations
 
 from dataclasses import dataclass
-from typing import List, Optional
+from typing import Dict, List, NamedTuple, Optional
 
 import torch
 from torch import nn
@@ -26,6 +26,21 @@ from hyperspot.ops.torch_ref import rope_cos_sin
 from hyperspot.parallel import (QKVParallelLinear, RowParallelLinear,
                                 MergedColumnParallelLinear)
 from hyperspot.parallel.state import get_tp_size
+
+
+class LatentSpan(NamedTuple):
+    """Work lists of latent attention in a prefill step, for one window.
+
+    Portions of more than ABSORB_TOKENS tokens attend over keys and values
+    expanded from the latents of kv rows: the tokens that the portion sees,
+    sequence after sequence.  The rows of shorter portions (`rows`) attend
+    over the latents themselves, as decoded tokens do."""
+
+    slots: torch.Tensor       # [n] int64 cache slot of every kv row, -1: none
+    start: torch.Tensor       # [num_seqs] int32 first kv row, multiple of 8
+    first: torch.Tensor       # [num_seqs] int32 position of that row's token
+    tiles: torch.Tensor       # [num_tiles, 2] int32, SPAN_TOKENS tokens each
+    rows: Optional[torch.Tensor]     # [r] int32 rows of the step
 
 
 @dataclass
@@ -60,18 +75,22 @@ class ForwardMeta:
     # a sequence's tiles consecutive; tile_start [num_seqs+1] int32
     tiles: Optional[torch.Tensor] = None
     tile_start: Optional[torch.Tensor] = None
+    # by window, for designs with latent attention
+    latent: Optional[Dict[int, LatentSpan]] = None
     # debugging: a list that collects the residual stream after every layer
     residual_trail: Optional[list] = None
 
 
 TILE_TOKENS = 64
+SPAN_TOKENS = 128       # query tokens per tile of expanded latent attention
+ABSORB_TOKENS = 16
 
 
-def prefill_tiles(lens) -> tuple:
+def prefill_tiles(lens, size: int = TILE_TOKENS) -> tuple:
     """(tiles, tile_start) as nested lists for portions of these lengths."""
     tiles, start = [], [0]
     for i, n in enumerate(lens):
-        tiles += [[i, a] for a in range(0, n, TILE_TOKENS)]
+        tiles += [[i, a] for a in range(0, n, size)]
         start.append(len(tiles))
     return tiles, start
 

@@ -1,4 +1,5 @@
-"""Layer parts of the hybrid designs: norms, mixers, feed-forward.
+"""Layer parts of the hybrid designs: norms, mixers, feed-forwards, token
+inputs.
 
 A mixer takes the normed input, the step's metadata and its layer's cache and
 returns the branch output before the post-norm.  Its sizes and constants come
@@ -15,12 +16,15 @@ from __future__ import annotations
 import torch
 from torch import nn
 
-from hyperspot.engine.layer_spec import DiffAttention, GatedLinear, MatrixLSTM
-from hyperspot.ops import hybrid
+from hyperspot.engine.layer_spec import (DiffAttention, Experts, GatedLinear,
+                                         LatentAttention, Lightning,
+                                         MatrixLSTM)
+from hyperspot.ops import experts, hybrid, latent
 from hyperspot.parallel import (MergedColumnParallelLinear,
                                 RowParallelLinear)
 from hyperspot.parallel.layers import _init_weight
-from hyperspot.parallel.state import get_tp_rank, get_tp_size
+from hyperspot.parallel.state import (get_ep_size, get_tp_rank, get_tp_size,
+                                      tensor_model_parallel_all_reduce)
 
 
 def _param(t: torch.Tensor) -> nn.Parameter:
@@ -53,6 +57,14 @@ def _put(param: nn.Parameter, tp: int = 1, r: int = 0):
     return put
 
 
+def _shard(param: nn.Parameter, dim: int, slices: list, full_shape: tuple):
+    """Mark a parameter as sharded over `dim` for checkpoint save."""
+    if get_tp_size() > 1:
+        param._tp_shard_dim, param._tp_slices = dim, slices
+        param._tp_full_shape = full_shape
+    return param
+
+
 def _part(layer, i: int):
     return lambda full: layer.load_part(i, full)
 
@@ -77,6 +89,20 @@ class DynamicTanh(nn.Module):
         yield name + ".alpha", (), _put(self.alpha)
 
 
+class RmsScale(nn.Module):
+    """RMS norm with a float weight; `stored` is what a checkpoint's weight
+    is short of the factor (1 for weights stored around zero)."""
+
+    def __init__(self, width: int, stored: float = 0.0):
+        super().__init__()
+        self.w = _param(torch.ones(width))
+        self.stored = stored
+
+    def tensors(self, name: str):
+        yield name, tuple(self.w.shape), \
+            lambda t: self.w.data.copy_(t.float() + self.stored)
+
+
 class GatedGelu(nn.Module):
     """down(gelu_tanh(gate x) * up x)."""
 
@@ -94,6 +120,104 @@ class GatedGelu(nn.Module):
         yield p + "gate", (self.ff, self.width), _part(self.gate_up, 0)
         yield p + "up", (self.ff, self.width), _part(self.gate_up, 1)
         yield p + "down", (self.width, self.ff), self.down.load_full_weight
+
+
+class ExpertMixture(nn.Module):
+    """Gated-SiLU experts chosen per token, and an optional shared one.
+
+    Under tensor parallelism every expert's inner size is divided over the
+    ranks, so all ranks run all experts and the sum is one all-reduce."""
+
+    def __init__(self, spec: Experts, width: int, dtype, tag: int):
+        super().__init__()
+        if get_ep_size() > 1:
+            raise ValueError("this design's experts are divided over the "
+                             "tensor-parallel group; ep_size must be 1")
+        self.spec, self.width = spec, width
+        m, tp, r = spec, get_tp_size(), get_tp_rank()
+
+        def pair(count, ff, tag):
+            """([count, gate | up, width], [count, width, ff]) of this rank"""
+            assert ff % tp == 0, (ff, tp)
+            n = ff // tp
+            a = _init_weight(count * 2 * ff, width, dtype, tag) \
+                .view(count, 2, ff, width)[:, :, r * n:(r + 1) * n]
+            b = _init_weight(count * width, ff, dtype, tag + 1) \
+                .view(count, width, ff)[:, :, r * n:(r + 1) * n]
+            up = _param(a.reshape(count, 2 * n, width).contiguous())
+            down = _param(b.contiguous())
+            return (_shard(up, 1, [(r * n, n, 0), (ff + r * n, n, n)],
+                           (count, 2 * ff, width)),
+                    _shard(down, 2, [(r * n, n, 0)], (count, width, ff)))
+
+        self.up, self.down = pair(m.experts, m.ff, tag)
+        self.shared_up = self.shared_down = None
+        if m.shared is not None:
+            self.shared_up, self.shared_down = pair(1, m.shared, tag + 2)
+        # router rows, then the shared expert's gate: one product
+        self.router = _param(_init_weight(
+            m.experts + (m.shared is not None), width, dtype, tag + 4))
+
+    @property
+    def args(self) -> tuple:
+        return (self.router, self.up, self.down, self.shared_up,
+                self.shared_down, self.spec.top)
+
+    def add_normed(self, x, residual, norm: RmsScale, eps: float):
+        """residual += norm(mixture of x); the residual in x's type."""
+        if get_tp_size() == 1:
+            return experts.mixture_add_rms(x, *self.args, residual, norm.w,
+                                           eps)
+        y = tensor_model_parallel_all_reduce(
+            experts.mixture(x, *self.args))
+        return hybrid.add_rms(y, residual, norm.w, eps, x.dtype)
+
+    def tensors(self, p: str):
+        m, w = self.spec, self.width
+        tp, r = get_tp_size(), get_tp_rank()
+
+        def expert(p, up, down, ff):
+            n = ff // tp
+            yield p + "gate", (ff, w), \
+                lambda t: up[:n].copy_(t[r * n:(r + 1) * n])
+            yield p + "up", (ff, w), \
+                lambda t: up[n:].copy_(t[r * n:(r + 1) * n])
+            yield p + "down", (w, ff), \
+                lambda t: down.copy_(t[:, r * n:(r + 1) * n])
+
+        for i in range(m.experts):
+            yield from expert(f"{p}e{i}.", self.up.data[i],
+                              self.down.data[i], m.ff)
+        yield p + "router", (m.experts, w), self.router.data[:m.experts].copy_
+        if m.shared is not None:
+            yield from expert(p + "shared.", self.shared_up.data[0],
+                              self.shared_down.data[0], m.shared)
+            yield p + "shared.sg", (1, w), self.router.data[m.experts:].copy_
+
+
+class TokenSide(nn.Module):
+    """A token's own input to one layer: the residual gates the token's entry
+    of a table, the product is projected, normed and added."""
+
+    def __init__(self, width: int, dim: int, column: int, dtype, tag: int):
+        super().__init__()
+        self.width, self.dim, self.column = width, dim, column
+        whole = lambda i, o, t: MergedColumnParallelLinear(
+            i, [o], dtype, seed_tag=t, replicated=(0,))
+        self.gate = whole(width, dim, tag)
+        self.proj = whole(dim, width, tag + 1)
+        self.norm = RmsScale(width)
+
+    def add(self, x, residual, table, ids, eps: float):
+        """residual += this layer's input; the residual in x's type."""
+        g = hybrid.gelu_gate(self.gate(x), table, ids, self.column)
+        return hybrid.add_rms(self.proj(g), residual, self.norm.w, eps,
+                              x.dtype)
+
+    def tensors(self, p: str):
+        yield p + "gate", (self.dim, self.width), _part(self.gate, 0)
+        yield p + "proj", (self.width, self.dim), _part(self.proj, 0)
+        yield from self.norm.tensors(p + "norm")
 
 
 class WindowDiffAttention(nn.Module):
@@ -210,6 +334,98 @@ class MatrixMemoryLSTM(nn.Module):
             yield p + n + ".b", (m.heads,), _put(b, tp, r)
 
 
+class WindowLatentAttention(nn.Module):
+    def __init__(self, spec: LatentAttention, width: int, eps: float, dtype,
+                 tag: int):
+        super().__init__()
+        self.spec, self.width, self.eps = spec, width, eps
+        m, tp, r = spec, get_tp_size(), get_tp_rank()
+        self.owner = m.kv_from is None
+        q = m.heads * (m.dim + m.rot_dim)
+        # q | latent, rotated key part (kept whole)
+        self.proj = MergedColumnParallelLinear(
+            width, [q] + [m.kv_rank + m.rot_dim] * self.owner, dtype,
+            seed_tag=tag, replicated=(1,))
+        self.o_proj = RowParallelLinear(m.heads * m.vdim, width, dtype,
+                                        seed_tag=tag + 2)
+        # [rank, H * D]: rows of a head's key expansion are columns here, the
+        # layout both the expansion and its absorption into q read
+        d, e = m.heads * m.dim // tp, m.heads * m.vdim // tp
+        uk = _init_weight(m.heads * m.dim, m.kv_rank, dtype, tag + 3)
+        self.uk = _shard(
+            _param(uk[r * d:(r + 1) * d].t().contiguous()), 1,
+            [(r * d, d, 0)], (m.kv_rank, m.heads * m.dim))
+        self.uv = _rows(_param(
+            _init_weight(m.heads * m.vdim, m.kv_rank, dtype, tag + 4)
+            [r * e:(r + 1) * e].contiguous()), tp, r, m.heads * m.vdim)
+        self.kv_norm = RmsScale(m.kv_rank) if self.owner else None
+        i = torch.arange(0, m.rot_dim, 2, dtype=torch.float64)
+        self.register_buffer(
+            "freqs", m.rot_base ** (-i / m.rot_dim) if m.rot_dim else i,
+            persistent=False)
+
+    def forward(self, x, meta, cache) -> torch.Tensor:
+        m = self.spec
+        heads = m.heads // get_tp_size()
+        parts = self.proj.split(self.proj(x))
+        q, kv = parts if self.owner else (parts[0], None)
+        latent.rope_append(q, kv, self.kv_norm.w if self.owner else None,
+                           meta, self.freqs, cache, heads, self.eps)
+        o = latent.attention(q, cache, meta, self.uk, self.uv, heads,
+                             m.window, m.scale)
+        return self.o_proj(o)
+
+    def tensors(self, p: str):
+        m, w = self.spec, self.width
+        tp, r = get_tp_size(), get_tp_rank()
+        d = m.heads * m.dim // tp
+        yield p + "q", (m.heads * (m.dim + m.rot_dim), w), _part(self.proj, 0)
+        if self.owner:
+            yield p + "dkv", (m.kv_rank + m.rot_dim, w), _part(self.proj, 1)
+            yield from self.kv_norm.tensors(p + "dkv.norm")
+        yield p + "uk", (m.heads * m.dim, m.kv_rank), \
+            lambda t: self.uk.data.copy_(t[r * d:(r + 1) * d].t())
+        yield p + "uv", (m.heads * m.vdim, m.kv_rank), _put(self.uv, tp, r)
+        yield p + "o", (w, m.heads * m.vdim), self.o_proj.load_full_weight
+
+
+class LightningAttention(nn.Module):
+    def __init__(self, spec: Lightning, width: int, eps: float, dtype,
+                 tag: int):
+        super().__init__()
+        self.spec, self.width, self.eps = spec, width, eps
+        m, tp, r = spec, get_tp_size(), get_tp_rank()
+        d, e = m.heads * m.dim, m.heads * m.vdim
+        self.proj = MergedColumnParallelLinear(width, [d, d, e, e], dtype,
+                                               seed_tag=tag)
+        self.o_proj = RowParallelLinear(e, width, dtype, seed_tag=tag + 4)
+        self.norm = _rows(_param(torch.ones(e // tp)), tp, r, e)
+        h = m.heads // tp
+        self.register_buffer("decay", torch.tensor(
+            m.decay[r * h:(r + 1) * h], dtype=torch.float32),
+            persistent=False)
+
+    def forward(self, x, meta, state) -> torch.Tensor:
+        q, k, v, g = self.proj.split(self.proj(x))
+        o = hybrid.lightning_mix(q, k, v, self.decay, state, meta)
+        ss = None
+        if get_tp_size() > 1:          # the norm spans the heads of all ranks
+            ss = tensor_model_parallel_all_reduce(o.pow(2).sum(-1))
+        return self.o_proj(hybrid.rms_gate(o, g, self.norm, self.eps, ss,
+                                           self.spec.heads * self.spec.vdim))
+
+    def tensors(self, p: str):
+        m, w = self.spec, self.width
+        d, e = m.heads * m.dim, m.heads * m.vdim
+        for i, (n, rows) in enumerate((("q", d), ("k", d), ("v", e),
+                                       ("g", e))):
+            yield p + n, (rows, w), _part(self.proj, i)
+        yield p + "o", (w, e), self.o_proj.load_full_weight
+        yield p + "norm", (e,), _put(self.norm, get_tp_size(), get_tp_rank())
+
+
 MIXERS = {DiffAttention: WindowDiffAttention,
           GatedLinear: GatedLinearAttention,
-          MatrixLSTM: MatrixMemoryLSTM}
+          MatrixLSTM: MatrixMemoryLSTM,
+          LatentAttention: WindowLatentAttention,
+          Lightning: LightningAttention}

@@ -12,16 +12,18 @@ import torch
 
 from hyperspot.engine.config import ModelSpec, get_model_spec
 
-from . import sumosun
+from . import sumosun, tefezen
 
 # config.json "architecture" -> (configuration reader, model class)
 DESIGNS = {
     sumosun.ARCHITECTURE: (sumosun.spec_from_folder,
                            sumosun.SumosunForCausalLM),
+    tefezen.ARCHITECTURE: (tefezen.spec_from_folder,
+                           tefezen.TefezenForCausalLM),
 }
 
 # presets of the designs (random-init), by canonical id
-DESIGN_PRESETS = dict(sumosun.PRESETS)
+DESIGN_PRESETS = {**sumosun.PRESETS, **tefezen.PRESETS}
 
 
 def spec_from_folder(folder: str) -> ModelSpec:

@@ -56,7 +56,8 @@ def spec_from_config(cfg: dict, shapes: dict, name: str) -> HybridSpec:
         layers.append(LayerSpec(_mixer(entry["type"], entry["mixer"], rank),
                                 None if mlp is None else mlp["ff"]))
     return hybrid_spec(name, ARCHITECTURE, cfg["width"], cfg["vocab"],
-                       float(cfg["norm"]["eps"]), layers)
+                       float(cfg["norm"]["eps"]), layers,
+                       norm_params=2 * cfg["width"] + 1)
 
 
 def preset(name: str, width: int, vocab: int, ff: int, heads: int,
@@ -69,7 +70,7 @@ def preset(name: str, width: int, vocab: int, ff: int, heads: int,
     gla = GatedLinear(state_heads, dim, 2 * dim, tau=8.0, rank=24)
     layers = [LayerSpec(attn, ff), LayerSpec(lstm), LayerSpec(gla, ff)]
     return hybrid_spec(name, ARCHITECTURE, width, vocab, 1e-5,
-                       layers * periods)
+                       layers * periods, norm_params=2 * width + 1)
 
 
 PRESETS = {

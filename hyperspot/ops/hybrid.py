@@ -1,11 +1,11 @@
 """Ops of the hybrid designs (models.mixers), dispatched like the rest of the
-op layer: a GPU tensor runs the gfx950 kernels of csrc/dyt.hip,
-csrc/attn_window.hip, csrc/recurrent.hip and csrc/recurrent_chunk.hip, a CPU tensor the PyTorch
-references.
+op layer: a GPU tensor runs the gfx950 kernels of csrc/dyt.hip, csrc/rms.hip,
+csrc/attn_window.hip, csrc/recurrent.hip and csrc/recurrent_chunk.hip, a CPU
+tensor the PyTorch references.
 
-Norm parameters travel as tuples (w, b, alpha) of float tensors.  q, k, v, g
-are column views of one projection buffer [T, ...]; the kernels take its row
-stride.
+Dynamic-tanh parameters travel as tuples (w, b, alpha) of float tensors.
+q, k, v, g are column views of one projection buffer [T, ...]; the kernels
+take its row stride.
 """
 
 from __future__ import annotations
@@ -37,6 +37,68 @@ def add_dyt(h: torch.Tensor, residual: torch.Tensor, post, pre):
         return out
     residual += torch_ref.dyt(h, post)
     return torch_ref.dyt(residual, pre).to(h.dtype)
+
+
+def embed_scaled(table: torch.Tensor, ids: torch.Tensor, scale: float):
+    """(x, residual): the scaled embedding as float residual, and the same in
+    the table's element type.  For a float table both are one tensor."""
+    if not table.is_cuda:
+        res = table[ids].float() * scale
+        return res.to(table.dtype), res
+    T, W = ids.numel(), table.shape[1]
+    res = torch.empty(T, W, dtype=torch.float32, device=table.device)
+    x = res if table.dtype == torch.float32 \
+        else torch.empty(T, W, dtype=table.dtype, device=table.device)
+    _native().embed_scaled(x, res, table, ids, scale)
+    return x, res
+
+
+def rms_scale(x: torch.Tensor, w: torch.Tensor, eps: float, dtype):
+    """RMS norm of float rows with a float weight, as `dtype`."""
+    if not x.is_cuda:
+        return torch_ref.rms_scale(x, w, eps).to(dtype)
+    out = torch.empty(x.shape, dtype=dtype, device=x.device)
+    _native().rms_scale(out, x, w, eps)
+    return out
+
+
+def add_rms(h: torch.Tensor, residual: torch.Tensor, w: torch.Tensor,
+            eps: float, dtype) -> torch.Tensor:
+    """residual += rms(h) * w in place; returns the residual as `dtype` (the
+    residual itself for float)."""
+    if not h.is_cuda:
+        residual += torch_ref.rms_scale(h, w, eps)
+        return residual.to(dtype)
+    out = residual if dtype == torch.float32 \
+        else torch.empty(h.shape, dtype=dtype, device=h.device)
+    _native().add_rms(out, residual, h, w, eps)
+    return out
+
+
+def rms_gate(o: torch.Tensor, g: torch.Tensor, w: torch.Tensor, eps: float,
+             ss, total: int) -> torch.Tensor:
+    """rms(o) * w * sigmoid(g) over the whole row of o [T, N] float.  `ss`
+    [T] is the sum of squares of all `total` columns where o holds only some
+    of them (None: o holds all)."""
+    if not o.is_cuda:
+        s = o.pow(2).sum(-1) if ss is None else ss
+        y = o / (s / total + eps).sqrt()[:, None] * w
+        return (y * torch.sigmoid(g.float())).to(g.dtype)
+    y = torch.empty(o.shape, dtype=g.dtype, device=o.device)
+    _native().rms_gate(y, o, g, w, ss, total, eps)
+    return y
+
+
+def gelu_gate(z: torch.Tensor, table: torch.Tensor, ids: torch.Tensor,
+              column: int) -> torch.Tensor:
+    """gelu_tanh(z) * table[ids, column : column + n] for z [T, n]."""
+    if not z.is_cuda:
+        e = table[ids, column:column + z.shape[1]].float()
+        return (torch.nn.functional.gelu(z.float(), approximate="tanh")
+                * e).to(z.dtype)
+    out = torch.empty_like(z)
+    _native().gelu_gate(out, z, table, ids, column)
+    return out
 
 
 def gelu_mul(gate_up: torch.Tensor) -> torch.Tensor:
@@ -177,6 +239,33 @@ def mlstm_mix(q, k, v, g, raw, ib, fb, w, state, meta, cap: float,
                      meta.seq_start, meta.positions, meta.state_slots, qscale)
     n.recurrent_out(y, o, g, w, H, True, eps)
     return y
+
+
+def lightning_mix(q, k, v, decay, state, meta) -> torch.Tensor:
+    """Lightning attention of one layer before its norm, [T, H*E] float; SiLU
+    is applied to q, k and v on the way in."""
+    _, H, D, E = state.S.shape
+    T = q.shape[0]
+    decode = meta.mode == "decode"
+    if not q.is_cuda:
+        return torch_ref.lightning_scan(
+            q, k, v, decay, state, None if decode else meta.seq_start,
+            meta.state_slots, meta.positions).view(T, H * E)
+    n = _native()
+    o = torch.empty(T, H * E, dtype=torch.float32, device=q.device)
+    if decode:
+        n.lightning_step(o, state.S, q, k, v, decay, meta.positions,
+                         meta.state_slots)
+    elif n.chunk_fits(state.S, q, k, v, v, 0):
+        U = torch.empty(meta.tiles.shape[0], H, E, D, dtype=torch.float32,
+                        device=q.device)
+        n.lightning_chunk(o, U, state.S, q, k, v, decay, meta.seq_start,
+                          meta.positions, meta.state_slots, meta.tiles,
+                          meta.tile_start)
+    else:
+        n.lightning_scan(o, state.S, q, k, v, decay, meta.seq_start,
+                         meta.positions, meta.state_slots)
+    return o
 
 
 def gate_projection(h: torch.Tensor, w: torch.Tensor) -> torch.Tensor:

@@ -1,0 +1,94 @@
+"""Windowed latent attention: keys and values of all heads come from one row
+[latent | rotated key part] per token in the pages.
+
+A GPU tensor runs the gfx950 kernels of csrc/attn_latent.hip, a CPU tensor the
+PyTorch references.  Two ways to compute the same scores on the GPU:
+
+  absorbed   the key expansion is applied to the query, W_uk^T q, and the head
+             attends over the latents; the value expansion follows.  Decoded
+             tokens and short portions: every cached row is read once for all
+             heads.
+  expanded   keys and values of the rows a portion sees are expanded per head
+             first.  Longer portions: a third of the attention's work.
+"""
+
+from __future__ import annotations
+
+import torch
+
+from . import _native, torch_ref
+
+
+def rope_append(q, kv, w, meta, freqs, cache, heads: int, eps: float) -> None:
+    """Rotate the last part of each head of q in place; append the normed
+    latent (weight w) and rotated key part of kv, if the layer has its own."""
+    rank = 0 if kv is None else w.numel()
+    f = _native().latent_rope_append if q.is_cuda \
+        else torch_ref.latent_rope_append
+    f(q, kv, w, meta.positions, freqs, meta.slot_mapping, cache.kv, heads,
+      rank, eps)
+
+
+def attention(q, cache, meta, uk, uv, heads: int, window: int,
+              scale: float) -> torch.Tensor:
+    """[T, H*E] for q [T, H*(D+R)]; uk [rank, H*D], uv [H*E, rank]."""
+    row_seq = meta.row_seq if meta.mode == "prefill" else None
+    if not q.is_cuda:
+        return torch_ref.latent_attention(
+            q, cache.kv, meta.block_tables, meta.positions, row_seq, uk, uv,
+            heads, window, scale)
+    out = torch.empty(q.shape[0], uv.shape[0], dtype=q.dtype,
+                      device=q.device)
+    span = None
+    fits = _native().latent_fits(q, cache.kv, uk, uv, heads)
+    if meta.mode == "prefill" and fits:
+        span = meta.latent[window]
+        if span.tiles.shape[0]:
+            _expanded(out, q, cache, meta, span, uk, uv, heads, window, scale)
+        if span.rows is None:
+            return out
+    _absorbed(out, q, cache, meta, row_seq,
+              None if span is None else span.rows, uk, uv, heads, window,
+              scale, fits)
+    return out
+
+
+def _expanded(out, q, cache, meta, span, uk, uv, heads, window, scale):
+    n, rank = _native(), uk.shape[0]
+    lat = torch.empty(span.slots.numel(), cache.kv.shape[-1], dtype=q.dtype,
+                      device=q.device)
+    n.latent_gather(lat, cache.kv, span.slots)
+    c = lat[:, :rank]
+    n.latent_attn_prefill(
+        out, q, c @ uk, lat, uv @ c.t(), meta.positions, meta.seq_start,
+        span.start, span.first, span.tiles, heads, window, scale)
+
+
+def _absorbed(out, q, cache, meta, row_seq, rows, uk, uv, heads, window,
+              scale, fits):
+    n, rank = _native(), uk.shape[0]
+    R = q.shape[0] if rows is None else rows.numel()
+    empty = lambda *s, dtype=q.dtype: torch.empty(*s, dtype=dtype,
+                                                  device=q.device)
+    qa = empty(R, heads, rank)
+    n.latent_absorb(qa, q, uk, rows, heads)
+    o = empty(R, heads, rank)
+    if fits:
+        reach = min(window, meta.block_tables.shape[1] * cache.kv.shape[1])
+        split = absorbed_split(R * -(-heads // 32), reach)
+        partial = None if split == 1 else empty(
+            R * heads * split * (rank + 2), dtype=torch.float32)
+        n.latent_attn_decode(o, qa, q, cache.kv, meta.block_tables,
+                             meta.positions, rows, row_seq, partial, split,
+                             window, scale)
+    else:
+        n.latent_attn_general(o, qa, q, cache.kv, meta.block_tables,
+                              meta.positions, rows, row_seq, window, scale)
+    n.latent_values(out, o, uv, rows)
+
+
+def absorbed_split(groups: int, reach: int) -> int:
+    """How many workgroups share one row's window: two for every compute unit
+    where the batch alone gives fewer, each with at least 64 tokens.  Depends
+    on shapes only, so a captured graph keeps it."""
+    return max(1, min(16, 512 // groups, reach // 64))

@@ -355,3 +355,107 @@ def recurrent_out(o, g, w, gate: str, eps: float, dtype) -> torch.Tensor:
     gf = torch.sigmoid(gf) if gate == "sigmoid" \
         else torch.nn.functional.silu(gf)
     return (y.reshape(T, H * E) * gf).to(dtype)
+
+
+# ---------------------------------------------------------------------------
+# RMS-normed float residual, latent attention, lightning attention, experts
+# ---------------------------------------------------------------------------
+
+def rms_scale(x: torch.Tensor, w: torch.Tensor, eps: float) -> torch.Tensor:
+    """Computed and returned in float."""
+    x = x.float()
+    return x / (x.pow(2).mean(-1, keepdim=True) + eps).sqrt() * w
+
+
+def latent_rope_append(q, kv, w, positions, freqs, slot_mapping, cache,
+                       heads: int, rank: int, eps: float) -> None:
+    """Rotate the last part of each head of q [T, H*(D+R)] in place; append
+    the normed latent and the rotated key part of kv [T, rank + R]."""
+    T, R = q.shape[0], 2 * freqs.numel()
+    if R:
+        a = positions.double()[:, None] * freqs[None, :]
+        c, s = a.cos().float()[:, None, :], a.sin().float()[:, None, :]
+
+    def rotate(x):                                  # [T, n, R]
+        if not R:
+            return x
+        x = x.float()
+        u, v = x[..., 0::2], x[..., 1::2]
+        return torch.stack([u * c - v * s, v * c + u * s], -1).flatten(-2)
+
+    qh = q.unflatten(-1, (heads, -1))
+    D = qh.shape[-1] - R
+    qh[..., D:] = rotate(qh[..., D:]).to(q.dtype)
+    if kv is None:
+        return
+    row = torch.cat([rms_scale(kv[:, :rank], w, eps),
+                     rotate(kv[:, None, rank:])[:, 0]], -1).to(cache.dtype)
+    ok = slot_mapping >= 0
+    cache.view(-1, cache.shape[-1])[slot_mapping[ok]] = row[ok]
+
+
+def latent_attention(q, cache, block_tables, positions, row_seq, uk, uv,
+                     heads: int, window: int, scale: float) -> torch.Tensor:
+    """q [T, H*(D+R)] rotated; uk [rank, H*D], uv [H*E, rank]."""
+    T, BS, rank = q.shape[0], cache.shape[1], uk.shape[0]
+    D, E = uk.shape[1] // heads, uv.shape[0] // heads
+    qh = q.float().view(T, heads, -1)
+    # queries in latent coordinates: one row per head against the cache
+    qa = torch.cat([torch.einsum("thd,rhd->thr", qh[..., :D],
+                                 uk.float().view(rank, heads, D)),
+                    qh[..., D:]], -1)
+    o = torch.empty(T, heads, rank, device=q.device)
+    for t in range(T):
+        s = int(row_seq[t]) if row_seq is not None else t
+        p = int(positions[t])
+        idx = torch.arange(max(0, p - window + 1), p + 1, device=q.device)
+        rows = cache[block_tables[s][idx // BS].long(), idx % BS].float()
+        att = (qa[t] @ rows.t() * scale).softmax(-1)
+        o[t] = att @ rows[:, :rank]
+    out = torch.einsum("thr,her->the", o, uv.float().view(heads, E, rank))
+    return out.reshape(T, heads * E).to(q.dtype)
+
+
+def lightning_scan(q, k, v, decay, state, seq_start, slots,
+                   positions) -> torch.Tensor:
+    """o [T, H, E] float; SiLU is applied to q, k and v here; the state pool
+    is updated."""
+    _, H, D, E = state.S.shape
+    T = q.shape[0]
+    silu = torch.nn.functional.silu
+    qf, kf = (silu(x.float()).reshape(T, H, D) for x in (q, k))
+    vf = silu(v.float()).reshape(T, H, E)
+    o = torch.zeros(T, H, E, device=q.device)
+    for t0, t1, slot, fresh in _sequences(seq_start, slots, positions):
+        S = torch.zeros(H, D, E, device=q.device) if fresh \
+            else state.S[slot].clone()
+        for t in range(t0, t1):
+            S = S * decay[:, None, None] \
+                + kf[t][:, :, None] * vf[t][:, None, :]
+            o[t] = (S * qf[t][:, :, None]).sum(1)
+        if slot >= 0:
+            state.S[slot] = S
+    return o
+
+
+def mixture(x, router, up, down, shared_up, shared_down, top: int):
+    """[T, W] float: chosen experts weighted by the softmax over the chosen
+    logits, plus the shared expert under its sigmoid gate."""
+    E = up.shape[0]
+    z = x.float() @ router.float().t()
+    s, ids = z[:, :E].topk(top, dim=-1)
+    weight = s.softmax(-1)
+
+    def expert(h, up, down):
+        return (silu_mul(h @ up.t()) @ down.t()).float()
+
+    out = torch.zeros(x.shape, dtype=torch.float32, device=x.device)
+    for e in range(E):
+        t, j = (ids == e).nonzero(as_tuple=True)
+        if t.numel():
+            out.index_add_(0, t, weight[t, j][:, None]
+                           * expert(x[t], up[e], down[e]))
+    if shared_up is not None:
+        out += torch.sigmoid(z[:, E:]) * expert(x, shared_up[0],
+                                                shared_down[0])
+    return out
