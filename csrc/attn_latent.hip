@@ -1,0 +1,843 @@
+// Windowed latent attention over the paged cache (gfx950).
+//
+// A token keeps one row [c (rank) | k_r (rot)] for all heads, c normed and
+// k_r rotated:                      cache [NB, 16, rank + rot]
+// Head h has k = [W_uk[h] c | k_r], v = W_uv[h] c and
+//   score(i, j) = (q_i . k_j) * scale,  i - window < j <= i.
+//
+//   q   [T, H, D + rot]  (token stride qs), the last rot of a head rotated
+//   uk  [rank, H * D]    (W_uk transposed)    uv [H * E, rank]
+//
+// Absorbed: qa = W_uk^T q_unrotated per head (head_gemm), attention of
+// [qa | q_r] over the rows themselves giving sum_j p_j c_j, then W_uv
+// (head_gemm).  Expanded: k and v of the visible rows are formed per head
+// with plain products, v transposed, and attended like ordinary ones.
+//
+// Matrix-core kernels (bf16): sizes are multiples of 8, padded with zeros in
+// registers and LDS.  The attention weights enter as a bf16 high and low
+// part.  Scores are formed transposed, S^T = K Q^T, so that a lane holds one
+// query column.  The general kernels take any sizes, bf16 or float.
+#include <float.h>
+
+#include <algorithm>
+
+#include "common.h"
+
+#define PAGE 16
+
+typedef __attribute__((ext_vector_type(4))) short short4_t;
+
+namespace {
+
+constexpr float LOG2E = 1.4426950408889634f;
+
+DEV float exp2_fast(float x) { return __builtin_amdgcn_exp2f(x); }
+
+// ---- rotation of q, norm and rotation of a token's row, append -----------
+// One workgroup a token.  freqs holds base^(-2i/rot) in double: angles stay
+// exact to float rounding at any position.
+template <typename T, int V>
+__global__ __launch_bounds__(256) void latent_rope_append_kernel(
+    T* __restrict__ q, const T* __restrict__ kv, const float* __restrict__ w,
+    const long* __restrict__ positions, const double* __restrict__ freqs,
+    const long* __restrict__ slot_mapping, T* __restrict__ cache, int H,
+    int D, int rank, int rot, long qs, long ks, float eps) {
+  extern __shared__ float cs[];        // (cos, sin) of each pair
+  __shared__ float scratch[4];
+  const long row = blockIdx.x;
+  const int half = rot / 2;
+  for (int i = threadIdx.x; i < half; i += 256) {
+    // angle in turns, reduced to [-1/2, 1/2]
+    double a = (double)positions[row] * freqs[i] * 0.15915494309189535;
+    a -= rint(a);
+    float s, c;
+    if constexpr (sizeof(T) == 2) {
+      s = __builtin_amdgcn_sinf((float)a);       // argument in turns
+      c = __builtin_amdgcn_cosf((float)a);
+    } else {
+      sincosf((float)(a * 6.283185307179586), &s, &c);
+    }
+    cs[2 * i] = c;
+    cs[2 * i + 1] = s;
+  }
+  __syncthreads();
+  for (int u = threadIdx.x; u < H * half; u += 256) {
+    const int h = u / half, i = u % half;
+    T* p = q + row * qs + (long)h * (D + rot) + D + 2 * i;
+    const float x = Elem<T>::ld(p), y = Elem<T>::ld(p + 1);
+    Elem<T>::st(p, x * cs[2 * i] - y * cs[2 * i + 1]);
+    Elem<T>::st(p + 1, y * cs[2 * i] + x * cs[2 * i + 1]);
+  }
+  if (!kv) return;
+  const long slot = slot_mapping[row];
+  if (slot < 0) return;                // the whole workgroup
+  const T* src = kv + row * ks;
+  T* dst = cache + slot * (rank + rot);
+  float ss = 0.f;
+  for (int c = threadIdx.x * V; c < rank; c += 256 * V) {
+    float f[V];
+    load_vec<T, V>(src + c, f);
+    #pragma unroll
+    for (int i = 0; i < V; ++i) ss += f[i] * f[i];
+  }
+  ss = block_reduce_sum_256(ss, scratch);
+  const float rs = 1.f / sqrtf(ss / rank + eps);
+  for (int c = threadIdx.x * V; c < rank; c += 256 * V) {
+    float f[V], wv[V];
+    load_vec<T, V>(src + c, f);
+    load_vec<float, V>(w + c, wv);
+    #pragma unroll
+    for (int i = 0; i < V; ++i) f[i] *= rs * wv[i];
+    store_vec<T, V>(dst + c, f);
+  }
+  for (int i = threadIdx.x; i < half; i += 256) {
+    const float x = Elem<T>::ld(src + rank + 2 * i);
+    const float y = Elem<T>::ld(src + rank + 2 * i + 1);
+    Elem<T>::st(dst + rank + 2 * i, x * cs[2 * i] - y * cs[2 * i + 1]);
+    Elem<T>::st(dst + rank + 2 * i + 1, y * cs[2 * i] + x * cs[2 * i + 1]);
+  }
+}
+
+// rows of the cache by slot, in units of 8 elements; slot -1 gives zeros
+__global__ __launch_bounds__(256) void latent_gather_kernel(
+    uint4* __restrict__ out, const uint4* __restrict__ cache,
+    const long* __restrict__ slots, long total, int units) {
+  const long u = (long)blockIdx.x * 256 + threadIdx.x;
+  if (u >= total) return;
+  const long row = u / units;
+  const long slot = slots[row];
+  out[u] = slot < 0 ? uint4{0, 0, 0, 0} : cache[slot * units + u % units];
+}
+
+// ---- a small product per head ---------------------------------------------
+// out[r, h, n] = sum_k x[r, h, k] w[h, n, k] with strides; `rows_in` and
+// `rows_out` map r to rows of x and out (null: r itself)
+struct HeadGemm {
+  const int* rows_in;
+  const int* rows_out;
+  long R;
+  int N, K;
+  long xr, xh, wn, wh, outr, outh;
+};
+
+template <typename T>
+__global__ __launch_bounds__(256) void head_gemm_general_kernel(
+    T* __restrict__ out, const T* __restrict__ x, const T* __restrict__ w,
+    HeadGemm a) {
+  const long r = blockIdx.x;
+  const int h = blockIdx.y, lane = threadIdx.x & 63;
+  const T* xp = x + (a.rows_in ? a.rows_in[r] : r) * a.xr + h * a.xh;
+  T* op = out + (a.rows_out ? a.rows_out[r] : r) * a.outr + h * a.outh;
+  for (int n = threadIdx.x >> 6; n < a.N; n += 4) {
+    const T* wp = w + h * a.wh + n * a.wn;
+    float s = 0.f;
+    for (int k = lane; k < a.K; k += 64)
+      s += Elem<T>::ld(xp + k) * Elem<T>::ld(wp + k);
+    s = wave_reduce_sum(s);
+    if (lane == 0) Elem<T>::st(op + n, s);
+  }
+}
+
+// a wave has 16 n and CT tiles of 16 rows
+template <int CT>
+__global__ __launch_bounds__(256) void head_gemm_kernel(
+    bf16* __restrict__ out, const bf16* __restrict__ x,
+    const bf16* __restrict__ w, HeadGemm a) {
+  const int lane = threadIdx.x & 63, col = lane & 15, gr = lane >> 4;
+  const int n0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * 16;
+  const int h = blockIdx.z;
+  if (n0 >= a.N) return;
+  const bool wn = n0 + col < a.N;
+  const bf16* wp = w + h * a.wh + (long)(n0 + col) * a.wn + gr * 8;
+  const bf16* xp[CT];
+  bool live[CT];
+  #pragma unroll
+  for (int t = 0; t < CT; ++t) {
+    const long r = ((long)blockIdx.y * CT + t) * 16 + col;
+    live[t] = r < a.R;
+    xp[t] = x + (live[t] && a.rows_in ? a.rows_in[r] : r) * a.xr + h * a.xh +
+            gr * 8;
+  }
+  f32x4_t acc[CT];
+  #pragma unroll
+  for (int t = 0; t < CT; ++t) acc[t] = f32x4_t(0.f);
+  #pragma unroll 4
+  for (int k = 0; k < a.K; k += 32) {
+    const bool in = k + gr * 8 < a.K;
+    const short8_t wf = in && wn
+        ? *reinterpret_cast<const short8_t*>(wp + k) : short8_t{};
+    #pragma unroll
+    for (int t = 0; t < CT; ++t) {
+      const short8_t xf = in && live[t]
+          ? *reinterpret_cast<const short8_t*>(xp[t] + k) : short8_t{};
+      acc[t] = mfma16(wf, xf, acc[t]);
+    }
+  }
+  const int n = n0 + gr * 4;
+  if (n >= a.N) return;                 // N is a multiple of 8
+  #pragma unroll
+  for (int t = 0; t < CT; ++t) {
+    if (!live[t]) continue;
+    const long r = ((long)blockIdx.y * CT + t) * 16 + col;
+    *reinterpret_cast<uint2*>(
+        out + (a.rows_out ? a.rows_out[r] : r) * a.outr + h * a.outh + n) =
+        uint2{cvt_pk_bf16(acc[t][0], acc[t][1]),
+              cvt_pk_bf16(acc[t][2], acc[t][3])};
+  }
+}
+
+// ---- absorbed attention, any sizes ------------------------------------------
+constexpr int TILE = 256;      // tokens per softmax step
+constexpr int MAX_RPT = 8;     // latent columns a thread: rank <= 2048
+
+template <typename T>
+__global__ __launch_bounds__(256) void latent_attn_general_kernel(
+    T* __restrict__ out, const T* __restrict__ qa, const T* __restrict__ q,
+    const T* __restrict__ cache, const int* __restrict__ block_tables,
+    const long* __restrict__ positions, const int* __restrict__ rows,
+    const int* __restrict__ row_seq, int max_blocks, int H, int D, int rank,
+    int rot, int window, float scale, long qs) {
+  extern __shared__ float general_lds[];
+  const int width = rank + rot;
+  float* q_lds = general_lds;          // [width]
+  float* p_lds = q_lds + width;        // [TILE]
+  __shared__ float scratch[4];
+  const long r = blockIdx.x;
+  const int h = blockIdx.y, tid = threadIdx.x;
+  const long row = rows ? rows[r] : r;
+  const int* bt = block_tables +
+                  (long)(row_seq ? row_seq[row] : (int)row) * max_blocks;
+  const long pos = positions[row];
+  const long lo = pos - window + 1 > 0 ? pos - window + 1 : 0;
+  for (int i = tid; i < width; i += 256)
+    q_lds[i] = i < rank
+        ? Elem<T>::ld(qa + (r * H + h) * rank + i)
+        : Elem<T>::ld(q + row * qs + (long)h * (D + rot) + D + i - rank);
+  __syncthreads();
+  float acc[MAX_RPT] = {};
+  float m = -FLT_MAX, l = 0.f;
+  for (long base = lo; base <= pos; base += TILE) {
+    const int n = (int)min((long)TILE, pos - base + 1);
+    float s = -FLT_MAX;
+    if (tid < n) {
+      const long p = base + tid;
+      const T* kp = cache + ((long)bt[p / PAGE] * PAGE + p % PAGE) * width;
+      float d = 0.f;
+      for (int i = 0; i < width; ++i) d += q_lds[i] * Elem<T>::ld(kp + i);
+      s = d * scale;
+    }
+    const float mn = fmaxf(m, block_reduce_max_256(s, scratch));
+    const float p = tid < n ? Fn<T>::exp(s - mn) : 0.f;
+    const float alpha = m == -FLT_MAX ? 0.f : Fn<T>::exp(m - mn);
+    l = l * alpha + block_reduce_sum_256(p, scratch);
+    m = mn;
+    p_lds[tid] = p;
+    __syncthreads();
+    #pragma unroll
+    for (int i = 0; i < MAX_RPT; ++i) {
+      const int e = tid + 256 * i;
+      if (e < rank) {
+        float a = acc[i] * alpha;
+        for (int t = 0; t < n; ++t) {
+          const long pt = base + t;
+          a += p_lds[t] * Elem<T>::ld(
+              cache + ((long)bt[pt / PAGE] * PAGE + pt % PAGE) * width + e);
+        }
+        acc[i] = a;
+      }
+    }
+    __syncthreads();
+  }
+  #pragma unroll
+  for (int i = 0; i < MAX_RPT; ++i)
+    if (tid + 256 * i < rank)
+      Elem<T>::st(out + (r * H + h) * rank + tid + 256 * i, acc[i] / l);
+}
+
+// ---- absorbed attention, matrix cores ---------------------------------------
+// A workgroup has one row, HT tiles of 16 heads and every split-th tile of
+// KT tokens.  A tile is staged once in LDS (two buffers): the score product
+// reads it row by row, the value product reads its transpose with the
+// transposing LDS load.  In the score product wave w has tokens
+// (w & 1) * 16 and head tile w >> 1 (one head tile: half of the columns); in
+// the value product every wave has all heads and a quarter of the latent.
+constexpr int KT = 32;
+constexpr int SS = KT + 4;         // row of the score tile
+
+// four rows of one column: in every 16 lanes, lane i passes the address of
+// row i / 4, columns 4 (i % 4), and receives column i
+DEV short4_t lds_read_tr(const short* p) {
+  return __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+      (__attribute__((address_space(3))) short4_t*)p);
+}
+
+constexpr int decode_lds(int RP, int XP) {
+  return 2 * KT * (RP + XP + 8) * 2 + 2 * 16 * SS * 4;
+}
+
+template <int RP, int XP, int HT>
+__global__ __launch_bounds__(256, 2) void latent_attn_decode_kernel(
+    bf16* __restrict__ out, float* __restrict__ partial,
+    const bf16* __restrict__ qa, const bf16* __restrict__ q,
+    const bf16* __restrict__ cache, const int* __restrict__ block_tables,
+    const long* __restrict__ positions, const int* __restrict__ rows,
+    const int* __restrict__ row_seq, int max_blocks, int H, int D, int rank,
+    int rot, int window, float scale2, long qs) {
+  constexpr int LS = RP + XP + 8;            // row of a staged tile
+  constexpr int KC = (RP + XP) / 32;         // steps of the score product
+  constexpr int QC = HT == 2 ? KC : (KC + 1) / 2;
+  constexpr int ET = RP / 64;                // 16-column tiles of a wave
+  constexpr int UPR = (RP + XP) / 8;         // 16-byte units of a row
+  constexpr int LOADS = (KT * UPR + 255) / 256;
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  short* kv_lds = reinterpret_cast<short*>(smem);            // [2][KT][LS]
+  float* s_lds = reinterpret_cast<float*>(kv_lds + 2 * KT * LS);
+
+  const long r = blockIdx.x;
+  const int h0 = blockIdx.y * HT * 16;
+  const int split = gridDim.z, z = blockIdx.z;
+  const long row = rows ? rows[r] : r;
+  const int* bt = block_tables +
+                  (long)(row_seq ? row_seq[row] : (int)row) * max_blocks;
+  const int pos = (int)positions[row];
+  const int lo = max(0, pos - window + 1);
+  const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+  const int col = lane & 15, gr = lane >> 4;
+  const int tg = wid & 1, part = wid >> 1;
+
+  // this wave's query columns: steps [c0, c0 + QC) of head tile `part`
+  const int c0 = HT == 2 ? 0 : part * QC;
+  short8_t qf[QC];
+  {
+    const int h = h0 + (HT == 2 ? part * 16 : 0) + col;
+    #pragma unroll
+    for (int c = 0; c < QC; ++c) {
+      const int d = (c0 + c) * 32 + gr * 8;
+      qf[c] = short8_t{};
+      if (h < H) {
+        if (d < RP) {
+          if (d < rank)
+            qf[c] = *reinterpret_cast<const short8_t*>(
+                qa + (r * H + h) * rank + d);
+        } else if (d - RP < rot) {
+          qf[c] = *reinterpret_cast<const short8_t*>(
+              q + row * qs + (long)h * (D + rot) + D + d - RP);
+        }
+      }
+    }
+  }
+  f32x4_t acc[HT][ET];
+  #pragma unroll
+  for (int t = 0; t < HT; ++t)
+    #pragma unroll
+    for (int e = 0; e < ET; ++e) acc[t][e] = f32x4_t(0.f);
+  float m[HT], l[HT];
+  #pragma unroll
+  for (int t = 0; t < HT; ++t) { m[t] = -FLT_MAX; l[t] = 0.f; }
+
+  uint4 kr[LOADS];
+  auto fetch = [&](int p0) {
+    const long b0 = bt[p0 / PAGE];
+    const long b1 = p0 + PAGE <= pos ? bt[p0 / PAGE + 1] : b0;
+    #pragma unroll
+    for (int i = 0; i < LOADS; ++i) {
+      const int u = tid + 256 * i;
+      const int t = u / UPR, d = (u % UPR) * 8;
+      kr[i] = uint4{0, 0, 0, 0};
+      const bool in = d < RP ? d < rank : d - RP < rot;
+      if (t < KT && in && p0 + t <= pos)
+        kr[i] = *reinterpret_cast<const uint4*>(
+            cache + ((t < PAGE ? b0 : b1) * PAGE + t % PAGE) * (rank + rot) +
+            (d < RP ? d : d - RP + rank));
+    }
+  };
+
+  int p0 = (lo / KT + z) * KT, buf = 0;
+  if (p0 <= pos) fetch(p0);
+  for (; p0 <= pos; p0 += split * KT, buf ^= 1) {
+    short* tile = kv_lds + buf * KT * LS;
+    #pragma unroll
+    for (int i = 0; i < LOADS; ++i) {
+      const int u = tid + 256 * i;
+      if (u < KT * UPR)
+        *reinterpret_cast<uint4*>(tile + (u / UPR) * LS + (u % UPR) * 8) =
+            kr[i];
+    }
+    __syncthreads();
+    if (p0 + split * KT <= pos) fetch(p0 + split * KT);
+    {
+      f32x4_t sc = f32x4_t(0.f);
+      #pragma unroll
+      for (int c = 0; c < QC; ++c)
+        if (c0 + c < KC)
+          sc = mfma16(*reinterpret_cast<const short8_t*>(
+                          tile + (tg * 16 + col) * LS + (c0 + c) * 32 +
+                          gr * 8),
+                      qf[c], sc);
+      *reinterpret_cast<f32x4_t*>(
+          s_lds + (part * 16 + col) * SS + tg * 16 + gr * 4) = sc;
+    }
+    __syncthreads();
+    short8_t ph[HT], pl[HT];
+    #pragma unroll
+    for (int t = 0; t < HT; ++t) {
+      float p[8], mx = m[t];
+      const float* sp = s_lds + (t * 16 + col) * SS + gr * 8;
+      *reinterpret_cast<float4*>(p) = *reinterpret_cast<const float4*>(sp);
+      *reinterpret_cast<float4*>(p + 4) =
+          *reinterpret_cast<const float4*>(sp + 4);
+      if constexpr (HT == 1) {
+        #pragma unroll
+        for (int i = 0; i < 8; ++i) p[i] += sp[16 * SS + i];
+      }
+      #pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const int at = p0 + gr * 8 + i;
+        p[i] = at >= lo && at <= pos ? p[i] * scale2 : -FLT_MAX;
+        mx = fmaxf(mx, p[i]);
+      }
+      mx = fmaxf(mx, __shfl_xor(mx, 16));
+      mx = fmaxf(mx, __shfl_xor(mx, 32));
+      if (!__all(mx == m[t])) {
+        const float alpha = m[t] == -FLT_MAX ? 0.f : exp2_fast(m[t] - mx);
+        #pragma unroll
+        for (int e = 0; e < ET; ++e)
+          #pragma unroll
+          for (int i = 0; i < 4; ++i) acc[t][e][i] *= alpha;
+        l[t] *= alpha;
+        m[t] = mx;
+      }
+      const float base = m[t] == -FLT_MAX ? 0.f : m[t];
+      #pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        p[i] = exp2_fast(p[i] - base);
+        l[t] += p[i];
+      }
+      split_bf16x8(p, &ph[t], &pl[t]);
+    }
+    const short* vp = tile + (gr * 8 + (col >> 2)) * LS + wid * (RP / 4) +
+                      (col & 3) * 4;
+    #pragma unroll
+    for (int e = 0; e < ET; ++e) {
+      const short4_t a = lds_read_tr(vp + e * 16);
+      const short4_t b = lds_read_tr(vp + 4 * LS + e * 16);
+      const short8_t vf{a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+      #pragma unroll
+      for (int t = 0; t < HT; ++t) {
+        acc[t][e] = mfma16(vf, ph[t], acc[t][e]);
+        acc[t][e] = mfma16(vf, pl[t], acc[t][e]);
+      }
+    }
+  }
+  #pragma unroll
+  for (int t = 0; t < HT; ++t) {
+    l[t] += __shfl_xor(l[t], 16);
+    l[t] += __shfl_xor(l[t], 32);
+    const int h = h0 + t * 16 + col;
+    if (h >= H) continue;
+    const float f = split > 1 ? 1.f : 1.f / l[t];
+    const long at = split > 1
+        ? ((r * H + h) * split + z) * (rank + 4) : (r * H + h) * rank;
+    #pragma unroll
+    for (int e = 0; e < ET; ++e) {
+      const int d = wid * (RP / 4) + e * 16 + gr * 4;
+      if (d >= rank) continue;
+      if (split > 1)
+        *reinterpret_cast<f32x4_t*>(partial + at + d) = acc[t][e];
+      else
+        *reinterpret_cast<uint2*>(out + at + d) =
+            uint2{cvt_pk_bf16(acc[t][e][0] * f, acc[t][e][1] * f),
+                  cvt_pk_bf16(acc[t][e][2] * f, acc[t][e][3] * f)};
+    }
+    if (split > 1 && wid == 0 && gr == 0) {
+      partial[at + rank] = m[t];
+      partial[at + rank + 1] = l[t];
+    }
+  }
+}
+
+// a wave per (row, head): split <= 64 partial results combined
+__global__ __launch_bounds__(64) void latent_merge_kernel(
+    bf16* __restrict__ out, const float* __restrict__ partial, int split,
+    int H, int rank) {
+  const long rh = (long)blockIdx.x * H + blockIdx.y;
+  const int lane = threadIdx.x;
+  const float* src = partial + rh * split * (rank + 4);
+  float m = -FLT_MAX, l = 0.f;
+  if (lane < split) {
+    m = src[(long)lane * (rank + 4) + rank];
+    l = src[(long)lane * (rank + 4) + rank + 1];
+  }
+  const float mx = wave_reduce_max(m);
+  float w = m == -FLT_MAX ? 0.f : exp2_fast(m - mx);
+  w /= wave_reduce_sum(w * l);
+  for (int c = lane * 4; c < rank; c += 256) {
+    float o[4] = {};
+    #pragma unroll 4
+    for (int p = 0; p < split; ++p) {
+      const float wp = __shfl(w, p);
+      const float4 x = *reinterpret_cast<const float4*>(
+          src + (long)p * (rank + 4) + c);
+      o[0] += wp * x.x;
+      o[1] += wp * x.y;
+      o[2] += wp * x.z;
+      o[3] += wp * x.w;
+    }
+    *reinterpret_cast<uint2*>(out + rh * rank + c) =
+        uint2{cvt_pk_bf16(o[0], o[1]), cvt_pk_bf16(o[2], o[3])};
+  }
+}
+
+// ---- expanded attention, matrix cores ---------------------------------------
+// 128 query rows of one head a workgroup, 32 a wave; kv rows come in steps
+// of 64.  kn [n, H*D] unrotated keys, lat [n, rank + rot] with the rotated
+// part, vt [H*E, n] values transposed.  Row r of sequence s is the token at
+// position first[s] + r - start[s]; start is a multiple of 8.
+constexpr int KV = 64;
+constexpr int VS = KV + 8;
+constexpr int QT = 128;
+
+constexpr int prefill_lds(int DP, int EP) {
+  return (KV * (DP + 8) + EP * VS) * 2;
+}
+
+template <int DP, int EP>
+__global__ __launch_bounds__(256, EP <= 128 ? 2 : 1)
+void latent_attn_prefill_kernel(
+    bf16* __restrict__ out, const bf16* __restrict__ q,
+    const bf16* __restrict__ kn, const bf16* __restrict__ lat,
+    const bf16* __restrict__ vt, const long* __restrict__ positions,
+    const int* __restrict__ seq_start, const int* __restrict__ kv_start,
+    const int* __restrict__ kv_first, const int* __restrict__ tiles, int H,
+    int D, int E, int rank, int rot, long nkv, int window, float scale2,
+    long qs) {
+  constexpr int KS = DP + 8;                     // K row in LDS
+  constexpr int KC = DP / 16, ET = EP / 32;
+  constexpr int KLOADS = KV * DP / 8 / 256;      // 16-byte units a thread
+  constexpr int VLOADS = KV * EP / 8 / 256;
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  short* k_lds = reinterpret_cast<short*>(smem);
+  short* v_lds = k_lds + KV * KS;
+
+  const int s = tiles[2 * blockIdx.x];
+  const int t0 = seq_start[s] + tiles[2 * blockIdx.x + 1];
+  const int n = min(QT, seq_start[s + 1] - t0);
+  if (n <= 0) return;
+  const int h = blockIdx.y;
+  const long kv0r = kv_start[s];                 // first kv row
+  // positions relative to the first kv row's token
+  const int p0 = (int)positions[t0] - kv_first[s];
+  const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+  const int col = lane & 31, hf = lane >> 5;
+  const int row = wid * 32 + col;                // this lane's query row
+  const int qp = p0 + row;
+
+  short8_t qf[KC];
+  {
+    const bf16* qr = q + (long)(t0 + row) * qs + (long)h * (D + rot);
+    #pragma unroll
+    for (int c = 0; c < KC; ++c) {
+      const int d = c * 16 + hf * 8;
+      qf[c] = row < n && d < D + rot
+          ? *reinterpret_cast<const short8_t*>(qr + d) : short8_t{};
+    }
+  }
+  f32x16_t acc[ET];
+  #pragma unroll
+  for (int e = 0; e < ET; ++e) acc[e] = f32x16_t(0.f);
+  float m = -FLT_MAX, l = 0.f;
+
+  const int last = p0 + n - 1;
+  const int lo = max(0, p0 - window + 1);
+  // first and last position of this wave's rows, for skipping whole steps
+  const int w_first = p0 + wid * 32, w_last = min(w_first + 31, last);
+
+  uint4 kr[KLOADS], vr[VLOADS];
+  auto fetch = [&](int kv) {
+    #pragma unroll
+    for (int i = 0; i < KLOADS; ++i) {
+      const int u = tid + 256 * i;
+      const int p = kv + u / (DP / 8), d = (u % (DP / 8)) * 8;
+      kr[i] = uint4{0, 0, 0, 0};
+      if (p <= last && d < D + rot)
+        kr[i] = *reinterpret_cast<const uint4*>(
+            d < D ? kn + (kv0r + p) * ((long)H * D) + (long)h * D + d
+                  : lat + (kv0r + p) * (rank + rot) + rank + d - D);
+    }
+    #pragma unroll
+    for (int i = 0; i < VLOADS; ++i) {
+      const int u = tid + 256 * i;
+      const int e = u / 8, p = kv + (u % 8) * 8;
+      vr[i] = uint4{0, 0, 0, 0};
+      if (e < E && p <= last)
+        vr[i] = *reinterpret_cast<const uint4*>(
+            vt + ((long)h * E + e) * nkv + kv0r + p);
+    }
+  };
+  auto stage = [&]() {
+    #pragma unroll
+    for (int i = 0; i < KLOADS; ++i) {
+      const int u = tid + 256 * i;
+      *reinterpret_cast<uint4*>(k_lds + (u / (DP / 8)) * KS +
+                                (u % (DP / 8)) * 8) = kr[i];
+    }
+    #pragma unroll
+    for (int i = 0; i < VLOADS; ++i) {
+      const int u = tid + 256 * i;
+      *reinterpret_cast<uint4*>(v_lds + (u / 8) * VS + (u % 8) * 8) = vr[i];
+    }
+  };
+
+  // matrix row i of a 32-token block takes this token's key, so that the
+  // scores a lane holds are 8 consecutive tokens
+  const int krow = (col & 16) + ((col >> 2) & 1) * 8 + ((col >> 3) & 1) * 4 +
+                   (col & 3);
+  const int kv_first_step = lo / KV * KV;
+  fetch(kv_first_step);
+  for (int kv = kv_first_step; kv <= last; kv += KV) {
+    stage();
+    __syncthreads();
+    if (kv + KV <= last) fetch(kv + KV);
+    const bool any = kv <= w_last && kv + KV - 1 > w_first - window &&
+                     w_first <= last;
+    if (any) {
+      f32x16_t sc[2];
+      #pragma unroll
+      for (int b = 0; b < 2; ++b) {
+        sc[b] = f32x16_t(0.f);
+        #pragma unroll
+        for (int c = 0; c < KC; ++c)
+          sc[b] = mfma32(*reinterpret_cast<const short8_t*>(
+                             k_lds + (b * 32 + krow) * KS + c * 16 + hf * 8),
+                         qf[c], sc[b]);
+      }
+      // token of sc[b][r]: kv + b*32 + (r>>3)*16 + hf*8 + (r&7)
+      const bool full = kv + KV - 1 <= w_first && kv > w_last - window;
+      float mx = m;
+      #pragma unroll
+      for (int b = 0; b < 2; ++b)
+        #pragma unroll
+        for (int r = 0; r < 16; ++r) {
+          float x = sc[b][r] * scale2;
+          if (!full) {
+            const int p = kv + b * 32 + (r >> 3) * 16 + hf * 8 + (r & 7);
+            if (p > qp || p <= qp - window) x = -FLT_MAX;
+          }
+          sc[b][r] = x;
+          mx = fmaxf(mx, x);
+        }
+      mx = fmaxf(mx, __shfl_xor(mx, 32));
+      if (!__all(mx == m)) {
+        const float alpha = m == -FLT_MAX ? 0.f : exp2_fast(m - mx);
+        #pragma unroll
+        for (int e = 0; e < ET; ++e)
+          #pragma unroll
+          for (int r = 0; r < 16; ++r) acc[e][r] *= alpha;
+        l *= alpha;
+        m = mx;
+      }
+      // a column without a visible key yet has m = -FLT_MAX: with base 0 its
+      // masked scores weigh exp2(-FLT_MAX) = 0
+      const float base = m == -FLT_MAX ? 0.f : m;
+      short8_t ph[4], pl[4];
+      #pragma unroll
+      for (int b = 0; b < 2; ++b)
+        #pragma unroll
+        for (int c = 0; c < 2; ++c) {
+          float p[8];
+          #pragma unroll
+          for (int j = 0; j < 8; ++j) {
+            p[j] = exp2_fast(sc[b][c * 8 + j] - base);
+            l += p[j];
+          }
+          split_bf16x8(p, &ph[b * 2 + c], &pl[b * 2 + c]);
+        }
+      #pragma unroll
+      for (int e = 0; e < ET; ++e)
+        #pragma unroll
+        for (int c = 0; c < 4; ++c) {
+          const short8_t vf = *reinterpret_cast<const short8_t*>(
+              v_lds + (e * 32 + col) * VS + c * 16 + hf * 8);
+          acc[e] = mfma32(vf, ph[c], acc[e]);
+          acc[e] = mfma32(vf, pl[c], acc[e]);
+        }
+    }
+    __syncthreads();
+  }
+  l += __shfl_xor(l, 32);
+  if (row >= n) return;
+  const float inv = 1.f / l;
+  bf16* orow = out + ((long)(t0 + row) * H + h) * E;
+  #pragma unroll
+  for (int e = 0; e < ET; ++e)
+    #pragma unroll
+    for (int r = 0; r < 16; r += 4) {
+      const int c = e * 32 + 8 * (r >> 2) + 4 * hf;
+      if (c < E)
+        *reinterpret_cast<uint2*>(orow + c) = uint2{
+            cvt_pk_bf16(acc[e][r] * inv, acc[e][r + 1] * inv),
+            cvt_pk_bf16(acc[e][r + 2] * inv, acc[e][r + 3] * inv)};
+    }
+}
+
+template <typename K> void allow_lds(K kernel, int bytes) {
+  if (bytes > 65536)
+    HIP_CHECK(hipFuncSetAttribute(
+        reinterpret_cast<const void*>(kernel),
+        hipFuncAttributeMaxDynamicSharedMemorySize, bytes));
+}
+
+}  // namespace
+
+bool latent_sizes_fit(int D, int E, int rank, int rot) {
+  return D % 8 == 0 && E % 8 == 0 && rank % 8 == 0 && rot % 8 == 0 &&
+         D + rot <= 256 && E <= 256 && rank <= 512 && rot <= 64;
+}
+
+template <typename T>
+void launch_latent_rope_append(T* q, const T* kv, const float* w,
+                               const long* positions, const double* freqs,
+                               const long* slot_mapping, T* cache, long rows,
+                               int H, int D, int rank, int rot, long qs,
+                               long ks, float eps, hipStream_t stream) {
+  if (rows == 0 || (rot == 0 && !kv)) return;
+  const size_t lds = (rot + 2) * sizeof(float);
+  const bool vec = rank % 4 == 0 && rot % 4 == 0 && ks % 4 == 0 &&
+                   reinterpret_cast<uintptr_t>(kv) % (4 * sizeof(T)) == 0;
+  if (vec)
+    latent_rope_append_kernel<T, 4><<<(unsigned)rows, 256, lds, stream>>>(
+        q, kv, w, positions, freqs, slot_mapping, cache, H, D, rank, rot, qs,
+        ks, eps);
+  else
+    latent_rope_append_kernel<T, 1><<<(unsigned)rows, 256, lds, stream>>>(
+        q, kv, w, positions, freqs, slot_mapping, cache, H, D, rank, rot, qs,
+        ks, eps);
+}
+
+void launch_latent_gather(bf16* out, const bf16* cache, const long* slots,
+                          long rows, int width, hipStream_t stream) {
+  if (rows == 0) return;
+  const long total = rows * (width / 8);
+  latent_gather_kernel<<<(unsigned)((total + 255) / 256), 256, 0, stream>>>(
+      reinterpret_cast<uint4*>(out), reinterpret_cast<const uint4*>(cache),
+      slots, total, width / 8);
+}
+
+// `fast`: bf16, N and K multiples of 8, 16-byte aligned rows
+template <typename T>
+void launch_head_gemm(T* out, const T* x, const T* w, const int* rows_in,
+                      const int* rows_out, long R, int H, int N, int K,
+                      long xr, long xh, long wn, long wh, long outr,
+                      long outh, bool fast, hipStream_t stream) {
+  if (R == 0) return;
+  const HeadGemm a{rows_in, rows_out, R, N, K, xr, xh, wn, wh, outr, outh};
+  if constexpr (sizeof(T) == 2) {
+    if (fast) {
+      const unsigned nx = (unsigned)((N + 63) / 64);
+      #define RUN(CT)                                                       \
+        head_gemm_kernel<CT>                                                \
+            <<<dim3(nx, (unsigned)((R + 16 * CT - 1) / (16 * CT)),          \
+                    (unsigned)H), 256, 0, stream>>>(out, x, w, a)
+      if (R <= 16) RUN(1);
+      else if (R <= 32) RUN(2);
+      else RUN(4);
+      #undef RUN
+      return;
+    }
+  }
+  head_gemm_general_kernel<T>
+      <<<dim3((unsigned)R, (unsigned)H), 256, 0, stream>>>(out, x, w, a);
+}
+
+template <typename T>
+void launch_latent_attn_general(T* out, const T* qa, const T* q,
+                                const T* cache, const int* block_tables,
+                                const long* positions, const int* rows,
+                                const int* row_seq, long R, int max_blocks,
+                                int H, int D, int rank, int rot, int window,
+                                float scale, long qs, hipStream_t stream) {
+  if (R == 0) return;
+  if (rank > 256 * MAX_RPT || rot > 4096)
+    throw std::runtime_error("latent_attn_general: latent size");
+  latent_attn_general_kernel<T>
+      <<<dim3((unsigned)R, (unsigned)H), 256,
+         (rank + rot + TILE) * sizeof(float), stream>>>(
+          out, qa, q, cache, block_tables, positions, rows, row_seq,
+          max_blocks, H, D, rank, rot, window, scale, qs);
+}
+
+void launch_latent_attn_decode(bf16* out, float* partial, const bf16* qa,
+                               const bf16* q, const bf16* cache,
+                               const int* block_tables, const long* positions,
+                               const int* rows, const int* row_seq, long R,
+                               int max_blocks, int H, int D, int rank,
+                               int rot, int window, float scale, long qs,
+                               int split, hipStream_t stream) {
+  if (R == 0) return;
+  #define RUN(RP, XP, HT)                                                   \
+    {                                                                       \
+      allow_lds(&latent_attn_decode_kernel<RP, XP, HT>,                     \
+                decode_lds(RP, XP));                                        \
+      latent_attn_decode_kernel<RP, XP, HT>                                 \
+          <<<dim3((unsigned)R, (unsigned)((H + 16 * HT - 1) / (16 * HT)),   \
+                  (unsigned)split), 256, decode_lds(RP, XP), stream>>>(     \
+              out, partial, qa, q, cache, block_tables, positions, rows,    \
+              row_seq, max_blocks, H, D, rank, rot, window, scale * LOG2E,  \
+              qs);                                                          \
+    }
+  #define CASE(RP, XP)                                                      \
+    if (!done && rank <= RP && rot <= XP) {                                 \
+      if (H <= 16) RUN(RP, XP, 1) else RUN(RP, XP, 2)                       \
+      done = true;                                                          \
+    }
+  bool done = false;
+  CASE(64, 32) CASE(64, 64) CASE(128, 32) CASE(128, 64) CASE(256, 32)
+  CASE(256, 64) CASE(512, 32) CASE(512, 64)
+  #undef CASE
+  #undef RUN
+  if (!done) throw std::runtime_error("latent_attn_decode: latent size");
+  if (split > 1)
+    latent_merge_kernel<<<dim3((unsigned)R, (unsigned)H), 64, 0, stream>>>(
+        out, partial, split, H, rank);
+}
+
+void launch_latent_attn_prefill(bf16* out, const bf16* q, const bf16* kn,
+                                const bf16* lat, const bf16* vt,
+                                const long* positions, const int* seq_start,
+                                const int* kv_start, const int* kv_first,
+                                const int* tiles, int num_tiles, int H, int D,
+                                int E, int rank, int rot, long nkv,
+                                int window, float scale, long qs,
+                                hipStream_t stream) {
+  if (num_tiles == 0) return;
+  #define CASE(DP, EP)                                                      \
+    if (D + rot <= DP && E <= EP) {                                         \
+      allow_lds(&latent_attn_prefill_kernel<DP, EP>, prefill_lds(DP, EP));  \
+      latent_attn_prefill_kernel<DP, EP>                                    \
+          <<<dim3((unsigned)num_tiles, (unsigned)H), 256,                   \
+             prefill_lds(DP, EP), stream>>>(                                \
+              out, q, kn, lat, vt, positions, seq_start, kv_start,          \
+              kv_first, tiles, H, D, E, rank, rot, nkv, window,             \
+              scale * LOG2E, qs);                                           \
+      return;                                                               \
+    }
+  CASE(64, 64) CASE(96, 64) CASE(64, 128) CASE(96, 128) CASE(128, 128)
+  CASE(192, 128) CASE(256, 128) CASE(128, 256) CASE(192, 256) CASE(256, 256)
+  #undef CASE
+  throw std::runtime_error("latent_attn_prefill: head sizes");
+}
+
+#define INSTANTIATE(T)                                                      \
+  template void launch_latent_rope_append<T>(                               \
+      T*, const T*, const float*, const long*, const double*, const long*,  \
+      T*, long, int, int, int, int, long, long, float, hipStream_t);        \
+  template void launch_head_gemm<T>(                                        \
+      T*, const T*, const T*, const int*, const int*, long, int, int, int,  \
+      long, long, long, long, long, long, bool, hipStream_t);               \
+  template void launch_latent_attn_general<T>(                              \
+      T*, const T*, const T*, const T*, const int*, const long*,            \
+      const int*, const int*, long, int, int, int, int, int, int, float,    \
+      long, hipStream_t);
+INSTANTIATE(bf16)
+INSTANTIATE(float)
+#undef INSTANTIATE

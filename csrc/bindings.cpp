@@ -2,16 +2,11 @@
 //
 // Host-side glue only — every kernel lives in a .hip translation unit and
 // is reached through a plain launcher so this file needs no device code.
-#include <torch/extension.h>
-
-#include <c10/hip/HIPStream.h>
-#include <hip/hip_bf16.h>
+#include "bindings.h"
 
 #include <array>
-#include <stdexcept>
-#include <type_traits>
 
-using bf16 = __hip_bfloat16;
+#include "recurrent.h"
 
 void launch_rmsnorm(bf16*, const bf16*, const bf16*, float, long, int,
                     hipStream_t);
@@ -64,7 +59,7 @@ void launch_gla_chunk_gates(float*, const bf16*, const bf16*, const float*,
 void launch_mlstm_chunk_gates(float*, float*, const float*, const float*,
                               const float*, const int*, const int*, int, int,
                               float, hipStream_t);
-void launch_recurrent_chunk(bf16*, float*, float*, float*, float*, float*,
+void launch_recurrent_chunk(Kind, bf16*, float*, float*, float*, float*, float*, float*,
                             float*, const bf16*, const bf16*, const bf16*,
                             const bf16*, const float*, const float*,
                             const float*, const int*, const long*,
@@ -76,7 +71,7 @@ void launch_gla_decay(float*, const T*, const T*, const float*, long, int,
 void launch_mlstm_gates(float*, const float*, const float*, const float*,
                         long, int, float, hipStream_t);
 template <typename T>
-void launch_recurrent_scan(float*, float*, float*, float*, float*, const T*,
+void launch_recurrent_scan(Kind, float*, float*, float*, float*, float*, const T*,
                            const T*, const T*, const float*, const int*,
                            const long*, const int*, int, int, int, int, long,
                            float, hipStream_t);
@@ -84,7 +79,8 @@ template <typename T>
 void launch_recurrent_out(T*, const float*, const T*, const float*, bool,
                           long, int, int, long, float, hipStream_t);
 template <typename T>
-void launch_recurrent_step(T*, float*, float*, float*, const T*, const T*,
+void launch_recurrent_step(Kind, T*, float*, float*, float*, float*,
+                           const T*, const T*,
                            const T*, const T*, const T*, const T*,
                            const float*, const float*, const float*,
                            const float*, const long*, const int*, long, int,
@@ -113,16 +109,6 @@ void launch_inv_cdf_sample(long*, const float*, const float*, long, int,
                            hipStream_t);
 
 namespace {
-
-hipStream_t stream() {
-  return c10::hip::getCurrentHIPStream().stream();
-}
-
-void check(const torch::Tensor& t, torch::ScalarType dt, const char* name) {
-  TORCH_CHECK(t.is_cuda(), name, " must be on GPU");
-  TORCH_CHECK(t.is_contiguous(), name, " must be contiguous");
-  TORCH_CHECK(t.scalar_type() == dt, name, " has wrong dtype");
-}
 
 bf16* bf(torch::Tensor& t) { return reinterpret_cast<bf16*>(t.data_ptr()); }
 const bf16* cbf(const torch::Tensor& t) {
@@ -245,37 +231,6 @@ void silu_mul(torch::Tensor out, torch::Tensor x) {
 }
 
 // ---- bf16 | float kernels ------------------------------------------------
-
-template <typename T> T* ptr(const torch::Tensor& t) {
-  return reinterpret_cast<T*>(t.data_ptr());
-}
-
-// run f with a null pointer of the element type that t has
-template <typename F> void by_dtype(const torch::Tensor& t, F f) {
-  if (t.scalar_type() == torch::kBFloat16)
-    f((bf16*)nullptr);
-  else if (t.scalar_type() == torch::kFloat32)
-    f((float*)nullptr);
-  else
-    TORCH_CHECK(false, "element type must be bfloat16 or float32");
-}
-
-#define ELEM(tag) std::remove_pointer_t<decltype(tag)>
-
-// [T, n] view with unit column stride of one projection buffer
-void check_rows(const torch::Tensor& t, torch::ScalarType dt, long rows,
-                long cols, long stride, const char* name) {
-  TORCH_CHECK(t.is_cuda() && t.scalar_type() == dt && t.dim() == 2 &&
-                  t.size(0) == rows && t.size(1) == cols &&
-                  t.stride(1) == 1 && t.stride(0) == stride,
-              name, " must be a [", rows, ", ", cols,
-              "] view of the projection buffer");
-}
-
-void check_param(const torch::Tensor& t, long numel, const char* name) {
-  check(t, torch::kFloat32, name);
-  TORCH_CHECK(t.numel() == numel, name, " must have ", numel, " elements");
-}
 
 void check_dyt(const torch::Tensor& w, const torch::Tensor& b,
                const torch::Tensor& a, long width) {
@@ -461,15 +416,6 @@ WindowDims check_window_fast(const torch::Tensor& out, const torch::Tensor& q,
   return {H, G, MD / 2, E};
 }
 
-// tiles [num_tiles, 2] of portions listed by seq_start; one table row each
-void check_tiles(const torch::Tensor& tiles, const torch::Tensor& seq_start,
-                 long seqs) {
-  check(tiles, torch::kInt32, "tiles");
-  check(seq_start, torch::kInt32, "seq_start");
-  TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 2, "tiles");
-  TORCH_CHECK(seq_start.numel() == seqs + 1, "seq_start");
-}
-
 void window_attn_prefill(torch::Tensor out, torch::Tensor q,
                          torch::Tensor k_cache, torch::Tensor v_cache,
                          torch::Tensor block_tables, torch::Tensor positions,
@@ -556,10 +502,6 @@ StateDims check_state(const torch::Tensor& S,
   return {S.size(0), S.size(1), S.size(2), S.size(3)};
 }
 
-float* opt(const c10::optional<torch::Tensor>& t) {
-  return t.has_value() ? ptr<float>(*t) : nullptr;
-}
-
 void recurrent_scan(torch::Tensor o, torch::Tensor S,
                     c10::optional<torch::Tensor> n,
                     c10::optional<torch::Tensor> m,
@@ -587,7 +529,7 @@ void recurrent_scan(torch::Tensor o, torch::Tensor S,
   by_dtype(q, [&](auto tag) {
     using T = ELEM(tag);
     launch_recurrent_scan<T>(
-        ptr<float>(o), ptr<float>(S), opt(n), opt(m), opt(nm_new), ptr<T>(q),
+        n.has_value() ? MLSTM : GLA, ptr<float>(o), ptr<float>(S), opt(n), opt(m), opt(nm_new), ptr<T>(q),
         ptr<T>(k), ptr<T>(v), ptr<float>(gates), seq_start.data_ptr<int>(),
         positions.data_ptr<long>(), slots.data_ptr<int>(), (int)B, (int)d.H,
         (int)d.D, (int)d.E, st, (float)qscale, stream());
@@ -677,7 +619,7 @@ void recurrent_chunk(torch::Tensor y, torch::Tensor U,
     check_param(*info, nt * d.H * 2, "info");
   }
   launch_recurrent_chunk(
-      bf(y), ptr<float>(U), opt(nU), opt(m_in), ptr<float>(S), opt(n),
+      mlstm ? MLSTM : GLA, bf(y), nullptr, ptr<float>(U), opt(nU), opt(m_in), ptr<float>(S), opt(n),
       opt(m), cbf(q), cbf(k), cbf(v), cbf(g), ptr<float>(gates), opt(info),
       ptr<float>(w), seq_start.data_ptr<int>(), positions.data_ptr<long>(),
       slots.data_ptr<int>(), tiles.data_ptr<int>(),
@@ -737,7 +679,7 @@ void gla_step(torch::Tensor y, torch::Tensor S, torch::Tensor q,
   by_dtype(q, [&](auto tag) {
     using T = ELEM(tag);
     launch_recurrent_step<T>(
-        ptr<T>(y), ptr<float>(S), nullptr, nullptr, ptr<T>(q), ptr<T>(k),
+        GLA, ptr<T>(y), nullptr, ptr<float>(S), nullptr, nullptr, ptr<T>(q), ptr<T>(k),
         ptr<T>(v), ptr<T>(g), ptr<T>(a1h), ptr<T>(a2), ptr<float>(a2b),
         nullptr, nullptr, ptr<float>(w), positions.data_ptr<long>(),
         slots.data_ptr<int>(), rows, (int)d.H, (int)d.D, (int)d.E, (int)R,
@@ -761,13 +703,93 @@ void mlstm_step(torch::Tensor y, torch::Tensor S, torch::Tensor n,
   by_dtype(q, [&](auto tag) {
     using T = ELEM(tag);
     launch_recurrent_step<T>(
-        ptr<T>(y), ptr<float>(S), ptr<float>(n), ptr<float>(m), ptr<T>(q),
+        MLSTM, ptr<T>(y), nullptr, ptr<float>(S), ptr<float>(n), ptr<float>(m), ptr<T>(q),
         ptr<T>(k), ptr<T>(v), ptr<T>(g), nullptr, nullptr, ptr<float>(ib),
         ptr<float>(fb), ptr<float>(raw), ptr<float>(w),
         positions.data_ptr<long>(), slots.data_ptr<int>(), rows, (int)d.H,
         (int)d.D, (int)d.E, 0, q.stride(0), (float)qscale, (float)cap,
         (float)eps, stream());
   });
+}
+
+// q, k, v rows of one buffer, o [T, H * E] float, one decay per head
+StateDims check_lightning(const torch::Tensor& o, const torch::Tensor& S,
+                          const torch::Tensor& q, const torch::Tensor& k,
+                          const torch::Tensor& v, const torch::Tensor& decay,
+                          const torch::Tensor& positions,
+                          const torch::Tensor& slots) {
+  const auto d = check_state(S, c10::nullopt, c10::nullopt);
+  const auto dt = q.scalar_type();
+  const long rows = q.size(0), st = q.stride(0);
+  check_rows(q, dt, rows, d.H * d.D, st, "q");
+  check_rows(k, dt, rows, d.H * d.D, st, "k");
+  check_rows(v, dt, rows, d.H * d.E, st, "v");
+  check_param(o, rows * d.H * d.E, "o");
+  check_param(decay, d.H, "decay");
+  check(positions, torch::kInt64, "positions");
+  check(slots, torch::kInt32, "slots");
+  TORCH_CHECK(positions.numel() == rows, "lightning: rows");
+  return d;
+}
+
+void lightning_step(torch::Tensor o, torch::Tensor S, torch::Tensor q,
+                    torch::Tensor k, torch::Tensor v, torch::Tensor decay,
+                    torch::Tensor positions, torch::Tensor slots) {
+  const auto d = check_lightning(o, S, q, k, v, decay, positions, slots);
+  TORCH_CHECK(slots.numel() == q.size(0), "lightning_step: slots");
+  by_dtype(q, [&](auto tag) {
+    using T = ELEM(tag);
+    launch_recurrent_step<T>(
+        LIGHTNING, nullptr, ptr<float>(o), ptr<float>(S), nullptr, nullptr,
+        ptr<T>(q), ptr<T>(k), ptr<T>(v), nullptr, nullptr, nullptr,
+        ptr<float>(decay), nullptr, nullptr, nullptr,
+        positions.data_ptr<long>(), slots.data_ptr<int>(), q.size(0),
+        (int)d.H, (int)d.D, (int)d.E, 0, q.stride(0), 1.f, 0.f, 0.f,
+        stream());
+  });
+}
+
+void lightning_scan(torch::Tensor o, torch::Tensor S, torch::Tensor q,
+                    torch::Tensor k, torch::Tensor v, torch::Tensor decay,
+                    torch::Tensor seq_start, torch::Tensor positions,
+                    torch::Tensor slots) {
+  const auto d = check_lightning(o, S, q, k, v, decay, positions, slots);
+  const long B = slots.numel();
+  check(seq_start, torch::kInt32, "seq_start");
+  TORCH_CHECK(seq_start.numel() == B + 1 && B <= 65535,
+              "lightning_scan: sequences");
+  by_dtype(q, [&](auto tag) {
+    using T = ELEM(tag);
+    launch_recurrent_scan<T>(
+        LIGHTNING, ptr<float>(o), ptr<float>(S), nullptr, nullptr, nullptr,
+        ptr<T>(q), ptr<T>(k), ptr<T>(v), ptr<float>(decay),
+        seq_start.data_ptr<int>(), positions.data_ptr<long>(),
+        slots.data_ptr<int>(), (int)B, (int)d.H, (int)d.D, (int)d.E,
+        q.stride(0), 1.f, stream());
+  });
+}
+
+void lightning_chunk(torch::Tensor o, torch::Tensor U, torch::Tensor S,
+                     torch::Tensor q, torch::Tensor k, torch::Tensor v,
+                     torch::Tensor decay, torch::Tensor seq_start,
+                     torch::Tensor positions, torch::Tensor slots,
+                     torch::Tensor tiles, torch::Tensor tile_start) {
+  const auto d = check_lightning(o, S, q, k, v, decay, positions, slots);
+  const long B = slots.numel(), nt = tiles.size(0);
+  TORCH_CHECK(chunk_fits(S, q, k, v, v, 0), "lightning_chunk: sizes");
+  check(tile_start, torch::kInt32, "tile_start");
+  check_tiles(tiles, seq_start, B);
+  TORCH_CHECK(tile_start.numel() == B + 1 && B <= 65535,
+              "lightning_chunk: sequences");
+  check_param(U, nt * d.H * d.D * d.E, "U");
+  launch_recurrent_chunk(
+      LIGHTNING, nullptr, ptr<float>(o), ptr<float>(U), nullptr, nullptr,
+      ptr<float>(S), nullptr, nullptr, ptr<bf16>(q), ptr<bf16>(k),
+      ptr<bf16>(v), nullptr, ptr<float>(decay), nullptr, nullptr,
+      seq_start.data_ptr<int>(), positions.data_ptr<long>(),
+      slots.data_ptr<int>(), tiles.data_ptr<int>(),
+      tile_start.data_ptr<int>(), (int)nt, (int)B, (int)d.H, (int)d.D,
+      (int)d.E, q.stride(0), 1.f, 0.f, stream());
 }
 
 void greedy_sample(torch::Tensor out, torch::Tensor logits) {
@@ -917,6 +939,8 @@ void moe_gemm_fp8(torch::Tensor out, torch::Tensor xq, torch::Tensor xs,
                       stream());
 }
 
+void register_latent(pybind11::module_& m);    // bindings_latent.cpp
+
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.doc() = "HyperSpot-AMD gfx950 (CDNA4) kernels";
   m.def("rmsnorm", &rmsnorm);
@@ -950,6 +974,10 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("recurrent_out", &recurrent_out);
   m.def("gla_step", &gla_step);
   m.def("mlstm_step", &mlstm_step);
+  m.def("lightning_step", &lightning_step);
+  m.def("lightning_scan", &lightning_scan);
+  m.def("lightning_chunk", &lightning_chunk);
+  register_latent(m);
   m.def("greedy_sample", &greedy_sample);
   m.def("inv_cdf_sample", &inv_cdf_sample);
 }

@@ -52,7 +52,7 @@ def _includes():
 def _needs_build(src: Path, obj: Path) -> bool:
     if not obj.exists():
         return True
-    deps = [src, CSRC / "common.h", Path(__file__)]
+    deps = [src, Path(__file__)] + list(CSRC.glob("*.h"))
     return any(d.stat().st_mtime > obj.stat().st_mtime for d in deps)
 
 
@@ -78,9 +78,9 @@ def build(force: bool = False, verbose: bool = False) -> Path:
     kernels = sorted(CSRC.glob("*.hip"))
     incs = _includes()
     with cf.ThreadPoolExecutor(max_workers=8) as ex:
-        futs = [ex.submit(_compile, k, DEVICE, verbose) for k in kernels]
-        futs.append(ex.submit(_compile, CSRC / "bindings.cpp",
-                              TORCH_DEFS + incs, verbose))
+        futs = [ex.submit(_compile, b, TORCH_DEFS + incs, verbose)
+                for b in sorted(CSRC.glob("bindings*.cpp"))]
+        futs += [ex.submit(_compile, k, DEVICE, verbose) for k in kernels]
         objs = [f.result() for f in futs]
     lib_dir = ce.library_paths("cuda")[0]
     if SO_PATH.exists() and not force and \

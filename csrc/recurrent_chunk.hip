@@ -8,6 +8,8 @@
 //   o_t   = (q_t exp(b_t)) S_in + sum_{s<=t} [q_t exp(b_t - b_s) . k_s] v_s
 //   S_out = exp(b_C) S_in + sum_s (k_s exp(b_C - b_s)) v_s^T
 //
+// Lightning attention is the scalar case with b_t = (t + 1) log(decay).
+//
 // The matrix LSTM adds the input gate i_s to the exponents and keeps every
 // sum divided by exp(m_t), m_t = F_t + max(m_in, max_{s<=t}(i_s - F_s)).
 //
@@ -24,12 +26,12 @@
 #include <float.h>
 
 #include "common.h"
+#include "recurrent.h"
 
 namespace {
 
 constexpr int C = 64;               // tokens per tile
 constexpr int TS = C + 8;           // row of a token-minor LDS tile
-constexpr float DEN_EPS = 1e-6f;
 
 DEV int pad32(int x) { return (x + 31) & ~31; }
 
@@ -48,10 +50,24 @@ DEV Tile load_tile(const int* tiles, const int* seq_start, int i) {
   return t;
 }
 
+// log of a constant decay; a decay of zero becomes one that vanishes in float
+DEV float log_decay_of(float decay) { return logf(fmaxf(decay, 1e-38f)); }
+
+DEV short8_t silu8(const short8_t& v) {
+  union { unsigned u[4]; short8_t v; } r;
+  #pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const float a = bf16x8_at(v, 2 * i), b = bf16x8_at(v, 2 * i + 1);
+    r.u[i] = cvt_pk_bf16(a / (1.f + __expf(-a)), b / (1.f + __expf(-b)));
+  }
+  return r.v;
+}
+
 // Rows [t0, t0+n) of src (column offset included, row stride `stride`) into
 // dst[column][token], columns padded to `cols_pad` and tokens to C with zeros.
-// f(token, column, 8 values in place) transforms each 8-column chunk.
-template <typename F>
+// ACT applies SiLU; f(token, column, 8 values in place) then transforms each
+// 8-column chunk.
+template <bool ACT, typename F>
 DEV void stage_transposed(short* dst, short* dst_lo, const bf16* src,
                           long stride, int n, int cols, int cols_pad, F f) {
   const int units = 32 * (cols_pad / 8);
@@ -65,6 +81,7 @@ DEV void stage_transposed(short* dst, short* dst_lo, const bf16* src,
       lo[k] = short8_t{};
       if (s < n && c < cols) {
         hi[k] = *reinterpret_cast<const short8_t*>(src + s * stride + c);
+        if constexpr (ACT) hi[k] = silu8(hi[k]);
         if (dst_lo) {
           float x[8];
           #pragma unroll
@@ -158,7 +175,7 @@ __global__ __launch_bounds__(64) void mlstm_chunk_gates_kernel(
 
 // ---- a tile's own state contribution --------------------------------------
 // U[tile, h, e, d] (transposed state) and, for the matrix LSTM, nU[tile, h, d]
-template <bool MLSTM>
+template <Kind K>
 __global__ __launch_bounds__(256) void chunk_state_kernel(
     float* __restrict__ U, float* __restrict__ nU, const bf16* __restrict__ k,
     const bf16* __restrict__ v, const float* __restrict__ gates,
@@ -177,12 +194,17 @@ __global__ __launch_bounds__(256) void chunk_state_kernel(
   const float* bh = gates + ((long)t.t0 * H + h) * D;     // GLA: [s][H*D]
   const float* gh = gates + (long)t.t0 * 2 * H + h;       // mLSTM: i, F
   float fc = 0.f, mu = 0.f;
-  if constexpr (MLSTM) { fc = info[2 * th]; mu = info[2 * th + 1]; }
-  stage_transposed(
+  if constexpr (K == MLSTM) { fc = info[2 * th]; mu = info[2 * th + 1]; }
+  if constexpr (K == LIGHTNING) fc = log_decay_of(gates[h]);
+  stage_transposed<K == LIGHTNING>(
       kt, kt_lo, k + (long)t.t0 * stride + (long)h * D, stride, t.n, D, DP,
       [&](int s, int c, float* x) {
-        if constexpr (MLSTM) {
+        if constexpr (K == MLSTM) {
           const float w = __expf(fc - gh[s * 2 * H + H] + gh[s * 2 * H] - mu);
+          #pragma unroll
+          for (int i = 0; i < 8; ++i) x[i] *= w;
+        } else if constexpr (K == LIGHTNING) {
+          const float w = __expf(fc * (t.n - 1 - s));
           #pragma unroll
           for (int i = 0; i < 8; ++i) x[i] *= w;
         } else {
@@ -192,11 +214,11 @@ __global__ __launch_bounds__(256) void chunk_state_kernel(
           for (int i = 0; i < 8; ++i) x[i] *= __expf(bc[i] - bs[i]);
         }
       });
-  stage_transposed(vt, nullptr, v + (long)t.t0 * stride + (long)h * E, stride,
+  stage_transposed<K == LIGHTNING>(vt, nullptr, v + (long)t.t0 * stride + (long)h * E, stride,
                    t.n, E, EP, [](int, int, float*) {});
   __syncthreads();
 
-  if constexpr (MLSTM) {
+  if constexpr (K == MLSTM) {
     for (int d = threadIdx.x; d < D; d += 256) {
       float s = 0.f;
       for (int i = 0; i < C; i += 8) {
@@ -238,7 +260,7 @@ __global__ __launch_bounds__(256) void chunk_state_kernel(
 // U[tile] becomes the state the tile starts from; the state after the last
 // tile goes to the pool.  A thread owns four neighbouring d of one e; the
 // matrix LSTM's extra block (blockIdx.x == gridDim.x - 1) carries n and m_in.
-template <bool MLSTM>
+template <Kind K>
 __global__ __launch_bounds__(256) void chunk_scan_kernel(
     float* __restrict__ U, float* __restrict__ nU, float* __restrict__ m_in,
     float* __restrict__ S, float* __restrict__ n_pool,
@@ -254,7 +276,7 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(
   if (t1 <= t0 || c1 <= c0) return;
   const int slot = slots[s];
   const bool fresh = slot < 0 || positions[t0] == 0;
-  const bool nblock = MLSTM && blockIdx.x == gridDim.x - 1;
+  const bool nblock = K == MLSTM && blockIdx.x == gridDim.x - 1;
   const int u = (nblock ? 0 : blockIdx.x * 1024) + threadIdx.x * 4;
   const int size = nblock ? D : D * E;
   if (u >= size) return;
@@ -270,7 +292,7 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(
   #pragma unroll
   for (int i = 0; i < 4; ++i) st[i] = fresh ? 0.f : pool[i * pstep];
   float m = 0.f;
-  if (MLSTM && !fresh) m = m_pool[(long)slot * H + h];
+  if (K == MLSTM && !fresh) m = m_pool[(long)slot * H + h];
 
   constexpr int AHEAD = 4;
   for (int c = c0; c < c1; c += AHEAD) {
@@ -279,10 +301,13 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(
     for (int j = 0; j < AHEAD; ++j) {
       if (c + j >= c1) break;
       x[j] = *reinterpret_cast<float4*>(p + j * step);
-      if constexpr (MLSTM) {
+      if constexpr (K == MLSTM) {
         const float* f = info + ((long)(c + j) * H + h) * 2;
         a[j].x = f[0];
         a[j].y = f[1];
+      } else if constexpr (K == LIGHTNING) {
+        const int n = min(t1 - t0 - (c + j - c0) * C, C);
+        a[j].x = log_decay_of(gates[h]) * n;
       } else {
         // the last token of the tile carries the tile's whole decay
         const int row = min(t0 + (c + j - c0 + 1) * C, t1) - 1;
@@ -295,7 +320,7 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(
       if (c + j >= c1) break;
       *reinterpret_cast<float4*>(p + j * step) =
           make_float4(st[0], st[1], st[2], st[3]);
-      if constexpr (MLSTM) {
+      if constexpr (K == MLSTM) {
         if (nblock && threadIdx.x == 0) m_in[(long)(c + j) * H + h] = m;
         const float mn = fmaxf(a[j].x + m, a[j].y);
         const float fs = expf(a[j].x + m - mn), us = expf(a[j].y - mn);
@@ -304,6 +329,12 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(
         st[1] = st[1] * fs + x[j].y * us;
         st[2] = st[2] * fs + x[j].z * us;
         st[3] = st[3] * fs + x[j].w * us;
+      } else if constexpr (K == LIGHTNING) {
+        const float f = expf(a[j].x);
+        st[0] = st[0] * f + x[j].x;
+        st[1] = st[1] * f + x[j].y;
+        st[2] = st[2] * f + x[j].z;
+        st[3] = st[3] * f + x[j].w;
       } else {
         st[0] = st[0] * expf(a[j].x) + x[j].x;
         st[1] = st[1] * expf(a[j].y) + x[j].y;
@@ -320,10 +351,10 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(
 
 // ---- outputs ----------------------------------------------------------------
 // ET: 32-column blocks of the value size per wave (E <= 128 * ET)
-template <int ET, bool MLSTM>
+template <int ET, Kind K>
 __global__ __launch_bounds__(256) void chunk_out_kernel(
-    bf16* __restrict__ y, const float* __restrict__ S,
-    const float* __restrict__ n_in, const float* __restrict__ m_in,
+    bf16* __restrict__ y, float* __restrict__ o_raw,
+    const float* __restrict__ S, const float* __restrict__ n_in, const float* __restrict__ m_in,
     float* __restrict__ m_pool, const bf16* __restrict__ q,
     const bf16* __restrict__ k, const bf16* __restrict__ v,
     const bf16* __restrict__ g, const float* __restrict__ gates,
@@ -359,10 +390,11 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(
       const long at = (long)(t.t0 + s) * stride + (long)h * D + c;
       a = *reinterpret_cast<const short8_t*>(q + at);
       b = *reinterpret_cast<const short8_t*>(k + at);
+      if constexpr (K == LIGHTNING) { a = silu8(a); b = silu8(b); }
     }
     *reinterpret_cast<short8_t*>(q_lds + s * DS + c) = a;
     *reinterpret_cast<short8_t*>(k_lds + s * DS + c) = b;
-    if constexpr (!MLSTM) {
+    if constexpr (K == GLA) {
       // rows past the end repeat the last one: every exponent stays finite
       const float* src = gates +
           ((long)(t.t0 + min(s, t.n - 1)) * H + h) * D + c;
@@ -375,10 +407,11 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(
       *reinterpret_cast<float4*>(b_lds + s * BS + c + 4) = z;
     }
   }
-  stage_transposed(vt, nullptr, v + (long)t.t0 * stride + (long)h * E, stride,
+  stage_transposed<K == LIGHTNING>(vt, nullptr, v + (long)t.t0 * stride + (long)h * E, stride,
                    t.n, E, EP, [](int, int, float*) {});
-  float mi = 0.f;
-  if constexpr (MLSTM) {
+  float mi = 0.f, ld = 0.f;
+  if constexpr (K == LIGHTNING) ld = log_decay_of(gates[h]);
+  if constexpr (K == MLSTM) {
     mi = m_in[th];
     if (wid == 0) {
       const int s = min(lane, t.n - 1);
@@ -408,7 +441,7 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(
     for (int J = 0; J < 4; ++J) {
       const int s = J * 16 + cl;
       float a[4] = {0.f, 0.f, 0.f, 0.f};
-      if (J < wid || (MLSTM && J == wid)) {
+      if (J < wid || (K != GLA && J == wid)) {
         f32x4_t acc = f32x4_t(0.f);
         for (int c = 0; c < DP; c += 32) {
           const int d = c + gr * 8;
@@ -416,7 +449,7 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(
               q_lds + (wid * 16 + cl) * DS + d);
           const short8_t kv = *reinterpret_cast<short8_t*>(
               k_lds + s * DS + d);
-          if constexpr (MLSTM) {
+          if constexpr (K != GLA) {
             acc = mfma16(qv, kv, acc);
           } else {
             const float* bq = b_lds + (wid * 16 + cl) * BS + d;
@@ -464,7 +497,8 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(
         float x = 0.f;
         if (s <= row) {
           x = a[r] * qscale;
-          if constexpr (MLSTM) {
+          if constexpr (K == LIGHTNING) x *= __expf(ld * (row - s));
+          if constexpr (K == MLSTM) {
             x *= __expf(tf[row] - tf[s] + ti[s] - tm[row]);
             den[r] += x;
           }
@@ -474,7 +508,7 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(
         a_lo[row * TS + s] = (short)f2bf(x - bf2f(hi));
       }
     }
-    if constexpr (MLSTM) {
+    if constexpr (K == MLSTM) {
       #pragma unroll
       for (int r = 0; r < 4; ++r) {
         float x = den[r];
@@ -485,7 +519,7 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(
     }
   }
   __syncthreads();
-  if constexpr (MLSTM) {
+  if constexpr (K == MLSTM) {
     // four threads a row finish the denominator with the incoming n
     const int row = tid >> 2, part = tid & 3;
     float x = 0.f;
@@ -515,7 +549,7 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(
     for (int tt = 0; tt < 2; ++tt) {
       const int row = tt * 32 + col;
       qh[tt] = *reinterpret_cast<short8_t*>(q_lds + row * DS + d);
-      if constexpr (!MLSTM) {
+      if constexpr (K == GLA) {
         float x[8];
         #pragma unroll
         for (int i = 0; i < 8; ++i)
@@ -540,7 +574,7 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(
       for (int tt = 0; tt < 2; ++tt) {
         acc[i][tt] = mfma32(sh, qh[tt], acc[i][tt]);
         acc[i][tt] = mfma32(sl, qh[tt], acc[i][tt]);
-        if constexpr (!MLSTM) acc[i][tt] = mfma32(sh, ql[tt], acc[i][tt]);
+        if constexpr (K == GLA) acc[i][tt] = mfma32(sh, ql[tt], acc[i][tt]);
       }
     }
   }
@@ -548,7 +582,8 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(
   for (int tt = 0; tt < 2; ++tt) {
     const int row = tt * 32 + col;
     float f = qscale;
-    if constexpr (MLSTM) f *= __expf(tf[row] + mi - tm[row]);
+    if constexpr (K == MLSTM) f *= __expf(tf[row] + mi - tm[row]);
+    if constexpr (K == LIGHTNING) f *= __expf(ld * (row + 1));
     #pragma unroll
     for (int i = 0; i < ET; ++i)
       #pragma unroll
@@ -567,17 +602,33 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(
         acc[i][tt] = mfma32(vf, al, acc[i][tt]);
       }
     }
+    if constexpr (K == LIGHTNING) {
+      if (row >= t.n) continue;
+      #pragma unroll
+      for (int i = 0; i < ET; ++i)
+        #pragma unroll
+        for (int r = 0; r < 16; r += 4) {
+          const int e = (wid + 4 * i) * 32 + 8 * (r >> 2) + 4 * hf;
+          if (e >= E) continue;
+          *reinterpret_cast<float4*>(
+              o_raw + ((long)(t.t0 + row) * H + h) * E + e) =
+              make_float4(acc[i][tt][r], acc[i][tt][r + 1],
+                          acc[i][tt][r + 2], acc[i][tt][r + 3]);
+        }
+      continue;
+    }
     float ss = 0.f;
     #pragma unroll
     for (int i = 0; i < ET; ++i)
       #pragma unroll
       for (int r = 0; r < 16; ++r) {
-        if constexpr (MLSTM) acc[i][tt][r] *= tinv[row];
+        if constexpr (K == MLSTM) acc[i][tt][r] *= tinv[row];
         ss += acc[i][tt][r] * acc[i][tt][r];    // columns past E are zero
       }
     ss += __shfl_xor(ss, 32);
     if (hf == 0) red[wid * C + row] = ss;
   }
+  if constexpr (K == LIGHTNING) return;
   __syncthreads();
   #pragma unroll
   for (int tt = 0; tt < 2; ++tt) {
@@ -595,7 +646,7 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(
         const int e = (wid + 4 * i) * 32 + 8 * (r >> 2) + 4 * hf;
         if (e >= E) continue;
         const float4 wv = *reinterpret_cast<const float4*>(
-            w + (MLSTM ? h * E : 0) + e);
+            w + (K == MLSTM ? h * E : 0) + e);
         float gv[4];
         load_vec<bf16, 4>(gr + e, gv);
         float o[4];
@@ -603,7 +654,7 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(
         for (int j = 0; j < 4; ++j) {
           const float sg = 1.f / (1.f + __expf(-gv[j]));
           o[j] = acc[i][tt][r + j] * rs * (&wv.x)[j] *
-                 (MLSTM ? sg : gv[j] * sg);
+                 (K == MLSTM ? sg : gv[j] * sg);
         }
         store_vec<bf16, 4>(yr + e, o);
       }
@@ -617,11 +668,11 @@ size_t state_lds(int D, int E) {
   return (size_t)(2 * dp + ep) * TS * 2;
 }
 
-size_t out_lds(int D, int E, bool mlstm) {
+size_t out_lds(int D, int E, bool gla) {
   const int dp = (D + 31) / 32 * 32, ep = (E + 31) / 32 * 32;
   size_t n = (size_t)(2 * C * (dp + 8) + (ep + 2 * C) * TS) * 2;
   n += (4 + 5) * C * 4;
-  if (!mlstm) n += (size_t)C * (dp + 4) * 4;
+  if (gla) n += (size_t)C * (dp + 4) * 4;
   return n;
 }
 
@@ -636,7 +687,7 @@ template <typename K> void allow_lds(K kernel, size_t bytes) {
 
 bool recurrent_chunk_fits(int D, int E, int rank) {
   return D % 8 == 0 && E % 8 == 0 && E <= 256 && rank <= 64 &&
-         state_lds(D, E) <= MAX_LDS && out_lds(D, E, false) <= MAX_LDS;
+         state_lds(D, E) <= MAX_LDS && out_lds(D, E, true) <= MAX_LDS;
 }
 
 void launch_gla_chunk_gates(float* b, const bf16* a1h, const bf16* a2,
@@ -669,9 +720,9 @@ void launch_mlstm_chunk_gates(float* gates, float* info, const float* raw,
                                        tiles, H, cap);
 }
 
-template <bool MLSTM>
-static void run_chunk(bf16* y, float* U, float* nU, float* m_in, float* S,
-                      float* n_pool, float* m_pool, const bf16* q,
+template <Kind K>
+static void run_chunk(bf16* y, float* o_raw, float* U, float* nU, float* m_in,
+                      float* S, float* n_pool, float* m_pool, const bf16* q,
                       const bf16* k, const bf16* v, const bf16* g,
                       const float* gates, const float* info, const float* w,
                       const int* seq_start, const long* positions,
@@ -680,33 +731,32 @@ static void run_chunk(bf16* y, float* U, float* nU, float* m_in, float* S,
                       int H, int D, int E, long stride, float qscale,
                       float eps, hipStream_t stream) {
   const dim3 grid((unsigned)num_tiles, (unsigned)H);
-  const size_t l1 = state_lds(D, E), l2 = out_lds(D, E, MLSTM);
-  allow_lds(&chunk_state_kernel<MLSTM>, l1);
-  chunk_state_kernel<MLSTM><<<grid, 256, l1, stream>>>(
+  const size_t l1 = state_lds(D, E), l2 = out_lds(D, E, K == GLA);
+  allow_lds(&chunk_state_kernel<K>, l1);
+  chunk_state_kernel<K><<<grid, 256, l1, stream>>>(
       U, nU, k, v, gates, info, seq_start, tiles, H, D, E, stride);
-  const dim3 sgrid((unsigned)((D * E + 1023) / 1024 + (MLSTM ? 1 : 0)),
+  const dim3 sgrid((unsigned)((D * E + 1023) / 1024 + (K == MLSTM ? 1 : 0)),
                    (unsigned)H, (unsigned)num_seqs);
-  chunk_scan_kernel<MLSTM><<<sgrid, 256, 0, stream>>>(
+  chunk_scan_kernel<K><<<sgrid, 256, 0, stream>>>(
       U, nU, m_in, S, n_pool, m_pool, gates, info, seq_start, positions,
       slots, tile_start, H, D, E);
+  #define OUT(ET)                                                           \
+    allow_lds(&chunk_out_kernel<ET, K>, l2);                                \
+    chunk_out_kernel<ET, K><<<grid, 256, l2, stream>>>(                     \
+        y, o_raw, U, nU, m_in, m_pool, q, k, v, g, gates, w, seq_start,     \
+        tiles, slots, H, D, E, stride, qscale, eps)
   if (E <= 128) {
-    allow_lds(&chunk_out_kernel<1, MLSTM>, l2);
-    chunk_out_kernel<1, MLSTM><<<grid, 256, l2, stream>>>(
-        y, U, nU, m_in, m_pool, q, k, v, g, gates, w, seq_start, tiles, slots,
-        H, D, E, stride, qscale, eps);
+    OUT(1);
   } else {
-    allow_lds(&chunk_out_kernel<2, MLSTM>, l2);
-    chunk_out_kernel<2, MLSTM><<<grid, 256, l2, stream>>>(
-        y, U, nU, m_in, m_pool, q, k, v, g, gates, w, seq_start, tiles, slots,
-        H, D, E, stride, qscale, eps);
+    OUT(2);
   }
+  #undef OUT
 }
 
-// n_pool == nullptr selects gated linear attention
-void launch_recurrent_chunk(bf16* y, float* U, float* nU, float* m_in,
-                            float* S, float* n_pool, float* m_pool,
-                            const bf16* q, const bf16* k, const bf16* v,
-                            const bf16* g, const float* gates,
+void launch_recurrent_chunk(Kind kind, bf16* y, float* o_raw, float* U,
+                            float* nU, float* m_in, float* S, float* n_pool,
+                            float* m_pool, const bf16* q, const bf16* k,
+                            const bf16* v, const bf16* g, const float* gates,
                             const float* info, const float* w,
                             const int* seq_start, const long* positions,
                             const int* slots, const int* tiles,
@@ -714,14 +764,12 @@ void launch_recurrent_chunk(bf16* y, float* U, float* nU, float* m_in,
                             int num_seqs, int H, int D, int E, long stride,
                             float qscale, float eps, hipStream_t stream) {
   if (num_tiles == 0 || num_seqs == 0) return;
-  if (n_pool)
-    run_chunk<true>(y, U, nU, m_in, S, n_pool, m_pool, q, k, v, g, gates,
-                    info, w, seq_start, positions, slots, tiles, tile_start,
-                    num_tiles, num_seqs, H, D, E, stride, qscale, eps,
-                    stream);
-  else
-    run_chunk<false>(y, U, nU, m_in, S, n_pool, m_pool, q, k, v, g, gates,
-                     info, w, seq_start, positions, slots, tiles, tile_start,
-                     num_tiles, num_seqs, H, D, E, stride, qscale, eps,
-                     stream);
+  #define RUN(K)                                                            \
+    if (kind == K)                                                          \
+      run_chunk<K>(y, o_raw, U, nU, m_in, S, n_pool, m_pool, q, k, v, g,    \
+                   gates, info, w, seq_start, positions, slots, tiles,      \
+                   tile_start, num_tiles, num_seqs, H, D, E, stride,        \
+                   qscale, eps, stream);
+  RUN(GLA) RUN(MLSTM) RUN(LIGHTNING)
+  #undef RUN
 }

@@ -93,7 +93,7 @@ def _tiles(n, x, up, down, ids):
     P, dev = tiles * MOE_BM, x.device
     i32 = lambda *s: torch.empty(*s, dtype=torch.int32, device=dev)
     order, expert, place = i32(P), i32(tiles), i32(T * top)
-    n.moe_align(order, expert, place, ids.view(-1), E)
+    n.experts_sort(order, expert, place, ids.view(-1), E, MOE_BM)
     h = torch.empty(P, F2, dtype=x.dtype, device=dev)
     s, ws = _moe_splitk(tiles * (F2 // 128), W // 64, P * F2, dev)
     n.moe_gemm(h, x, up, order, expert, top, s, ws)

@@ -77,7 +77,7 @@ def _absorbed(out, q, cache, meta, row_seq, rows, uk, uv, heads, window,
         reach = min(window, meta.block_tables.shape[1] * cache.kv.shape[1])
         split = absorbed_split(R * -(-heads // 32), reach)
         partial = None if split == 1 else empty(
-            R * heads * split * (rank + 2), dtype=torch.float32)
+            R * heads * split * (rank + 4), dtype=torch.float32)
         n.latent_attn_decode(o, qa, q, cache.kv, meta.block_tables,
                              meta.positions, rows, row_seq, partial, split,
                              window, scale)
