@@ -568,15 +568,31 @@ def engine_direct(args, rank, world, on_gpu):
     }
 
 
-# ------------------------------------------- hybrid design vs. plain decoder
+# --------------------------------------- hybrid design vs. the closest model
 
-def _compare_specs(width):
-    """The hybrid design and a plain decoder with equal width, feed-forwards,
-    vocabulary and number of feed-forward layers."""
+def _compare_specs(design, width):
+    """A hybrid design and the closest other model at equal size."""
     from hyperspot.engine.config import ModelSpec
+    heads, vocab = width // 128, 32768
+    if design == "tefezen":
+        # equal width, layers, attention heads, experts, choices per token
+        # and expert size; the design's shared expert and token inputs have
+        # no counterpart in the other model
+        from hyperspot.engine.layer_spec import Experts
+        from hyperspot.models.tefezen import preset
+        experts, ff = 65536 // width, width // 2
+        hybrid = preset(f"tefezen-w{width}", width=width, vocab=vocab,
+                        heads=heads, dim=128, rot_dim=64, kv_rank=512,
+                        window=1024, state_heads=heads, state_dim=128,
+                        experts=Experts(experts, 4, ff, ff), side_dim=128,
+                        periods=2)
+        plain = ModelSpec(f"mixtral-w{width}", width, 8, heads, heads // 4,
+                          128, ff, vocab, max_position=16384,
+                          num_experts=experts, num_experts_per_tok=4)
+        return hybrid, plain
+    # equal width, feed-forwards, vocabulary and number of feed-forwards
     from hyperspot.models.sumosun import preset
-    heads = width // 128
-    ff, vocab = width * 7 // 2, 32768
+    ff = width * 7 // 2
     hybrid = preset(f"sumosun-w{width}", width=width, vocab=vocab, ff=ff,
                     heads=heads, kv_heads=heads // 4, dim=64, window=1024,
                     periods=4, state_heads=heads // 2)
@@ -603,7 +619,7 @@ def compare_designs(args):
 
     for width in args.compare:
         engines = {}
-        for spec in _compare_specs(width):
+        for spec in _compare_specs(args.compare_design, width):
             if only and not spec.name.startswith(only):
                 continue
             C._PRESETS[spec.name] = spec
@@ -699,9 +715,13 @@ def main():
     ap.add_argument("--device", default=None)
     ap.add_argument("--compare", nargs="*", type=int, metavar="WIDTH",
                     default=None,
-                    help="instead: prefill and decode throughput of the "
-                         "Sumosun design beside a plain decoder of equal "
-                         "size, at these widths (default 2048 4096)")
+                    help="instead: prefill and decode throughput of a "
+                         "hybrid design beside the closest other model of "
+                         "equal size, at these widths (default 2048 4096)")
+    ap.add_argument("--compare-design", default="sumosun",
+                    choices=["sumosun", "tefezen"],
+                    help="with --compare: Sumosun beside a plain decoder, or "
+                         "Tefezen beside a Mixtral-like one")
     ap.add_argument("--compare-model", default=None, metavar="PREFIX",
                     help="with --compare: only models of this name prefix")
     ap.add_argument("--compare-reps", type=int, default=3)

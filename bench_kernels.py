@@ -1,7 +1,7 @@
 #!/usr/bin/env python3
 """Isolated kernel microbenchmarks (GPU only) — us/call + achieved GB/s.
 
-Usage: python bench_kernels.py [--which attn|gemm|fp8|hybrid|all] [--iters N]
+Usage: python bench_kernels.py [--which attn|gemm|fp8|hybrid|latent|all] [--iters N]
 
 Shapes mirror the flagship bench (Llama-3-8B bf16, bs=256 ctx=512 decode):
 the numbers here are the per-kernel budget lines behind bench.py's step
@@ -124,43 +124,64 @@ def bench_fp8_gemm(iters):
             "us_fp8_mm_only": round(us_fp8_mm, 1)}), flush=True)
 
 
+DEV = "cuda:0"
+
+
+def timed_graph(fn, iters, calls=10):
+    """us/call inside a replayed graph: no host time between the kernels."""
+    fn()
+    torch.cuda.synchronize()
+    g = torch.cuda.CUDAGraph()
+    with torch.cuda.graph(g):
+        for _ in range(calls):
+            fn()
+    return timed(g.replay, max(1, iters // calls), warmup=3) / calls
+
+
+def report_kernel(iters, name, shape, fn, nbytes, flops=0, timer=timed):
+    """Time against the larger of the HBM floor (8 TB/s) and the bf16 matrix
+    floor (2.5 PFLOP/s)."""
+    us = timer(fn, iters)
+    roof = max(nbytes / 8e12, flops / 2.5e15) * 1e6
+    print(json.dumps({"kernel": name, "shape": shape, "us": round(us, 1),
+                      "roofline_us": round(roof, 2),
+                      "x_roofline": round(us / roof, 2)}), flush=True)
+
+
+def meta_for(lens, mode="prefill", ctx=0):
+    """(metadata, pages) of portions of these lengths after ctx tokens."""
+    from hyperspot.models.llama import ForwardMeta, prefill_tiles
+    n = len(lens)
+    starts = [0]
+    for x in lens:
+        starts.append(starts[-1] + x)
+    i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=DEV)
+    pos = [ctx + p for x in lens for p in range(x)]
+    nblk = (max(lens) + ctx + 15) // 16
+    tiles, ts = prefill_tiles(lens)
+    bt = torch.randperm(n * nblk, device=DEV).int().view(n, nblk)
+    p = torch.tensor(pos, device=DEV)
+    seq = torch.tensor([i for i, x in enumerate(lens) for _ in range(x)],
+                       device=DEV)
+    slots = bt[seq, p // 16].long() * 16 + p % 16
+    return ForwardMeta(
+        mode=mode, positions=p, slot_mapping=slots, seq_start=i32(starts),
+        max_seqlen=max(lens), row_seq=seq.int(), ctx_lens=(p + 1).int(),
+        block_tables=bt, seq_lens=(p + 1).int(),
+        state_slots=i32(list(range(n))), tiles=i32(tiles),
+        tile_start=i32(ts)), n * nblk
+
+
 def bench_hybrid(iters):
     """Kernels of the hybrid design and the like kernels of the plain decoder
     at width 4096: time against the larger of the HBM floor (8 TB/s) and the
     bf16 matrix floor (2.5 PFLOP/s)."""
     import hyperspot.ops as ops
     from hyperspot.engine.kv_cache import KVPages, RecurrentState
-    from hyperspot.models.llama import ForwardMeta, prefill_tiles
     from hyperspot.ops import hybrid
     dev, bf = "cuda:0", torch.bfloat16
-
-    def report(name, shape, fn, nbytes, flops=0):
-        us = timed(fn, iters)
-        roof = max(nbytes / 8e12, flops / 2.5e15) * 1e6
-        print(json.dumps({"kernel": name, "shape": shape,
-                          "us": round(us, 1), "roofline_us": round(roof, 2),
-                          "x_roofline": round(us / roof, 2)}), flush=True)
-
-    def meta_for(lens, mode="prefill", ctx=0):
-        T, n = sum(lens), len(lens)
-        starts = [0]
-        for x in lens:
-            starts.append(starts[-1] + x)
-        i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=dev)
-        pos = [ctx + p for x in lens for p in range(x)]
-        nblk = (max(lens) + ctx + 15) // 16
-        tiles, ts = prefill_tiles(lens)
-        bt = torch.randperm(n * nblk, device=dev).int().view(n, nblk)
-        p = torch.tensor(pos, device=dev)
-        seq = torch.tensor([i for i, x in enumerate(lens)
-                            for _ in range(x)], device=dev)
-        slots = bt[seq, p // 16].long() * 16 + p % 16
-        return ForwardMeta(
-            mode=mode, positions=p, slot_mapping=slots,
-            seq_start=i32(starts), max_seqlen=max(lens),
-            row_seq=seq.int(), ctx_lens=(p + 1).int(), block_tables=bt,
-            seq_lens=(p + 1).int(), state_slots=i32(list(range(n))),
-            tiles=i32(tiles), tile_start=i32(ts)), n * nblk
+    dev, bf = DEV, torch.bfloat16
+    report = lambda *a: report_kernel(iters, *a)
 
     W, H, G, D, E, win = 4096, 32, 8, 64, 128, 1024
     HS = 16                                     # recurrent heads
@@ -283,6 +304,160 @@ def bench_hybrid(iters):
         report("silu_mul", tag, lambda: ops.silu_mul(gu), B * 14336 * 6)
 
 
+def bench_latent(iters, W):
+    """Kernels of the Tefezen design at width W and the like kernels of the
+    Mixtral-like model."""
+    import hyperspot.ops as ops
+    from hyperspot.engine.kv_cache import LatentKV, RecurrentState
+    from hyperspot.models.llama import (SPAN_TOKENS, LatentSpan,
+                                        prefill_tiles)
+    from hyperspot.ops import experts, hybrid, latent
+    dev, bf, f32 = DEV, torch.bfloat16, torch.float32
+    n_ = ops._native()
+    report = lambda name, tag, fn, nbytes, flops=0: report_kernel(
+        iters, name, f"w{W}_{tag}", fn, nbytes, flops, timed_graph)
+    rnd = lambda *s, d=bf: (torch.randn(*s, device=dev) * 0.3).to(d)
+    i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=dev)
+    H, D, R, E, rank, win = W // 128, 128, 64, 128, 512, 1024
+    G, NE, top, F, side = H // 4, 65536 // W, 4, W // 2, 128
+    uk, uv, kw = rnd(rank, H * D), rnd(H * E, rank), rnd(rank, d=f32)
+    fr = 1e4 ** (-torch.arange(0, R, 2, device=dev).double() / R)
+    decay = torch.linspace(0.5, 0.999, H, device=dev)
+    up, down = rnd(NE, 2 * F, W) * 0.1, rnd(NE, W, F) * 0.1
+    su, sd, router = rnd(1, 2 * F, W), rnd(1, W, F), rnd(NE + 1, W)
+    nw, table = torch.ones(W, device=dev), rnd(1000, side)
+    w2 = torch.ones(W, dtype=bf, device=dev)
+
+    def common(T, tag):
+        x, r = rnd(T, W), rnd(T, W, d=f32)
+        report("add_rms", tag, lambda: hybrid.add_rms(x, r, nw, 1e-5, bf),
+               T * W * 12)
+        r2 = rnd(T, W)
+        report("fused_add_rmsnorm", tag, lambda: ops.fused_add_rmsnorm(
+            x, r2, w2, 1e-5), T * W * 8)
+        o, g = rnd(T, W, d=f32), rnd(T, W)
+        report("rms_gate", tag, lambda: hybrid.rms_gate(
+            o, g, nw, 1e-5, None, W), T * W * 8)
+        z, ids = rnd(T, side), torch.randint(0, 1000, (T,), device=dev)
+        report("gelu_gate", tag, lambda: hybrid.gelu_gate(z, table, ids, 0),
+               T * side * 6)
+        gu = rnd(T, 2 * F)
+        report("silu_mul", tag, lambda: ops.silu_mul(gu), T * F * 6)
+        # experts: every chosen expert's weights once, rows in and out
+        used = min(NE, T * top)
+        per = 3 * W * F
+        nbytes = 2 * (used * per + T * W) + 6 * T * W
+        report("experts (with shared, norm, add)", tag,
+               lambda: experts.mixture_add_rms(
+                   x, router, up, down, su, sd, top, r, nw, 1e-5),
+               nbytes + 2 * per + 8 * T * W, T * (top + 1) * 2 * per)
+        report("experts (routed only, sum)", tag, lambda: experts.mixture(
+            x, router[:NE], up, down, None, None, top), nbytes,
+            T * top * 2 * per)
+
+        def other():
+            p = (x.float() @ router[:NE].float().t()).softmax(-1)
+            wt, ids = p.topk(top, dim=-1)
+            wt = wt / wt.sum(-1, keepdim=True)
+            ops.moe_ffn(x, up, down, wt.to(bf), ids.int())
+        report("moe (route, moe_ffn)", tag, other, nbytes, T * top * 2 * per)
+
+    for lens in ([2048], [8192], [1024] * 8):
+        m, nb = meta_for(lens)
+        T, tag = sum(lens), "x".join(map(str, (len(lens), lens[0])))
+        m.latent = {win: LatentSpan(
+            m.slot_mapping, m.seq_start[:-1].contiguous(),
+            i32([0] * len(lens)), i32(prefill_tiles(lens, SPAN_TOKENS)[0]),
+            None)}
+        q, kv = rnd(T, H * (D + R) + rank + R).split(
+            [H * (D + R), rank + R], -1)
+        cache = LatentKV(torch.zeros(nb, 16, rank + R, dtype=bf, device=dev))
+        report("latent_rope_append", tag, lambda: latent.rope_append(
+            q, kv, kw, m, fr, cache, H, 1e-5),
+            T * (4 * H * R + 4 * (rank + R)))
+        pairs = sum(min(p + 1, win) for x in lens for p in range(x))
+        lat, out = rnd(T, rank + R), rnd(T, H * E)
+        kn, vt, sp = lat[:, :rank] @ uk, uv @ lat[:, :rank].t(), m.latent[win]
+        report("latent_gather", tag, lambda: n_.latent_gather(
+            lat, cache.kv, sp.slots), T * (rank + R) * 4)
+        report("latent_attn_prefill", tag, lambda: n_.latent_attn_prefill(
+            out, q, kn, lat, vt, m.positions, m.seq_start, sp.start, sp.first,
+            sp.tiles, H, win, 0.07), 2 * T * H * (2 * D + R + 2 * E),
+            pairs * H * 2 * (D + R + E))
+        report("latent attention, with expansion", tag,
+               lambda: latent.attention(q, cache, m, uk, uv, H, win, 0.07),
+               2 * T * (H * (D + R + E) + rank + R),
+               pairs * H * 2 * (D + R + E) + T * rank * H * (D + E) * 2)
+        q2, k2, v2 = (x.view(T, -1, 128) for x in rnd(
+            T, (H + 2 * G) * 128).split([H * 128, G * 128, G * 128], -1))
+        kc = torch.zeros(2, nb, G, 16, 128, dtype=bf, device=dev)
+        cs = torch.randn(max(lens), 128, device=dev)
+        report("rope_kv_append", tag, lambda: ops.rope_kv_append(
+            q2, k2, v2, m.positions, cs, m.slot_mapping, kc[0], kc[1]),
+            2 * T * 128 * (2 * H + 4 * G))
+        report("attn_prefill_mfma", tag, lambda: ops.attention(
+            q2, k2, v2, kc[0], kc[1], m, 0.088),
+            2 * T * 128 * (2 * H + 2 * G),
+            sum(x * (x + 1) // 2 for x in lens) * H * 4 * 128)
+        lq, lk, lv, lg = rnd(T, 4 * W).split([W] * 4, -1)
+        st = RecurrentState(torch.zeros(len(lens), H, 128, 128, device=dev))
+        report("lightning_prefill", tag, lambda: hybrid.lightning_mix(
+            lq, lk, lv, decay, st, m), T * W * 10,
+            T * H * 2 * (2 * 128 * 128 + 32 * 256))
+        ga, a2 = rnd(T, 4 * W + 24), rnd(W, 24)
+        gq, gk, gv, gg, ga = ga.split([W] * 4 + [24], -1)
+        a2b, wn = torch.zeros(W, device=dev), torch.ones(128, device=dev)
+        report("gla_prefill", tag, lambda: hybrid.gla_mix(
+            gq, gk, gv, gg, ga, a2, a2b, wn, st, m, 8.0, 1e-5),
+            2 * T * (5 * W + 24), T * H * 2 * (2 * 128 * 128 + 32 * 256))
+        common(T, tag)
+    for B in (1, 32, 256):
+        ctx = 1024
+        m, nb = meta_for([1] * B, "decode", ctx)
+        tag = f"b{B}_ctx{ctx}"
+        q, kv = rnd(B, H * (D + R) + rank + R).split(
+            [H * (D + R), rank + R], -1)
+        cache = LatentKV(rnd(nb, 16, rank + R))
+        report("latent_rope_append", tag, lambda: latent.rope_append(
+            q, kv, kw, m, fr, cache, H, 1e-5),
+            B * (4 * H * R + 4 * (rank + R)))
+        qa, out = rnd(B, H, rank), rnd(B, H * E)
+        report("latent_absorb", tag, lambda: n_.latent_absorb(
+            qa, q, uk, None, H), 2 * H * (D * rank + B * (D + rank)),
+            2 * B * H * D * rank)
+        nbytes = 2 * B * (win * (rank + R) + H * (2 * rank + R))
+        flops = 2 * B * win * H * (2 * rank + R)
+        split = latent.absorbed_split(B * -(-H // 32), win)
+        part = torch.empty(B, H, split, rank + 4, device=dev)
+        report("latent_attn_decode", f"{tag}_split{split}",
+               lambda: n_.latent_attn_decode(
+                   part, qa, q, cache.kv, m.block_tables, m.positions, None,
+                   None, split, win, 0.07), nbytes, flops)
+        report("latent_merge_values", tag, lambda: n_.latent_merge_values(
+            out, part, uv, None, B, H, split),
+            2 * H * (E * rank + B * (E + 2 * split * rank)),
+            2 * B * H * E * rank)
+        report("latent attention, absorbed", tag, lambda: latent.attention(
+            q, cache, m, uk, uv, H, win, 0.07),
+            nbytes + 2 * H * rank * (D + E),
+            flops + 2 * B * H * rank * (D + E))
+        q2, k2, v2 = (x.view(B, -1, 128) for x in rnd(
+            B, (H + 2 * G) * 128).split([H * 128, G * 128, G * 128], -1))
+        kc = rnd(2, nb, G, 16, 128)
+        cs = torch.randn(ctx + 1, 128, device=dev)
+        report("rope_kv_append", tag, lambda: ops.rope_kv_append(
+            q2, k2, v2, m.positions, cs, m.slot_mapping, kc[0], kc[1]),
+            2 * B * 128 * (2 * H + 4 * G))
+        report("paged_attn_decode", tag, lambda: ops.paged_attn_decode(
+            q2, kc[0], kc[1], m.block_tables, m.seq_lens, 0.088),
+            4 * B * (ctx + 1) * G * 128)
+        lq, lk, lv, lg = rnd(B, 4 * W).split([W] * 4, -1)
+        st = RecurrentState(torch.zeros(B, H, 128, 128, device=dev))
+        report("lightning_step", tag, lambda: hybrid.lightning_mix(
+            lq, lk, lv, decay, st, m), B * H * 128 * 128 * 8)
+        common(B, tag)
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--which", default="attn")
@@ -295,6 +470,9 @@ def main():
         bench_gemm(args.iters)
     if args.which in ("hybrid", "all"):
         bench_hybrid(args.iters)
+    if args.which in ("latent", "all"):
+        for width in (2048, 4096):
+            bench_latent(args.iters, width)
     if args.which in ("fp8", "all"):
         bench_fp8_gemm(args.iters)
 

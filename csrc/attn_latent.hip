@@ -161,7 +161,7 @@ __global__ __launch_bounds__(256) void head_gemm_kernel(
   f32x4_t acc[CT];
   #pragma unroll
   for (int t = 0; t < CT; ++t) acc[t] = f32x4_t(0.f);
-  #pragma unroll 4
+  #pragma unroll 8
   for (int k = 0; k < a.K; k += 32) {
     const bool in = k + gr * 8 < a.K;
     const short8_t wf = in && wn
@@ -275,7 +275,8 @@ constexpr int decode_lds(int RP, int XP) {
   return 2 * KT * (RP + XP + 8) * 2 + 2 * 16 * SS * 4;
 }
 
-template <int RP, int XP, int HT>
+// EXACT: rank == RP and rot == XP, a row is staged as it is
+template <int RP, int XP, int HT, bool EXACT>
 __global__ __launch_bounds__(256, 2) void latent_attn_decode_kernel(
     bf16* __restrict__ out, float* __restrict__ partial,
     const bf16* __restrict__ qa, const bf16* __restrict__ q,
@@ -288,7 +289,7 @@ __global__ __launch_bounds__(256, 2) void latent_attn_decode_kernel(
   constexpr int QC = HT == 2 ? KC : (KC + 1) / 2;
   constexpr int ET = RP / 64;                // 16-column tiles of a wave
   constexpr int UPR = (RP + XP) / 8;         // 16-byte units of a row
-  constexpr int LOADS = (KT * UPR + 255) / 256;
+  constexpr int LOADS = (UPR + 7) / 8;       // units a thread: 8 share a row
   extern __shared__ __attribute__((aligned(16))) char smem[];
   short* kv_lds = reinterpret_cast<short*>(smem);            // [2][KT][LS]
   float* s_lds = reinterpret_cast<float*>(kv_lds + 2 * KT * LS);
@@ -335,34 +336,45 @@ __global__ __launch_bounds__(256, 2) void latent_attn_decode_kernel(
   #pragma unroll
   for (int t = 0; t < HT; ++t) { m[t] = -FLT_MAX; l[t] = 0.f; }
 
-  uint4 kr[LOADS];
+  // This thread stages units tid % 8 + 8 i of token tid / 8.  Tokens past the
+  // row's own read its own again (their weight is zero); padding columns are
+  // zeros.  A page id is read one tile ahead of its rows.
+  const int tok = tid >> 3;
+  int off[LOADS];                    // column in the cache row, -1: zeros
+  #pragma unroll
+  for (int i = 0; i < LOADS; ++i) {
+    const int d = ((tid & 7) + 8 * i) * 8;
+    off[i] = d < RP ? (d < rank ? d : -1)
+                    : d - RP < rot ? d - RP + rank : -1;
+  }
+  short8_t kr[LOADS];
+  long page = 0;
   auto fetch = [&](int p0) {
-    const long b0 = bt[p0 / PAGE];
-    const long b1 = p0 + PAGE <= pos ? bt[p0 / PAGE + 1] : b0;
+    const int p = min(p0 + tok, pos);
+    const bf16* src = cache + (page * PAGE + p % PAGE) * (rank + rot);
+    page = bt[min(p0 + split * KT + tok, pos) / PAGE];
     #pragma unroll
     for (int i = 0; i < LOADS; ++i) {
-      const int u = tid + 256 * i;
-      const int t = u / UPR, d = (u % UPR) * 8;
-      kr[i] = uint4{0, 0, 0, 0};
-      const bool in = d < RP ? d < rank : d - RP < rot;
-      if (t < KT && in && p0 + t <= pos)
-        kr[i] = *reinterpret_cast<const uint4*>(
-            cache + ((t < PAGE ? b0 : b1) * PAGE + t % PAGE) * (rank + rot) +
-            (d < RP ? d : d - RP + rank));
+      if constexpr (EXACT)
+        kr[i] = *reinterpret_cast<const short8_t*>(src + (tid & 7) * 8 + 64 * i);
+      else
+        kr[i] = off[i] >= 0 ? *reinterpret_cast<const short8_t*>(src + off[i])
+                            : short8_t{};
     }
   };
 
   int p0 = (lo / KT + z) * KT, buf = 0;
-  if (p0 <= pos) fetch(p0);
+  if (p0 <= pos) {
+    page = bt[min(p0 + tok, pos) / PAGE];
+    fetch(p0);
+  }
   for (; p0 <= pos; p0 += split * KT, buf ^= 1) {
     short* tile = kv_lds + buf * KT * LS;
     #pragma unroll
-    for (int i = 0; i < LOADS; ++i) {
-      const int u = tid + 256 * i;
-      if (u < KT * UPR)
-        *reinterpret_cast<uint4*>(tile + (u / UPR) * LS + (u % UPR) * 8) =
+    for (int i = 0; i < LOADS; ++i)
+      if ((tid & 7) + 8 * i < UPR)
+        *reinterpret_cast<short8_t*>(tile + tok * LS + (tid & 7) * 8 + 64 * i) =
             kr[i];
-    }
     __syncthreads();
     if (p0 + split * KT <= pos) fetch(p0 + split * KT);
     {
@@ -379,6 +391,7 @@ __global__ __launch_bounds__(256, 2) void latent_attn_decode_kernel(
     }
     __syncthreads();
     short8_t ph[HT], pl[HT];
+    const bool full = p0 >= lo && p0 + KT - 1 <= pos;
     #pragma unroll
     for (int t = 0; t < HT; ++t) {
       float p[8], mx = m[t];
@@ -391,11 +404,16 @@ __global__ __launch_bounds__(256, 2) void latent_attn_decode_kernel(
         for (int i = 0; i < 8; ++i) p[i] += sp[16 * SS + i];
       }
       #pragma unroll
-      for (int i = 0; i < 8; ++i) {
-        const int at = p0 + gr * 8 + i;
-        p[i] = at >= lo && at <= pos ? p[i] * scale2 : -FLT_MAX;
-        mx = fmaxf(mx, p[i]);
+      for (int i = 0; i < 8; ++i) p[i] *= scale2;
+      if (!full) {
+        #pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          const int at = p0 + gr * 8 + i;
+          if (at < lo || at > pos) p[i] = -FLT_MAX;
+        }
       }
+      #pragma unroll
+      for (int i = 0; i < 8; ++i) mx = fmaxf(mx, p[i]);
       mx = fmaxf(mx, __shfl_xor(mx, 16));
       mx = fmaxf(mx, __shfl_xor(mx, 32));
       if (!__all(mx == m[t])) {
@@ -456,35 +474,82 @@ __global__ __launch_bounds__(256, 2) void latent_attn_decode_kernel(
   }
 }
 
-// a wave per (row, head): split <= 64 partial results combined
-__global__ __launch_bounds__(64) void latent_merge_kernel(
-    bf16* __restrict__ out, const float* __restrict__ partial, int split,
-    int H, int rank) {
-  const long rh = (long)blockIdx.x * H + blockIdx.y;
-  const int lane = threadIdx.x;
-  const float* src = partial + rh * split * (rank + 4);
-  float m = -FLT_MAX, l = 0.f;
-  if (lane < split) {
-    m = src[(long)lane * (rank + 4) + rank];
-    l = src[(long)lane * (rank + 4) + rank + 1];
+// Partial results of 16 rows and one head combined, then W_uv of that head:
+// out[row, h] = W_uv[h] sum_p weight_p o_p.  split <= 16.
+__global__ __launch_bounds__(256) void latent_merge_values_kernel(
+    bf16* __restrict__ out, const float* __restrict__ partial,
+    const bf16* __restrict__ uv, const int* __restrict__ rows, long R,
+    int split, int H, int E, int rank) {
+  extern __shared__ __attribute__((aligned(16))) short merged[];
+  __shared__ float weight[16][17];
+  const int h = blockIdx.y, tid = threadIdx.x;
+  const long r0 = (long)blockIdx.x * 16;
+  const int XS = rank + 8;
+  {
+    const int i = tid >> 4, p = tid & 15;
+    const bool in = r0 + i < R && p < split;
+    const float* src = partial +
+        (((r0 + i) * H + h) * split + p) * (rank + 4) + rank;
+    const float m = in ? src[0] : -FLT_MAX, l = in ? src[1] : 0.f;
+    float mx = m;
+    #pragma unroll
+    for (int o = 1; o < 16; o <<= 1) mx = fmaxf(mx, __shfl_xor(mx, o));
+    const float w = m == -FLT_MAX ? 0.f : exp2_fast(m - mx);
+    float sum = w * l;
+    #pragma unroll
+    for (int o = 1; o < 16; o <<= 1) sum += __shfl_xor(sum, o);
+    weight[i][p] = sum > 0.f ? w / sum : 0.f;
   }
-  const float mx = wave_reduce_max(m);
-  float w = m == -FLT_MAX ? 0.f : exp2_fast(m - mx);
-  w /= wave_reduce_sum(w * l);
-  for (int c = lane * 4; c < rank; c += 256) {
-    float o[4] = {};
-    #pragma unroll 4
-    for (int p = 0; p < split; ++p) {
-      const float wp = __shfl(w, p);
-      const float4 x = *reinterpret_cast<const float4*>(
-          src + (long)p * (rank + 4) + c);
-      o[0] += wp * x.x;
-      o[1] += wp * x.y;
-      o[2] += wp * x.z;
-      o[3] += wp * x.w;
+  __syncthreads();
+  // a wave has a quarter of the columns, four rows at a time
+  const int lane = tid & 63, wid = tid >> 6, quarter = rank / 4;
+  const int live = (int)min(16L, R - r0);
+  for (int c = wid * quarter + lane * 2; c < (wid + 1) * quarter; c += 128)
+    for (int i0 = 0; i0 < live; i0 += 4) {
+      float2 o[4] = {};
+      const float* src[4];
+      #pragma unroll
+      for (int k = 0; k < 4; ++k)
+        src[k] = partial + ((r0 + min(i0 + k, live - 1)) * H + h) * split *
+                               (rank + 4) + c;
+      #pragma unroll 8
+      for (int p = 0; p < split; ++p)
+        #pragma unroll
+        for (int k = 0; k < 4; ++k) {
+          const float w = weight[i0 + k][p];
+          const float2 x = *reinterpret_cast<const float2*>(
+              src[k] + (long)p * (rank + 4));
+          o[k].x += w * x.x;
+          o[k].y += w * x.y;
+        }
+      #pragma unroll
+      for (int k = 0; k < 4; ++k)
+        *reinterpret_cast<unsigned*>(merged + (i0 + k) * XS + c) =
+            cvt_pk_bf16(o[k].x, o[k].y);
     }
-    *reinterpret_cast<uint2*>(out + rh * rank + c) =
-        uint2{cvt_pk_bf16(o[0], o[1]), cvt_pk_bf16(o[2], o[3])};
+  __syncthreads();
+  const int col = lane & 15, gr = lane >> 4;
+  const long r = r0 + col;
+  for (int n0 = wid * 16; n0 < E; n0 += 64) {
+    const bool wn = n0 + col < E;
+    const bf16* wp = uv + ((long)h * E + n0 + col) * rank + gr * 8;
+    f32x4_t acc = f32x4_t(0.f);
+    #pragma unroll 8
+    for (int k = 0; k < rank; k += 32) {
+      const bool in = k + gr * 8 < rank;
+      const short8_t wf = in && wn
+          ? *reinterpret_cast<const short8_t*>(wp + k) : short8_t{};
+      // columns past the last row are left out below
+      const short8_t xf = in && r < R
+          ? *reinterpret_cast<const short8_t*>(merged + col * XS + k + gr * 8)
+          : short8_t{};
+      acc = mfma16(wf, xf, acc);
+    }
+    const int n = n0 + gr * 4;
+    if (n < E && r < R)
+      *reinterpret_cast<uint2*>(
+          out + ((rows ? rows[r] : r) * H + h) * E + n) =
+          uint2{cvt_pk_bf16(acc[0], acc[1]), cvt_pk_bf16(acc[2], acc[3])};
   }
 }
 
@@ -739,8 +804,7 @@ void launch_head_gemm(T* out, const T* x, const T* w, const int* rows_in,
             <<<dim3(nx, (unsigned)((R + 16 * CT - 1) / (16 * CT)),          \
                     (unsigned)H), 256, 0, stream>>>(out, x, w, a)
       if (R <= 16) RUN(1);
-      else if (R <= 32) RUN(2);
-      else RUN(4);
+      else RUN(2);
       #undef RUN
       return;
     }
@@ -774,31 +838,41 @@ void launch_latent_attn_decode(bf16* out, float* partial, const bf16* qa,
                                int rot, int window, float scale, long qs,
                                int split, hipStream_t stream) {
   if (R == 0) return;
-  #define RUN(RP, XP, HT)                                                   \
+  #define RUN(RP, XP, HT, EXACT)                                            \
     {                                                                       \
-      allow_lds(&latent_attn_decode_kernel<RP, XP, HT>,                     \
+      allow_lds(&latent_attn_decode_kernel<RP, XP, HT, EXACT>,              \
                 decode_lds(RP, XP));                                        \
-      latent_attn_decode_kernel<RP, XP, HT>                                 \
+      latent_attn_decode_kernel<RP, XP, HT, EXACT>                          \
           <<<dim3((unsigned)R, (unsigned)((H + 16 * HT - 1) / (16 * HT)),   \
                   (unsigned)split), 256, decode_lds(RP, XP), stream>>>(     \
               out, partial, qa, q, cache, block_tables, positions, rows,    \
               row_seq, max_blocks, H, D, rank, rot, window, scale * LOG2E,  \
               qs);                                                          \
+      done = true;                                                          \
     }
   #define CASE(RP, XP)                                                      \
     if (!done && rank <= RP && rot <= XP) {                                 \
-      if (H <= 16) RUN(RP, XP, 1) else RUN(RP, XP, 2)                       \
-      done = true;                                                          \
+      if (H <= 16) RUN(RP, XP, 1, false) else RUN(RP, XP, 2, false)         \
     }
   bool done = false;
+  if (rank == 512 && rot == 64) {
+    if (H <= 16) RUN(512, 64, 1, true) else RUN(512, 64, 2, true)
+  }
   CASE(64, 32) CASE(64, 64) CASE(128, 32) CASE(128, 64) CASE(256, 32)
   CASE(256, 64) CASE(512, 32) CASE(512, 64)
   #undef CASE
   #undef RUN
   if (!done) throw std::runtime_error("latent_attn_decode: latent size");
-  if (split > 1)
-    latent_merge_kernel<<<dim3((unsigned)R, (unsigned)H), 64, 0, stream>>>(
-        out, partial, split, H, rank);
+}
+
+void launch_latent_merge_values(bf16* out, const float* partial,
+                                const bf16* uv, const int* rows, long R,
+                                int split, int H, int E, int rank,
+                                hipStream_t stream) {
+  if (R == 0) return;
+  latent_merge_values_kernel<<<dim3((unsigned)((R + 15) / 16), (unsigned)H),
+                               256, 16 * (rank + 8) * 2, stream>>>(
+      out, partial, uv, rows, R, split, H, E, rank);
 }
 
 void launch_latent_attn_prefill(bf16* out, const bf16* q, const bf16* kn,

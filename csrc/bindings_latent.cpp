@@ -37,6 +37,8 @@ void launch_latent_attn_decode(bf16*, float*, const bf16*, const bf16*,
                                const bf16*, const int*, const long*,
                                const int*, const int*, long, int, int, int,
                                int, int, int, float, long, int, hipStream_t);
+void launch_latent_merge_values(bf16*, const float*, const bf16*, const int*,
+                                long, int, int, int, int, hipStream_t);
 void launch_latent_attn_prefill(bf16*, const bf16*, const bf16*, const bf16*,
                                 const bf16*, const long*, const int*,
                                 const int*, const int*, const int*, int, int,
@@ -321,29 +323,48 @@ void latent_attn_general(Tensor o, Tensor qa, Tensor q, Tensor cache,
   });
 }
 
+// split 1: o [R, H, rank] bf16; otherwise o is the partial results of
+// latent_merge_values, [R, H, split, rank + 4] float
 void latent_attn_decode(Tensor o, Tensor qa, Tensor q, Tensor cache,
                         Tensor block_tables, Tensor positions, Maybe rows,
-                        Maybe row_seq, Maybe partial, long split, long window,
+                        Maybe row_seq, long split, long window,
                         double scale) {
-  const auto d = check_absorbed(o, qa, q, cache, block_tables, positions,
-                                rows, row_seq, window);
+  const auto d = check_absorbed(split > 1 ? qa : o, qa, q, cache,
+                                block_tables, positions, rows, row_seq,
+                                window);
   TORCH_CHECK(q.scalar_type() == torch::kBFloat16 && q.stride(0) % 8 == 0 &&
                   aligned16(q) &&
                   latent_sizes_fit((int)d.D, 8, (int)d.rank, (int)d.rot),
               "latent_attn_decode: sizes");
-  TORCH_CHECK(split >= 1 && split <= 64, "latent_attn_decode: split");
-  if (split > 1) {
-    TORCH_CHECK(partial.has_value(), "latent_attn_decode: partial");
-    check_param(*partial, qa.size(0) * d.H * split * (d.rank + 4),
-                "partial");
-  }
+  TORCH_CHECK(split >= 1 && split <= 16, "latent_attn_decode: split");
+  if (split > 1)
+    check_param(o, qa.size(0) * d.H * split * (d.rank + 4), "partial");
   launch_latent_attn_decode(
-      ptr<bf16>(o), split > 1 ? ptr<float>(*partial) : nullptr, ptr<bf16>(qa),
-      ptr<bf16>(q), ptr<bf16>(cache), block_tables.data_ptr<int>(),
-      positions.data_ptr<long>(), opt_int(rows), opt_int(row_seq),
-      qa.size(0), (int)block_tables.size(1), (int)d.H, (int)d.D, (int)d.rank,
-      (int)d.rot, (int)window, (float)scale, q.stride(0), (int)split,
-      stream());
+      split > 1 ? nullptr : ptr<bf16>(o), split > 1 ? ptr<float>(o) : nullptr,
+      ptr<bf16>(qa), ptr<bf16>(q), ptr<bf16>(cache),
+      block_tables.data_ptr<int>(), positions.data_ptr<long>(),
+      opt_int(rows), opt_int(row_seq), qa.size(0),
+      (int)block_tables.size(1), (int)d.H, (int)d.D, (int)d.rank, (int)d.rot,
+      (int)window, (float)scale, q.stride(0), (int)split, stream());
+}
+
+// out[rows[r], h] = W_uv[h] (combined partial results of r and h)
+void latent_merge_values(Tensor out, Tensor partial, Tensor uv, Maybe rows,
+                         long R, long heads, long split) {
+  check(out, torch::kBFloat16, "out");
+  check(uv, torch::kBFloat16, "uv");
+  const long E = uv.size(0) / heads, rank = uv.size(1);
+  TORCH_CHECK(uv.size(0) == heads * E && out.size(1) == heads * E &&
+                  latent_sizes_fit(8, (int)E, (int)rank, 8) && split >= 1 &&
+                  split <= 16, "latent_merge_values: sizes");
+  check_param(partial, R * heads * split * (rank + 4), "partial");
+  if (rows.has_value())
+    check_ints(*rows, R, "rows");
+  else
+    TORCH_CHECK(R == out.size(0), "latent_merge_values: rows");
+  launch_latent_merge_values(ptr<bf16>(out), ptr<float>(partial),
+                             ptr<bf16>(uv), opt_int(rows), R, (int)split,
+                             (int)heads, (int)E, (int)rank, stream());
 }
 
 void latent_attn_prefill(Tensor out, Tensor q, Tensor kn, Tensor lat,
@@ -542,6 +563,7 @@ void register_latent(pybind11::module_& m) {
   m.def("latent_values", &latent_values);
   m.def("latent_attn_general", &latent_attn_general);
   m.def("latent_attn_decode", &latent_attn_decode);
+  m.def("latent_merge_values", &latent_merge_values);
   m.def("latent_attn_prefill", &latent_attn_prefill);
   m.def("experts_route", &experts_route);
   m.def("experts_sort", &experts_sort);

@@ -72,23 +72,27 @@ def _absorbed(out, q, cache, meta, row_seq, rows, uk, uv, heads, window,
                                                   device=q.device)
     qa = empty(R, heads, rank)
     n.latent_absorb(qa, q, uk, rows, heads)
-    o = empty(R, heads, rank)
-    if fits:
-        reach = min(window, meta.block_tables.shape[1] * cache.kv.shape[1])
-        split = absorbed_split(R * -(-heads // 32), reach)
-        partial = None if split == 1 else empty(
-            R * heads * split * (rank + 4), dtype=torch.float32)
-        n.latent_attn_decode(o, qa, q, cache.kv, meta.block_tables,
-                             meta.positions, rows, row_seq, partial, split,
-                             window, scale)
+    where = (cache.kv, meta.block_tables, meta.positions, rows, row_seq)
+    if not fits:
+        o = empty(R, heads, rank)
+        n.latent_attn_general(o, qa, q, *where, window, scale)
+        n.latent_values(out, o, uv, rows)
+        return
+    reach = min(window, meta.block_tables.shape[1] * cache.kv.shape[1])
+    split = absorbed_split(R * -(-heads // 32), reach)
+    if split == 1:
+        o = empty(R, heads, rank)
+        n.latent_attn_decode(o, qa, q, *where, 1, window, scale)
+        n.latent_values(out, o, uv, rows)
     else:
-        n.latent_attn_general(o, qa, q, cache.kv, meta.block_tables,
-                              meta.positions, rows, row_seq, window, scale)
-    n.latent_values(out, o, uv, rows)
+        part = empty(R, heads, split, rank + 4, dtype=torch.float32)
+        n.latent_attn_decode(part, qa, q, *where, split, window, scale)
+        n.latent_merge_values(out, part, uv, rows, R, heads, split)
 
 
 def absorbed_split(groups: int, reach: int) -> int:
-    """How many workgroups share one row's window: two for every compute unit
-    where the batch alone gives fewer, each with at least 64 tokens.  Depends
-    on shapes only, so a captured graph keeps it."""
-    return max(1, min(16, 512 // groups, reach // 64))
+    """How many workgroups share one row's window, each with at least 64
+    tokens: one for every compute unit where the batch alone gives fewer, two
+    otherwise.  Depends on shapes only, so a captured graph keeps it."""
+    fill = 256 if groups < 256 else 512
+    return max(1, min(16, fill // groups, reach // 64))
