@@ -61,12 +61,31 @@ __global__ __launch_bounds__(256) void latent_rope_append_kernel(
     cs[2 * i + 1] = s;
   }
   __syncthreads();
-  for (int u = threadIdx.x; u < H * half; u += 256) {
-    const int h = u / half, i = u % half;
-    T* p = q + row * qs + (long)h * (D + rot) + D + 2 * i;
-    const float x = Elem<T>::ld(p), y = Elem<T>::ld(p + 1);
-    Elem<T>::st(p, x * cs[2 * i] - y * cs[2 * i + 1]);
-    Elem<T>::st(p + 1, y * cs[2 * i] + x * cs[2 * i + 1]);
+  // W elements of a head at a time
+  constexpr int W = V == 1 ? 2 : V;
+  const int units = rot / W;
+  for (int u = threadIdx.x; u < H * units; u += 256) {
+    const int h = u / units, d = u % units * W;
+    T* p = q + row * qs + (long)h * (D + rot) + D + d;
+    float x[W];
+    if constexpr (V == 1) {
+      x[0] = Elem<T>::ld(p);
+      x[1] = Elem<T>::ld(p + 1);
+    } else {
+      load_vec<T, V>(p, x);
+    }
+    #pragma unroll
+    for (int i = 0; i < W; i += 2) {
+      const float c = cs[d + i], s = cs[d + i + 1], a = x[i], b = x[i + 1];
+      x[i] = a * c - b * s;
+      x[i + 1] = b * c + a * s;
+    }
+    if constexpr (V == 1) {
+      Elem<T>::st(p, x[0]);
+      Elem<T>::st(p + 1, x[1]);
+    } else {
+      store_vec<T, V>(p, x);
+    }
   }
   if (!kv) return;
   const long slot = slot_mapping[row];
@@ -474,20 +493,37 @@ __global__ __launch_bounds__(256, 2) void latent_attn_decode_kernel(
   }
 }
 
-// Partial results of 16 rows and one head combined, then W_uv of that head:
-// out[row, h] = W_uv[h] sum_p weight_p o_p.  split <= 16.
+// Partial results of RB <= 16 rows and one head combined, then W_uv of that
+// head: out[row, h] = W_uv[h] sum_p weight_p o_p.  split <= 16, rank <= 512.
+// A wave has 16 of every gridDim.z * 64 values; its first weights are on their
+// way while the results are combined.
+template <int RB>
 __global__ __launch_bounds__(256) void latent_merge_values_kernel(
     bf16* __restrict__ out, const float* __restrict__ partial,
     const bf16* __restrict__ uv, const int* __restrict__ rows, long R,
     int split, int H, int E, int rank) {
   extern __shared__ __attribute__((aligned(16))) short merged[];
   __shared__ float weight[16][17];
+  constexpr int RK = RB < 4 ? RB : 4;        // rows combined together
   const int h = blockIdx.y, tid = threadIdx.x;
-  const long r0 = (long)blockIdx.x * 16;
+  const long r0 = (long)blockIdx.x * RB;
+  const int live = (int)min((long)RB, R - r0);
   const int XS = rank + 8;
+  const int lane = tid & 63, wid = tid >> 6, col = lane & 15, gr = lane >> 4;
+  int n0 = (blockIdx.z * 4 + wid) * 16;
+  short8_t wf[16];
+  auto weights = [&]() {
+    const bool wn = n0 + col < E;
+    const bf16* wp = uv + ((long)h * E + n0 + col) * rank + gr * 8;
+    #pragma unroll
+    for (int k = 0; k < 16; ++k)
+      wf[k] = wn && k * 32 + gr * 8 < rank
+          ? *reinterpret_cast<const short8_t*>(wp + k * 32) : short8_t{};
+  };
+  weights();
   {
     const int i = tid >> 4, p = tid & 15;
-    const bool in = r0 + i < R && p < split;
+    const bool in = i < live && p < split;
     const float* src = partial +
         (((r0 + i) * H + h) * split + p) * (rank + 4) + rank;
     const float m = in ? src[0] : -FLT_MAX, l = in ? src[1] : 0.f;
@@ -501,21 +537,20 @@ __global__ __launch_bounds__(256) void latent_merge_values_kernel(
     weight[i][p] = sum > 0.f ? w / sum : 0.f;
   }
   __syncthreads();
-  // a wave has a quarter of the columns, four rows at a time
-  const int lane = tid & 63, wid = tid >> 6, quarter = rank / 4;
-  const int live = (int)min(16L, R - r0);
+  // a wave has a quarter of the columns
+  const int quarter = rank / 4;
   for (int c = wid * quarter + lane * 2; c < (wid + 1) * quarter; c += 128)
-    for (int i0 = 0; i0 < live; i0 += 4) {
-      float2 o[4] = {};
-      const float* src[4];
+    for (int i0 = 0; i0 < live; i0 += RK) {
+      float2 o[RK] = {};
+      const float* src[RK];
       #pragma unroll
-      for (int k = 0; k < 4; ++k)
+      for (int k = 0; k < RK; ++k)
         src[k] = partial + ((r0 + min(i0 + k, live - 1)) * H + h) * split *
                                (rank + 4) + c;
       #pragma unroll 8
       for (int p = 0; p < split; ++p)
         #pragma unroll
-        for (int k = 0; k < 4; ++k) {
+        for (int k = 0; k < RK; ++k) {
           const float w = weight[i0 + k][p];
           const float2 x = *reinterpret_cast<const float2*>(
               src[k] + (long)p * (rank + 4));
@@ -523,33 +558,31 @@ __global__ __launch_bounds__(256) void latent_merge_values_kernel(
           o[k].y += w * x.y;
         }
       #pragma unroll
-      for (int k = 0; k < 4; ++k)
+      for (int k = 0; k < RK; ++k)
         *reinterpret_cast<unsigned*>(merged + (i0 + k) * XS + c) =
             cvt_pk_bf16(o[k].x, o[k].y);
     }
   __syncthreads();
-  const int col = lane & 15, gr = lane >> 4;
   const long r = r0 + col;
-  for (int n0 = wid * 16; n0 < E; n0 += 64) {
-    const bool wn = n0 + col < E;
-    const bf16* wp = uv + ((long)h * E + n0 + col) * rank + gr * 8;
+  while (n0 < E) {
     f32x4_t acc = f32x4_t(0.f);
-    #pragma unroll 8
-    for (int k = 0; k < rank; k += 32) {
-      const bool in = k + gr * 8 < rank;
-      const short8_t wf = in && wn
-          ? *reinterpret_cast<const short8_t*>(wp + k) : short8_t{};
+    #pragma unroll
+    for (int k = 0; k < 16; ++k) {
+      if (k * 32 >= rank) break;
       // columns past the last row are left out below
-      const short8_t xf = in && r < R
-          ? *reinterpret_cast<const short8_t*>(merged + col * XS + k + gr * 8)
+      const short8_t xf = k * 32 + gr * 8 < rank && col < live
+          ? *reinterpret_cast<const short8_t*>(merged + col * XS + k * 32 +
+                                               gr * 8)
           : short8_t{};
-      acc = mfma16(wf, xf, acc);
+      acc = mfma16(wf[k], xf, acc);
     }
     const int n = n0 + gr * 4;
-    if (n < E && r < R)
+    if (n < E && col < live)
       *reinterpret_cast<uint2*>(
           out + ((rows ? rows[r] : r) * H + h) * E + n) =
           uint2{cvt_pk_bf16(acc[0], acc[1]), cvt_pk_bf16(acc[2], acc[3])};
+    n0 += gridDim.z * 64;
+    if (n0 < E) weights();
   }
 }
 
@@ -767,8 +800,11 @@ void launch_latent_rope_append(T* q, const T* kv, const float* w,
                                long ks, float eps, hipStream_t stream) {
   if (rows == 0 || (rot == 0 && !kv)) return;
   const size_t lds = (rot + 2) * sizeof(float);
-  const bool vec = rank % 4 == 0 && rot % 4 == 0 && ks % 4 == 0 &&
-                   reinterpret_cast<uintptr_t>(kv) % (4 * sizeof(T)) == 0;
+  auto aligned = [](const T* p) {
+    return reinterpret_cast<uintptr_t>(p) % (4 * sizeof(T)) == 0;
+  };
+  const bool vec = rank % 4 == 0 && rot % 4 == 0 && D % 4 == 0 &&
+                   qs % 4 == 0 && ks % 4 == 0 && aligned(q) && aligned(kv);
   if (vec)
     latent_rope_append_kernel<T, 4><<<(unsigned)rows, 256, lds, stream>>>(
         q, kv, w, positions, freqs, slot_mapping, cache, H, D, rank, rot, qs,
@@ -870,9 +906,18 @@ void launch_latent_merge_values(bf16* out, const float* partial,
                                 int split, int H, int E, int rank,
                                 hipStream_t stream) {
   if (R == 0) return;
-  latent_merge_values_kernel<<<dim3((unsigned)((R + 15) / 16), (unsigned)H),
-                               256, 16 * (rank + 8) * 2, stream>>>(
-      out, partial, uv, rows, R, split, H, E, rank);
+  // few rows: fewer a workgroup, then fewer values a workgroup
+  int rb = 16;
+  while (rb > 1 && (R + rb - 1) / rb * H < 512) rb /= 2;
+  const unsigned nz = R * H < 128 ? (unsigned)((E + 63) / 64) : 1;
+  const dim3 grid((unsigned)((R + rb - 1) / rb), (unsigned)H, nz);
+  #define CASE(RB)                                                          \
+    if (rb == RB)                                                           \
+      latent_merge_values_kernel<RB>                                        \
+          <<<grid, 256, 16 * (rank + 8) * 2, stream>>>(                     \
+              out, partial, uv, rows, R, split, H, E, rank);
+  CASE(1) CASE(2) CASE(4) CASE(8) CASE(16)
+  #undef CASE
 }
 
 void launch_latent_attn_prefill(bf16* out, const bf16* q, const bf16* kn,

@@ -135,21 +135,28 @@ __global__ __launch_bounds__(256) void rms_gate_kernel(
 }
 
 // out[t, j] = gelu_tanh(z[t, j]) * table[ids[t], column + j]
-template <typename T>
+template <typename T, int V>
 __global__ __launch_bounds__(256) void gelu_gate_kernel(
     T* __restrict__ out, const T* __restrict__ z, const T* __restrict__ table,
-    const long* __restrict__ ids, long total, int n, long cols, long column,
+    const long* __restrict__ ids, long rows, int n, long cols, long column,
     long vocab) {
+  const int units = n / V;
   const long u = (long)blockIdx.x * 256 + threadIdx.x;
-  if (u >= total) return;
-  const long row = u / n;
-  const int j = (int)(u - row * n);
+  const long row = u / units;
+  if (row >= rows) return;
+  const int j = (int)(u - row * units) * V;
   long id = ids[row];
   id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
-  const float v = Elem<T>::ld(z + u);
-  const float s = 0.7978845608028654f * (v + 0.044715f * v * v * v);
-  Elem<T>::st(out + u, 0.5f * v * (1.f + Fn<T>::tanh(s)) *
-                           Elem<T>::ld(table + id * cols + column + j));
+  float v[V], e[V];
+  load_vec<T, V>(z + row * n + j, v);
+  load_vec<T, V>(table + id * cols + column + j, e);
+  #pragma unroll
+  for (int i = 0; i < V; ++i) {
+    const float s = 0.7978845608028654f *
+                    (v[i] + 0.044715f * v[i] * v[i] * v[i]);
+    v[i] = 0.5f * v[i] * (1.f + Fn<T>::tanh(s)) * e[i];
+  }
+  store_vec<T, V>(out + row * n + j, v);
 }
 
 bool by4(const void* p, size_t elem) {
@@ -215,8 +222,14 @@ void launch_gelu_gate(T* out, const T* z, const T* table, const long* ids,
                       long rows, int n, long cols, long column, long vocab,
                       hipStream_t stream) {
   if (rows == 0 || n == 0) return;
-  gelu_gate_kernel<T><<<(unsigned)((rows * n + 255) / 256), 256, 0, stream>>>(
-      out, z, table, ids, rows * n, n, cols, column, vocab);
+  if (n % 4 == 0 && cols % 4 == 0 && column % 4 == 0)
+    gelu_gate_kernel<T, 4>
+        <<<(unsigned)((rows * (n / 4) + 255) / 256), 256, 0, stream>>>(
+            out, z, table, ids, rows, n, cols, column, vocab);
+  else
+    gelu_gate_kernel<T, 1>
+        <<<(unsigned)((rows * n + 255) / 256), 256, 0, stream>>>(
+            out, z, table, ids, rows, n, cols, column, vocab);
 }
 
 #define INSTANTIATE(T)                                                      \
