@@ -401,9 +401,8 @@ class LightningAttention(nn.Module):
         self.o_proj = RowParallelLinear(e, width, dtype, seed_tag=tag + 4)
         self.norm = _rows(_param(torch.ones(e // tp)), tp, r, e)
         h = m.heads // tp
-        self.register_buffer("decay", torch.tensor(
-            m.decay[r * h:(r + 1) * h], dtype=torch.float32),
-            persistent=False)
+        self.decay = _rows(_param(torch.tensor(
+            m.decay[r * h:(r + 1) * h], dtype=torch.float32)), tp, r, m.heads)
 
     def forward(self, x, meta, state) -> torch.Tensor:
         q, k, v, g = self.proj.split(self.proj(x))
