@@ -14,6 +14,7 @@ void launch_add_rms(T*, float*, const T*, const float*, long, int, float,
 template <typename T>
 void launch_rms_gate(T*, const float*, const T*, const float*, const float*,
                      long, int, long, long, float, hipStream_t);
+void launch_row_squares(float*, const float*, long, int, hipStream_t);
 template <typename T>
 void launch_gelu_gate(T*, const T*, const T*, const long*, long, int, long,
                       long, long, hipStream_t);
@@ -142,6 +143,13 @@ void rms_gate(Tensor y, Tensor o, Tensor g, Tensor w, Maybe ss, long total,
                        opt(ss), rows, (int)n, total, g.stride(0), (float)eps,
                        stream());
   });
+}
+
+void row_squares(Tensor ss, Tensor x) {
+  check_param(x, x.numel(), "x");
+  check_param(ss, x.size(0), "ss");
+  launch_row_squares(ptr<float>(ss), ptr<float>(x), x.size(0),
+                     (int)x.size(1), stream());
 }
 
 void gelu_gate(Tensor out, Tensor z, Tensor table, Tensor ids, long column) {
@@ -555,6 +563,7 @@ void register_latent(pybind11::module_& m) {
   m.def("rms_scale", &rms_scale);
   m.def("add_rms", &add_rms);
   m.def("rms_gate", &rms_gate);
+  m.def("row_squares", &row_squares);
   m.def("gelu_gate", &gelu_gate);
   m.def("latent_fits", &latent_fits);
   m.def("latent_rope_append", &latent_rope_append);

@@ -134,6 +134,17 @@ __global__ __launch_bounds__(256) void rms_gate_kernel(
   });
 }
 
+// ss[t] = sum of squares of row t
+__global__ __launch_bounds__(256) void row_squares_kernel(
+    float* __restrict__ ss, const float* __restrict__ x, int n) {
+  __shared__ float scratch[4];
+  const float* row = x + (long)blockIdx.x * n;
+  float s = 0.f;
+  for (int c = threadIdx.x; c < n; c += 256) s += row[c] * row[c];
+  s = block_reduce_sum_256(s, scratch);
+  if (threadIdx.x == 0) ss[blockIdx.x] = s;
+}
+
 // out[t, j] = gelu_tanh(z[t, j]) * table[ids[t], column + j]
 template <typename T, int V>
 __global__ __launch_bounds__(256) void gelu_gate_kernel(
@@ -215,6 +226,12 @@ void launch_rms_gate(T* y, const float* o, const T* g, const float* w,
   else
     rms_gate_kernel<T, 1><<<(unsigned)rows, 256, 0, stream>>>(
         y, o, g, w, ss, n, total, stride, eps);
+}
+
+void launch_row_squares(float* ss, const float* x, long rows, int n,
+                        hipStream_t stream) {
+  if (rows == 0) return;
+  row_squares_kernel<<<(unsigned)rows, 256, 0, stream>>>(ss, x, n);
 }
 
 template <typename T>

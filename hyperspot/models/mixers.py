@@ -409,7 +409,7 @@ class LightningAttention(nn.Module):
         o = hybrid.lightning_mix(q, k, v, self.decay, state, meta)
         ss = None
         if get_tp_size() > 1:          # the norm spans the heads of all ranks
-            ss = tensor_model_parallel_all_reduce(o.pow(2).sum(-1))
+            ss = tensor_model_parallel_all_reduce(hybrid.row_squares(o))
         return self.o_proj(hybrid.rms_gate(o, g, self.norm, self.eps, ss,
                                            self.spec.heads * self.spec.vdim))
 

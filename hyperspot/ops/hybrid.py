@@ -89,6 +89,15 @@ def rms_gate(o: torch.Tensor, g: torch.Tensor, w: torch.Tensor, eps: float,
     return y
 
 
+def row_squares(x: torch.Tensor) -> torch.Tensor:
+    """Sum of squares of every row of x [T, N] float."""
+    if not x.is_cuda:
+        return x.pow(2).sum(-1)
+    ss = torch.empty(x.shape[0], dtype=torch.float32, device=x.device)
+    _native().row_squares(ss, x)
+    return ss
+
+
 def gelu_gate(z: torch.Tensor, table: torch.Tensor, ids: torch.Tensor,
               column: int) -> torch.Tensor:
     """gelu_tanh(z) * table[ids, column : column + n] for z [T, n]."""

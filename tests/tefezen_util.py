@@ -96,9 +96,10 @@ def shapes(cfg):
     return out
 
 
-def weights(cfg, seed=0):
+def weights(cfg, seed=0, sharp=2.0):
     """bf16 weights under which single keys stand out: queries and latents
-    are scaled up, and the residual does not just follow the token."""
+    are scaled up (`sharp`), and the residual does not just follow the
+    token.  Rounding grows with `sharp` as well."""
     gen = torch.Generator().manual_seed(seed)
     out = {}
     for name, shape in shapes(cfg).items():
@@ -112,10 +113,32 @@ def weights(cfg, seed=0):
         elif name == "head":
             x = x / shape[1] ** 0.5
         elif name != "side.embed":
-            gain = 2.0 if name.endswith(("mix.q", "mix.uk", "router")) else 1.0
+            gain = sharp if name.endswith(("mix.q", "mix.uk", "router")) else 1.0
             x = gain * x / shape[1] ** 0.5
         out[name] = x.to(torch.bfloat16)
     return out
+
+
+def errors(got, want):
+    """Per-position RMS difference (mean removed), relative to the RMS of all
+    wanted logits."""
+    d = got.double() - want
+    d = d - d.mean(-1, keepdim=True)
+    return d.pow(2).mean(-1).sqrt() / want.pow(2).mean().sqrt()
+
+
+def rounding_limits(forward, cfg, w, toks, times=3.0):
+    """What 16-bit rounding may cost at every position: a multiple of the
+    plain implementation's answer to noise of that size on all weights (some
+    positions of a small random model amplify it a hundredfold)."""
+    want, worst = forward(cfg, w, toks)[0], 0.0
+    for seed in range(8):
+        g = torch.Generator().manual_seed(seed)
+        noisy = {n: t.double() * (1 + 2 ** -8.5 * torch.randn(
+            t.shape, generator=g, dtype=torch.float64)) for n, t in w.items()}
+        e = errors(forward(cfg, noisy, toks)[0], want)
+        worst = torch.maximum(e, torch.as_tensor(worst, dtype=e.dtype))
+    return times * worst.clamp_min(float(worst.mean()))
 
 
 def write(folder, cfg, w):
