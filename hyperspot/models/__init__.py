@@ -2,3 +2,4 @@ from .llama import LlamaForCausalLM
 from .mixtral import MixtralForCausalLM
 from .registry import build_model
 from .sumosun import SumosunForCausalLM
+from .tefezen import TefezenForCausalLM

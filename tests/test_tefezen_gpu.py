@@ -202,7 +202,7 @@ def attention_case(H, D, R, E, rank, window, starts, lens, dtype,
     return got, torch.stack(want)
 
 
-SIZES = [(2, 8, 8, 8, 16), (4, 64, 32, 64, 96), (3, 48, 16, 40, 72),
+SIZES = [(2, 8, 8, 8, 16), (5, 64, 32, 48, 104), (3, 48, 16, 40, 72),
          (16, 24, 8, 32, 128), (17, 16, 24, 128, 200), (2, 128, 64, 128, 512),
          (33, 32, 64, 16, 256), (1, 192, 64, 256, 512), (2, 96, 32, 256, 64),
          (3, 7, 6, 9, 11), (1, 1, 2, 1, 1), (2, 16, 80, 24, 600)]
