@@ -205,7 +205,7 @@ __global__ __launch_bounds__(256) void head_gemm_kernel(
   }
 }
 
-// ---- absorbed attention, any sizes ------------------------------------------
+// ---- absorbed attention, any sizes ----------------------------------------
 constexpr int TILE = 256;      // tokens per softmax step
 constexpr int MAX_RPT = 8;     // latent columns a thread: rank <= 2048
 
@@ -273,7 +273,7 @@ __global__ __launch_bounds__(256) void latent_attn_general_kernel(
       Elem<T>::st(out + (r * H + h) * rank + tid + 256 * i, acc[i] / l);
 }
 
-// ---- absorbed attention, matrix cores ---------------------------------------
+// ---- absorbed attention, matrix cores -------------------------------------
 // A workgroup has one row, HT tiles of 16 heads and every split-th tile of
 // KT tokens.  A tile is staged once in LDS (two buffers): the score product
 // reads it row by row, the value product reads its transpose with the
@@ -375,7 +375,8 @@ __global__ __launch_bounds__(256, 2) void latent_attn_decode_kernel(
     #pragma unroll
     for (int i = 0; i < LOADS; ++i) {
       if constexpr (EXACT)
-        kr[i] = *reinterpret_cast<const short8_t*>(src + (tid & 7) * 8 + 64 * i);
+        kr[i] = *reinterpret_cast<const short8_t*>(src + (tid & 7) * 8 +
+                                                   64 * i);
       else
         kr[i] = off[i] >= 0 ? *reinterpret_cast<const short8_t*>(src + off[i])
                             : short8_t{};
@@ -392,8 +393,8 @@ __global__ __launch_bounds__(256, 2) void latent_attn_decode_kernel(
     #pragma unroll
     for (int i = 0; i < LOADS; ++i)
       if ((tid & 7) + 8 * i < UPR)
-        *reinterpret_cast<short8_t*>(tile + tok * LS + (tid & 7) * 8 + 64 * i) =
-            kr[i];
+        *reinterpret_cast<short8_t*>(tile + tok * LS + (tid & 7) * 8 +
+                                     64 * i) = kr[i];
     __syncthreads();
     if (p0 + split * KT <= pos) fetch(p0 + split * KT);
     {
@@ -586,7 +587,7 @@ __global__ __launch_bounds__(256) void latent_merge_values_kernel(
   }
 }
 
-// ---- expanded attention, matrix cores ---------------------------------------
+// ---- expanded attention, matrix cores -------------------------------------
 // 128 query rows of one head a workgroup, 32 a wave; kv rows come in steps
 // of 64.  kn [n, H*D] unrotated keys, lat [n, rank + rot] with the rotated
 // part, vt [H*E, n] values transposed.  Row r of sequence s is the token at

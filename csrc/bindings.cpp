@@ -59,8 +59,8 @@ void launch_gla_chunk_gates(float*, const bf16*, const bf16*, const float*,
 void launch_mlstm_chunk_gates(float*, float*, const float*, const float*,
                               const float*, const int*, const int*, int, int,
                               float, hipStream_t);
-void launch_recurrent_chunk(Kind, bf16*, float*, float*, float*, float*, float*, float*,
-                            float*, const bf16*, const bf16*, const bf16*,
+void launch_recurrent_chunk(Kind, bf16*, float*, float*, float*, float*,
+                            float*, float*, float*, const bf16*, const bf16*, const bf16*,
                             const bf16*, const float*, const float*,
                             const float*, const int*, const long*,
                             const int*, const int*, const int*, int, int,
@@ -71,8 +71,8 @@ void launch_gla_decay(float*, const T*, const T*, const float*, long, int,
 void launch_mlstm_gates(float*, const float*, const float*, const float*,
                         long, int, float, hipStream_t);
 template <typename T>
-void launch_recurrent_scan(Kind, float*, float*, float*, float*, float*, const T*,
-                           const T*, const T*, const float*, const int*,
+void launch_recurrent_scan(Kind, float*, float*, float*, float*, float*,
+                           const T*, const T*, const T*, const float*, const int*,
                            const long*, const int*, int, int, int, int, long,
                            float, hipStream_t);
 template <typename T>
@@ -529,7 +529,8 @@ void recurrent_scan(torch::Tensor o, torch::Tensor S,
   by_dtype(q, [&](auto tag) {
     using T = ELEM(tag);
     launch_recurrent_scan<T>(
-        n.has_value() ? MLSTM : GLA, ptr<float>(o), ptr<float>(S), opt(n), opt(m), opt(nm_new), ptr<T>(q),
+        n.has_value() ? MLSTM : GLA, ptr<float>(o), ptr<float>(S), opt(n),
+        opt(m), opt(nm_new), ptr<T>(q),
         ptr<T>(k), ptr<T>(v), ptr<float>(gates), seq_start.data_ptr<int>(),
         positions.data_ptr<long>(), slots.data_ptr<int>(), (int)B, (int)d.H,
         (int)d.D, (int)d.E, st, (float)qscale, stream());
@@ -619,7 +620,8 @@ void recurrent_chunk(torch::Tensor y, torch::Tensor U,
     check_param(*info, nt * d.H * 2, "info");
   }
   launch_recurrent_chunk(
-      mlstm ? MLSTM : GLA, bf(y), nullptr, ptr<float>(U), opt(nU), opt(m_in), ptr<float>(S), opt(n),
+      mlstm ? MLSTM : GLA, bf(y), nullptr, ptr<float>(U), opt(nU),
+      opt(m_in), ptr<float>(S), opt(n),
       opt(m), cbf(q), cbf(k), cbf(v), cbf(g), ptr<float>(gates), opt(info),
       ptr<float>(w), seq_start.data_ptr<int>(), positions.data_ptr<long>(),
       slots.data_ptr<int>(), tiles.data_ptr<int>(),
@@ -679,7 +681,8 @@ void gla_step(torch::Tensor y, torch::Tensor S, torch::Tensor q,
   by_dtype(q, [&](auto tag) {
     using T = ELEM(tag);
     launch_recurrent_step<T>(
-        GLA, ptr<T>(y), nullptr, ptr<float>(S), nullptr, nullptr, ptr<T>(q), ptr<T>(k),
+        GLA, ptr<T>(y), nullptr, ptr<float>(S), nullptr, nullptr, ptr<T>(q),
+        ptr<T>(k),
         ptr<T>(v), ptr<T>(g), ptr<T>(a1h), ptr<T>(a2), ptr<float>(a2b),
         nullptr, nullptr, ptr<float>(w), positions.data_ptr<long>(),
         slots.data_ptr<int>(), rows, (int)d.H, (int)d.D, (int)d.E, (int)R,
@@ -703,7 +706,8 @@ void mlstm_step(torch::Tensor y, torch::Tensor S, torch::Tensor n,
   by_dtype(q, [&](auto tag) {
     using T = ELEM(tag);
     launch_recurrent_step<T>(
-        MLSTM, ptr<T>(y), nullptr, ptr<float>(S), ptr<float>(n), ptr<float>(m), ptr<T>(q),
+        MLSTM, ptr<T>(y), nullptr, ptr<float>(S), ptr<float>(n),
+        ptr<float>(m), ptr<T>(q),
         ptr<T>(k), ptr<T>(v), ptr<T>(g), nullptr, nullptr, ptr<float>(ib),
         ptr<float>(fb), ptr<float>(raw), ptr<float>(w),
         positions.data_ptr<long>(), slots.data_ptr<int>(), rows, (int)d.H,

@@ -78,7 +78,7 @@ bool aligned16(const Tensor& t) {
   return reinterpret_cast<uintptr_t>(t.data_ptr()) % 16 == 0;
 }
 
-// ---- residual ---------------------------------------------------------------
+// ---- residual -------------------------------------------------------------
 
 void embed_scaled(Tensor out, Tensor residual, Tensor table, Tensor ids,
                   double scale) {
@@ -169,7 +169,7 @@ void gelu_gate(Tensor out, Tensor z, Tensor table, Tensor ids, long column) {
   });
 }
 
-// ---- latent attention ---------------------------------------------------------
+// ---- latent attention -----------------------------------------------------
 
 struct LatentDims {
   long H, D, E, rank, rot;
@@ -411,7 +411,7 @@ void latent_attn_prefill(Tensor out, Tensor q, Tensor kn, Tensor lat,
       stream());
 }
 
-// ---- experts --------------------------------------------------------------------
+// ---- experts --------------------------------------------------------------
 
 // logits [T, E] or, with a shared expert, [T, E + 1]; true: shared
 bool check_route(const Tensor& weight, const Tensor& logits, long E,

@@ -153,7 +153,7 @@ __global__ __launch_bounds__(1024) void sort_kernel(
   }
 }
 
-// ---- products ---------------------------------------------------------------
+// ---- products -------------------------------------------------------------
 // UP:   out[p, f] = silu(x . w[e, f]) * (x . w[e, N + f]), x row order[p]/div
 // else: out[p, n] = x . w[e, n], x row p
 // w [E, UP ? 2N : N, K]; the shared expert (e == E) has ws, Ns, Ks.
@@ -288,7 +288,7 @@ __global__ __launch_bounds__(256) void experts_general_kernel(
   }
 }
 
-// ---- weighted sum, norm, residual -------------------------------------------
+// ---- weighted sum, norm, residual -----------------------------------------
 // h[t] = sum_k weight[t, k] y[place[t, k]]  (+ weight[t, n] shared[t])
 // without a residual out = h, otherwise residual += rms(h) * w and out = the
 // residual (null: none).  One workgroup a token.

@@ -96,7 +96,8 @@ __global__ __launch_bounds__(64) void recurrent_scan_kernel(
   for (int r = 0; r < RPL; ++r) {
     const int d = lane + 64 * r;
     nv[r] = 0.f;
-    if (K == MLSTM && !fresh && d < D) nv[r] = n_pool[((long)slot * H + h) * D + d];
+    if (K == MLSTM && !fresh && d < D)
+      nv[r] = n_pool[((long)slot * H + h) * D + d];
     #pragma unroll
     for (int c = 0; c < COLS; ++c)
       st[r][c] = (!fresh && d < D && e0 + c < E)

@@ -113,8 +113,9 @@ def weights(cfg, seed=0, sharp=2.0):
         elif name == "head":
             x = x / shape[1] ** 0.5
         elif name != "side.embed":
-            gain = sharp if name.endswith(("mix.q", "mix.uk", "router")) else 1.0
-            x = gain * x / shape[1] ** 0.5
+            x = x / shape[1] ** 0.5
+            if name.endswith(("mix.q", "mix.uk", "router")):
+                x = sharp * x
         out[name] = x.to(torch.bfloat16)
     return out
 
