@@ -944,6 +944,7 @@ void moe_gemm_fp8(torch::Tensor out, torch::Tensor xq, torch::Tensor xs,
 }
 
 void register_latent(pybind11::module_& m);    // bindings_latent.cpp
+void register_sublayer(pybind11::module_& m);  // bindings_sublayer.cpp
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.doc() = "HyperSpot-AMD gfx950 (CDNA4) kernels";
@@ -982,6 +983,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("lightning_scan", &lightning_scan);
   m.def("lightning_chunk", &lightning_chunk);
   register_latent(m);
+  register_sublayer(m);
   m.def("greedy_sample", &greedy_sample);
   m.def("inv_cdf_sample", &inv_cdf_sample);
 }

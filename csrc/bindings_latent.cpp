@@ -46,19 +46,20 @@ void launch_latent_attn_prefill(bf16*, const bf16*, const bf16*, const bf16*,
                                 int, int, int, int, long, int, float, long,
                                 hipStream_t);
 void launch_experts_route(float*, int*, const float*, int, int, int, bool,
-                          bool, hipStream_t);
+                          bool, int, const float*, hipStream_t);
 void launch_experts_sort(int*, int*, int*, const int*, int, int, int, int,
                          hipStream_t);
 void launch_experts_route_sort(float*, int*, int*, int*, int*, const float*,
-                               int, int, int, bool, int, int, hipStream_t);
+                               int, int, int, bool, int, int, int,
+                               const float*, hipStream_t);
 template <typename T>
 void launch_experts_gemm(bool, T*, const T*, const T*, const T*, const int*,
                          const int*, int, int, int, int, int, int, int, long,
-                         long, int, hipStream_t);
+                         long, int, bool, float, hipStream_t);
 template <typename T>
-void launch_experts_sum(T*, float*, const T*, const T*, const float*,
-                        const int*, const float*, long, int, int, float,
-                        hipStream_t);
+void launch_experts_sum(T*, float*, const T*, const T*, const T*,
+                        const float*, const int*, const float*, long, int,
+                        int, float, hipStream_t);
 
 namespace {
 
@@ -80,17 +81,20 @@ bool aligned16(const Tensor& t) {
 
 // ---- residual -------------------------------------------------------------
 
-void embed_scaled(Tensor out, Tensor residual, Tensor table, Tensor ids,
+void embed_scaled(Maybe out, Tensor residual, Tensor table, Tensor ids,
                   double scale) {
   const long rows = ids.numel(), width = table.size(1);
   check(table, table.scalar_type(), "table");
-  check(out, table.scalar_type(), "out");
   check(ids, torch::kInt64, "ids");
   check_param(residual, rows * width, "residual");
-  TORCH_CHECK(out.numel() == rows * width, "embed_scaled: out");
+  if (out.has_value()) {
+    check(*out, table.scalar_type(), "out");
+    TORCH_CHECK(out->numel() == rows * width, "embed_scaled: out");
+  }
   by_dtype(table, [&](auto tag) {
     using T = ELEM(tag);
-    T* o = out.data_ptr() == residual.data_ptr() ? nullptr : ptr<T>(out);
+    T* o = !out.has_value() || out->data_ptr() == residual.data_ptr()
+        ? nullptr : ptr<T>(*out);
     launch_embed_scaled<T>(o, ptr<float>(residual), ptr<T>(table),
                            ids.data_ptr<long>(), (float)scale, rows,
                            (int)width, table.size(0), stream());
@@ -413,26 +417,32 @@ void latent_attn_prefill(Tensor out, Tensor q, Tensor kn, Tensor lat,
 
 // ---- experts --------------------------------------------------------------
 
-// logits [T, E] or, with a shared expert, [T, E + 1]; true: shared
-bool check_route(const Tensor& weight, const Tensor& logits, long E,
-                 long top) {
+// logits [T, N] or, with a shared expert, [T, N + 1], N = E + identity; true:
+// shared
+bool check_route(const Tensor& weight, const Tensor& logits, long E, long top,
+                 const Maybe& correction, long identity) {
   check(logits, torch::kFloat32, "logits");
   TORCH_CHECK(logits.dim() == 2, "experts: logits");
-  const long T = logits.size(0), extra = logits.size(1) - E;
+  const long N = E + identity;
+  const long T = logits.size(0), extra = logits.size(1) - N;
   TORCH_CHECK(extra == 0 || extra == 1, "experts: logits");
-  TORCH_CHECK(E >= 1 && E <= 1024 && top >= 1 && top <= 63 && top <= E,
+  TORCH_CHECK(E >= 1 && identity >= 0 && N <= 1024 && top >= 1 && top <= 63 &&
+                  top <= N,
               "experts: at most 1024 experts, of which at most 63 at once");
+  if (correction.has_value()) check_param(*correction, N, "correction");
   check_param(weight, T * (top + extra), "weight");
   return extra == 1;
 }
 
-void experts_route(Tensor weight, Tensor ids, Tensor logits, long E,
-                   long top) {
-  const bool shared = check_route(weight, logits, E, top);
+void experts_route(Tensor weight, Tensor ids, Tensor logits, long E, long top,
+                   Maybe correction, long identity) {
+  const bool shared = check_route(weight, logits, E, top, correction,
+                                  identity);
   check_ints(ids, logits.size(0) * top, "ids");
   launch_experts_route(ptr<float>(weight), ids.data_ptr<int>(),
                        ptr<float>(logits), (int)logits.size(0), (int)E,
-                       (int)top, shared, false, stream());
+                       (int)top, shared, false, (int)identity,
+                       opt(correction), stream());
 }
 
 void check_sorted(const Tensor& order, const Tensor& expert,
@@ -458,9 +468,10 @@ void experts_sort(Tensor order, Tensor expert, Tensor place, Tensor ids,
 }
 
 void experts_route_sort(Tensor weight, Tensor ids, Tensor place, Tensor order,
-                        Tensor expert, Tensor logits, long E, long top,
-                        long bm) {
-  const bool shared = check_route(weight, logits, E, top);
+                        Tensor expert, Tensor logits, long bm, long E,
+                        long top, Maybe correction, long identity) {
+  const bool shared = check_route(weight, logits, E, top, correction,
+                                  identity);
   const long T = logits.size(0), choices = T * (top + shared);
   check_ints(ids, choices, "ids");
   check_sorted(order, expert, place, choices, E + shared, bm);
@@ -468,12 +479,13 @@ void experts_route_sort(Tensor weight, Tensor ids, Tensor place, Tensor order,
       ptr<float>(weight), ids.data_ptr<int>(), place.data_ptr<int>(),
       order.data_ptr<int>(), expert.data_ptr<int>(), ptr<float>(logits),
       (int)T, (int)E, (int)top, shared, (int)bm, (int)expert.numel(),
-      stream());
+      (int)identity, opt(correction), stream());
 }
 
 void experts_gemm(bool up, const Tensor& out, const Tensor& x,
                   const Tensor& w, const Maybe& ws, const Tensor& order,
-                  const Tensor& expert, long div, long bm) {
+                  const Tensor& expert, long div, c10::optional<double> limit,
+                  long bm) {
   const auto dt = x.scalar_type();
   check(out, dt, "out");
   check(x, dt, "x");
@@ -510,22 +522,25 @@ void experts_gemm(bool up, const Tensor& out, const Tensor& x,
                            order.data_ptr<int>(), expert.data_ptr<int>(),
                            (int)tiles, (int)E, (int)N, (int)K, (int)Ns,
                            (int)Ks, (int)div, x.size(1), out.size(1), (int)bm,
+                           limit.has_value(), (float)limit.value_or(0.),
                            stream());
   });
 }
 
 void experts_up(Tensor h, Tensor x, Tensor w, Maybe ws, Tensor order,
-                Tensor expert, long div, long bm) {
-  experts_gemm(true, h, x, w, ws, order, expert, div, bm);
+                Tensor expert, long div, c10::optional<double> limit,
+                long bm) {
+  experts_gemm(true, h, x, w, ws, order, expert, div, limit, bm);
 }
 
 void experts_down(Tensor y, Tensor h, Tensor w, Maybe ws, Tensor order,
                   Tensor expert, long bm) {
-  experts_gemm(false, y, h, w, ws, order, expert, 1, bm);
+  experts_gemm(false, y, h, w, ws, order, expert, 1, c10::nullopt, bm);
 }
 
 void experts_sum(Tensor out, Tensor y, Tensor place, Tensor weight,
-                 Maybe shared, Maybe residual, Maybe w, double eps) {
+                 Maybe shared, Maybe identity, Maybe residual, Maybe w,
+                 double eps) {
   const auto dt = y.scalar_type();
   check(y, dt, "y");
   check(out, dt, "out");
@@ -539,6 +554,10 @@ void experts_sum(Tensor out, Tensor y, Tensor place, Tensor weight,
     check(*shared, dt, "shared");
     TORCH_CHECK(shared->numel() == rows * width, "experts_sum: shared");
   }
+  if (identity.has_value()) {
+    check(*identity, dt, "identity");
+    TORCH_CHECK(identity->numel() == rows * width, "experts_sum: identity");
+  }
   if (residual.has_value()) {
     check_param(*residual, rows * width, "residual");
     TORCH_CHECK(w.has_value(), "experts_sum: norm weight");
@@ -550,9 +569,10 @@ void experts_sum(Tensor out, Tensor y, Tensor place, Tensor weight,
         ? nullptr : ptr<T>(out);
     launch_experts_sum<T>(
         o, opt(residual), ptr<T>(y),
-        shared.has_value() ? ptr<T>(*shared) : nullptr, ptr<float>(weight),
-        place.data_ptr<int>(), opt(w), rows, (int)n, (int)width, (float)eps,
-        stream());
+        shared.has_value() ? ptr<T>(*shared) : nullptr,
+        identity.has_value() ? ptr<T>(*identity) : nullptr,
+        ptr<float>(weight), place.data_ptr<int>(), opt(w), rows, (int)n,
+        (int)width, (float)eps, stream());
   });
 }
 
@@ -574,7 +594,10 @@ void register_latent(pybind11::module_& m) {
   m.def("latent_attn_decode", &latent_attn_decode);
   m.def("latent_merge_values", &latent_merge_values);
   m.def("latent_attn_prefill", &latent_attn_prefill);
-  m.def("experts_route", &experts_route);
+  namespace py = pybind11;
+  m.def("experts_route", &experts_route, py::arg("weight"), py::arg("ids"),
+        py::arg("logits"), py::arg("E"), py::arg("top"),
+        py::arg("correction") = py::none(), py::arg("identity") = 0);
   m.def("experts_sort", &experts_sort);
   m.def("experts_route_sort", &experts_route_sort);
   m.def("experts_up", &experts_up);

@@ -115,6 +115,14 @@ template <> struct Fn<float> {
   static DEV float tanh(float x) { return tanhf(x); }
 };
 
+// clamped gated unit: g sigmoid(1.702 g) (u + 1) with g = min(gate, limit) and
+// u clamped to +-limit
+template <typename T> DEV float clamped_unit(float g, float u, float limit) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g / (1.f + Fn<T>::exp(-1.702f * g)) * (u + 1.f);
+}
+
 // log(sigmoid(z)) without overflow for either sign of z
 DEV float log_sigmoid(float z) {
   return fminf(z, 0.f) - log1pf(expf(-fabsf(z)));

@@ -1,14 +1,19 @@
-// Mixture of gated-SiLU experts with an optional shared expert (gfx950).
+// Mixture of gated experts with an optional shared expert (gfx950).
 //
-//   route   router logits -> chosen experts, softmax over the chosen, sigmoid
-//           of the shared expert's gate
+//   route   router logits -> chosen experts and their weights: the softmax
+//           over the chosen, or with a correction the softmax over all, the
+//           correction added for the choice only; sigmoid of the shared
+//           expert's gate.  Outputs after the E experts are identity experts
+//           (choice -1)
 //   sort    choices by expert, in tiles of `bm` rows; for few tokens routing
 //           and sorting are one kernel.  The shared expert may be expert
 //           number E, chosen by every token
-//   up      h = silu(x W_gate) * (x W_up) of every choice
+//   up      h = silu(x W_gate) * (x W_up) of every choice, or the clamped
+//           g sigmoid(1.702 g) (u + 1)
 //   down    y = h W_down of every choice
 //   sum     weighted sum of a token's choices, and either the sum itself or
-//           its RMS norm added to the float residual
+//           its RMS norm added to the float residual; or the whole step to
+//           the next sublayer's input (sublayer.h)
 //
 // Every grid depends on shapes only.  up and down stream each expert's
 // weights once per tile: weights are the A operand straight from memory, the
@@ -18,23 +23,51 @@
 
 #include <algorithm>
 
-#include "common.h"
+#include "sublayer.h"
 
 namespace {
 
 constexpr int ROUTE_TOGETHER = 64;   // tokens routed by the sorting workgroup
 
-// One wave: the `top` <= 64 largest of E <= 64 * LE logits by repeated
-// maximum, lowest index first among equals; a logit that is not a number
-// ranks last.  Lane k returns choice k (-1: none) and its weight.
+struct Route {
+  float* weight;           // [T, n]
+  int* ids;                // [T, n] or null
+  const float* logits;     // [T, N (+ 1)], N = E + identity
+  int T, E, top, shared;   // n = top + shared where ids has the shared expert
+  int with_shared;         // ids lists the shared expert
+  int N;
+  const float* correction; // [N] or null
+};
+
+// One wave: the `top` <= 64 largest of N <= 64 * LE logits (or corrected
+// shares) by repeated maximum, lowest index first among equals; a logit that
+// is not a number ranks last.  Lane k returns choice k (-1: an identity
+// expert) and its weight.
 template <int LE>
-DEV void route_token(const float* z, int E, int top, bool shared, int* id,
-                     float* weight) {
-  const int lane = threadIdx.x & 63;
-  float v[LE];
+DEV void route_token(const Route& r, const float* z, int* id, float* weight) {
+  const int lane = threadIdx.x & 63, E = r.N, top = r.top;
+  float v[LE], share[LE];
   #pragma unroll
   for (int i = 0; i < LE; ++i)       // the maximum drops NaN
     v[i] = lane + 64 * i < E ? fmaxf(z[lane + 64 * i], -FLT_MAX) : 0.f;
+  if (r.correction) {
+    float mx = -FLT_MAX, sum = 0.f;
+    #pragma unroll
+    for (int i = 0; i < LE; ++i)
+      if (lane + 64 * i < E) mx = fmaxf(mx, v[i]);
+    mx = wave_reduce_max(mx);
+    #pragma unroll
+    for (int i = 0; i < LE; ++i) {
+      share[i] = lane + 64 * i < E ? expf(v[i] - mx) : 0.f;
+      sum += share[i];
+    }
+    sum = wave_reduce_sum(sum);
+    #pragma unroll
+    for (int i = 0; i < LE; ++i) {
+      share[i] /= sum;
+      if (lane + 64 * i < E) v[i] = share[i] + r.correction[lane + 64 * i];
+    }
+  }
   unsigned taken = 0;
   float first = 0.f;
   *id = -1;
@@ -61,33 +94,31 @@ DEV void route_token(const float* z, int E, int top, bool shared, int* id,
     }
     if ((at & 63) == lane) taken |= 1u << (at >> 6);
     if (k == 0) first = best;
+    float s = 0.f;
+    if (r.correction) {
+      #pragma unroll
+      for (int i = 0; i < LE; ++i)
+        if (at >> 6 == i) s = share[i];
+      s = __shfl(s, at & 63);
+    }
     if (lane == k) {
-      *id = at;
-      *weight = expf(best - first);
+      *id = at < r.E ? at : -1;
+      *weight = r.correction ? s : expf(best - first);
     }
   }
-  *weight /= wave_reduce_sum(*weight);
-  if (shared && lane == top) {
-    *id = E;
+  if (!r.correction) *weight /= wave_reduce_sum(*weight);
+  if (r.shared && lane == top) {
+    *id = r.E;
     *weight = 1.f / (1.f + expf(-z[E]));
   }
 }
-
-struct Route {
-  float* weight;           // [T, n]
-  int* ids;                // [T, n] or null
-  const float* logits;     // [T, E (+ 1)]
-  int T, E, top, shared;   // n = top + shared where ids has the shared expert
-  int with_shared;         // ids lists the shared expert
-};
 
 template <int LE>
 DEV void route_row(const Route& r, int t) {
   const int lane = threadIdx.x & 63, n = r.top + r.shared;
   int id;
   float w;
-  route_token<LE>(r.logits + (long)t * (r.E + r.shared), r.E, r.top,
-                  r.shared != 0, &id, &w);
+  route_token<LE>(r, r.logits + (long)t * (r.N + r.shared), &id, &w);
   if (lane < n) r.weight[(long)t * n + lane] = w;
   const int m = r.top + r.with_shared;
   if (lane < m) r.ids[(long)t * m + lane] = id;
@@ -100,7 +131,8 @@ __global__ __launch_bounds__(256) void route_kernel(Route r) {
 }
 
 // One workgroup.  order[pos] = choice (-1: padding), expert[tile] (-1: none),
-// place[choice] = pos.  ROUTE: the choices are made here first.
+// place[choice] = pos (-1: an identity expert).  ROUTE: the choices are made
+// here first.
 template <int LE, bool ROUTE>
 __global__ __launch_bounds__(1024) void sort_kernel(
     Route r, int* __restrict__ order, int* __restrict__ expert,
@@ -118,7 +150,8 @@ __global__ __launch_bounds__(1024) void sort_kernel(
     for (int t = wid; t < r.T; t += 16) route_row<LE>(r, t);
   __threadfence_block();
   __syncthreads();
-  for (int p = tid; p < choices; p += 1024) atomicAdd(&cnt[ids[p]], 1);
+  for (int p = tid; p < choices; p += 1024)
+    if (ids[p] >= 0) atomicAdd(&cnt[ids[p]], 1);
   __syncthreads();
   // exclusive sums of tiles: kinds <= 1024 + 1, one or two a thread
   int base = 0;
@@ -147,14 +180,14 @@ __global__ __launch_bounds__(1024) void sort_kernel(
     __syncthreads();
   }
   for (int p = tid; p < choices; p += 1024) {
-    const int pos = atomicAdd(&cur[ids[p]], 1);
-    order[pos] = p;
+    const int pos = ids[p] < 0 ? -1 : atomicAdd(&cur[ids[p]], 1);
+    if (pos >= 0) order[pos] = p;
     place[p] = pos;
   }
 }
 
 // ---- products -------------------------------------------------------------
-// UP:   out[p, f] = silu(x . w[e, f]) * (x . w[e, N + f]), x row order[p]/div
+// UP:   out[p, f] = act(x . w[e, f], x . w[e, N + f]), x row order[p]/div
 // else: out[p, n] = x . w[e, n], x row p
 // w [E, UP ? 2N : N, K]; the shared expert (e == E) has ws, Ns, Ks.
 struct Grouped {
@@ -162,7 +195,14 @@ struct Grouped {
   const int* expert;
   int E, N, K, Ns, Ks, div;
   long xs, os;                       // row strides of x and out
+  int clamped;
+  float limit;
 };
+
+template <typename T> DEV float gate_act(const Grouped& a, float g, float u) {
+  return a.clamped ? clamped_unit<T>(g, u, a.limit)
+                   : g / (1.f + Fn<T>::exp(-g)) * u;
+}
 
 template <int CT, int NA, bool UP>
 __global__ __launch_bounds__(256) void experts_rows_kernel(
@@ -252,7 +292,7 @@ __global__ __launch_bounds__(256) void experts_rows_kernel(
     if constexpr (UP) {
       const f32x4_t z = total(i + NA / 2, t);
       #pragma unroll
-      for (int j = 0; j < 4; ++j) y[j] = y[j] / (1.f + __expf(-y[j])) * z[j];
+      for (int j = 0; j < 4; ++j) y[j] = gate_act<bf16>(a, y[j], z[j]);
     }
     *reinterpret_cast<uint2*>(out + p * a.os + n) =
         uint2{cvt_pk_bf16(y[0], y[1]), cvt_pk_bf16(y[2], y[3])};
@@ -282,39 +322,54 @@ __global__ __launch_bounds__(256) void experts_general_kernel(
     s = wave_reduce_sum(s);
     if constexpr (UP) {
       z = wave_reduce_sum(z);
-      s = s / (1.f + Fn<T>::exp(-s)) * z;
+      s = gate_act<T>(a, s, z);
     }
     if (lane == 0) Elem<T>::st(out + p * a.os + n, s);
   }
 }
 
 // ---- weighted sum, norm, residual -----------------------------------------
-// h[t] = sum_k weight[t, k] y[place[t, k]]  (+ weight[t, n] shared[t])
-// without a residual out = h, otherwise residual += rms(h) * w and out = the
-// residual (null: none).  One workgroup a token.
-template <typename T, int V>
-__global__ __launch_bounds__(256) void experts_sum_kernel(
-    T* __restrict__ out, float* __restrict__ residual,
-    const T* __restrict__ y, const T* __restrict__ shared,
-    const float* __restrict__ weight, const int* __restrict__ place,
-    const float* __restrict__ w, int n, int width, float eps) {
-  constexpr int HELD = 4;
-  __shared__ float scratch[4];
-  const long t = blockIdx.x, at = t * width;
-  const int tid = threadIdx.x, nw = n + (shared ? 1 : 0);
-  auto value = [&](int c, float* h) {
+// h[t] = sum_k weight[t, k] y[place[t, k]]  (+ weight[t, n] shared[t]), with
+// identity[t] where place is -1 (null: that part is added elsewhere)
+template <typename T> struct Sum {
+  const T* y;
+  const T* shared;
+  const T* identity;
+  const float* weight;
+  const int* place;
+  int n, width;
+
+  template <int V> DEV void value(long t, int c, float* h) const {
+    const int nw = n + (shared ? 1 : 0);
     #pragma unroll
     for (int i = 0; i < V; ++i) h[i] = 0.f;
     for (int k = 0; k < nw; ++k) {
-      const T* row = k < n ? y + (long)place[t * n + k] * width
-                           : shared + at;
+      const T* row = shared + t * width;
+      if (k < n) {
+        const int p = place[t * n + k];
+        if (p < 0 && !identity) continue;
+        row = p < 0 ? identity + t * width : y + (long)p * width;
+      }
       const float wk = weight[t * nw + k];
       float f[V];
       load_vec<T, V>(row + c, f);
       #pragma unroll
       for (int i = 0; i < V; ++i) h[i] += wk * f[i];
     }
-  };
+  }
+};
+
+// without a residual out = h, otherwise residual += rms(h) * w and out = the
+// residual (null: none).  One workgroup a token.
+template <typename T, int V>
+__global__ __launch_bounds__(256) void experts_sum_kernel(
+    T* __restrict__ out, float* __restrict__ residual, Sum<T> s,
+    const float* __restrict__ w, float eps) {
+  constexpr int HELD = 4;
+  __shared__ float scratch[4];
+  const int tid = threadIdx.x, width = s.width;
+  const long t = blockIdx.x, at = t * width;
+  auto value = [&](int c, float* h) { s.template value<V>(t, c, h); };
   if (!residual) {
     for (int c = tid * V; c < width; c += 256 * V) {
       float h[V];
@@ -362,19 +417,32 @@ __global__ __launch_bounds__(256) void experts_sum_kernel(
   }
 }
 
+template <typename T, int V>
+__global__ __launch_bounds__(256) void experts_sum_next_kernel(Between<T> a,
+                                                               Sum<T> s) {
+  __shared__ float scratch[4];
+  const long t = blockIdx.x;
+  between_sublayers<T, V, true>(a, t, scratch, [&](int c, float* x) {
+    s.template value<V>(t, c, x);
+  });
+}
+
 }  // namespace
 
 #define BY_EXPERTS(RUN)                                                     \
-  if (r.E <= 64) RUN(1);                                                    \
-  else if (r.E <= 256) RUN(4);                                              \
+  if (r.N <= 64) RUN(1);                                                    \
+  else if (r.N <= 256) RUN(4);                                              \
   else RUN(16)
 
-// ids lists [T, top] or, with_shared, [T, top + 1]; E <= 1024, top <= 63
+// ids lists [T, top] or, with_shared, [T, top + 1]; at most 1024 outputs,
+// top <= 63
 void launch_experts_route(float* weight, int* ids, const float* logits, int T,
                           int E, int top, bool shared, bool with_shared,
+                          int identity, const float* correction,
                           hipStream_t stream) {
   if (T == 0) return;
-  const Route r{weight, ids, logits, T, E, top, shared, with_shared};
+  const Route r{weight, ids, logits, T, E, top, shared, with_shared,
+                E + identity, correction};
   #define RUN(LE)                                                           \
     route_kernel<LE><<<(unsigned)((T + 3) / 4), 256, 0, stream>>>(r)
   BY_EXPERTS(RUN);
@@ -391,17 +459,19 @@ void launch_experts_sort(int* order, int* expert, int* place, const int* ids,
 void launch_experts_route_sort(float* weight, int* ids, int* place,
                                int* order, int* expert, const float* logits,
                                int T, int E, int top, bool shared, int bm,
-                               int tiles, hipStream_t stream) {
+                               int tiles, int identity,
+                               const float* correction, hipStream_t stream) {
   if (T == 0) return;
   const int kinds = E + shared, choices = T * (top + shared);
   if (T > ROUTE_TOGETHER) {
     launch_experts_route(weight, ids, logits, T, E, top, shared, shared,
-                         stream);
+                         identity, correction, stream);
     launch_experts_sort(order, expert, place, ids, choices, kinds, bm, tiles,
                         stream);
     return;
   }
-  const Route r{weight, ids, logits, T, E, top, shared, shared};
+  const Route r{weight, ids, logits, T, E, top, shared, shared, E + identity,
+                correction};
   #define RUN(LE)                                                           \
     sort_kernel<LE, true><<<1, 1024, 2 * kinds * sizeof(int), stream>>>(    \
         r, order, expert, place, ids, choices, kinds, bm, tiles)
@@ -414,9 +484,10 @@ template <typename T>
 void launch_experts_gemm(bool up, T* out, const T* x, const T* w, const T* ws,
                          const int* order, const int* expert, int tiles,
                          int E, int N, int K, int Ns, int Ks, int div,
-                         long xs, long os, int bm, hipStream_t stream) {
+                         long xs, long os, int bm, bool clamped, float limit,
+                        hipStream_t stream) {
   if (tiles == 0) return;
-  const Grouped a{order, expert, E, N, K, Ns, Ks, div, xs, os};
+  const Grouped a{order, expert, E, N, K, Ns, Ks, div, xs, os, clamped, limit};
   const int n = std::max(N, Ns);
   if (bm == 1) {
     const dim3 grid((unsigned)tiles, (unsigned)((n + 63) / 64));
@@ -452,25 +523,43 @@ void launch_experts_gemm(bool up, T* out, const T* x, const T* w, const T* ws,
 
 template <typename T>
 void launch_experts_sum(T* out, float* residual, const T* y, const T* shared,
-                        const float* weight, const int* place, const float* w,
-                        long rows, int n, int width, float eps,
-                        hipStream_t stream) {
+                        const T* identity, const float* weight,
+                        const int* place, const float* w, long rows, int n,
+                        int width, float eps, hipStream_t stream) {
   if (rows == 0) return;
+  const Sum<T> s{y, shared, identity, weight, place, n, width};
   if (width % 4 == 0)
     experts_sum_kernel<T, 4><<<(unsigned)rows, 256, 0, stream>>>(
-        out, residual, y, shared, weight, place, w, n, width, eps);
+        out, residual, s, w, eps);
   else
     experts_sum_kernel<T, 1><<<(unsigned)rows, 256, 0, stream>>>(
-        out, residual, y, shared, weight, place, w, n, width, eps);
+        out, residual, s, w, eps);
+}
+
+template <typename T>
+void launch_experts_sum_next(const Between<T>& a, const T* y, const T* shared,
+                             const T* identity, const float* weight,
+                             const int* place, long rows, int n,
+                             hipStream_t stream) {
+  if (rows == 0) return;
+  const Sum<T> s{y, shared, identity, weight, place, n, a.width};
+  if (a.width % 4 == 0)
+    experts_sum_next_kernel<T, 4><<<(unsigned)rows, 256, 0, stream>>>(a, s);
+  else
+    experts_sum_next_kernel<T, 1><<<(unsigned)rows, 256, 0, stream>>>(a, s);
 }
 
 #define INSTANTIATE(T)                                                      \
   template void launch_experts_gemm<T>(                                     \
       bool, T*, const T*, const T*, const T*, const int*, const int*, int,  \
-      int, int, int, int, int, int, long, long, int, hipStream_t);          \
+      int, int, int, int, int, int, long, long, int, bool, float,           \
+      hipStream_t);                                                         \
   template void launch_experts_sum<T>(                                      \
-      T*, float*, const T*, const T*, const float*, const int*,             \
-      const float*, long, int, int, float, hipStream_t);
+      T*, float*, const T*, const T*, const T*, const float*, const int*,   \
+      const float*, long, int, int, float, hipStream_t);                    \
+  template void launch_experts_sum_next<T>(                                 \
+      const Between<T>&, const T*, const T*, const T*, const float*,        \
+      const int*, long, int, hipStream_t);
 INSTANTIATE(bf16)
 INSTANTIATE(float)
 #undef INSTANTIATE

@@ -310,37 +310,52 @@ class RecurrentState(NamedTuple):
     m: Optional[torch.Tensor] = None
 
 
+class LayerCache(NamedTuple):
+    """A layer with input convolutions: its mixer's cache, and per sublayer
+    the last inputs [slots, rows, width], indexed like a recurrent state."""
+
+    mixer: object
+    tails: tuple
+
+
 def allocate_caches(spec, config, num_blocks: int, num_slots: int,
                     dtype: torch.dtype, device) -> list:
     """Per-layer caches following the model's layout."""
-    from .layer_spec import LatentPages, SharedCache, StateSlots
+    from .layer_spec import LatentPages, MixerAndTails, SharedCache, StateSlots
     layout = spec.cache_layout(max(config.tp_size, 1))
     bs = config.block_size
     caches = []
-    for c in layout:
+
+    def part(c):
+        if isinstance(c, MixerAndTails):
+            return LayerCache(part(c.mixer), tuple(
+                torch.zeros(num_slots, t.rows, t.width, dtype=dtype,
+                            device=device) for t in c.tails))
         if isinstance(c, SharedCache):
-            caches.append(caches[c.layer])
-        elif isinstance(c, LatentPages):
-            caches.append(LatentKV(torch.zeros(num_blocks, bs, c.width,
-                                               dtype=dtype, device=device)))
-        elif isinstance(c, StateSlots):
+            owner = caches[c.layer]
+            return owner.mixer if isinstance(owner, LayerCache) else owner
+        if isinstance(c, LatentPages):
+            return LatentKV(torch.zeros(num_blocks, bs, c.width, dtype=dtype,
+                                        device=device))
+        if isinstance(c, StateSlots):
             z = lambda *shape: torch.zeros(num_slots, *shape,
                                            dtype=torch.float32, device=device)
-            caches.append(
-                RecurrentState(z(c.heads, c.dim, c.vdim),
-                               z(c.heads, c.dim), z(c.heads))
-                if c.normalizer
-                else RecurrentState(z(c.heads, c.dim, c.vdim)))
-        elif c.v_transposed:
-            caches.append(KVPages(
+            return RecurrentState(z(c.heads, c.dim, c.vdim),
+                                  z(c.heads, c.dim), z(c.heads)) \
+                if c.normalizer \
+                else RecurrentState(z(c.heads, c.dim, c.vdim))
+        if c.v_transposed:
+            return KVPages(
                 torch.zeros(num_blocks, c.kv_heads, bs, c.k_dim,
                             dtype=dtype, device=device),
                 torch.zeros(num_blocks, c.kv_heads, c.v_dim, bs,
-                            dtype=dtype, device=device)))
-        else:
-            assert c.k_dim == c.v_dim, c
-            caches += allocate_kv_caches(1, num_blocks, c.kv_heads, bs,
-                                         c.k_dim, dtype, device)
+                            dtype=dtype, device=device))
+        assert c.k_dim == c.v_dim, c
+        return allocate_kv_caches(1, num_blocks, c.kv_heads, bs, c.k_dim,
+                                  dtype, device)[0]
+
+    for c in layout:
+        caches.append(part(c))
     return caches
 
 
@@ -353,15 +368,15 @@ def compute_num_gpu_blocks(spec, config, device, safety_frac: float = None,
     frac = safety_frac if safety_frac is not None else config.gpu_memory_utilization
     if device == "cpu" or (hasattr(device, "type") and device.type == "cpu"):
         return 512
-    from .layer_spec import StateSlots
+    from .layer_spec import ConvTail, StateSlots, cache_parts
     free, total = torch.cuda.mem_get_info(device)
     budget = int(total * frac) - (total - free)
     elem_bytes = 1 if getattr(config, "kv_dtype", "bfloat16") == "fp8" \
         else 4 if config.dtype == "float32" else 2
     per_block = 0
-    for c in spec.cache_layout(max(config.tp_size, 1)):
-        if isinstance(c, StateSlots):
-            budget -= num_slots * c.bytes_per_slot()
+    for c in cache_parts(spec.cache_layout(max(config.tp_size, 1))):
+        if isinstance(c, (StateSlots, ConvTail)):
+            budget -= num_slots * c.bytes_per_slot(elem_bytes)
         else:
             per_block += config.block_size * c.bytes_per_token(elem_bytes)
     if budget <= 0:

@@ -1,16 +1,17 @@
 """Per-layer descriptions for models whose layers are not all alike.
 
 A ``HybridSpec`` is a ``ModelSpec`` with an explicit list of layers, each one
-mixer (windowed differential attention, windowed latent attention, gated
-linear attention, matrix LSTM, lightning attention) and an optional
-feed-forward (dense, or a mixture of experts).  Every size and constant of a
-layer part is a field here; the layer classes in ``hyperspot.models.mixers``
-read nothing else.
+mixer (windowed differential attention, windowed latent attention, chunked
+sigmoid attention, gated linear attention, matrix LSTM, lightning attention)
+and an optional feed-forward (dense, or a mixture of experts).  Every size and
+constant of a layer part is a field here; the layer classes in
+``hyperspot.models.mixers`` read nothing else.
 
 ``cache_layout`` tells the cache manager what a layer keeps per sequence:
 pages that grow with the tokens (``PagedKV``, ``LatentPages``), a fixed-size
-recurrent state (``StateSlots``), or nothing of its own (``SharedCache``), all
-already divided over the tensor-parallel ranks.
+recurrent state (``StateSlots``), the last inputs of a convolution
+(``ConvTail``), or nothing of its own (``SharedCache``), all already divided
+over the tensor-parallel ranks.
 """
 
 from __future__ import annotations
@@ -68,11 +69,40 @@ class StateSlots:
     vdim: int
     normalizer: bool = False
 
-    def bytes_per_slot(self) -> int:
+    def bytes_per_slot(self, elem: int = 4) -> int:
         n = self.heads * self.dim * self.vdim
         if self.normalizer:
             n += self.heads * (self.dim + 1)
         return 4 * n
+
+
+@dataclass(frozen=True)
+class ConvTail:
+    """The last `rows` inputs of a convolution over time per sequence, in the
+    model's element type (every tensor-parallel rank keeps all channels)."""
+
+    rows: int
+    width: int
+
+    def bytes_per_slot(self, elem: int) -> int:
+        return elem * self.rows * self.width
+
+
+@dataclass(frozen=True)
+class MixerAndTails:
+    """What a layer with input convolutions keeps: its mixer's part and one
+    tail per sublayer."""
+
+    mixer: Union[PagedKV, LatentPages, SharedCache, StateSlots]
+    tails: Tuple[ConvTail, ...]
+
+
+def cache_parts(layout: list) -> list:
+    """The single parts of a layout."""
+    out = []
+    for c in layout:
+        out += [c.mixer, *c.tails] if isinstance(c, MixerAndTails) else [c]
+    return out
 
 
 # ------------------------------------------------------------------- mixers
@@ -213,29 +243,86 @@ class Lightning:
             raise ValueError("lightning: decays must be within [0, 1]")
 
 
+@dataclass(frozen=True)
+class SigmoidAttention:
+    """Attention within chunks of `chunk` positions: a key weighs the sigmoid
+    of its capped score plus a bias per head, without normalization over keys.
+    Queries and keys are normed per head; positions do not enter."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    cap: float          # scores are cap * tanh(score / cap)
+    chunk: int
+
+    def cache(self, tp: int) -> PagedKV:
+        return PagedKV(self.kv_heads // tp, self.dim, self.vdim,
+                       v_transposed=True)
+
+    def params(self, width: int) -> int:
+        return (width * (self.heads + self.kv_heads) * (self.dim + self.vdim)
+                + 2 * self.dim + self.heads)
+
+    def check(self) -> None:
+        if self.heads % self.kv_heads:
+            raise ValueError("attention: heads must be a multiple of kv_heads")
+        if self.chunk < 1:
+            raise ValueError("attention: chunks must be at least 1 long")
+        if not self.cap > 0:
+            raise ValueError("attention: the score cap must be positive")
+
+
 Mixer = Union[DiffAttention, GatedLinear, MatrixLSTM, LatentAttention,
-              Lightning]
+              Lightning, SigmoidAttention]
+
+
+# ------------------------------------------------------------- feed-forward
+
+@dataclass(frozen=True)
+class SquaredRelu:
+    """Dense feed-forward without a gate: down(relu(up x)^2)."""
+
+    ff: int
+
+    def params(self, width: int) -> int:
+        return 2 * width * self.ff
+
+    def check(self) -> None:
+        pass
 
 
 @dataclass(frozen=True)
 class Experts:
-    """Mixture of gated-SiLU experts; `shared` is the size of an expert that
-    every token also passes, weighted by a sigmoid gate (None: there is
-    none)."""
+    """Mixture of gated experts.
+
+    `shared` is the size of an expert that every token also passes, weighted
+    by a sigmoid gate (None: there is none).  `identity` further outputs of
+    the router stand for experts that return their input.  With `limit` an
+    expert computes g sigmoid(1.702 g) (u + 1) from g = min(gate, limit) and
+    u = up clamped to +-limit; without, silu(gate) * up.  `over_all`: weights are the softmax over all router
+    outputs, and a correction is added to it for the choice only; otherwise
+    the softmax over the chosen."""
 
     experts: int
     top: int
     ff: int
     shared: Optional[int] = None
+    identity: int = 0
+    over_all: bool = False
+    limit: Optional[float] = None
 
     def params(self, width: int) -> int:
-        n = width * self.experts * (1 + 3 * self.ff)
+        n = width * (self.experts * (1 + 3 * self.ff) + self.identity)
+        if self.over_all:
+            n += self.experts + self.identity
         if self.shared is not None:
             n += width * (1 + 3 * self.shared)
         return n
 
     def check(self) -> None:
-        if not 1 <= self.top <= self.experts:
+        if not 1 <= self.top <= self.experts + self.identity:
             raise ValueError("experts: top must be between 1 and the number "
                              "of experts")
 
@@ -243,8 +330,11 @@ class Experts:
 @dataclass(frozen=True)
 class LayerSpec:
     mixer: Mixer
-    # dense feed-forward size, experts, or None for no feed-forward
-    ff: Union[None, int, Experts] = None
+    # size of a dense gated feed-forward, a description of another kind, or
+    # None for no feed-forward
+    ff: Union[None, int, SquaredRelu, Experts] = None
+    # the layer whose tensors this one uses, with a cache of its own
+    weights_of: Optional[int] = None
 
 
 @dataclass
@@ -259,23 +349,33 @@ class HybridSpec(ModelSpec):
     embed_scale: float = 1.0
     # size of a token's own input to every layer (0: there is none)
     side_dim: int = 0
+    # taps of the convolution over time on every sublayer's input (0: none)
+    conv_taps: int = 0
 
     def param_count(self) -> int:
         h = self.hidden_size
         n = self.vocab_size * h * (1 if self.tie_embeddings else 2)
         n += self.norm_params
+        sublayer = self.norms * self.norm_params + h * self.conv_taps
         for layer in self.layers:
-            n += layer.mixer.params(h) + self.norms * self.norm_params
+            if layer.weights_of is not None:
+                continue
+            n += layer.mixer.params(h) + sublayer
             if layer.ff is not None:
-                n += layer.ff.params(h) if isinstance(layer.ff, Experts) \
-                    else 3 * h * layer.ff
-                n += self.norms * self.norm_params
+                n += 3 * h * layer.ff if isinstance(layer.ff, int) \
+                    else layer.ff.params(h)
+                n += sublayer
             if self.side_dim:
                 n += (self.vocab_size + 2 * h) * self.side_dim + h
         return n
 
     def cache_layout(self, tp: int) -> list:
-        return [layer.mixer.cache(tp) for layer in self.layers]
+        if not self.conv_taps:
+            return [layer.mixer.cache(tp) for layer in self.layers]
+        tail = ConvTail(self.conv_taps - 1, self.hidden_size)
+        return [MixerAndTails(layer.mixer.cache(tp),
+                              (tail,) * (1 if layer.ff is None else 2))
+                for layer in self.layers]
 
     @property
     def is_hybrid(self) -> bool:
@@ -283,7 +383,8 @@ class HybridSpec(ModelSpec):
 
     @property
     def has_state(self) -> bool:
-        return any(isinstance(c, StateSlots) for c in self.cache_layout(1))
+        return any(isinstance(c, (StateSlots, ConvTail))
+                   for c in cache_parts(self.cache_layout(1)))
 
     @property
     def latent_windows(self) -> List[int]:
@@ -300,9 +401,10 @@ def hybrid_spec(name: str, architecture: str, width: int, vocab: int,
     layers = tuple(layers)
     for i, layer in enumerate(layers):
         layer.mixer.check()
-        if isinstance(layer.ff, Experts):
+        if layer.ff is not None and not isinstance(layer.ff, int):
             layer.ff.check()
         _check_shared_cache(layers, i)
+        _check_shared_weights(layers, i)
     return HybridSpec(
         name=name, hidden_size=width, num_layers=len(layers), num_heads=0,
         num_kv_heads=0, head_dim=0, intermediate_size=0, vocab_size=vocab,
@@ -324,3 +426,16 @@ def _check_shared_cache(layers, i: int) -> None:
                                               m.rot_base):
         raise ValueError(f"layer {i}: latent sizes and rotation differ from "
                          f"layer {j}'s")
+
+
+def _check_shared_weights(layers, i: int) -> None:
+    j = layers[i].weights_of
+    if j is None:
+        return
+    o = layers[j] if 0 <= j < len(layers) else None
+    if o is None or o.weights_of is not None:
+        raise ValueError(f"layer {i}: weights_of must name a layer with "
+                         "tensors of its own")
+    if (o.mixer, o.ff) != (layers[i].mixer, layers[i].ff):
+        raise ValueError(f"layer {i}: sizes differ from those of layer {j}, "
+                         "whose tensors it uses")

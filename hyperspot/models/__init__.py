@@ -1,5 +1,6 @@
 from .llama import LlamaForCausalLM
 from .mixtral import MixtralForCausalLM
+from .mutusun import MutusunForCausalLM
 from .registry import build_model
 from .sumosun import SumosunForCausalLM
 from .tefezen import TefezenForCausalLM

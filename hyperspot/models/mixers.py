@@ -18,7 +18,8 @@ from torch import nn
 
 from hyperspot.engine.layer_spec import (DiffAttention, Experts, GatedLinear,
                                          LatentAttention, Lightning,
-                                         MatrixLSTM)
+                                         MatrixLSTM, SigmoidAttention,
+                                         SquaredRelu)
 from hyperspot.ops import experts, hybrid, latent
 from hyperspot.parallel import (MergedColumnParallelLinear,
                                 RowParallelLinear)
@@ -122,8 +123,28 @@ class GatedGelu(nn.Module):
         yield p + "down", (self.width, self.ff), self.down.load_full_weight
 
 
+class SquaredReluMLP(nn.Module):
+    """down(relu(up x)^2)."""
+
+    def __init__(self, spec: SquaredRelu, width: int, dtype, tag: int):
+        super().__init__()
+        self.up = MergedColumnParallelLinear(width, [spec.ff], dtype,
+                                             seed_tag=tag)
+        self.down = RowParallelLinear(spec.ff, width, dtype, seed_tag=tag + 1)
+        self.width, self.ff = width, spec.ff
+
+    def add_next(self, x, residual, norm: RmsScale, nxt, meta):
+        """residual += norm(self(x)); the next sublayer's input."""
+        y = self.down(hybrid.squared_relu(self.up(x)))
+        return hybrid.add_rms_next(y, residual, norm.w, nxt, meta)
+
+    def tensors(self, p: str):
+        yield p + "up", (self.ff, self.width), _part(self.up, 0)
+        yield p + "down", (self.width, self.ff), self.down.load_full_weight
+
+
 class ExpertMixture(nn.Module):
-    """Gated-SiLU experts chosen per token, and an optional shared one.
+    """Gated experts chosen per token, and an optional shared one.
 
     Under tensor parallelism every expert's inner size is divided over the
     ranks, so all ranks run all experts and the sum is one all-reduce."""
@@ -155,22 +176,39 @@ class ExpertMixture(nn.Module):
         if m.shared is not None:
             self.shared_up, self.shared_down = pair(1, m.shared, tag + 2)
         # router rows, then the shared expert's gate: one product
+        self.routes = m.experts + m.identity
         self.router = _param(_init_weight(
-            m.experts + (m.shared is not None), width, dtype, tag + 4))
+            self.routes + (m.shared is not None), width, dtype, tag + 4))
+        self.correction = _param(torch.zeros(self.routes)) if m.over_all \
+            else None
 
     @property
     def args(self) -> tuple:
         return (self.router, self.up, self.down, self.shared_up,
                 self.shared_down, self.spec.top)
 
+    @property
+    def rules(self) -> experts.Rules:
+        return experts.Rules(self.correction, self.spec.identity,
+                             self.spec.limit, get_tp_rank() == 0)
+
     def add_normed(self, x, residual, norm: RmsScale, eps: float):
         """residual += norm(mixture of x); the residual in x's type."""
         if get_tp_size() == 1:
             return experts.mixture_add_rms(x, *self.args, residual, norm.w,
-                                           eps)
+                                           eps, self.rules)
         y = tensor_model_parallel_all_reduce(
-            experts.mixture(x, *self.args))
+            experts.mixture(x, *self.args, self.rules))
         return hybrid.add_rms(y, residual, norm.w, eps, x.dtype)
+
+    def add_next(self, x, residual, norm: RmsScale, nxt, meta):
+        """residual += norm(mixture of x); the next sublayer's input."""
+        if get_tp_size() == 1:
+            return experts.mixture_add_next(x, *self.args, self.rules,
+                                            residual, norm.w, nxt, meta)
+        y = tensor_model_parallel_all_reduce(
+            experts.mixture(x, *self.args, self.rules))
+        return hybrid.add_rms_next(y, residual, norm.w, nxt, meta)
 
     def tensors(self, p: str):
         m, w = self.spec, self.width
@@ -188,11 +226,27 @@ class ExpertMixture(nn.Module):
         for i in range(m.experts):
             yield from expert(f"{p}e{i}.", self.up.data[i],
                               self.down.data[i], m.ff)
-        yield p + "router", (m.experts, w), self.router.data[:m.experts].copy_
+        n = self.routes
+        yield p + "router", (n, w), self.router.data[:n].copy_
+        if self.correction is not None:
+            yield p + "correction", (n,), self.correction.data.copy_
         if m.shared is not None:
             yield from expert(p + "shared.", self.shared_up.data[0],
                               self.shared_down.data[0], m.shared)
-            yield p + "shared.sg", (1, w), self.router.data[m.experts:].copy_
+            yield p + "shared.sg", (1, w), self.router.data[n:].copy_
+
+
+class InputConv(nn.Module):
+    """Causal convolution over time on each channel of a sublayer's input,
+    added to it; weights in float, kept [taps, width]."""
+
+    def __init__(self, width: int, taps: int, tag: int):
+        super().__init__()
+        self.w = _param(_random((taps, width), tag, 0.1))
+
+    def tensors(self, name: str):
+        yield name, tuple(self.w.t().shape), \
+            lambda t: self.w.data.copy_(t.t())
 
 
 class TokenSide(nn.Module):
@@ -334,6 +388,42 @@ class MatrixMemoryLSTM(nn.Module):
             yield p + n + ".b", (m.heads,), _put(b, tp, r)
 
 
+class ChunkedSigmoidAttention(nn.Module):
+    def __init__(self, spec: SigmoidAttention, width: int, eps: float, dtype,
+                 tag: int):
+        super().__init__()
+        self.spec, self.width, self.eps = spec, width, eps
+        m, tp, r = spec, get_tp_size(), get_tp_rank()
+        self.qkv = MergedColumnParallelLinear(
+            width, [m.heads * m.dim, m.kv_heads * m.dim,
+                    m.kv_heads * m.vdim], dtype, seed_tag=tag)
+        self.o_proj = RowParallelLinear(m.heads * m.vdim, width, dtype,
+                                        seed_tag=tag + 3)
+        self.q_norm, self.k_norm = RmsScale(m.dim), RmsScale(m.dim)
+        # added to the scores of a head
+        self.bias = _rows(_param(torch.zeros(m.heads // tp)), tp, r, m.heads)
+
+    def forward(self, x, meta, cache) -> torch.Tensor:
+        m = self.spec
+        q, k, v = self.qkv.split(self.qkv(x))
+        hybrid.norm_append(q, k, v, self.q_norm.w, self.k_norm.w, meta, cache,
+                           self.eps)
+        o = hybrid.sigmoid_attention(q, cache, meta, self.bias, m.chunk,
+                                     m.scale, m.cap)
+        return self.o_proj(o)
+
+    def tensors(self, p: str):
+        m, w = self.spec, self.width
+        yield p + "q", (m.heads * m.dim, w), _part(self.qkv, 0)
+        yield p + "k", (m.kv_heads * m.dim, w), _part(self.qkv, 1)
+        yield p + "v", (m.kv_heads * m.vdim, w), _part(self.qkv, 2)
+        yield p + "o", (w, m.heads * m.vdim), self.o_proj.load_full_weight
+        yield from self.q_norm.tensors(p + "q.norm")
+        yield from self.k_norm.tensors(p + "k.norm")
+        yield p + "pb", (m.heads,), _put(self.bias, get_tp_size(),
+                                         get_tp_rank())
+
+
 class WindowLatentAttention(nn.Module):
     def __init__(self, spec: LatentAttention, width: int, eps: float, dtype,
                  tag: int):
@@ -427,4 +517,5 @@ MIXERS = {DiffAttention: WindowDiffAttention,
           GatedLinear: GatedLinearAttention,
           MatrixLSTM: MatrixMemoryLSTM,
           LatentAttention: WindowLatentAttention,
-          Lightning: LightningAttention}
+          Lightning: LightningAttention,
+          SigmoidAttention: ChunkedSigmoidAttention}

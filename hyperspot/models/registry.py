@@ -12,7 +12,7 @@ import torch
 
 from hyperspot.engine.config import ModelSpec, get_model_spec
 
-from . import sumosun, tefezen
+from . import mutusun, sumosun, tefezen
 
 # config.json "architecture" -> (configuration reader, model class)
 DESIGNS = {
@@ -20,10 +20,12 @@ DESIGNS = {
                            sumosun.SumosunForCausalLM),
     tefezen.ARCHITECTURE: (tefezen.spec_from_folder,
                            tefezen.TefezenForCausalLM),
+    mutusun.ARCHITECTURE: (mutusun.spec_from_folder,
+                           mutusun.MutusunForCausalLM),
 }
 
 # presets of the designs (random-init), by canonical id
-DESIGN_PRESETS = {**sumosun.PRESETS, **tefezen.PRESETS}
+DESIGN_PRESETS = {**sumosun.PRESETS, **tefezen.PRESETS, **mutusun.PRESETS}
 
 
 def spec_from_folder(folder: str) -> ModelSpec:

@@ -1,7 +1,7 @@
 """Ops of the hybrid designs (models.mixers), dispatched like the rest of the
 op layer: a GPU tensor runs the gfx950 kernels of csrc/dyt.hip, csrc/rms.hip,
-csrc/attn_window.hip, csrc/recurrent.hip and csrc/recurrent_chunk.hip, a CPU
-tensor the PyTorch references.
+csrc/conv.hip, csrc/attn_window.hip, csrc/attn_sigmoid.hip, csrc/recurrent.hip
+and csrc/recurrent_chunk.hip, a CPU tensor the PyTorch references.
 
 Dynamic-tanh parameters travel as tuples (w, b, alpha) of float tensors.
 q, k, v, g are column views of one projection buffer [T, ...]; the kernels
@@ -9,6 +9,8 @@ take its row stride.
 """
 
 from __future__ import annotations
+
+from typing import NamedTuple, Optional
 
 import torch
 
@@ -53,6 +55,16 @@ def embed_scaled(table: torch.Tensor, ids: torch.Tensor, scale: float):
     return x, res
 
 
+def embed_residual(table: torch.Tensor, ids: torch.Tensor) -> torch.Tensor:
+    """Token embedding as float residual only."""
+    if not table.is_cuda:
+        return table[ids].float()
+    res = torch.empty(ids.numel(), table.shape[1], dtype=torch.float32,
+                      device=table.device)
+    _native().embed_scaled(None, res, table, ids, 1.0)
+    return res
+
+
 def rms_scale(x: torch.Tensor, w: torch.Tensor, eps: float, dtype):
     """RMS norm of float rows with a float weight, as `dtype`."""
     if not x.is_cuda:
@@ -72,6 +84,75 @@ def add_rms(h: torch.Tensor, residual: torch.Tensor, w: torch.Tensor,
     out = residual if dtype == torch.float32 \
         else torch.empty(h.shape, dtype=dtype, device=h.device)
     _native().add_rms(out, residual, h, w, eps)
+    return out
+
+
+class NextInput(NamedTuple):
+    """How a sublayer's input is made of the residual: an RMS norm with
+    weight `w` [W] and, if there is one, a causal convolution over time that
+    is added to it.  `conv` [taps, W] float has the token's own tap last,
+    `tail` [slots, taps - 1, W] the last inputs of every sequence."""
+
+    w: torch.Tensor
+    eps: float
+    conv: Optional[torch.Tensor] = None
+    tail: Optional[torch.Tensor] = None
+
+    def row_args(self, meta):
+        """Kernel arguments where a row is a sequence of its own."""
+        if self.conv is None or meta.mode == "prefill":
+            return None, None, None, None
+        return self.conv, self.tail, meta.state_slots, meta.positions
+
+    def finish(self, h, meta):
+        """The convolution where the rows of a sequence meet each other."""
+        if self.conv is None or meta.mode == "decode":
+            return h
+        return causal_conv(h, self.conv, self.tail, meta)
+
+
+def next_input(residual: torch.Tensor, nxt: NextInput, meta,
+               dtype) -> torch.Tensor:
+    """The first sublayer's input."""
+    if not residual.is_cuda:
+        h = torch_ref.rms_scale(residual, nxt.w, nxt.eps).to(dtype)
+        return _conv_ref(h, nxt, meta)
+    h = torch.empty(residual.shape, dtype=dtype, device=residual.device)
+    _native().add_rms_next(h, residual, None, None, nxt.w, nxt.eps,
+                           *nxt.row_args(meta))
+    return nxt.finish(h, meta)
+
+
+def add_rms_next(y: torch.Tensor, residual: torch.Tensor, w: torch.Tensor,
+                 nxt: NextInput, meta) -> torch.Tensor:
+    """residual += rms(y) * w in place; returns the next sublayer's input in
+    y's type."""
+    if not y.is_cuda:
+        residual += torch_ref.rms_scale(y, w, nxt.eps)
+        h = torch_ref.rms_scale(residual, nxt.w, nxt.eps).to(y.dtype)
+        return _conv_ref(h, nxt, meta)
+    h = torch.empty_like(y)
+    _native().add_rms_next(h, residual, y, w, nxt.w, nxt.eps,
+                           *nxt.row_args(meta))
+    return nxt.finish(h, meta)
+
+
+def _conv_ref(h, nxt: NextInput, meta):
+    return h if nxt.conv is None \
+        else causal_conv(h, nxt.conv, nxt.tail, meta)
+
+
+def causal_conv(h: torch.Tensor, w: torch.Tensor, tail: torch.Tensor,
+                meta) -> torch.Tensor:
+    """h [T, W] plus its convolution over time within every sequence; the
+    tails are renewed."""
+    if not h.is_cuda:
+        return torch_ref.causal_conv(
+            h, w, tail, None if meta.mode == "decode" else meta.seq_start,
+            meta.state_slots, meta.positions)
+    out = torch.empty_like(h)
+    _native().causal_conv(out, h, w, tail, meta.seq_start, meta.positions,
+                          meta.state_slots, meta.tiles)
     return out
 
 
@@ -120,6 +201,25 @@ def gelu_mul(gate_up: torch.Tensor) -> torch.Tensor:
     return torch_ref.gelu_mul(gate_up)
 
 
+def squared_relu(x: torch.Tensor) -> torch.Tensor:
+    """relu(x)^2; in place on the GPU."""
+    if x.is_cuda:
+        _native().squared_relu(x)
+        return x
+    return x.float().clamp(min=0).square().to(x.dtype)
+
+
+def clamped_glu(gate_up: torch.Tensor, limit: float) -> torch.Tensor:
+    """g sigmoid(1.702 g) (u + 1) of a merged [gate | up] projection, with
+    g = min(gate, limit) and u = up clamped to +-limit."""
+    if not gate_up.is_cuda:
+        return torch_ref.clamped_glu(gate_up, limit)
+    out = torch.empty(*gate_up.shape[:-1], gate_up.shape[-1] // 2,
+                      dtype=gate_up.dtype, device=gate_up.device)
+    _native().clamped_glu(out, gate_up, limit)
+    return out
+
+
 # ---------------------------------------------------------------- attention
 
 def rope_pairs_append(q, k, v, meta, freqs, cache, head_dim: int) -> None:
@@ -160,6 +260,44 @@ def window_diff_attention(q, cache, meta, lam, window: int, scale: float,
         n.window_attn_decode(
             out, q, cache.k, cache.v, meta.block_tables, meta.positions, lam,
             partial, split, window, scale, diff, eps)
+    return out
+
+
+def norm_append(q, k, v, qw, kw, meta, cache, eps: float) -> None:
+    """RMS norm of every head of q (in place) and k, append k and v."""
+    f = _native().norm_append if q.is_cuda else torch_ref.norm_append
+    f(q, k, v, qw, kw, meta.slot_mapping, cache.k, cache.v, eps)
+
+
+def sigmoid_attention(q, cache, meta, bias, chunk: int, scale: float,
+                      cap: float) -> torch.Tensor:
+    """[T, H * E]: the keys of a row's chunk up to itself, each weighing
+    sigmoid(cap tanh(q.k scale / cap) + bias[h]); keys come from the pages."""
+    row_seq = meta.row_seq if meta.mode == "prefill" else None
+    if not q.is_cuda:
+        return torch_ref.sigmoid_attention(
+            q, cache.k, cache.v, meta.block_tables, meta.positions, row_seq,
+            bias, chunk, scale, cap)
+    n, T = _native(), q.shape[0]
+    G, E = cache.v.shape[1], cache.v.shape[2]
+    H = q.shape[1] // cache.k.shape[3]
+    out = torch.empty(T, H * E, dtype=q.dtype, device=q.device)
+    if not n.sigmoid_attn_fits(q, cache.k, cache.v):
+        n.sigmoid_attn_general(
+            out, q, cache.k, cache.v, meta.block_tables, meta.positions,
+            row_seq, bias, chunk, scale, cap)
+    elif meta.mode == "prefill":
+        n.sigmoid_attn_prefill(
+            out, q, cache.k, cache.v, meta.block_tables, meta.positions,
+            meta.seq_start, meta.tiles, bias, chunk, scale, cap)
+    else:
+        reach = min(chunk, meta.block_tables.shape[1] * cache.k.shape[2])
+        split = decode_split(T * G * -(-(H // G) // 16), reach)
+        partial = None if split == 1 else torch.empty(
+            T * H * split * E, dtype=torch.float32, device=q.device)
+        n.sigmoid_attn_decode(
+            out, q, cache.k, cache.v, meta.block_tables, meta.positions, bias,
+            partial, split, chunk, scale, cap)
     return out
 
 

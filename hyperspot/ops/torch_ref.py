@@ -438,24 +438,98 @@ def lightning_scan(q, k, v, decay, state, seq_start, slots,
     return o
 
 
-def mixture(x, router, up, down, shared_up, shared_down, top: int):
-    """[T, W] float: chosen experts weighted by the softmax over the chosen
-    logits, plus the shared expert under its sigmoid gate."""
+def clamped_glu(gate_up: torch.Tensor, limit: float) -> torch.Tensor:
+    """g sigmoid(1.702 g) (u + 1) of a merged [gate | up] projection, with
+    g = min(gate, limit) and u = up clamped to +-limit."""
+    g, u = gate_up.float().chunk(2, -1)
+    g, u = g.clamp(max=limit), u.clamp(-limit, limit)
+    return (g * torch.sigmoid(1.702 * g) * (u + 1)).to(gate_up.dtype)
+
+
+def mixture(x, router, up, down, shared_up, shared_down, top: int,
+            rules=(None, 0, None, True)):
+    """[T, W] float: chosen experts under their weights, plus the shared
+    expert under its sigmoid gate; `rules` as in ops.experts."""
+    correction, identity, limit, identity_here = rules
     E = up.shape[0]
+    n = E + identity
     z = x.float() @ router.float().t()
-    s, ids = z[:, :E].topk(top, dim=-1)
-    weight = s.softmax(-1)
+    if correction is None:
+        s, ids = z[:, :n].topk(top, dim=-1)
+        weight = s.softmax(-1)
+    else:
+        s = z[:, :n].softmax(-1)
+        ids = (s + correction).topk(top, dim=-1).indices
+        weight = s.gather(1, ids)
 
     def expert(h, up, down):
-        return (silu_mul(h @ up.t()) @ down.t()).float()
+        y = h @ up.t()
+        y = silu_mul(y) if limit is None else clamped_glu(y, limit)
+        return (y @ down.t()).float()
 
-    out = torch.zeros(x.shape, dtype=torch.float32, device=x.device)
+    out = x.float() * (weight * (ids >= E)).sum(-1, keepdim=True) \
+        * identity_here
     for e in range(E):
         t, j = (ids == e).nonzero(as_tuple=True)
         if t.numel():
             out.index_add_(0, t, weight[t, j][:, None]
                            * expert(x[t], up[e], down[e]))
     if shared_up is not None:
-        out += torch.sigmoid(z[:, E:]) * expert(x, shared_up[0],
+        out += torch.sigmoid(z[:, n:]) * expert(x, shared_up[0],
                                                 shared_down[0])
+    return out
+
+
+# ---------------------------------------------------------------------------
+# Convolved sublayer inputs, chunked sigmoid attention
+# ---------------------------------------------------------------------------
+
+def causal_conv(h, w, tail, seq_start, slots, positions) -> torch.Tensor:
+    """h [T, W] plus its convolution over time; w [taps, W] float with the
+    token's own tap last; tail [slots, taps - 1, W] is read and renewed."""
+    taps = w.shape[0]
+    out = torch.empty_like(h)
+    for a, b, slot, fresh in _sequences(seq_start, slots, positions):
+        past = torch.zeros(taps - 1, h.shape[1], dtype=h.dtype,
+                           device=h.device) if fresh else tail[slot]
+        x = torch.cat([past, h[a:b]])
+        y = h[a:b].float()
+        for j in range(taps):
+            y = y + w[j] * x[j:j + b - a].float()
+        out[a:b] = y.to(h.dtype)
+        if slot >= 0:
+            tail[slot] = x[b - a:]
+    return out
+
+
+def norm_append(q, k, v, qw, kw, slot_mapping, k_cache, v_cache,
+                eps: float) -> None:
+    """RMS norm of every head of q [T, H*D] in place; append normed k and
+    transposed v."""
+    _, G, BS, D = k_cache.shape
+    norm = lambda x, w: rms_scale(x.unflatten(-1, (-1, D)), w, eps).flatten(1)
+    q.copy_(norm(q, qw))
+    ok = slot_mapping >= 0
+    blk, off = slot_mapping[ok] // BS, slot_mapping[ok] % BS
+    k_cache[blk, :, off] = norm(k, kw)[ok].view(-1, G, D).to(k_cache.dtype)
+    v_cache[blk, :, :, off] = v[ok].reshape(int(ok.sum()), G, -1)
+
+
+def sigmoid_attention(q, k_cache, v_cache, block_tables, positions, row_seq,
+                      bias, chunk: int, scale: float, cap: float):
+    T = q.shape[0]
+    _, G, BS, D = k_cache.shape
+    H = q.shape[1] // D
+    out = torch.empty(T, H * v_cache.shape[2], dtype=q.dtype, device=q.device)
+    for t in range(T):
+        s = int(row_seq[t]) if row_seq is not None else t
+        p = int(positions[t])
+        idx = torch.arange(p // chunk * chunk, p + 1, device=q.device)
+        blk, off = block_tables[s][idx // BS].long(), idx % BS
+        k = k_cache[blk, :, off].float()                       # [n, G, D]
+        v = v_cache[blk, :, :, off].float()                    # [n, G, E]
+        z = torch.einsum("gxd,ngd->gxn", q[t].float().view(G, H // G, D), k)
+        z = cap * torch.tanh(z * scale / cap) + bias.view(G, H // G, 1)
+        out[t] = torch.einsum("gxn,nge->gxe", z.sigmoid(),
+                              v).reshape(-1).to(q.dtype)
     return out
