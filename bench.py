@@ -574,21 +574,35 @@ def _compare_specs(design, width):
     """A hybrid design and the closest other model at equal size."""
     from hyperspot.engine.config import ModelSpec
     heads, vocab = width // 128, 32768
+    if design in ("tefezen", "mutusun"):
+        experts, ff = 65536 // width, width // 2
+        plain = ModelSpec(f"mixtral-w{width}", width, 8, heads, heads // 4,
+                          128, ff, vocab, max_position=16384,
+                          num_experts=experts, num_experts_per_tok=4)
+    if design == "mutusun":
+        # equal width, layers, attention heads, experts, choices per token
+        # and expert size; the first layer's dense feed-forward has the work
+        # of four experts; one chunk holds every prompt, so both models
+        # attend to all earlier tokens.  One in nine of the router's outputs
+        # is an identity expert
+        from hyperspot.engine.layer_spec import Experts
+        from hyperspot.models.mutusun import preset
+        return preset(f"mutusun-w{width}", width=width, vocab=vocab,
+                      heads=heads, kv_heads=heads // 4, dim=128, chunk=16384,
+                      ff=6 * ff, experts=Experts(
+                          experts, 4, ff, identity=experts // 8,
+                          over_all=True, limit=7.0), layers=8), plain
     if design == "tefezen":
         # equal width, layers, attention heads, experts, choices per token
         # and expert size; the design's shared expert and token inputs have
         # no counterpart in the other model
         from hyperspot.engine.layer_spec import Experts
         from hyperspot.models.tefezen import preset
-        experts, ff = 65536 // width, width // 2
         hybrid = preset(f"tefezen-w{width}", width=width, vocab=vocab,
                         heads=heads, dim=128, rot_dim=64, kv_rank=512,
                         window=1024, state_heads=heads, state_dim=128,
                         experts=Experts(experts, 4, ff, ff), side_dim=128,
                         periods=2)
-        plain = ModelSpec(f"mixtral-w{width}", width, 8, heads, heads // 4,
-                          128, ff, vocab, max_position=16384,
-                          num_experts=experts, num_experts_per_tok=4)
         return hybrid, plain
     # equal width, feed-forwards, vocabulary and number of feed-forwards
     from hyperspot.models.sumosun import preset
@@ -719,9 +733,9 @@ def main():
                          "hybrid design beside the closest other model of "
                          "equal size, at these widths (default 2048 4096)")
     ap.add_argument("--compare-design", default="sumosun",
-                    choices=["sumosun", "tefezen"],
+                    choices=["sumosun", "tefezen", "mutusun"],
                     help="with --compare: Sumosun beside a plain decoder, or "
-                         "Tefezen beside a Mixtral-like one")
+                         "Tefezen or Mutusun beside a Mixtral-like one")
     ap.add_argument("--compare-model", default=None, metavar="PREFIX",
                     help="with --compare: only models of this name prefix")
     ap.add_argument("--compare-reps", type=int, default=3)

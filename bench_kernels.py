@@ -1,7 +1,8 @@
 #!/usr/bin/env python3
 """Isolated kernel microbenchmarks (GPU only) — us/call + achieved GB/s.
 
-Usage: python bench_kernels.py [--which attn|gemm|fp8|hybrid|latent|all] [--iters N]
+Usage: python bench_kernels.py [--iters N]
+           [--which attn|gemm|fp8|hybrid|latent|sigmoid|all]
 
 Shapes mirror the flagship bench (Llama-3-8B bf16, bs=256 ctx=512 decode):
 the numbers here are the per-kernel budget lines behind bench.py's step
@@ -458,6 +459,114 @@ def bench_latent(iters, W):
         common(B, tag)
 
 
+def bench_sigmoid(iters, W):
+    """Kernels of the Mutusun design at width W and the like kernels of the
+    Mixtral-like model."""
+    import hyperspot.ops as ops
+    from hyperspot.engine.kv_cache import KVPages
+    from hyperspot.ops import experts, hybrid
+    dev, bf, f32 = DEV, torch.bfloat16, torch.float32
+    report = lambda name, tag, fn, nbytes, flops=0: report_kernel(
+        iters, name, f"w{W}_{tag}", fn, nbytes, flops, timed_graph)
+    rnd = lambda *s, d=bf: (torch.randn(*s, device=dev) * 0.3).to(d)
+    H, G, D, chunk, taps = W // 128, W // 512, 128, 16384, 4
+    NE, top, F = 65536 // W, 4, W // 2
+    NI = NE // 8
+    rules = experts.Rules(torch.zeros(NE + NI, device=dev), NI, 7.0)
+    qw, kw, bias = rnd(D, d=f32), rnd(D, d=f32), rnd(H, d=f32)
+    up, down = rnd(NE, 2 * F, W) * 0.1, rnd(NE, W, F) * 0.1
+    router, conv = rnd(NE + NI, W), rnd(taps, W, d=f32)
+    nw, w2 = torch.ones(W, device=dev), torch.ones(W, dtype=bf, device=dev)
+
+    def common(m, T, seqs, tag):
+        x, r, y = rnd(T, W), rnd(T, W, d=f32), rnd(T, W)
+        nxt = hybrid.NextInput(nw, 1e-5, conv, rnd(seqs, taps - 1, W))
+        decode = m.mode == "decode"
+        tail = 4 * seqs * (taps - 1) * W
+        report("add_rms_next" + " (with conv)" * decode, tag,
+               lambda: hybrid.add_rms_next(x, r, nw, nxt if decode else
+                                           hybrid.NextInput(nw, 1e-5), m),
+               T * W * 12 + tail * decode)
+        report("fused_add_rmsnorm", tag, lambda: ops.fused_add_rmsnorm(
+            x, y, w2, 1e-5), T * W * 8)
+        if not decode:
+            report("causal_conv", tag, lambda: hybrid.causal_conv(
+                x, conv, nxt.tail, m), T * W * 4 + tail)
+        u, gu = rnd(T, 6 * F), rnd(T, 12 * F)
+        report("squared_relu", tag, lambda: hybrid.squared_relu(u),
+               T * F * 24)
+        report("clamped_glu", tag, lambda: hybrid.clamped_glu(gu, 7.0),
+               T * F * 36)
+        report("silu_mul", tag, lambda: ops.silu_mul(gu), T * F * 36)
+        # experts: every chosen expert's weights once, rows in and out; one
+        # choice in nine needs no expert
+        real = T * top * NE / (NE + NI)
+        per = 3 * W * F
+        nbytes = 2 * (min(NE, real) * per + T * W) + 6 * T * W
+        report("experts (with norms, add, conv)", tag,
+               lambda: experts.mixture_add_next(
+                   x, router, up, down, None, None, top, rules, r, nw, nxt,
+                   m), nbytes + 8 * T * W, real * 2 * per)
+        report("experts (sum only)", tag, lambda: experts.mixture(
+            x, router, up, down, None, None, top, rules), nbytes,
+            real * 2 * per)
+
+        def other():
+            p = (x.float() @ router[:NE].float().t()).softmax(-1)
+            wt, ids = p.topk(top, dim=-1)
+            wt = wt / wt.sum(-1, keepdim=True)
+            ops.moe_ffn(x, up, down, wt.to(bf), ids.int())
+        report("moe (route, moe_ffn)", tag, other,
+               2 * (min(NE, T * top) * per + T * W) + 6 * T * W,
+               T * top * 2 * per)
+
+    def heads(T):
+        return rnd(T, (H + 2 * G) * D).split([H * D, G * D, G * D], -1)
+
+    for lens in ([2048], [8192], [1024] * 8):
+        m, nb = meta_for(lens)
+        T, tag = sum(lens), "x".join(map(str, (len(lens), lens[0])))
+        q, k, v = heads(T)
+        cache = KVPages(torch.zeros(nb, G, 16, D, dtype=bf, device=dev),
+                        torch.zeros(nb, G, D, 16, dtype=bf, device=dev))
+        pairs = sum(x * (x + 1) // 2 for x in lens)
+        report("norm_append", tag, lambda: hybrid.norm_append(
+            q, k, v, qw, kw, m, cache, 1e-5), 2 * T * D * (2 * H + 4 * G))
+        q2, k2, v2 = (x.view(T, -1, D) for x in heads(T))
+        kc = torch.zeros(2, nb, G, 16, D, dtype=bf, device=dev)
+        cs = torch.randn(max(lens), D, device=dev)
+        report("rope_kv_append", tag, lambda: ops.rope_kv_append(
+            q2, k2, v2, m.positions, cs, m.slot_mapping, kc[0], kc[1]),
+            2 * T * D * (2 * H + 4 * G))
+        nbytes = 2 * T * D * (2 * H + 2 * G)
+        report("sigmoid_attn_prefill", tag, lambda: hybrid.sigmoid_attention(
+            q, cache, m, bias, chunk, 0.09, 30.0), nbytes,
+            pairs * H * 4 * D)
+        report("attn_prefill_mfma", tag, lambda: ops.attention(
+            q2, k2, v2, kc[0], kc[1], m, 0.088), nbytes, pairs * H * 4 * D)
+        common(m, T, len(lens), tag)
+    for B in (1, 32, 256):
+        ctx = 1024
+        m, nb = meta_for([1] * B, "decode", ctx)
+        tag = f"b{B}_ctx{ctx}"
+        q, k, v = heads(B)
+        cache = KVPages(rnd(nb, G, 16, D), rnd(nb, G, D, 16))
+        report("norm_append", tag, lambda: hybrid.norm_append(
+            q, k, v, qw, kw, m, cache, 1e-5), 2 * B * D * (2 * H + 4 * G))
+        q2, k2, v2 = (x.view(B, -1, D) for x in heads(B))
+        kc = rnd(2, nb, G, 16, D)
+        cs = torch.randn(ctx + 1, D, device=dev)
+        report("rope_kv_append", tag, lambda: ops.rope_kv_append(
+            q2, k2, v2, m.positions, cs, m.slot_mapping, kc[0], kc[1]),
+            2 * B * D * (2 * H + 4 * G))
+        nbytes = 4 * B * (ctx + 1) * G * D
+        report("sigmoid_attn_decode", tag, lambda: hybrid.sigmoid_attention(
+            q, cache, m, bias, chunk, 0.09, 30.0), nbytes)
+        report("paged_attn_decode", tag, lambda: ops.paged_attn_decode(
+            q2, kc[0], kc[1], m.block_tables, m.seq_lens, 0.088), nbytes)
+        common(m, B, B, tag)
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--which", default="attn")
@@ -473,6 +582,9 @@ def main():
     if args.which in ("latent", "all"):
         for width in (2048, 4096):
             bench_latent(args.iters, width)
+    if args.which in ("sigmoid", "all"):
+        for width in (2048, 4096):
+            bench_sigmoid(args.iters, width)
     if args.which in ("fp8", "all"):
         bench_fp8_gemm(args.iters)
 

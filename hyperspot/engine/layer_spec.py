@@ -383,7 +383,8 @@ class HybridSpec(ModelSpec):
 
     @property
     def has_state(self) -> bool:
-        return any(isinstance(c, (StateSlots, ConvTail))
+        return any(isinstance(c, StateSlots)
+                   or isinstance(c, ConvTail) and c.rows > 0
                    for c in cache_parts(self.cache_layout(1)))
 
     @property

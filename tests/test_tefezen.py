@@ -303,7 +303,8 @@ def test_key_leaves_the_window_at_its_edge(tmp_path, cuts):
     assert d[39] > 0.1 and d[40:].max() == 0
 
 
-def mixed_run(r, cfg, w, lens, seed=0, limits=lambda toks: TOL):
+def mixed_run(r, cfg, w, lens, seed=0, limits=lambda toks: TOL,
+              forward=O.forward):
     """Requests of these lengths through random portions, single tokens and
     pauses, at most four live, each checked against itself alone; the largest
     error over its limit."""
@@ -311,7 +312,7 @@ def mixed_run(r, cfg, w, lens, seed=0, limits=lambda toks: TOL):
     rnd = lambda n: int(torch.randint(0, n, (1,), generator=g))
     todo = [(f"r{i}", U.tokens(n, cfg["vocab"], seed=i))
             for i, n in enumerate(lens)]
-    want = {i: O.forward(cfg, w, t)[0] for i, t in todo}
+    want = {i: forward(cfg, w, t)[0] for i, t in todo}
     lim = {i: torch.as_tensor(limits(t)).expand(len(t)) for i, t in todo}
     live, worst = [], 0.0
     while todo or live:
