@@ -23,6 +23,8 @@
 // which is the operand P^T of O^T = V^T P^T: weights never leave their
 // registers, and V^T comes straight from the transposed pages.  The weights
 // enter as a bf16 high and low part.
+#include <type_traits>
+
 #include "common.h"
 
 #define PAGE 16
@@ -225,35 +227,33 @@ void sigmoid_attn_prefill_kernel(
   // matrix row i of a 32-token block takes this token's key
   const int krow = (col & 16) + ((col >> 2) & 1) * 8 + ((col >> 3) & 1) * 4 +
                    (col & 3);
-  const int kv_first = (p0 - p0 % chunk) / KV * KV;
-  pages(kv_first);
-  fetch(kv_first);
-  for (int kv0 = kv_first; kv0 <= last; kv0 += KV) {
-    stage();
-    __syncthreads();
-    if (kv0 + KV <= last) fetch(kv0 + KV);
+  // NB blocks from token kb on; FULL: every row sees all of them
+  auto step = [&](int kb, auto full) {
+    constexpr bool FULL = decltype(full)::value;
+    const int b0 = HW == 2 ? 0 : half;           // first block in LDS
+    f32x16_t sc[NB];
     #pragma unroll
     for (int i = 0; i < NB; ++i) {
-      const int b = HW == 2 ? i : half;
-      const int kb = kv0 + b * 32;               // first token of the block
-      if (w_first > last || kb > w_last || kb + 31 < w_lo) continue;
-      f32x16_t sc = f32x16_t(0.f);
+      sc[i] = f32x16_t(0.f);
       #pragma unroll
       for (int c = 0; c < KC; ++c)
-        sc = mfma32(*reinterpret_cast<const short8_t*>(
-                        k_lds + (b * 32 + krow) * KS + c * 16 + hf * 8),
-                    qf[c], sc);
-      // token of sc[r]: kb + (r>>3)*16 + hf*8 + (r&7)
-      const bool full = kb + 31 <= w_first && kb >= w_hi;
+        sc[i] = mfma32(*reinterpret_cast<const short8_t*>(
+                           k_lds + ((b0 + i) * 32 + krow) * KS + c * 16 +
+                           hf * 8),
+                       qf[c], sc[i]);
+    }
+    #pragma unroll
+    for (int i = 0; i < NB; ++i) {
+      // token of sc[i][r]: kb + i*32 + (r>>3)*16 + hf*8 + (r&7)
       short8_t ph[2], pl[2];
       #pragma unroll
       for (int c = 0; c < 2; ++c) {
         float p[8];
         #pragma unroll
         for (int j = 0; j < 8; ++j) {
-          p[j] = weigh(sc[c * 8 + j]);
-          if (!full) {
-            const int at = kb + c * 16 + hf * 8 + j;
+          p[j] = weigh(sc[i][c * 8 + j]);
+          if constexpr (!FULL) {
+            const int at = kb + i * 32 + c * 16 + hf * 8 + j;
             if (at > qp || at < q_lo) p[j] = 0.f;
           }
         }
@@ -264,10 +264,25 @@ void sigmoid_attn_prefill_kernel(
         #pragma unroll
         for (int c = 0; c < 2; ++c) {
           const short8_t vf = *reinterpret_cast<const short8_t*>(
-              v_lds + (e * 32 + col) * VS + b * 32 + c * 16 + hf * 8);
+              v_lds + (e * 32 + col) * VS + (b0 + i) * 32 + c * 16 + hf * 8);
           acc[e] = mfma32(vf, ph[c], acc[e]);
           acc[e] = mfma32(vf, pl[c], acc[e]);
         }
+    }
+  };
+  const int kv_first = (p0 - p0 % chunk) / KV * KV;
+  pages(kv_first);
+  fetch(kv_first);
+  for (int kv0 = kv_first; kv0 <= last; kv0 += KV) {
+    stage();
+    __syncthreads();
+    if (kv0 + KV <= last) fetch(kv0 + KV);
+    const int kb = kv0 + (HW == 2 ? 0 : half * 32);    // first token
+    if (w_first <= last && kb <= w_last && kb + NB * 32 > w_lo) {
+      if (kb + NB * 32 <= w_first + 1 && kb >= w_hi)
+        step(kb, std::true_type{});
+      else
+        step(kb, std::false_type{});
     }
     __syncthreads();
   }
@@ -470,7 +485,8 @@ void launch_sigmoid_attn_prefill(bf16* out, const bf16* q,
                                  int D, int E, int chunk, float scale,
                                  float cap, long qs, hipStream_t stream) {
   if (num_tiles == 0) return;
-  const int hw = H / G % 2 == 0 ? 2 : 1;
+  // two heads share a tile's keys where enough workgroups remain
+  const int hw = H / G % 2 == 0 && (long)H / 2 * num_tiles >= 512 ? 2 : 1;
   const dim3 grid((unsigned)(H / hw), (unsigned)num_tiles);
   #define RUN(DP, EP, HW)                                                   \
     sigmoid_attn_prefill_kernel<DP, EP, HW><<<grid, 256, 0, stream>>>(      \

@@ -85,9 +85,12 @@ template <> struct Elem<float> {
   }
 };
 
-// V consecutive elements (V = 1 or 4; 4 needs 4-element alignment)
+// V consecutive elements (V = 1, 4 or 8, which need alignment to V elements)
 template <typename T, int V> DEV void load_vec(const T* p, float* f) {
-  if constexpr (V == 4) {
+  if constexpr (V == 8) {
+    load_vec<T, 4>(p, f);
+    load_vec<T, 4>(p + 4, f + 4);
+  } else if constexpr (V == 4) {
     const float4 v = Elem<T>::ld4(p);
     f[0] = v.x; f[1] = v.y; f[2] = v.z; f[3] = v.w;
   } else {
@@ -95,7 +98,10 @@ template <typename T, int V> DEV void load_vec(const T* p, float* f) {
   }
 }
 template <typename T, int V> DEV void store_vec(T* p, const float* f) {
-  if constexpr (V == 4)
+  if constexpr (V == 8) {
+    store_vec<T, 4>(p, f);
+    store_vec<T, 4>(p + 4, f + 4);
+  } else if constexpr (V == 4)
     Elem<T>::st4(p, make_float4(f[0], f[1], f[2], f[3]));
   else
     Elem<T>::st(p, f[0]);

@@ -12,18 +12,17 @@
 
 namespace {
 
-template <typename T, int V, bool ADD>
-__global__ __launch_bounds__(256) void add_rms_next_kernel(
+template <typename T, int V, int NT, bool CONV, bool ADD>
+__global__ __launch_bounds__(NT) void add_rms_next_kernel(
     Between<T> a, const T* __restrict__ y) {
-  __shared__ float scratch[4];
   const long t = blockIdx.x;
-  between_sublayers<T, V, ADD>(a, t, scratch, [&](int c, float* x) {
+  between_sublayers<T, V, NT, CONV, ADD>(a, t, [&](int c, float* x) {
     load_vec<T, V>(y + t * a.width + c, x);
   });
 }
 
 constexpr int TILE = 64;            // rows of a tile of the list
-constexpr int ROWS = 8;             // of these per workgroup
+constexpr int ROWS = 4;             // of these per workgroup
 
 template <typename T> struct Conv {
   T* out;
@@ -55,12 +54,16 @@ template <typename T, int V> struct Rows {
 };
 
 template <typename T, int V>
-DEV Rows<T, V> rows_of(const Conv<T>& a, int s, int c) {
-  const int t0 = a.seq_start[s], slot = a.slots[s];
-  return {a.h + (long)t0 * a.width + c,
-          slot < 0 ? nullptr
-                   : a.tail + (long)slot * (a.taps - 1) * a.width + c,
-          a.positions[t0], a.taps - 1, a.width};
+DEV Rows<T, V> rows_of(const Conv<T>& a, int s, int c, bool start) {
+  const int t0 = a.seq_start[s];
+  Rows<T, V> rows{a.h + (long)t0 * a.width + c, nullptr, 0, a.taps - 1,
+                  a.width};
+  if (start) {
+    const int slot = a.slots[s];
+    if (slot >= 0) rows.tail = a.tail + (long)slot * rows.past * a.width + c;
+    rows.first = a.positions[t0];
+  }
+  return rows;
 }
 
 // the last inputs of a portion of n rows, oldest first: row i is read from
@@ -80,13 +83,17 @@ DEV void renew_tail(const Conv<T>& a, const Rows<T, V>& rows, int s, int n,
 // TAPS 0: any number, every row is read again for every tap
 template <typename T, int V, int TAPS>
 __global__ __launch_bounds__(256) void conv_kernel(Conv<T> a) {
-  const int tile = blockIdx.x / (TILE / ROWS);
+  // neighbouring rows on the same one of the 8 dies: they share past rows
+  // through its cache (the grid is a multiple of 8)
+  const unsigned b = blockIdx.x % 8 * (gridDim.x / 8) + blockIdx.x / 8;
+  const int tile = b / (TILE / ROWS);
   const int s = a.tiles[2 * tile];
-  const int r0 = a.tiles[2 * tile + 1] + blockIdx.x % (TILE / ROWS) * ROWS;
+  const int r0 = a.tiles[2 * tile + 1] + b % (TILE / ROWS) * ROWS;
   const int n = a.seq_start[s + 1] - a.seq_start[s];
   const int c = (blockIdx.y * 256 + threadIdx.x) * V;
   if (r0 >= n || c >= a.width) return;
-  const Rows<T, V> rows = rows_of<T, V>(a, s, c);
+  const bool start = r0 < max(a.taps - 1, 1);    // these meet the tail
+  const Rows<T, V> rows = rows_of<T, V>(a, s, c, start);
   T* out = a.out + (long)a.seq_start[s] * a.width + c;
   const int r1 = min(r0 + ROWS, n);
   if constexpr (TAPS > 0) {
@@ -133,7 +140,7 @@ __global__ __launch_bounds__(256) void conv_tail_kernel(Conv<T> a) {
   const int s = blockIdx.x, c = (blockIdx.y * 256 + threadIdx.x) * V;
   const int n = a.seq_start[s + 1] - a.seq_start[s];
   if (n <= 0 || c >= a.width) return;
-  renew_tail(a, rows_of<T, V>(a, s, c), s, n, c);
+  renew_tail(a, rows_of<T, V>(a, s, c, true), s, n, c);
 }
 
 template <typename T, int V>
@@ -156,13 +163,14 @@ template <typename T>
 void launch_add_rms_next(const Between<T>& a, const T* y, long rows,
                          hipStream_t stream) {
   if (rows == 0) return;
-  #define RUN(V, ADD)                                                       \
-    add_rms_next_kernel<T, V, ADD><<<(unsigned)rows, 256, 0, stream>>>(a, y)
-  if (a.width % 4 == 0) {
-    if (y) RUN(4, true); else RUN(4, false);
-  } else {
-    if (y) RUN(1, true); else RUN(1, false);
-  }
+  #define RUN(V, NT, CONV)                                                  \
+    if (y)                                                                  \
+      add_rms_next_kernel<T, V, NT, CONV, true>                             \
+          <<<(unsigned)rows, NT, 0, stream>>>(a, y);                        \
+    else                                                                    \
+      add_rms_next_kernel<T, V, NT, CONV, false>                            \
+          <<<(unsigned)rows, NT, 0, stream>>>(a, y)
+  BY_WIDTH(RUN);
   #undef RUN
 }
 

@@ -417,12 +417,11 @@ __global__ __launch_bounds__(256) void experts_sum_kernel(
   }
 }
 
-template <typename T, int V>
-__global__ __launch_bounds__(256) void experts_sum_next_kernel(Between<T> a,
-                                                               Sum<T> s) {
-  __shared__ float scratch[4];
+template <typename T, int V, int NT, bool CONV>
+__global__ __launch_bounds__(NT) void experts_sum_next_kernel(Between<T> a,
+                                                              Sum<T> s) {
   const long t = blockIdx.x;
-  between_sublayers<T, V, true>(a, t, scratch, [&](int c, float* x) {
+  between_sublayers<T, V, NT, CONV, true>(a, t, [&](int c, float* x) {
     s.template value<V>(t, c, x);
   });
 }
@@ -543,10 +542,11 @@ void launch_experts_sum_next(const Between<T>& a, const T* y, const T* shared,
                              hipStream_t stream) {
   if (rows == 0) return;
   const Sum<T> s{y, shared, identity, weight, place, n, a.width};
-  if (a.width % 4 == 0)
-    experts_sum_next_kernel<T, 4><<<(unsigned)rows, 256, 0, stream>>>(a, s);
-  else
-    experts_sum_next_kernel<T, 1><<<(unsigned)rows, 256, 0, stream>>>(a, s);
+  #define RUN(V, NT, CONV)                                                  \
+    experts_sum_next_kernel<T, V, NT, CONV>                                 \
+        <<<(unsigned)rows, NT, 0, stream>>>(a, s)
+  BY_WIDTH(RUN);
+  #undef RUN
 }
 
 #define INSTANTIATE(T)                                                      \

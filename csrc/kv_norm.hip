@@ -13,23 +13,6 @@
 
 namespace {
 
-template <typename T, int V> DEV void load_wide(const T* p, float* x) {
-  if constexpr (V == 8) {
-    load_vec<T, 4>(p, x);
-    load_vec<T, 4>(p + 4, x + 4);
-  } else {
-    load_vec<T, V>(p, x);
-  }
-}
-template <typename T, int V> DEV void store_wide(T* p, const float* x) {
-  if constexpr (V == 8) {
-    store_vec<T, 4>(p, x);
-    store_vec<T, 4>(p + 4, x + 4);
-  } else {
-    store_vec<T, V>(p, x);
-  }
-}
-
 // one head by `lanes` lanes (this one is `l`); dst may be x
 template <typename T, int V>
 DEV void norm_head(T* dst, const T* x, const float* w, int D, int l,
@@ -37,7 +20,7 @@ DEV void norm_head(T* dst, const T* x, const float* w, int D, int l,
   float ss = 0.f;
   for (int d = l * V; d < D; d += lanes * V) {
     float f[V];
-    load_wide<T, V>(x + d, f);
+    load_vec<T, V>(x + d, f);
     #pragma unroll
     for (int i = 0; i < V; ++i) ss += f[i] * f[i];
   }
@@ -45,11 +28,11 @@ DEV void norm_head(T* dst, const T* x, const float* w, int D, int l,
   const float rs = 1.f / sqrtf(ss / D + eps);
   for (int d = l * V; d < D; d += lanes * V) {
     float f[V], g[V];
-    load_wide<T, V>(x + d, f);
-    load_wide<float, V>(w + d, g);
+    load_vec<T, V>(x + d, f);
+    load_vec<float, V>(w + d, g);
     #pragma unroll
     for (int i = 0; i < V; ++i) f[i] *= rs * g[i];
-    if (dst) store_wide<T, V>(dst + d, f);
+    if (dst) store_vec<T, V>(dst + d, f);
   }
 }
 
@@ -90,7 +73,7 @@ __global__ __launch_bounds__(256) void norm_append_kernel(
     const long blk = slot_of[b] / block_size, off = slot_of[b] % block_size;
     T* dst = v_cache + (blk * G * E + c) * block_size + off;
     float x[V];
-    load_wide<T, V>(v + (row0 + b) * vs + c, x);
+    load_vec<T, V>(v + (row0 + b) * vs + c, x);
     #pragma unroll
     for (int i = 0; i < V; ++i) Elem<T>::st(dst + (long)i * block_size, x[i]);
   }

@@ -253,10 +253,19 @@ def test_attention_prefill(dtype, H, G, D, E):
 @pytest.mark.parametrize("dtype", [BF, F32])
 @pytest.mark.parametrize("chunk", [1, 2, 31, 32, 64, 65, 200, 5000, 1 << 30])
 def test_attention_prefill_chunks(dtype, chunk):
-    for H in (2, 3):               # both ways to divide a tile among waves
-        got, want = attention_case(H, 1, 16, 24, chunk, [0, 130], [300, 140],
-                                   dtype)
-        assert rel(got, want) < tol(dtype)
+    got, want = attention_case(2, 1, 16, 24, chunk, [0, 130], [300, 140],
+                               dtype)
+    assert rel(got, want) < tol(dtype)
+
+
+@pytest.mark.parametrize("D,E", [(16, 24), (40, 128), (128, 128), (64, 200),
+                                 (104, 256), (256, 256)])
+@pytest.mark.parametrize("chunk", [45, 300])
+def test_attention_prefill_by_pairs_of_heads(D, E, chunk):
+    """Enough tiles and heads that one workgroup takes two heads."""
+    got, want = attention_case(64, 2, D, E, chunk, [0, 333, 70],
+                               [700, 300, 30], BF)
+    assert rel(got, want) < 2e-2
 
 
 @pytest.mark.parametrize("dtype", [BF, F32])
