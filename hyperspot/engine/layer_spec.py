@@ -301,9 +301,9 @@ class Experts:
     by a sigmoid gate (None: there is none).  `identity` further outputs of
     the router stand for experts that return their input.  With `limit` an
     expert computes g sigmoid(1.702 g) (u + 1) from g = min(gate, limit) and
-    u = up clamped to +-limit; without, silu(gate) * up.  `over_all`: weights are the softmax over all router
-    outputs, and a correction is added to it for the choice only; otherwise
-    the softmax over the chosen."""
+    u = up clamped to +-limit; without, silu(gate) * up.  `over_all`: weights
+    are the softmax over all router outputs, and a correction is added to it
+    for the choice only; otherwise the softmax over the chosen."""
 
     experts: int
     top: int
