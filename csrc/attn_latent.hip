@@ -4,6 +4,9 @@
 // k_r rotated:                      cache [NB, 16, rank + rot]
 // Head h has k = [W_uk[h] c | k_r], v = W_uv[h] c and
 //   score(i, j) = (q_i . k_j) * scale,  i - window < j <= i.
+// The softmax denominator of head h also has exp(sink[h]), once, without a
+// value, and the head's output is multiplied by sigmoid(gate[i, h]) (null:
+// nothing).
 //
 //   q   [T, H, D + rot]  (token stride qs), the last rot of a head rotated
 //   uk  [rank, H * D]    (W_uk transposed)    uv [H * E, rank]
@@ -21,7 +24,8 @@
 
 #include <algorithm>
 
-#include "common.h"
+#include "rotary.h"
+#include "side.h"
 
 #define PAGE 16
 
@@ -34,31 +38,29 @@ constexpr float LOG2E = 1.4426950408889634f;
 DEV float exp2_fast(float x) { return __builtin_amdgcn_exp2f(x); }
 
 // ---- rotation of q, norm and rotation of a token's row, append -----------
-// One workgroup a token.  freqs holds base^(-2i/rot) in double: angles stay
-// exact to float rounding at any position.
+// One workgroup a token, blockIdx.y 0; the others have an activation of the
+// same rows.  freqs holds the angle per position of every pair; cosine and
+// sine are multiplied by `gain`.
 template <typename T, int V>
 __global__ __launch_bounds__(256) void latent_rope_append_kernel(
     T* __restrict__ q, const T* __restrict__ kv, const float* __restrict__ w,
     const long* __restrict__ positions, const double* __restrict__ freqs,
     const long* __restrict__ slot_mapping, T* __restrict__ cache, int H,
-    int D, int rank, int rot, long qs, long ks, float eps) {
+    int D, int rank, int rot, long qs, long ks, float eps, float gain,
+    SideRelu<T> side) {
   extern __shared__ float cs[];        // (cos, sin) of each pair
   __shared__ float scratch[4];
   const long row = blockIdx.x;
+  if (blockIdx.y > 0) {
+    side_relu(side, row, 1, blockIdx.y - 1);
+    return;
+  }
   const int half = rot / 2;
   for (int i = threadIdx.x; i < half; i += 256) {
-    // angle in turns, reduced to [-1/2, 1/2]
-    double a = (double)positions[row] * freqs[i] * 0.15915494309189535;
-    a -= rint(a);
-    float s, c;
-    if constexpr (sizeof(T) == 2) {
-      s = __builtin_amdgcn_sinf((float)a);       // argument in turns
-      c = __builtin_amdgcn_cosf((float)a);
-    } else {
-      sincosf((float)(a * 6.283185307179586), &s, &c);
-    }
-    cs[2 * i] = c;
-    cs[2 * i + 1] = s;
+    float c, s;
+    angle<T>(positions[row], freqs[i], &c, &s);
+    cs[2 * i] = c * gain;
+    cs[2 * i + 1] = s * gain;
   }
   __syncthreads();
   // W elements of a head at a time
@@ -74,12 +76,7 @@ __global__ __launch_bounds__(256) void latent_rope_append_kernel(
     } else {
       load_vec<T, V>(p, x);
     }
-    #pragma unroll
-    for (int i = 0; i < W; i += 2) {
-      const float c = cs[d + i], s = cs[d + i + 1], a = x[i], b = x[i + 1];
-      x[i] = a * c - b * s;
-      x[i + 1] = b * c + a * s;
-    }
+    turn_pairs<W>(x, cs + d);
     if constexpr (V == 1) {
       Elem<T>::st(p, x[0]);
       Elem<T>::st(p + 1, x[1]);
@@ -110,10 +107,11 @@ __global__ __launch_bounds__(256) void latent_rope_append_kernel(
     store_vec<T, V>(dst + c, f);
   }
   for (int i = threadIdx.x; i < half; i += 256) {
-    const float x = Elem<T>::ld(src + rank + 2 * i);
-    const float y = Elem<T>::ld(src + rank + 2 * i + 1);
-    Elem<T>::st(dst + rank + 2 * i, x * cs[2 * i] - y * cs[2 * i + 1]);
-    Elem<T>::st(dst + rank + 2 * i + 1, y * cs[2 * i] + x * cs[2 * i + 1]);
+    float x[2] = {Elem<T>::ld(src + rank + 2 * i),
+                  Elem<T>::ld(src + rank + 2 * i + 1)};
+    turn_pairs<2>(x, cs + 2 * i);
+    Elem<T>::st(dst + rank + 2 * i, x[0]);
+    Elem<T>::st(dst + rank + 2 * i + 1, x[1]);
   }
 }
 
@@ -129,8 +127,20 @@ __global__ __launch_bounds__(256) void latent_gather_kernel(
 }
 
 // ---- a small product per head ---------------------------------------------
-// out[r, h, n] = sum_k x[r, h, k] w[h, n, k] with strides; `rows_in` and
-// `rows_out` map r to rows of x and out (null: r itself)
+// sigmoid(g[row, h]), null: 1
+template <typename T> struct Gate {
+  const T* g;
+  long stride;
+
+  DEV float operator()(long row, int h) const {
+    return g ? 1.f / (1.f + Fn<T>::exp(-Elem<T>::ld(g + row * stride + h)))
+             : 1.f;
+  }
+};
+
+// out[r, h, n] = sum_k x[r, h, k] w[h, n, k] with strides, times the gate of
+// out's row; `rows_in` and `rows_out` map r to rows of x and out (null: r
+// itself)
 struct HeadGemm {
   const int* rows_in;
   const int* rows_out;
@@ -142,18 +152,20 @@ struct HeadGemm {
 template <typename T>
 __global__ __launch_bounds__(256) void head_gemm_general_kernel(
     T* __restrict__ out, const T* __restrict__ x, const T* __restrict__ w,
-    HeadGemm a) {
+    HeadGemm a, Gate<T> gate) {
   const long r = blockIdx.x;
   const int h = blockIdx.y, lane = threadIdx.x & 63;
   const T* xp = x + (a.rows_in ? a.rows_in[r] : r) * a.xr + h * a.xh;
-  T* op = out + (a.rows_out ? a.rows_out[r] : r) * a.outr + h * a.outh;
+  const long row = a.rows_out ? a.rows_out[r] : r;
+  T* op = out + row * a.outr + h * a.outh;
+  const float f = gate(row, h);
   for (int n = threadIdx.x >> 6; n < a.N; n += 4) {
     const T* wp = w + h * a.wh + n * a.wn;
     float s = 0.f;
     for (int k = lane; k < a.K; k += 64)
       s += Elem<T>::ld(xp + k) * Elem<T>::ld(wp + k);
     s = wave_reduce_sum(s);
-    if (lane == 0) Elem<T>::st(op + n, s);
+    if (lane == 0) Elem<T>::st(op + n, s * f);
   }
 }
 
@@ -161,7 +173,7 @@ __global__ __launch_bounds__(256) void head_gemm_general_kernel(
 template <int CT>
 __global__ __launch_bounds__(256) void head_gemm_kernel(
     bf16* __restrict__ out, const bf16* __restrict__ x,
-    const bf16* __restrict__ w, HeadGemm a) {
+    const bf16* __restrict__ w, HeadGemm a, Gate<bf16> gate) {
   const int lane = threadIdx.x & 63, col = lane & 15, gr = lane >> 4;
   const int n0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * 16;
   const int h = blockIdx.z;
@@ -198,10 +210,11 @@ __global__ __launch_bounds__(256) void head_gemm_kernel(
   for (int t = 0; t < CT; ++t) {
     if (!live[t]) continue;
     const long r = ((long)blockIdx.y * CT + t) * 16 + col;
-    *reinterpret_cast<uint2*>(
-        out + (a.rows_out ? a.rows_out[r] : r) * a.outr + h * a.outh + n) =
-        uint2{cvt_pk_bf16(acc[t][0], acc[t][1]),
-              cvt_pk_bf16(acc[t][2], acc[t][3])};
+    const long row = a.rows_out ? a.rows_out[r] : r;
+    const float f = gate(row, h);
+    *reinterpret_cast<uint2*>(out + row * a.outr + h * a.outh + n) =
+        uint2{cvt_pk_bf16(acc[t][0] * f, acc[t][1] * f),
+              cvt_pk_bf16(acc[t][2] * f, acc[t][3] * f)};
   }
 }
 
@@ -214,8 +227,9 @@ __global__ __launch_bounds__(256) void latent_attn_general_kernel(
     T* __restrict__ out, const T* __restrict__ qa, const T* __restrict__ q,
     const T* __restrict__ cache, const int* __restrict__ block_tables,
     const long* __restrict__ positions, const int* __restrict__ rows,
-    const int* __restrict__ row_seq, int max_blocks, int H, int D, int rank,
-    int rot, int window, float scale, long qs) {
+    const int* __restrict__ row_seq, const float* __restrict__ sink,
+    int max_blocks, int H, int D, int rank, int rot, int window, float scale,
+    long qs) {
   extern __shared__ float general_lds[];
   const int width = rank + rot;
   float* q_lds = general_lds;          // [width]
@@ -234,7 +248,7 @@ __global__ __launch_bounds__(256) void latent_attn_general_kernel(
         : Elem<T>::ld(q + row * qs + (long)h * (D + rot) + D + i - rank);
   __syncthreads();
   float acc[MAX_RPT] = {};
-  float m = -FLT_MAX, l = 0.f;
+  float m = sink ? sink[h] : -FLT_MAX, l = sink ? 1.f : 0.f;
   for (long base = lo; base <= pos; base += TILE) {
     const int n = (int)min((long)TILE, pos - base + 1);
     float s = -FLT_MAX;
@@ -301,8 +315,9 @@ __global__ __launch_bounds__(256, 2) void latent_attn_decode_kernel(
     const bf16* __restrict__ qa, const bf16* __restrict__ q,
     const bf16* __restrict__ cache, const int* __restrict__ block_tables,
     const long* __restrict__ positions, const int* __restrict__ rows,
-    const int* __restrict__ row_seq, int max_blocks, int H, int D, int rank,
-    int rot, int window, float scale2, long qs) {
+    const int* __restrict__ row_seq, const float* __restrict__ sink,
+    int max_blocks, int H, int D, int rank, int rot, int window, float scale2,
+    long qs) {
   constexpr int LS = RP + XP + 8;            // row of a staged tile
   constexpr int KC = (RP + XP) / 32;         // steps of the score product
   constexpr int QC = HT == 2 ? KC : (KC + 1) / 2;
@@ -353,7 +368,14 @@ __global__ __launch_bounds__(256, 2) void latent_attn_decode_kernel(
     for (int e = 0; e < ET; ++e) acc[t][e] = f32x4_t(0.f);
   float m[HT], l[HT];
   #pragma unroll
-  for (int t = 0; t < HT; ++t) { m[t] = -FLT_MAX; l[t] = 0.f; }
+  for (int t = 0; t < HT; ++t) {
+    m[t] = -FLT_MAX;
+    l[t] = 0.f;
+    if (sink && z == 0) {            // counted once: by a quarter of the lanes
+      m[t] = sink[min(h0 + t * 16 + col, H - 1)] * LOG2E;
+      l[t] = gr == 0 ? 1.f : 0.f;
+    }
+  }
 
   // This thread stages units tid % 8 + 8 i of token tid / 8.  Tokens past the
   // row's own read its own again (their weight is zero); padding columns are
@@ -502,7 +524,7 @@ template <int RB>
 __global__ __launch_bounds__(256) void latent_merge_values_kernel(
     bf16* __restrict__ out, const float* __restrict__ partial,
     const bf16* __restrict__ uv, const int* __restrict__ rows, long R,
-    int split, int H, int E, int rank) {
+    int split, int H, int E, int rank, long os, Gate<bf16> gate) {
   extern __shared__ __attribute__((aligned(16))) short merged[];
   __shared__ float weight[16][17];
   constexpr int RK = RB < 4 ? RB : 4;        // rows combined together
@@ -522,6 +544,8 @@ __global__ __launch_bounds__(256) void latent_merge_values_kernel(
           ? *reinterpret_cast<const short8_t*>(wp + k * 32) : short8_t{};
   };
   weights();
+  const long r = rows && col < live ? rows[r0 + col] : r0 + col;
+  const float f = col < live ? gate(r, h) : 0.f;
   {
     const int i = tid >> 4, p = tid & 15;
     const bool in = i < live && p < split;
@@ -564,7 +588,6 @@ __global__ __launch_bounds__(256) void latent_merge_values_kernel(
             cvt_pk_bf16(o[k].x, o[k].y);
     }
   __syncthreads();
-  const long r = r0 + col;
   while (n0 < E) {
     f32x4_t acc = f32x4_t(0.f);
     #pragma unroll
@@ -579,9 +602,9 @@ __global__ __launch_bounds__(256) void latent_merge_values_kernel(
     }
     const int n = n0 + gr * 4;
     if (n < E && col < live)
-      *reinterpret_cast<uint2*>(
-          out + ((rows ? rows[r] : r) * H + h) * E + n) =
-          uint2{cvt_pk_bf16(acc[0], acc[1]), cvt_pk_bf16(acc[2], acc[3])};
+      *reinterpret_cast<uint2*>(out + r * os + (long)h * E + n) =
+          uint2{cvt_pk_bf16(acc[0] * f, acc[1] * f),
+                cvt_pk_bf16(acc[2] * f, acc[3] * f)};
     n0 += gridDim.z * 64;
     if (n0 < E) weights();
   }
@@ -607,9 +630,9 @@ void latent_attn_prefill_kernel(
     const bf16* __restrict__ kn, const bf16* __restrict__ lat,
     const bf16* __restrict__ vt, const long* __restrict__ positions,
     const int* __restrict__ seq_start, const int* __restrict__ kv_start,
-    const int* __restrict__ kv_first, const int* __restrict__ tiles, int H,
-    int D, int E, int rank, int rot, long nkv, int window, float scale2,
-    long qs) {
+    const int* __restrict__ kv_first, const int* __restrict__ tiles,
+    const float* __restrict__ sink, int H, int D, int E, int rank, int rot,
+    long nkv, int window, float scale2, long qs, long os, Gate<bf16> gate) {
   constexpr int KS = DP + 8;                     // K row in LDS
   constexpr int KC = DP / 16, ET = EP / 32;
   constexpr int KLOADS = KV * DP / 8 / 256;      // 16-byte units a thread
@@ -645,6 +668,10 @@ void latent_attn_prefill_kernel(
   #pragma unroll
   for (int e = 0; e < ET; ++e) acc[e] = f32x16_t(0.f);
   float m = -FLT_MAX, l = 0.f;
+  if (sink) {                        // counted once: by half of the lanes
+    m = sink[h] * LOG2E;
+    l = hf == 0 ? 1.f : 0.f;
+  }
 
   const int last = p0 + n - 1;
   const int lo = max(0, p0 - window + 1);
@@ -765,8 +792,8 @@ void latent_attn_prefill_kernel(
   }
   l += __shfl_xor(l, 32);
   if (row >= n) return;
-  const float inv = 1.f / l;
-  bf16* orow = out + ((long)(t0 + row) * H + h) * E;
+  const float inv = gate(t0 + row, h) / l;
+  bf16* orow = out + (long)(t0 + row) * os + (long)h * E;
   #pragma unroll
   for (int e = 0; e < ET; ++e)
     #pragma unroll
@@ -798,8 +825,10 @@ void launch_latent_rope_append(T* q, const T* kv, const float* w,
                                const long* positions, const double* freqs,
                                const long* slot_mapping, T* cache, long rows,
                                int H, int D, int rank, int rot, long qs,
-                               long ks, float eps, hipStream_t stream) {
-  if (rows == 0 || (rot == 0 && !kv)) return;
+                               long ks, float eps, float gain,
+                               const SideRelu<T>& side, hipStream_t stream) {
+  if (rows == 0 || (rot == 0 && !kv && !side.n)) return;
+  const dim3 grid((unsigned)rows, 1 + side_blocks(side.n));
   const size_t lds = (rot + 2) * sizeof(float);
   auto aligned = [](const T* p) {
     return reinterpret_cast<uintptr_t>(p) % (4 * sizeof(T)) == 0;
@@ -807,13 +836,13 @@ void launch_latent_rope_append(T* q, const T* kv, const float* w,
   const bool vec = rank % 4 == 0 && rot % 4 == 0 && D % 4 == 0 &&
                    qs % 4 == 0 && ks % 4 == 0 && aligned(q) && aligned(kv);
   if (vec)
-    latent_rope_append_kernel<T, 4><<<(unsigned)rows, 256, lds, stream>>>(
+    latent_rope_append_kernel<T, 4><<<grid, 256, lds, stream>>>(
         q, kv, w, positions, freqs, slot_mapping, cache, H, D, rank, rot, qs,
-        ks, eps);
+        ks, eps, gain, side);
   else
-    latent_rope_append_kernel<T, 1><<<(unsigned)rows, 256, lds, stream>>>(
+    latent_rope_append_kernel<T, 1><<<grid, 256, lds, stream>>>(
         q, kv, w, positions, freqs, slot_mapping, cache, H, D, rank, rot, qs,
-        ks, eps);
+        ks, eps, gain, side);
 }
 
 void launch_latent_gather(bf16* out, const bf16* cache, const long* slots,
@@ -830,8 +859,10 @@ template <typename T>
 void launch_head_gemm(T* out, const T* x, const T* w, const int* rows_in,
                       const int* rows_out, long R, int H, int N, int K,
                       long xr, long xh, long wn, long wh, long outr,
-                      long outh, bool fast, hipStream_t stream) {
+                      long outh, const T* g, long gs, bool fast,
+                      hipStream_t stream) {
   if (R == 0) return;
+  const Gate<T> gate{g, gs};
   const HeadGemm a{rows_in, rows_out, R, N, K, xr, xh, wn, wh, outr, outh};
   if constexpr (sizeof(T) == 2) {
     if (fast) {
@@ -839,7 +870,7 @@ void launch_head_gemm(T* out, const T* x, const T* w, const int* rows_in,
       #define RUN(CT)                                                       \
         head_gemm_kernel<CT>                                                \
             <<<dim3(nx, (unsigned)((R + 16 * CT - 1) / (16 * CT)),          \
-                    (unsigned)H), 256, 0, stream>>>(out, x, w, a)
+                    (unsigned)H), 256, 0, stream>>>(out, x, w, a, gate)
       if (R <= 16) RUN(1);
       else RUN(2);
       #undef RUN
@@ -847,33 +878,36 @@ void launch_head_gemm(T* out, const T* x, const T* w, const int* rows_in,
     }
   }
   head_gemm_general_kernel<T>
-      <<<dim3((unsigned)R, (unsigned)H), 256, 0, stream>>>(out, x, w, a);
+      <<<dim3((unsigned)R, (unsigned)H), 256, 0, stream>>>(out, x, w, a,
+                                                           gate);
 }
 
 template <typename T>
 void launch_latent_attn_general(T* out, const T* qa, const T* q,
                                 const T* cache, const int* block_tables,
                                 const long* positions, const int* rows,
-                                const int* row_seq, long R, int max_blocks,
-                                int H, int D, int rank, int rot, int window,
-                                float scale, long qs, hipStream_t stream) {
+                                const int* row_seq, const float* sink,
+                                long R, int max_blocks, int H, int D,
+                                int rank, int rot, int window, float scale,
+                                long qs, hipStream_t stream) {
   if (R == 0) return;
   if (rank > 256 * MAX_RPT || rot > 4096)
     throw std::runtime_error("latent_attn_general: latent size");
   latent_attn_general_kernel<T>
       <<<dim3((unsigned)R, (unsigned)H), 256,
          (rank + rot + TILE) * sizeof(float), stream>>>(
-          out, qa, q, cache, block_tables, positions, rows, row_seq,
+          out, qa, q, cache, block_tables, positions, rows, row_seq, sink,
           max_blocks, H, D, rank, rot, window, scale, qs);
 }
 
 void launch_latent_attn_decode(bf16* out, float* partial, const bf16* qa,
                                const bf16* q, const bf16* cache,
                                const int* block_tables, const long* positions,
-                               const int* rows, const int* row_seq, long R,
-                               int max_blocks, int H, int D, int rank,
-                               int rot, int window, float scale, long qs,
-                               int split, hipStream_t stream) {
+                               const int* rows, const int* row_seq,
+                               const float* sink, long R, int max_blocks,
+                               int H, int D, int rank, int rot, int window,
+                               float scale, long qs, int split,
+                               hipStream_t stream) {
   if (R == 0) return;
   #define RUN(RP, XP, HT, EXACT)                                            \
     {                                                                       \
@@ -883,8 +917,8 @@ void launch_latent_attn_decode(bf16* out, float* partial, const bf16* qa,
           <<<dim3((unsigned)R, (unsigned)((H + 16 * HT - 1) / (16 * HT)),   \
                   (unsigned)split), 256, decode_lds(RP, XP), stream>>>(     \
               out, partial, qa, q, cache, block_tables, positions, rows,    \
-              row_seq, max_blocks, H, D, rank, rot, window, scale * LOG2E,  \
-              qs);                                                          \
+              row_seq, sink, max_blocks, H, D, rank, rot, window,           \
+              scale * LOG2E, qs);                                           \
       done = true;                                                          \
     }
   #define CASE(RP, XP)                                                      \
@@ -904,8 +938,8 @@ void launch_latent_attn_decode(bf16* out, float* partial, const bf16* qa,
 
 void launch_latent_merge_values(bf16* out, const float* partial,
                                 const bf16* uv, const int* rows, long R,
-                                int split, int H, int E, int rank,
-                                hipStream_t stream) {
+                                int split, int H, int E, int rank, long os,
+                                const bf16* g, long gs, hipStream_t stream) {
   if (R == 0) return;
   // few rows: fewer a workgroup, then fewer values a workgroup
   int rb = 16;
@@ -916,7 +950,8 @@ void launch_latent_merge_values(bf16* out, const float* partial,
     if (rb == RB)                                                           \
       latent_merge_values_kernel<RB>                                        \
           <<<grid, 256, 16 * (rank + 8) * 2, stream>>>(                     \
-              out, partial, uv, rows, R, split, H, E, rank);
+              out, partial, uv, rows, R, split, H, E, rank, os,             \
+              Gate<bf16>{g, gs});
   CASE(1) CASE(2) CASE(4) CASE(8) CASE(16)
   #undef CASE
 }
@@ -925,9 +960,10 @@ void launch_latent_attn_prefill(bf16* out, const bf16* q, const bf16* kn,
                                 const bf16* lat, const bf16* vt,
                                 const long* positions, const int* seq_start,
                                 const int* kv_start, const int* kv_first,
-                                const int* tiles, int num_tiles, int H, int D,
-                                int E, int rank, int rot, long nkv,
-                                int window, float scale, long qs,
+                                const int* tiles, const float* sink,
+                                int num_tiles, int H, int D, int E, int rank,
+                                int rot, long nkv, int window, float scale,
+                                long qs, long os, const bf16* g, long gs,
                                 hipStream_t stream) {
   if (num_tiles == 0) return;
   #define CASE(DP, EP)                                                      \
@@ -937,8 +973,8 @@ void launch_latent_attn_prefill(bf16* out, const bf16* q, const bf16* kn,
           <<<dim3((unsigned)num_tiles, (unsigned)H), 256,                   \
              prefill_lds(DP, EP), stream>>>(                                \
               out, q, kn, lat, vt, positions, seq_start, kv_start,          \
-              kv_first, tiles, H, D, E, rank, rot, nkv, window,             \
-              scale * LOG2E, qs);                                           \
+              kv_first, tiles, sink, H, D, E, rank, rot, nkv, window,       \
+              scale * LOG2E, qs, os, Gate<bf16>{g, gs});                    \
       return;                                                               \
     }
   CASE(64, 64) CASE(96, 64) CASE(64, 128) CASE(96, 128) CASE(128, 128)
@@ -950,14 +986,16 @@ void launch_latent_attn_prefill(bf16* out, const bf16* q, const bf16* kn,
 #define INSTANTIATE(T)                                                      \
   template void launch_latent_rope_append<T>(                               \
       T*, const T*, const float*, const long*, const double*, const long*,  \
-      T*, long, int, int, int, int, long, long, float, hipStream_t);        \
+      T*, long, int, int, int, int, long, long, float, float,               \
+      const SideRelu<T>&, hipStream_t);                                     \
   template void launch_head_gemm<T>(                                        \
       T*, const T*, const T*, const int*, const int*, long, int, int, int,  \
-      long, long, long, long, long, long, bool, hipStream_t);               \
+      long, long, long, long, long, long, const T*, long, bool,             \
+      hipStream_t);                                                         \
   template void launch_latent_attn_general<T>(                              \
       T*, const T*, const T*, const T*, const int*, const long*,            \
-      const int*, const int*, long, int, int, int, int, int, int, float,    \
-      long, hipStream_t);
+      const int*, const int*, const float*, long, int, int, int, int, int,  \
+      int, float, long, hipStream_t);
 INSTANTIATE(bf16)
 INSTANTIATE(float)
 #undef INSTANTIATE

@@ -9,6 +9,8 @@
 #include <stdexcept>
 #include <type_traits>
 
+#include "side.h"
+
 using bf16 = __hip_bfloat16;
 
 inline hipStream_t stream() {
@@ -63,4 +65,18 @@ inline void check_tiles(const torch::Tensor& tiles, const torch::Tensor& seq_sta
 
 inline float* opt(const c10::optional<torch::Tensor>& t) {
   return t.has_value() ? ptr<float>(*t) : nullptr;
+}
+
+// side activation: x and out [rows, n] column views, or neither
+template <typename T>
+SideRelu<T> side_of(const c10::optional<torch::Tensor>& x,
+                    const c10::optional<torch::Tensor>& out, long rows,
+                    torch::ScalarType dt) {
+  TORCH_CHECK(x.has_value() == out.has_value(), "side activation");
+  if (!x.has_value()) return {};
+  const long n = x->size(1);
+  check_rows(*x, dt, rows, n, x->stride(0), "side x");
+  check_rows(*out, dt, rows, n, out->stride(0), "side out");
+  return make_side<T>(ptr<T>(*x), ptr<T>(*out), x->stride(0), out->stride(0),
+                      (int)n);
 }

@@ -22,29 +22,33 @@ bool latent_sizes_fit(int, int, int, int);
 template <typename T>
 void launch_latent_rope_append(T*, const T*, const float*, const long*,
                                const double*, const long*, T*, long, int, int,
-                               int, int, long, long, float, hipStream_t);
+                               int, int, long, long, float, float,
+                               const SideRelu<T>&, hipStream_t);
 void launch_latent_gather(bf16*, const bf16*, const long*, long, int,
                           hipStream_t);
 template <typename T>
 void launch_head_gemm(T*, const T*, const T*, const int*, const int*, long,
-                      int, int, int, long, long, long, long, long, long, bool,
-                      hipStream_t);
+                      int, int, int, long, long, long, long, long, long,
+                      const T*, long, bool, hipStream_t);
 template <typename T>
 void launch_latent_attn_general(T*, const T*, const T*, const T*, const int*,
-                                const long*, const int*, const int*, long,
-                                int, int, int, int, int, int, float, long,
-                                hipStream_t);
+                                const long*, const int*, const int*,
+                                const float*, long, int, int, int, int, int,
+                                int, float, long, hipStream_t);
 void launch_latent_attn_decode(bf16*, float*, const bf16*, const bf16*,
                                const bf16*, const int*, const long*,
-                               const int*, const int*, long, int, int, int,
-                               int, int, int, float, long, int, hipStream_t);
+                               const int*, const int*, const float*, long,
+                               int, int, int, int, int, int, float, long, int,
+                               hipStream_t);
 void launch_latent_merge_values(bf16*, const float*, const bf16*, const int*,
-                                long, int, int, int, int, hipStream_t);
+                                long, int, int, int, int, long, const bf16*,
+                                long, hipStream_t);
 void launch_latent_attn_prefill(bf16*, const bf16*, const bf16*, const bf16*,
                                 const bf16*, const long*, const int*,
-                                const int*, const int*, const int*, int, int,
-                                int, int, int, int, long, int, float, long,
-                                hipStream_t);
+                                const int*, const int*, const int*,
+                                const float*, int, int, int, int, int, int,
+                                long, int, float, long, long, const bf16*,
+                                long, hipStream_t);
 void launch_experts_route(float*, int*, const float*, int, int, int, bool,
                           bool, int, const float*, hipStream_t);
 void launch_experts_sort(int*, int*, int*, const int*, int, int, int, int,
@@ -179,6 +183,22 @@ struct LatentDims {
   long H, D, E, rank, rot;
 };
 
+const float* sink_of(const Maybe& sink, long heads) {
+  if (sink.has_value()) check_param(*sink, heads, "sink");
+  return opt(sink);
+}
+
+// gate [rows, H], a column view
+template <typename T>
+const T* gate_of(const Maybe& gate, torch::ScalarType dt, long rows,
+                 long heads) {
+  if (!gate.has_value()) return nullptr;
+  check_rows(*gate, dt, rows, heads, gate->stride(0), "gate");
+  return ptr<T>(*gate);
+}
+
+long stride_of(const Maybe& t) { return t.has_value() ? t->stride(0) : 0; }
+
 // q [T, H * (D + rot)], cache [NB, 16, rank + rot], uk [rank, H * D]
 LatentDims latent_dims(const Tensor& q, const Tensor& cache, long rank,
                        long heads, long D, long E) {
@@ -191,17 +211,25 @@ LatentDims latent_dims(const Tensor& q, const Tensor& cache, long rank,
   return {heads, D, E, rank, rot};
 }
 
-bool latent_fits(Tensor q, Tensor cache, Tensor uk, Tensor uv, long heads) {
+// out [T, H * E] as a column view: rows and base for 8-byte stores
+bool out_fits(const Tensor& out) {
+  return out.stride(0) % 4 == 0 &&
+         reinterpret_cast<uintptr_t>(out.data_ptr()) % 8 == 0;
+}
+
+bool latent_fits(Tensor q, Tensor cache, Tensor uk, Tensor uv, Tensor out,
+                 long heads) {
   const long rank = uk.size(0);
   return q.scalar_type() == torch::kBFloat16 && q.stride(0) % 8 == 0 &&
-         aligned16(q) &&
+         aligned16(q) && out_fits(out) &&
          latent_sizes_fit((int)(uk.size(1) / heads), (int)(uv.size(0) / heads),
                           (int)rank, (int)(cache.size(2) - rank));
 }
 
 void latent_rope_append(Tensor q, Maybe kv, Maybe w, Tensor positions,
                         Tensor freqs, Tensor slot_mapping, Tensor cache,
-                        long heads, long rank, double eps) {
+                        long heads, long rank, double eps, double gain,
+                        Maybe side_x, Maybe side_out) {
   const long rows = q.size(0), rot = 2 * freqs.numel();
   const auto dt = q.scalar_type();
   TORCH_CHECK(heads >= 1 && q.size(1) % heads == 0 &&
@@ -226,8 +254,8 @@ void latent_rope_append(Tensor q, Maybe kv, Maybe w, Tensor positions,
         ptr<T>(q), kv.has_value() ? ptr<T>(*kv) : nullptr, opt(w),
         positions.data_ptr<long>(), freqs.data_ptr<double>(),
         slot_mapping.data_ptr<long>(), ptr<T>(cache), rows, (int)heads,
-        (int)D, (int)rank, (int)rot, q.stride(0),
-        kv.has_value() ? kv->stride(0) : 0, (float)eps, stream());
+        (int)D, (int)rank, (int)rot, q.stride(0), stride_of(kv), (float)eps,
+        (float)gain, side_of<T>(side_x, side_out, rows, dt), stream());
   });
 }
 
@@ -266,15 +294,16 @@ void latent_absorb(Tensor qa, Tensor q, Tensor uk, Maybe rows, long heads) {
     launch_head_gemm<T>(ptr<T>(qa), ptr<T>(q), ptr<T>(uk), opt_int(rows),
                         nullptr, R, (int)heads, (int)rank, (int)D,
                         q.stride(0), head, heads * D, D, heads * rank, rank,
-                        fast, stream());
+                        nullptr, 0, fast, stream());
   });
 }
 
-// out[rows[r], h] = W_uv[h] o[r, h];  o [R, H, rank], uv [H * E, rank]
-void latent_values(Tensor out, Tensor o, Tensor uv, Maybe rows) {
+// out[rows[r], h] = W_uv[h] o[r, h] sigmoid(gate[rows[r], h]);
+// o [R, H, rank], uv [H * E, rank]
+void latent_values(Tensor out, Tensor o, Tensor uv, Maybe rows, Maybe gate) {
   const auto dt = o.scalar_type();
   const long R = o.size(0), H = o.size(1), rank = o.size(2);
-  check(out, dt, "out");
+  check_rows(out, dt, out.size(0), uv.size(0), out.stride(0), "out");
   check(o, dt, "o");
   check(uv, dt, "uv");
   TORCH_CHECK(uv.size(0) % H == 0 && uv.size(1) == rank &&
@@ -288,8 +317,10 @@ void latent_values(Tensor out, Tensor o, Tensor uv, Maybe rows) {
     using T = ELEM(tag);
     launch_head_gemm<T>(ptr<T>(out), ptr<T>(o), ptr<T>(uv), nullptr,
                         opt_int(rows), R, (int)H, (int)E, (int)rank, H * rank,
-                        rank, rank, E * rank, H * E, E,
-                        E % 8 == 0 && rank % 8 == 0, stream());
+                        rank, rank, E * rank, out.stride(0), E,
+                        gate_of<T>(gate, dt, out.size(0), H), stride_of(gate),
+                        E % 8 == 0 && rank % 8 == 0 && out_fits(out),
+                        stream());
   });
 }
 
@@ -321,7 +352,8 @@ LatentDims check_absorbed(const Tensor& o, const Tensor& qa, const Tensor& q,
 
 void latent_attn_general(Tensor o, Tensor qa, Tensor q, Tensor cache,
                          Tensor block_tables, Tensor positions, Maybe rows,
-                         Maybe row_seq, long window, double scale) {
+                         Maybe row_seq, long window, double scale,
+                         Maybe sink) {
   const auto d = check_absorbed(o, qa, q, cache, block_tables, positions,
                                 rows, row_seq, window);
   by_dtype(q, [&](auto tag) {
@@ -329,7 +361,7 @@ void latent_attn_general(Tensor o, Tensor qa, Tensor q, Tensor cache,
     launch_latent_attn_general<T>(
         ptr<T>(o), ptr<T>(qa), ptr<T>(q), ptr<T>(cache),
         block_tables.data_ptr<int>(), positions.data_ptr<long>(),
-        opt_int(rows), opt_int(row_seq), qa.size(0),
+        opt_int(rows), opt_int(row_seq), sink_of(sink, d.H), qa.size(0),
         (int)block_tables.size(1), (int)d.H, (int)d.D, (int)d.rank,
         (int)d.rot, (int)window, (float)scale, q.stride(0), stream());
   });
@@ -339,8 +371,8 @@ void latent_attn_general(Tensor o, Tensor qa, Tensor q, Tensor cache,
 // latent_merge_values, [R, H, split, rank + 4] float
 void latent_attn_decode(Tensor o, Tensor qa, Tensor q, Tensor cache,
                         Tensor block_tables, Tensor positions, Maybe rows,
-                        Maybe row_seq, long split, long window,
-                        double scale) {
+                        Maybe row_seq, long split, long window, double scale,
+                        Maybe sink) {
   const auto d = check_absorbed(split > 1 ? qa : o, qa, q, cache,
                                 block_tables, positions, rows, row_seq,
                                 window);
@@ -355,18 +387,20 @@ void latent_attn_decode(Tensor o, Tensor qa, Tensor q, Tensor cache,
       split > 1 ? nullptr : ptr<bf16>(o), split > 1 ? ptr<float>(o) : nullptr,
       ptr<bf16>(qa), ptr<bf16>(q), ptr<bf16>(cache),
       block_tables.data_ptr<int>(), positions.data_ptr<long>(),
-      opt_int(rows), opt_int(row_seq), qa.size(0),
+      opt_int(rows), opt_int(row_seq), sink_of(sink, d.H), qa.size(0),
       (int)block_tables.size(1), (int)d.H, (int)d.D, (int)d.rank, (int)d.rot,
       (int)window, (float)scale, q.stride(0), (int)split, stream());
 }
 
 // out[rows[r], h] = W_uv[h] (combined partial results of r and h)
+//                   sigmoid(gate[rows[r], h])
 void latent_merge_values(Tensor out, Tensor partial, Tensor uv, Maybe rows,
-                         long R, long heads, long split) {
-  check(out, torch::kBFloat16, "out");
-  check(uv, torch::kBFloat16, "uv");
+                         long R, long heads, long split, Maybe gate) {
+  const auto dt = torch::kBFloat16;
+  check_rows(out, dt, out.size(0), uv.size(0), out.stride(0), "out");
+  check(uv, dt, "uv");
   const long E = uv.size(0) / heads, rank = uv.size(1);
-  TORCH_CHECK(uv.size(0) == heads * E && out.size(1) == heads * E &&
+  TORCH_CHECK(uv.size(0) == heads * E && out_fits(out) &&
                   latent_sizes_fit(8, (int)E, (int)rank, 8) && split >= 1 &&
                   split <= 16, "latent_merge_values: sizes");
   check_param(partial, R * heads * split * (rank + 4), "partial");
@@ -376,15 +410,17 @@ void latent_merge_values(Tensor out, Tensor partial, Tensor uv, Maybe rows,
     TORCH_CHECK(R == out.size(0), "latent_merge_values: rows");
   launch_latent_merge_values(ptr<bf16>(out), ptr<float>(partial),
                              ptr<bf16>(uv), opt_int(rows), R, (int)split,
-                             (int)heads, (int)E, (int)rank, stream());
+                             (int)heads, (int)E, (int)rank, out.stride(0),
+                             gate_of<bf16>(gate, dt, out.size(0), heads),
+                             stride_of(gate), stream());
 }
 
 void latent_attn_prefill(Tensor out, Tensor q, Tensor kn, Tensor lat,
                          Tensor vt, Tensor positions, Tensor seq_start,
                          Tensor kv_start, Tensor kv_first, Tensor tiles,
-                         long heads, long window, double scale) {
+                         long heads, long window, double scale, Maybe sink,
+                         Maybe gate) {
   const auto dt = torch::kBFloat16;
-  check(out, dt, "out");
   check(kn, dt, "kn");
   check(lat, dt, "lat");
   check(vt, dt, "vt");
@@ -398,8 +434,8 @@ void latent_attn_prefill(Tensor out, Tensor q, Tensor kn, Tensor lat,
                   latent_sizes_fit((int)D, (int)E, (int)rank, (int)rot),
               "latent_attn_prefill: sizes");
   check_rows(q, dt, q.size(0), heads * (D + rot), q.stride(0), "q");
-  TORCH_CHECK(out.numel() == q.size(0) * heads * E && window >= 1,
-              "latent_attn_prefill: out");
+  check_rows(out, dt, q.size(0), heads * E, out.stride(0), "out");
+  TORCH_CHECK(out_fits(out) && window >= 1, "latent_attn_prefill: out");
   check(positions, torch::kInt64, "positions");
   TORCH_CHECK(positions.numel() == q.size(0), "latent_attn_prefill: rows");
   const long B = seq_start.numel() - 1;
@@ -410,9 +446,10 @@ void latent_attn_prefill(Tensor out, Tensor q, Tensor kn, Tensor lat,
       ptr<bf16>(out), ptr<bf16>(q), ptr<bf16>(kn), ptr<bf16>(lat),
       ptr<bf16>(vt), positions.data_ptr<long>(), seq_start.data_ptr<int>(),
       kv_start.data_ptr<int>(), kv_first.data_ptr<int>(),
-      tiles.data_ptr<int>(), (int)tiles.size(0), (int)heads, (int)D, (int)E,
-      (int)rank, (int)rot, nkv, (int)window, (float)scale, q.stride(0),
-      stream());
+      tiles.data_ptr<int>(), sink_of(sink, heads), (int)tiles.size(0),
+      (int)heads, (int)D, (int)E, (int)rank, (int)rot, nkv, (int)window,
+      (float)scale, q.stride(0), out.stride(0),
+      gate_of<bf16>(gate, dt, q.size(0), heads), stride_of(gate), stream());
 }
 
 // ---- experts --------------------------------------------------------------

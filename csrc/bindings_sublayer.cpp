@@ -1,6 +1,7 @@
-// Bindings of sublayer inputs, head norms and chunked sigmoid attention
-// (conv.hip, kv_norm.hip, attn_sigmoid.hip, the activations of act.hip and
-// the closing step of experts.hip).
+// Bindings of sublayer inputs, head norms, chunked sigmoid attention and
+// windowed attention with kept tokens (conv.hip, kv_norm.hip, rope_norm.hip,
+// attn_sigmoid.hip, attn_kept.hip, the activations of act.hip and the closing
+// step of experts.hip).
 #include "bindings.h"
 #include "sublayer.h"
 
@@ -32,6 +33,27 @@ void launch_sigmoid_attn_decode(bf16*, const bf16*, const bf16*, const bf16*,
                                 const int*, const long*, const float*, float*,
                                 long, int, int, int, int, int, int, float,
                                 float, long, int, hipStream_t);
+template <typename T>
+void launch_rope_norm_append(T*, const T*, const T*, const long*,
+                             const double*, const double*, const long*, T*,
+                             T*, long, int, int, int, int, int, int, int,
+                             long, long, long, float, float, bool,
+                             const SideRelu<T>&, hipStream_t);
+template <typename T>
+void launch_kept_attn_general(T*, const T*, const T*, const T*, const int*,
+                              const long*, const int*, const double*,
+                              const float*, long, int, int, int, int, int,
+                              int, int, float, long, long, hipStream_t);
+void launch_kept_attn_prefill(bf16*, const bf16*, const bf16*, const bf16*,
+                              const int*, const long*, const int*, const int*,
+                              const double*, const float*, int, int, int, int,
+                              int, int, int, int, float, long, long,
+                              hipStream_t);
+void launch_kept_attn_decode(bf16*, const bf16*, const bf16*, const bf16*,
+                             const int*, const long*, const double*,
+                             const float*, float*, long, int, int, int, int,
+                             int, int, int, float, long, long, int,
+                             hipStream_t);
 template <typename T>
 void launch_clamped_glu(T*, const T*, long, int, float, hipStream_t);
 template <typename T> void launch_squared_relu(T*, long, hipStream_t);
@@ -88,7 +110,7 @@ Between<T> between(const Tensor& out, const Tensor& residual, const Maybe& w,
 void add_rms_next(Tensor out, Tensor residual, Maybe y, Maybe w, Tensor pre,
                   double eps, Maybe conv, Maybe tail, Maybe slots,
                   Maybe positions) {
-  TORCH_CHECK(y.has_value() == w.has_value(), "add_rms_next: y");
+  TORCH_CHECK(y.has_value() || !w.has_value(), "add_rms_next: y");
   if (y.has_value()) {
     check(*y, out.scalar_type(), "y");
     TORCH_CHECK(y->numel() == residual.numel(), "add_rms_next: y");
@@ -307,6 +329,140 @@ void sigmoid_attn_decode(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
       (float)cap, q.stride(0), (int)split, stream());
 }
 
+// freqs [rot / 2] and turn [E / 2 or none] float64
+void rope_norm_append(Tensor q, Tensor k, Tensor v, Tensor positions,
+                      Tensor freqs, Tensor turn, Tensor slot_mapping,
+                      Tensor k_cache, Tensor v_cache, double gain,
+                      c10::optional<double> eps, Maybe side_x,
+                      Maybe side_out) {
+  const auto dt = q.scalar_type();
+  const auto d = check_heads(q, k_cache, v_cache);
+  const long rows = q.size(0);
+  check_rows(k, dt, rows, (long)d.G * d.D, k.stride(0), "k");
+  check_rows(v, dt, rows, (long)d.G * d.E, v.stride(0), "v");
+  check(positions, torch::kInt64, "positions");
+  check(slot_mapping, torch::kInt64, "slot_mapping");
+  check(freqs, torch::kFloat64, "freqs");
+  check(turn, torch::kFloat64, "turn");
+  const long rot = 2 * freqs.numel(), vrot = 2 * turn.numel();
+  TORCH_CHECK(positions.numel() == rows && slot_mapping.numel() == rows,
+              "rope_norm_append: rows");
+  TORCH_CHECK(rot <= d.D && (vrot == 0 || vrot == d.E) && rot + vrot <= 8192,
+              "rope_norm_append: rotated sizes");
+  by_dtype(q, [&](auto tag) {
+    using T = ELEM(tag);
+    launch_rope_norm_append<T>(
+        ptr<T>(q), ptr<T>(k), ptr<T>(v), positions.data_ptr<long>(),
+        freqs.data_ptr<double>(), turn.data_ptr<double>(),
+        slot_mapping.data_ptr<long>(), ptr<T>(k_cache), ptr<T>(v_cache), rows,
+        d.H, d.G, d.D, d.E, (int)rot, (int)vrot, 16, q.stride(0), k.stride(0),
+        v.stride(0), (float)gain, (float)eps.value_or(0.0), eps.has_value(),
+        side_of<T>(side_x, side_out, rows, dt), stream());
+  });
+}
+
+// 16-byte loads of q and 8-byte stores of out (rows and bases), sizes of the
+// padded kernels
+bool kept_attn_fits(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache) {
+  return sigmoid_attn_fits(q, k_cache, v_cache) && out.stride(0) % 4 == 0 &&
+         reinterpret_cast<uintptr_t>(out.data_ptr()) % 8 == 0;
+}
+
+struct KeptArgs {
+  HeadDims d;
+  const double* turn;
+  const float* sink;
+};
+
+KeptArgs check_kept(const Tensor& out, const Tensor& q, const Tensor& k_cache,
+                    const Tensor& v_cache, const Tensor& block_tables,
+                    const Tensor& positions, const Tensor& turn,
+                    const Maybe& sink, long window, long keep) {
+  const auto d = check_heads(q, k_cache, v_cache);
+  check_rows(out, q.scalar_type(), q.size(0), (long)d.H * d.E, out.stride(0),
+             "out");
+  check(block_tables, torch::kInt32, "block_tables");
+  check(positions, torch::kInt64, "positions");
+  check(turn, torch::kFloat64, "turn");
+  TORCH_CHECK(turn.numel() == 0 || 2 * turn.numel() == d.E,
+              "kept_attn: turn");
+  constexpr long most = 1L << 30;
+  TORCH_CHECK(positions.numel() == q.size(0) && window >= 1 &&
+                  window <= most && keep >= 0 && keep <= most,
+              "kept_attn: rows, window");
+  if (sink.has_value()) check_param(*sink, d.H, "sink");
+  return {d, turn.numel() ? turn.data_ptr<double>() : nullptr, opt(sink)};
+}
+
+void kept_attn_general(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
+                       Tensor block_tables, Tensor positions, Maybe row_seq,
+                       Tensor turn, Maybe sink, long window, long keep,
+                       double scale) {
+  const auto a = check_kept(out, q, k_cache, v_cache, block_tables, positions,
+                            turn, sink, window, keep);
+  const long rows = q.size(0);
+  TORCH_CHECK(a.d.E <= 1024 && a.d.D <= 8192, "kept_attn: head sizes");
+  const int* rs = nullptr;
+  if (row_seq.has_value()) {
+    check(*row_seq, torch::kInt32, "row_seq");
+    TORCH_CHECK(row_seq->numel() == rows, "kept_attn: row_seq");
+    rs = row_seq->data_ptr<int>();
+  } else {
+    TORCH_CHECK(block_tables.size(0) >= rows, "kept_attn: block_tables");
+  }
+  by_dtype(q, [&](auto tag) {
+    using T = ELEM(tag);
+    launch_kept_attn_general<T>(
+        ptr<T>(out), ptr<T>(q), ptr<T>(k_cache), ptr<T>(v_cache),
+        block_tables.data_ptr<int>(), positions.data_ptr<long>(), rs, a.turn,
+        a.sink, rows, (int)block_tables.size(1), a.d.H, a.d.G, a.d.D, a.d.E,
+        (int)window, (int)keep, (float)scale, q.stride(0), out.stride(0),
+        stream());
+  });
+}
+
+void kept_attn_prefill(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
+                       Tensor block_tables, Tensor positions,
+                       Tensor seq_start, Tensor tiles, Tensor turn,
+                       Maybe sink, long window, long keep, double scale) {
+  const auto a = check_kept(out, q, k_cache, v_cache, block_tables, positions,
+                            turn, sink, window, keep);
+  TORCH_CHECK(kept_attn_fits(out, q, k_cache, v_cache), "kept_attn: sizes");
+  check_tiles(tiles, seq_start, block_tables.size(0));
+  TORCH_CHECK(tiles.size(0) <= 65535, "kept_attn: tiles");
+  launch_kept_attn_prefill(
+      ptr<bf16>(out), ptr<bf16>(q), ptr<bf16>(k_cache), ptr<bf16>(v_cache),
+      block_tables.data_ptr<int>(), positions.data_ptr<long>(),
+      seq_start.data_ptr<int>(), tiles.data_ptr<int>(), a.turn, a.sink,
+      (int)tiles.size(0), (int)block_tables.size(1), a.d.H, a.d.G, a.d.D,
+      a.d.E, (int)window, (int)keep, (float)scale, q.stride(0),
+      out.stride(0), stream());
+}
+
+// partial [rows, H, split, E + 4] float where split > 1
+void kept_attn_decode(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
+                      Tensor block_tables, Tensor positions, Tensor turn,
+                      Maybe sink, Maybe partial, long split, long window,
+                      long keep, double scale) {
+  const auto a = check_kept(out, q, k_cache, v_cache, block_tables, positions,
+                            turn, sink, window, keep);
+  const long rows = q.size(0);
+  TORCH_CHECK(kept_attn_fits(out, q, k_cache, v_cache), "kept_attn: sizes");
+  TORCH_CHECK(block_tables.size(0) >= rows && split >= 1 && split <= 64,
+              "kept_attn_decode: rows, split");
+  if (split > 1) {
+    TORCH_CHECK(partial.has_value(), "kept_attn_decode: partial");
+    check_param(*partial, rows * a.d.H * split * (a.d.E + 4), "partial");
+  }
+  launch_kept_attn_decode(
+      ptr<bf16>(out), ptr<bf16>(q), ptr<bf16>(k_cache), ptr<bf16>(v_cache),
+      block_tables.data_ptr<int>(), positions.data_ptr<long>(), a.turn,
+      a.sink, split > 1 ? ptr<float>(*partial) : nullptr, rows,
+      (int)block_tables.size(1), a.d.H, a.d.G, a.d.D, a.d.E, (int)window,
+      (int)keep, (float)scale, q.stride(0), out.stride(0), (int)split,
+      stream());
+}
+
 }  // namespace
 
 void register_sublayer(pybind11::module_& m) {
@@ -316,6 +472,11 @@ void register_sublayer(pybind11::module_& m) {
   m.def("clamped_glu", &clamped_glu);
   m.def("squared_relu", &squared_relu);
   m.def("norm_append", &norm_append);
+  m.def("rope_norm_append", &rope_norm_append);
+  m.def("kept_attn_fits", &kept_attn_fits);
+  m.def("kept_attn_general", &kept_attn_general);
+  m.def("kept_attn_prefill", &kept_attn_prefill);
+  m.def("kept_attn_decode", &kept_attn_decode);
   m.def("sigmoid_attn_fits", &sigmoid_attn_fits);
   m.def("sigmoid_attn_general", &sigmoid_attn_general);
   m.def("sigmoid_attn_prefill", &sigmoid_attn_prefill);

@@ -12,7 +12,7 @@
 
 namespace {
 
-template <typename T, int V, int NT, bool CONV, bool ADD>
+template <typename T, int V, int NT, bool CONV, int ADD>
 __global__ __launch_bounds__(NT) void add_rms_next_kernel(
     Between<T> a, const T* __restrict__ y) {
   const long t = blockIdx.x;
@@ -163,15 +163,16 @@ template <typename T>
 void launch_add_rms_next(const Between<T>& a, const T* y, long rows,
                          hipStream_t stream) {
   if (rows == 0) return;
+  #define ADD(V, NT, CONV, HOW)                                             \
+    add_rms_next_kernel<T, V, NT, CONV, HOW>                                \
+        <<<(unsigned)rows, NT, 0, stream>>>(a, y)
   #define RUN(V, NT, CONV)                                                  \
-    if (y)                                                                  \
-      add_rms_next_kernel<T, V, NT, CONV, true>                             \
-          <<<(unsigned)rows, NT, 0, stream>>>(a, y);                        \
-    else                                                                    \
-      add_rms_next_kernel<T, V, NT, CONV, false>                            \
-          <<<(unsigned)rows, NT, 0, stream>>>(a, y)
+    if (!y) ADD(V, NT, CONV, ADD_NOTHING);                                  \
+    else if (a.post) ADD(V, NT, CONV, ADD_NORMED);                          \
+    else ADD(V, NT, CONV, ADD_PLAIN)
   BY_WIDTH(RUN);
   #undef RUN
+  #undef ADD
 }
 
 template <typename T>

@@ -421,7 +421,7 @@ template <typename T, int V, int NT, bool CONV>
 __global__ __launch_bounds__(NT) void experts_sum_next_kernel(Between<T> a,
                                                               Sum<T> s) {
   const long t = blockIdx.x;
-  between_sublayers<T, V, NT, CONV, true>(a, t, [&](int c, float* x) {
+  between_sublayers<T, V, NT, CONV, ADD_NORMED>(a, t, [&](int c, float* x) {
     s.template value<V>(t, c, x);
   });
 }

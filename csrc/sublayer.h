@@ -1,6 +1,7 @@
 // Between two sublayers, one row by a workgroup:
 //
-//   residual += rms(y) * post          (not before the first sublayer)
+//   residual += rms(y) * post          (not before the first sublayer), or
+//   residual += y                      (no norm after a sublayer)
 //   h = rms(residual) * pre, rounded to T
 //   out = h, or for a decoded token h + sum_j conv[j] * (input taps-1-j ago)
 //
@@ -131,7 +132,10 @@ template <typename T, int V> struct NoConv {
   DEV void apply(int, float*, bool) const {}
 };
 
-template <typename T, int V, int NT, bool CONV, bool ADD, typename Value>
+// how y enters the residual
+enum { ADD_NOTHING, ADD_NORMED, ADD_PLAIN };
+
+template <typename T, int V, int NT, bool CONV, int ADD, typename Value>
 DEV void between_sublayers(const Between<T>& a, long t, Value value) {
   constexpr int HELD = CONV ? 1 : 4;
   const int tid = threadIdx.x, n = a.width;
@@ -143,7 +147,7 @@ DEV void between_sublayers(const Between<T>& a, long t, Value value) {
       a, t, tid * V);
   if (CONV && tid * V < n) {
     load_vec<float, V>(a.pre + tid * V, pre0);
-    if (ADD) load_vec<float, V>(a.post + tid * V, post0);
+    if (ADD == ADD_NORMED) load_vec<float, V>(a.post + tid * V, post0);
     load_vec<float, V>(res + tid * V, res0);
   }
   auto squares = [&](const float* x) {
@@ -171,7 +175,7 @@ DEV void between_sublayers(const Between<T>& a, long t, Value value) {
       body(c, x, false);
     }
   };
-  if constexpr (ADD) {
+  if constexpr (ADD == ADD_NORMED) {
     columns([&](int c, float* x, bool) {
       value(c, x);
       squares(x);
@@ -191,6 +195,13 @@ DEV void between_sublayers(const Between<T>& a, long t, Value value) {
   } else {
     columns([&](int c, float* x, bool is_held) {
       fetch(res, res0, c, is_held, x);
+      if constexpr (ADD == ADD_PLAIN) {
+        float y[V];
+        value(c, y);
+        #pragma unroll
+        for (int j = 0; j < V; ++j) x[j] += y[j];
+        store_vec<float, V>(res + c, x);
+      }
       squares(x);
     });
   }

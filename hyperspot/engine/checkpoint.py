@@ -87,6 +87,17 @@ def _full_from_shards(param: torch.Tensor, group) -> torch.Tensor:
     return full
 
 
+def _without_padding(param: torch.Tensor) -> torch.Tensor:
+    """The full tensor of a parameter that is not divided."""
+    t = param.detach().contiguous().cpu()
+    if tuple(t.shape) == tuple(param._tp_full_shape):
+        return t
+    full, dim = t.new_empty(param._tp_full_shape), param._tp_shard_dim
+    for f0, ln, s0 in param._tp_slices:
+        full.narrow(dim, f0, ln).copy_(t.narrow(dim, s0, ln))
+    return full
+
+
 def _slices_for_rank(param: torch.Tensor, r: int):
     """Derive rank r's slices from this rank's slice pattern.  Within
     each section the full_start is section_base + r*length; section_base
@@ -112,7 +123,7 @@ def save_checkpoint(model, path: str, meta: Dict = None) -> None:
         if getattr(v, "_tp_slices", None) is not None:
             group, _, size = _shard_group_of(v)
             state[k] = (_full_from_shards(v, group) if size > 1
-                        else v.detach().contiguous().cpu())
+                        else _without_padding(v))
         else:
             state[k] = v.detach().contiguous().cpu()
     if dist.is_initialized() and dist.get_rank() != 0:

@@ -1,11 +1,12 @@
 """Per-layer descriptions for models whose layers are not all alike.
 
 A ``HybridSpec`` is a ``ModelSpec`` with an explicit list of layers, each one
-mixer (windowed differential attention, windowed latent attention, chunked
-sigmoid attention, gated linear attention, matrix LSTM, lightning attention)
-and an optional feed-forward (dense, or a mixture of experts).  Every size and
-constant of a layer part is a field here; the layer classes in
-``hyperspot.models.mixers`` read nothing else.
+mixer (windowed differential attention, windowed latent attention, windowed
+softmax attention with kept first tokens, chunked sigmoid attention, gated
+linear attention, matrix LSTM, lightning attention) and an optional
+feed-forward (dense, or a mixture of experts).  Every size and constant of a
+layer part is a field here; the layer classes in ``hyperspot.models.mixers``
+read nothing else.
 
 ``cache_layout`` tells the cache manager what a layer keeps per sequence:
 pages that grow with the tokens (``PagedKV``, ``LatentPages``), a fixed-size
@@ -16,10 +17,14 @@ over the tensor-parallel ranks.
 
 from __future__ import annotations
 
-from dataclasses import dataclass, field
+from dataclasses import dataclass, field, replace
 from typing import List, Optional, Tuple, Union
 
 from .config import ModelSpec
+from .rotary import Stretch, Yarn
+
+# a window that holds every position
+UNBOUNDED = 1 << 30
 
 
 # ------------------------------------------------------------- cache layout
@@ -188,7 +193,10 @@ class MatrixLSTM:
 class LatentAttention:
     """Sliding-window attention whose keys and values are expanded per head
     from one latent per token; a rotated key part is shared by all heads.
-    With `kv_from` the latents are those of an earlier layer."""
+    With `kv_from` the latents are those of an earlier layer.  `halves`: a
+    checkpoint's rotated pairs lie half the rotated size apart; `sink`: every
+    head's softmax has a learned score without a value in its denominator;
+    `gate`: a sigmoid of the input scales every head's output."""
 
     heads: int
     dim: int            # unrotated query/key size per head
@@ -199,6 +207,10 @@ class LatentAttention:
     window: int
     rot_base: float
     kv_from: Optional[int] = None
+    stretch: Stretch = 1.0
+    halves: bool = False
+    sink: bool = False
+    gate: bool = False
 
     def cache(self, tp: int) -> Union[LatentPages, SharedCache]:
         if self.kv_from is not None:
@@ -210,13 +222,14 @@ class LatentAttention:
              + self.kv_rank * self.heads * (self.dim + self.vdim))
         if self.kv_from is None:
             n += width * (self.kv_rank + self.rot_dim) + self.kv_rank
-        return n
+        return n + self.heads * (self.sink + width * self.gate)
 
     def check(self) -> None:
         if self.rot_dim % 2:
             raise ValueError("latent attention: rotary size must be even")
         if self.window < 1:
             raise ValueError("latent attention: window must be at least 1")
+        check_rotation(self.rot_base, self.stretch)
 
 
 @dataclass(frozen=True)
@@ -274,8 +287,65 @@ class SigmoidAttention:
             raise ValueError("attention: the score cap must be positive")
 
 
+@dataclass(frozen=True)
+class WindowAttention:
+    """Grouped-query softmax attention over a sliding window and the first
+    `keep_first` tokens of the sequence.
+
+    The first `rot_dims` dimensions of queries and keys are rotated, in pairs
+    half that size apart with `halves`; with `qk_norm` every head of both is
+    then divided by its root mean square.  With `turn_values` the value of
+    position j is turned by j over all its dimensions before it is kept, and
+    position i's output back by i.  `sink` is a fixed score without a value in
+    the softmax denominator (None: there is none)."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    window: int
+    rot_dims: int
+    rot_base: float
+    keep_first: int = 0
+    stretch: Stretch = 1.0
+    halves: bool = False
+    qk_norm: bool = False
+    turn_values: bool = False
+    sink: Optional[float] = None
+
+    def cache(self, tp: int) -> PagedKV:
+        return PagedKV(self.kv_heads // tp, self.dim, self.vdim,
+                       v_transposed=True)
+
+    def params(self, width: int) -> int:
+        return width * (self.heads + self.kv_heads) * (self.dim + self.vdim)
+
+    def check(self) -> None:
+        if self.heads % self.kv_heads:
+            raise ValueError("attention: heads must be a multiple of kv_heads")
+        if self.rot_dims % 2 or not 0 <= self.rot_dims <= self.dim:
+            raise ValueError("attention: rotary dims must be even and <= dim")
+        if self.turn_values and self.vdim % 2:
+            raise ValueError("attention: turned values must have an even size")
+        if self.window < 1 or self.keep_first < 0:
+            raise ValueError("attention: window must be at least 1, kept "
+                             "tokens at least 0")
+        check_rotation(self.rot_base, self.stretch)
+
+
+def check_rotation(base: float, stretch: Stretch) -> None:
+    if base <= 0 or isinstance(stretch, Yarn) and base == 1:
+        raise ValueError("rotation: the base must be positive, with YaRN "
+                         "other than 1")
+    if isinstance(stretch, Yarn):
+        stretch.check()
+    elif not stretch > 0:
+        raise ValueError("rotation: the factor must be positive")
+
+
 Mixer = Union[DiffAttention, GatedLinear, MatrixLSTM, LatentAttention,
-              Lightning, SigmoidAttention]
+              Lightning, SigmoidAttention, WindowAttention]
 
 
 # ------------------------------------------------------------- feed-forward
@@ -346,6 +416,8 @@ class HybridSpec(ModelSpec):
     layers: Tuple[LayerSpec, ...] = field(default_factory=tuple)
     norm_params: int = 0          # parameters of one norm
     norms: int = 2                # norms per sublayer
+    # mixer and feed-forward read one normed input; both are added at once
+    parallel: bool = False
     embed_scale: float = 1.0
     # size of a token's own input to every layer (0: there is none)
     side_dim: int = 0
@@ -364,7 +436,7 @@ class HybridSpec(ModelSpec):
             if layer.ff is not None:
                 n += 3 * h * layer.ff if isinstance(layer.ff, int) \
                     else layer.ff.params(h)
-                n += sublayer
+                n += 0 if self.parallel else sublayer
             if self.side_dim:
                 n += (self.vocab_size + 2 * h) * self.side_dim + h
         return n
@@ -414,6 +486,17 @@ def hybrid_spec(name: str, architecture: str, width: int, vocab: int,
         layers=layers, **kw)
 
 
+def looped(layers, start: int, stop: int, times: int) -> List[LayerSpec]:
+    """Layer runs in which layers start ... stop - 1 come `times` times in a
+    row, later passes with the tensors of the first and caches of their
+    own."""
+    if not 0 <= start <= stop <= len(layers) or times < 1:
+        raise ValueError(f"loop: layers {start} ... {stop - 1}, {times} times, "
+                         f"of {len(layers)}")
+    again = [replace(layers[i], weights_of=i) for i in range(start, stop)]
+    return [*layers[:stop], *again * (times - 1), *layers[stop:]]
+
+
 def _check_shared_cache(layers, i: int) -> None:
     m = layers[i].mixer
     j = getattr(m, "kv_from", None)
@@ -423,8 +506,8 @@ def _check_shared_cache(layers, i: int) -> None:
     if not isinstance(o, LatentAttention) or o.kv_from is not None:
         raise ValueError(f"layer {i}: kv_from must name an earlier "
                          "latent-attention layer with latents of its own")
-    if (o.kv_rank, o.rot_dim, o.rot_base) != (m.kv_rank, m.rot_dim,
-                                              m.rot_base):
+    rotated = lambda x: (x.kv_rank, x.rot_dim, x.rot_base, x.stretch, x.halves)
+    if rotated(o) != rotated(m):
         raise ValueError(f"layer {i}: latent sizes and rotation differ from "
                          f"layer {j}'s")
 

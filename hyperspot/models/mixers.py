@@ -19,10 +19,12 @@ from torch import nn
 from hyperspot.engine.layer_spec import (DiffAttention, Experts, GatedLinear,
                                          LatentAttention, Lightning,
                                          MatrixLSTM, SigmoidAttention,
-                                         SquaredRelu)
+                                         SquaredRelu, WindowAttention)
+from hyperspot.engine.rotary import (frequencies, gain, head_order,
+                                     pair_order)
 from hyperspot.ops import experts, hybrid, latent
 from hyperspot.parallel import (MergedColumnParallelLinear,
-                                RowParallelLinear)
+                                MergedRowParallelLinear, RowParallelLinear)
 from hyperspot.parallel.layers import _init_weight
 from hyperspot.parallel.state import (get_ep_size, get_tp_rank, get_tp_size,
                                       tensor_model_parallel_all_reduce)
@@ -424,59 +426,154 @@ class ChunkedSigmoidAttention(nn.Module):
                                          get_tp_rank())
 
 
-class WindowLatentAttention(nn.Module):
-    def __init__(self, spec: LatentAttention, width: int, eps: float, dtype,
-                 tag: int):
+class JoinedMixer(nn.Module):
+    """A mixer that may have a dense feed-forward beside it, both reading one
+    input and their outputs added: one product makes all projections of the
+    input, one reduces the joined results [mixer | feed-forward], which adds
+    them.  The activation rides along with the kernel that rotates."""
+
+    def _join(self, width: int, parts: list, out: int, ff, dtype, tag: int,
+              replicated: tuple = ()) -> None:
+        if ff is not None and not isinstance(ff, SquaredRelu):
+            raise ValueError("only a dense squared-ReLU feed-forward runs "
+                             "beside a mixer")
+        self.width, self.ff, self.out_size = width, ff, out
+        hidden = [] if ff is None else [ff.ff]
+        self.proj = MergedColumnParallelLinear(
+            width, parts + hidden, dtype, seed_tag=tag,
+            replicated=replicated, align=8)
+        self.o_proj = MergedRowParallelLinear([out] + hidden, width, dtype,
+                                              seed_tag=tag + len(parts) + 1)
+
+    def enter(self, x: torch.Tensor):
+        """The mixer's projections, its place in the joined results, these,
+        and the activation to ride along (None: no feed-forward)."""
+        parts = self.proj.split(self.proj(x))
+        n = sum(self.o_proj.shard_sizes)
+        joined = x.new_empty(x.shape[0], (n + 7) // 8 * 8)[:, :n]
+        if self.ff is None:
+            return parts, joined, joined, None
+        m = self.o_proj.shard_sizes[0]
+        return (parts[:-1], joined[:, :m], joined,
+                hybrid.SideRelu(parts[-1], joined[:, m:]))
+
+    def ff_tensors(self, p: str):
+        if self.ff is not None:
+            n, i = self.ff.ff, len(self.proj.out_sizes) - 1
+            yield p + "up", (n, self.width), _part(self.proj, i)
+            yield p + "down", (self.width, n), _part(self.o_proj, 1)
+
+    def in_rows(self, name: str, i: int, order=None):
+        """Tensor of the i-th projection; `order` of its rows."""
+        yield name, (self.proj.out_sizes[i], self.width), \
+            lambda t: self.proj.load_part(i, t if order is None else t[order])
+
+    def out_columns(self, name: str, order=None):
+        yield name, (self.width, self.out_size), \
+            lambda t: self.o_proj.load_part(0, t if order is None
+                                            else t[:, order])
+
+
+class KeptWindowAttention(JoinedMixer):
+    def __init__(self, spec: WindowAttention, width: int, eps: float, dtype,
+                 tag: int, ff=None):
         super().__init__()
-        self.spec, self.width, self.eps = spec, width, eps
+        self.spec, self.eps = spec, eps
+        m = spec
+        self._join(width, [m.heads * m.dim, m.kv_heads * m.dim,
+                           m.kv_heads * m.vdim], m.heads * m.vdim, ff, dtype,
+                   tag)
+        buffer = lambda name, t: self.register_buffer(name, t,
+                                                      persistent=False)
+        buffer("freqs", frequencies(m.rot_dims, m.rot_base, m.stretch))
+        buffer("turn", frequencies(m.vdim if m.turn_values else 0,
+                                   m.rot_base))
+        tp, r = get_tp_size(), get_tp_rank()
+        self.sink = None if m.sink is None else _rows(_param(
+            torch.full((m.heads // tp,), float(m.sink))), tp, r, m.heads)
+
+    def forward(self, x, meta, cache) -> torch.Tensor:
+        m = self.spec
+        (q, k, v), out, joined, side = self.enter(x)
+        hybrid.rope_norm_append(q, k, v, meta, self.freqs, self.turn, cache,
+                                gain(m.stretch),
+                                self.eps if m.qk_norm else None, side)
+        hybrid.window_attention(out, q, cache, meta, self.turn, self.sink,
+                                m.window, m.keep_first, m.scale)
+        return self.o_proj(joined)
+
+    def tensors(self, p: str):
+        m = self.spec
+        qk = pair_order(m.dim, m.rot_dims, m.halves)
+        v = pair_order(m.vdim, m.vdim, m.halves and m.turn_values)
+        yield from self.in_rows(p + "q", 0, head_order(m.heads, m.dim, qk))
+        yield from self.in_rows(p + "k", 1, head_order(m.kv_heads, m.dim, qk))
+        yield from self.in_rows(p + "v", 2, head_order(m.kv_heads, m.vdim, v))
+        yield from self.out_columns(p + "o", head_order(m.heads, m.vdim, v))
+
+
+class WindowLatentAttention(JoinedMixer):
+    def __init__(self, spec: LatentAttention, width: int, eps: float, dtype,
+                 tag: int, ff=None):
+        super().__init__()
+        self.spec, self.eps = spec, eps
         m, tp, r = spec, get_tp_size(), get_tp_rank()
         self.owner = m.kv_from is None
-        q = m.heads * (m.dim + m.rot_dim)
-        # q | latent, rotated key part (kept whole)
-        self.proj = MergedColumnParallelLinear(
-            width, [q] + [m.kv_rank + m.rot_dim] * self.owner, dtype,
-            seed_tag=tag, replicated=(1,))
-        self.o_proj = RowParallelLinear(m.heads * m.vdim, width, dtype,
-                                        seed_tag=tag + 2)
+        # q | latent, rotated key part (kept whole) | gate
+        self._join(width, [m.heads * (m.dim + m.rot_dim)]
+                   + [m.kv_rank + m.rot_dim] * self.owner
+                   + [m.heads] * m.gate, m.heads * m.vdim, ff, dtype, tag,
+                   replicated=(1,) * self.owner)
         # [rank, H * D]: rows of a head's key expansion are columns here, the
         # layout both the expansion and its absorption into q read
         d, e = m.heads * m.dim // tp, m.heads * m.vdim // tp
-        uk = _init_weight(m.heads * m.dim, m.kv_rank, dtype, tag + 3)
+        uk = _init_weight(m.heads * m.dim, m.kv_rank, dtype, tag + 6)
         self.uk = _shard(
             _param(uk[r * d:(r + 1) * d].t().contiguous()), 1,
             [(r * d, d, 0)], (m.kv_rank, m.heads * m.dim))
         self.uv = _rows(_param(
-            _init_weight(m.heads * m.vdim, m.kv_rank, dtype, tag + 4)
+            _init_weight(m.heads * m.vdim, m.kv_rank, dtype, tag + 7)
             [r * e:(r + 1) * e].contiguous()), tp, r, m.heads * m.vdim)
         self.kv_norm = RmsScale(m.kv_rank) if self.owner else None
-        i = torch.arange(0, m.rot_dim, 2, dtype=torch.float64)
+        self.sink = _rows(_param(torch.zeros(m.heads // tp)), tp, r,
+                          m.heads) if m.sink else None
         self.register_buffer(
-            "freqs", m.rot_base ** (-i / m.rot_dim) if m.rot_dim else i,
+            "freqs", frequencies(m.rot_dim, m.rot_base, m.stretch),
             persistent=False)
 
     def forward(self, x, meta, cache) -> torch.Tensor:
         m = self.spec
         heads = m.heads // get_tp_size()
-        parts = self.proj.split(self.proj(x))
-        q, kv = parts if self.owner else (parts[0], None)
-        latent.rope_append(q, kv, self.kv_norm.w if self.owner else None,
-                           meta, self.freqs, cache, heads, self.eps)
-        o = latent.attention(q, cache, meta, self.uk, self.uv, heads,
-                             m.window, m.scale)
-        return self.o_proj(o)
+        parts, out, joined, side = self.enter(x)
+        kv = parts[1] if self.owner else None
+        latent.rope_append(parts[0], kv,
+                           self.kv_norm.w if self.owner else None, meta,
+                           self.freqs, cache, heads, self.eps,
+                           gain(m.stretch), side)
+        latent.attention(parts[0], cache, meta, self.uk, self.uv, heads,
+                         m.window, m.scale, self.sink,
+                         parts[-1] if m.gate else None, out)
+        return self.o_proj(joined)
 
     def tensors(self, p: str):
-        m, w = self.spec, self.width
+        m = self.spec
         tp, r = get_tp_size(), get_tp_rank()
         d = m.heads * m.dim // tp
-        yield p + "q", (m.heads * (m.dim + m.rot_dim), w), _part(self.proj, 0)
+        rotated = lambda first: pair_order(first + m.rot_dim, m.rot_dim,
+                                           m.halves, first)
+        yield from self.in_rows(p + "q", 0, head_order(
+            m.heads, m.dim + m.rot_dim, rotated(m.dim)))
         if self.owner:
-            yield p + "dkv", (m.kv_rank + m.rot_dim, w), _part(self.proj, 1)
+            yield from self.in_rows(p + "dkv", 1, rotated(m.kv_rank))
             yield from self.kv_norm.tensors(p + "dkv.norm")
         yield p + "uk", (m.heads * m.dim, m.kv_rank), \
             lambda t: self.uk.data.copy_(t[r * d:(r + 1) * d].t())
         yield p + "uv", (m.heads * m.vdim, m.kv_rank), _put(self.uv, tp, r)
-        yield p + "o", (w, m.heads * m.vdim), self.o_proj.load_full_weight
+        if m.sink:
+            yield p + "sink", (m.heads,), _put(self.sink, tp, r)
+        if m.gate:
+            yield from self.in_rows(p + "g", 1 + self.owner)
+        yield from self.out_columns(p + "o")
 
 
 class LightningAttention(nn.Module):
@@ -518,4 +615,5 @@ MIXERS = {DiffAttention: WindowDiffAttention,
           MatrixLSTM: MatrixMemoryLSTM,
           LatentAttention: WindowLatentAttention,
           Lightning: LightningAttention,
-          SigmoidAttention: ChunkedSigmoidAttention}
+          SigmoidAttention: ChunkedSigmoidAttention,
+          WindowAttention: KeptWindowAttention}

@@ -12,7 +12,7 @@ import torch
 
 from hyperspot.engine.config import ModelSpec, get_model_spec
 
-from . import mutusun, sumosun, tefezen
+from . import mutusun, radenex, sumosun, tefezen
 
 # config.json "architecture" -> (configuration reader, model class)
 DESIGNS = {
@@ -22,10 +22,13 @@ DESIGNS = {
                            tefezen.TefezenForCausalLM),
     mutusun.ARCHITECTURE: (mutusun.spec_from_folder,
                            mutusun.MutusunForCausalLM),
+    radenex.ARCHITECTURE: (radenex.spec_from_folder,
+                           radenex.RadenexForCausalLM),
 }
 
 # presets of the designs (random-init), by canonical id
-DESIGN_PRESETS = {**sumosun.PRESETS, **tefezen.PRESETS, **mutusun.PRESETS}
+DESIGN_PRESETS = {**sumosun.PRESETS, **tefezen.PRESETS, **mutusun.PRESETS,
+                  **radenex.PRESETS}
 
 
 def spec_from_folder(folder: str) -> ModelSpec:

@@ -1,7 +1,8 @@
 """Ops of the hybrid designs (models.mixers), dispatched like the rest of the
 op layer: a GPU tensor runs the gfx950 kernels of csrc/dyt.hip, csrc/rms.hip,
-csrc/conv.hip, csrc/attn_window.hip, csrc/attn_sigmoid.hip, csrc/recurrent.hip
-and csrc/recurrent_chunk.hip, a CPU tensor the PyTorch references.
+csrc/conv.hip, csrc/rope_norm.hip, csrc/attn_window.hip, csrc/attn_kept.hip,
+csrc/attn_sigmoid.hip, csrc/recurrent.hip and csrc/recurrent_chunk.hip, a CPU
+tensor the PyTorch references.
 
 Dynamic-tanh parameters travel as tuples (w, b, alpha) of float tensors.
 q, k, v, g are column views of one projection buffer [T, ...]; the kernels
@@ -137,6 +138,20 @@ def add_rms_next(y: torch.Tensor, residual: torch.Tensor, w: torch.Tensor,
     return nxt.finish(h, meta)
 
 
+def add_next(y: torch.Tensor, residual: torch.Tensor, nxt: NextInput,
+             meta) -> torch.Tensor:
+    """residual += y in place; returns the next sublayer's input in y's
+    type."""
+    if not y.is_cuda:
+        residual += y.float()
+        h = torch_ref.rms_scale(residual, nxt.w, nxt.eps).to(y.dtype)
+        return _conv_ref(h, nxt, meta)
+    h = torch.empty_like(y)
+    _native().add_rms_next(h, residual, y, None, nxt.w, nxt.eps,
+                           *nxt.row_args(meta))
+    return nxt.finish(h, meta)
+
+
 def _conv_ref(h, nxt: NextInput, meta):
     return h if nxt.conv is None \
         else causal_conv(h, nxt.conv, nxt.tail, meta)
@@ -209,6 +224,21 @@ def squared_relu(x: torch.Tensor) -> torch.Tensor:
     return x.float().clamp(min=0).square().to(x.dtype)
 
 
+class SideRelu(NamedTuple):
+    """out = relu(x)^2 for column views x, out [T, n] of two buffers, done by
+    a kernel that has the same rows."""
+
+    x: torch.Tensor
+    out: torch.Tensor
+
+    def run_ref(self) -> None:
+        self.out.copy_(self.x.float().clamp(min=0).square())
+
+
+def side_args(side: Optional[SideRelu]) -> tuple:
+    return (None, None) if side is None else side
+
+
 def clamped_glu(gate_up: torch.Tensor, limit: float) -> torch.Tensor:
     """g sigmoid(1.702 g) (u + 1) of a merged [gate | up] projection, with
     g = min(gate, limit) and u = up clamped to +-limit."""
@@ -261,6 +291,54 @@ def window_diff_attention(q, cache, meta, lam, window: int, scale: float,
             out, q, cache.k, cache.v, meta.block_tables, meta.positions, lam,
             partial, split, window, scale, diff, eps)
     return out
+
+
+def rope_norm_append(q, k, v, meta, freqs, turn, cache, gain: float,
+                     eps: Optional[float], side: Optional[SideRelu]) -> None:
+    """Interleaved rotary on q (in place) and k, each head then divided by its
+    root mean square (eps None: not); v turned over all its dimensions by the
+    frequencies `turn` [E / 2] (empty: not); append k and v to pages."""
+    if not q.is_cuda:
+        torch_ref.rope_norm_append(q, k, v, meta.positions, freqs, turn,
+                                   meta.slot_mapping, cache.k, cache.v, gain,
+                                   eps)
+        if side is not None:
+            side.run_ref()
+        return
+    _native().rope_norm_append(q, k, v, meta.positions, freqs, turn,
+                               meta.slot_mapping, cache.k, cache.v, gain, eps,
+                               *side_args(side))
+
+
+def window_attention(out, q, cache, meta, turn, sink, window: int, keep: int,
+                     scale: float) -> None:
+    """out [T, H * E] (a column view): softmax attention over the last
+    `window` positions and the first `keep`, `sink` [H] float in the
+    denominators (None: nothing); outputs turned back by `turn`."""
+    row_seq = meta.row_seq if meta.mode == "prefill" else None
+    if not q.is_cuda:
+        torch_ref.window_attention(
+            out, q, cache.k, cache.v, meta.block_tables, meta.positions,
+            row_seq, turn, sink, window, keep, scale)
+        return
+    n, T = _native(), q.shape[0]
+    G, E = cache.v.shape[1], cache.v.shape[2]
+    H = q.shape[1] // cache.k.shape[3]
+    where = (cache.k, cache.v, meta.block_tables, meta.positions)
+    if not n.kept_attn_fits(out, q, cache.k, cache.v):
+        n.kept_attn_general(out, q, *where, row_seq, turn, sink, window, keep,
+                            scale)
+    elif meta.mode == "prefill":
+        n.kept_attn_prefill(out, q, *where, meta.seq_start, meta.tiles, turn,
+                            sink, window, keep, scale)
+    else:
+        reach = min(window + keep,
+                    meta.block_tables.shape[1] * cache.k.shape[2])
+        split = decode_split(T * G * -(-(H // G) // 16), reach)
+        partial = None if split == 1 else torch.empty(
+            T * H * split * (E + 4), dtype=torch.float32, device=q.device)
+        n.kept_attn_decode(out, q, *where, turn, sink, partial, split, window,
+                           keep, scale)
 
 
 def norm_append(q, k, v, qw, kw, meta, cache, eps: float) -> None:

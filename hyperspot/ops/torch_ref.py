@@ -368,13 +368,15 @@ def rms_scale(x: torch.Tensor, w: torch.Tensor, eps: float) -> torch.Tensor:
 
 
 def latent_rope_append(q, kv, w, positions, freqs, slot_mapping, cache,
-                       heads: int, rank: int, eps: float) -> None:
+                       heads: int, rank: int, eps: float,
+                       gain: float = 1.0) -> None:
     """Rotate the last part of each head of q [T, H*(D+R)] in place; append
     the normed latent and the rotated key part of kv [T, rank + R]."""
     T, R = q.shape[0], 2 * freqs.numel()
     if R:
         a = positions.double()[:, None] * freqs[None, :]
-        c, s = a.cos().float()[:, None, :], a.sin().float()[:, None, :]
+        c, s = (gain * a.cos()).float()[:, None, :], \
+            (gain * a.sin()).float()[:, None, :]
 
     def rotate(x):                                  # [T, n, R]
         if not R:
@@ -394,9 +396,20 @@ def latent_rope_append(q, kv, w, positions, freqs, slot_mapping, cache,
     cache.view(-1, cache.shape[-1])[slot_mapping[ok]] = row[ok]
 
 
+def softmax_with_sink(s, sink):
+    """Softmax over the last axis; `sink` broadcasts against the rest and adds
+    exp(sink) to the denominator (None: a plain softmax)."""
+    if sink is None:
+        return s.softmax(-1)
+    both = torch.cat([s, sink.expand(s.shape[:-1])[..., None]], -1)
+    return both.softmax(-1)[..., :-1]
+
+
 def latent_attention(q, cache, block_tables, positions, row_seq, uk, uv,
-                     heads: int, window: int, scale: float) -> torch.Tensor:
-    """q [T, H*(D+R)] rotated; uk [rank, H*D], uv [H*E, rank]."""
+                     heads: int, window: int, scale: float, sink=None,
+                     gate=None) -> torch.Tensor:
+    """q [T, H*(D+R)] rotated; uk [rank, H*D], uv [H*E, rank]; sink [H], gate
+    [T, H] before its sigmoid."""
     T, BS, rank = q.shape[0], cache.shape[1], uk.shape[0]
     D, E = uk.shape[1] // heads, uv.shape[0] // heads
     qh = q.float().view(T, heads, -1)
@@ -410,9 +423,11 @@ def latent_attention(q, cache, block_tables, positions, row_seq, uk, uv,
         p = int(positions[t])
         idx = torch.arange(max(0, p - window + 1), p + 1, device=q.device)
         rows = cache[block_tables[s][idx // BS].long(), idx % BS].float()
-        att = (qa[t] @ rows.t() * scale).softmax(-1)
+        att = softmax_with_sink(qa[t] @ rows.t() * scale, sink)
         o[t] = att @ rows[:, :rank]
     out = torch.einsum("thr,her->the", o, uv.float().view(heads, E, rank))
+    if gate is not None:
+        out = out * torch.sigmoid(gate.float())[:, :, None]
     return out.reshape(T, heads * E).to(q.dtype)
 
 
@@ -533,3 +548,59 @@ def sigmoid_attention(q, k_cache, v_cache, block_tables, positions, row_seq,
         out[t] = torch.einsum("gxn,nge->gxe", z.sigmoid(),
                               v).reshape(-1).to(q.dtype)
     return out
+
+
+# ---------------------------------------------------------------------------
+# Windowed attention with kept first tokens, sinks and turned values
+# ---------------------------------------------------------------------------
+
+def turn_pairs(x, positions, freqs, gain: float = 1.0) -> torch.Tensor:
+    """x [T, n, D] float with the neighbouring pairs of the first
+    2 * len(freqs) dimensions turned by position times frequency."""
+    a = positions.double()[:, None] * freqs[None, :]
+    c, s = (gain * a.cos()).float()[:, None], (gain * a.sin()).float()[:, None]
+    r = 2 * freqs.numel()
+    u, v = x[..., 0:r:2], x[..., 1:r:2]
+    return torch.cat([torch.stack([u * c - v * s, v * c + u * s], -1)
+                      .flatten(-2), x[..., r:]], -1)
+
+
+def rope_norm_append(q, k, v, positions, freqs, turn, slot_mapping, k_cache,
+                     v_cache, gain: float, eps) -> None:
+    T, (_, G, BS, D) = q.shape[0], k_cache.shape
+
+    def heads(x):
+        x = turn_pairs(x.float().unflatten(-1, (-1, D)), positions, freqs,
+                       gain)
+        return x if eps is None else rms_scale(x, 1.0, eps)
+
+    q.copy_(heads(q).flatten(1))
+    ok = slot_mapping >= 0
+    blk, off = slot_mapping[ok] // BS, slot_mapping[ok] % BS
+    k_cache[blk, :, off] = heads(k)[ok].to(k_cache.dtype)
+    v = turn_pairs(v.float().unflatten(-1, (G, -1)), positions, turn)
+    v_cache[blk, :, :, off] = v[ok].to(v_cache.dtype)
+
+
+def window_attention(out, q, k_cache, v_cache, block_tables, positions,
+                     row_seq, turn, sink, window: int, keep: int,
+                     scale: float) -> None:
+    T = q.shape[0]
+    _, G, BS, D = k_cache.shape
+    H, E = q.shape[1] // D, v_cache.shape[2]
+    o = torch.empty(T, H, E, device=q.device)
+    if sink is not None:
+        sink = sink.view(G, H // G)
+    for t in range(T):
+        s = int(row_seq[t]) if row_seq is not None else t
+        p = int(positions[t])
+        lo = max(0, p - window + 1)
+        idx = torch.cat([torch.arange(min(keep, lo), device=q.device),
+                         torch.arange(lo, p + 1, device=q.device)])
+        blk, off = block_tables[s][idx // BS].long(), idx % BS
+        k = k_cache[blk, :, off].float()                       # [n, G, D]
+        v = v_cache[blk, :, :, off].float()                    # [n, G, E]
+        z = torch.einsum("gxd,ngd->gxn", q[t].float().view(G, H // G, D), k)
+        o[t] = torch.einsum("gxn,nge->gxe", softmax_with_sink(z * scale, sink),
+                            v).reshape(H, E)
+    out.copy_(turn_pairs(o, -positions, turn).flatten(1))

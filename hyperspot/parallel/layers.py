@@ -155,10 +155,12 @@ class MergedColumnParallelLinear(_LinearCompute):
     """Several column-parallel projections fused into one GEMM
     (gate_proj | up_proj).  Each sub-projection is sharded independently so
     the shard layout matches per-projection splits downstream; those named
-    in `replicated` are kept whole on every rank."""
+    in `replicated` are kept whole on every rank.  Every projection and the
+    rows of the output begin at a multiple of `align` columns; zero rows fill
+    the weight up."""
 
     def __init__(self, in_features: int, out_sizes: list, dtype: torch.dtype,
-                 seed_tag: int = 0, replicated: tuple = ()):
+                 seed_tag: int = 0, replicated: tuple = (), align: int = 1):
         super().__init__()
         tp, r = get_tp_size(), get_tp_rank()
         self.out_sizes = out_sizes
@@ -180,6 +182,9 @@ class MergedColumnParallelLinear(_LinearCompute):
             slices.append((off_full + first, sh, off_shard))
             off_full += o
             off_shard += sh
+            if off_shard % align:
+                parts.append(full.new_zeros(-off_shard % align, in_features))
+                off_shard += -off_shard % align
         self._finalize_weight(torch.cat(parts, 0), shard_dim=0,
                               slices=slices,
                               full_shape=(sum(out_sizes), in_features))
@@ -190,7 +195,8 @@ class MergedColumnParallelLinear(_LinearCompute):
 
     def split(self, y: torch.Tensor) -> tuple:
         """Column views of the merged output, one per projection."""
-        return y.split(self.shard_sizes, dim=-1)
+        return tuple(y[..., s0:s0 + n]
+                     for _, n, s0 in self.weight._tp_slices)
 
 
 class QKVParallelLinear(_LinearCompute):
@@ -251,3 +257,36 @@ class RowParallelLinear(_LinearCompute):
     def forward(self, x: torch.Tensor) -> torch.Tensor:
         out = self._mm(x)
         return tensor_model_parallel_all_reduce(out)
+
+
+class MergedRowParallelLinear(_LinearCompute):
+    """The sum of several row-parallel projections as one GEMM over their
+    joined inputs, with one all-reduce.  Each is sharded by itself, so a rank's
+    input is its shard of the first one, then of the second, ..."""
+
+    def __init__(self, in_sizes: list, out_features: int, dtype: torch.dtype,
+                 seed_tag: int = 0):
+        super().__init__()
+        tp, r = get_tp_size(), get_tp_rank()
+        self.in_sizes = in_sizes
+        self.shard_sizes = [n // tp for n in in_sizes]
+        parts, slices, off_full, off_shard = [], [], 0, 0
+        for i, (n, sh) in enumerate(zip(in_sizes, self.shard_sizes)):
+            assert n % tp == 0, (n, tp)
+            full = _init_weight(out_features, n, dtype, seed_tag + i)
+            parts.append(full[:, r * sh:(r + 1) * sh])
+            slices.append((off_full + r * sh, sh, off_shard))
+            off_full += n
+            off_shard += sh
+        self._finalize_weight(torch.cat(parts, 1), shard_dim=1, slices=slices,
+                              full_shape=(out_features, sum(in_sizes)))
+
+    def load_part(self, i: int, w: torch.Tensor) -> None:
+        """Copy this rank's columns of the i-th projection's FULL weight into
+        place (bf16/float storage only)."""
+        f0, ln, s0 = self.weight._tp_slices[i]
+        start = f0 - sum(self.in_sizes[:i])
+        self.weight.data[:, s0:s0 + ln].copy_(w[:, start:start + ln])
+
+    def forward(self, x: torch.Tensor) -> torch.Tensor:
+        return tensor_model_parallel_all_reduce(self._mm(x))
