@@ -604,6 +604,20 @@ def _compare_specs(design, width):
                         experts=Experts(experts, 4, ff, ff), side_dim=128,
                         periods=2)
         return hybrid, plain
+    if design == "radenex":
+        # equal width, layers, attention heads and vocabulary; the
+        # feed-forward without a gate is half as large again, so both have
+        # the same number of weights
+        from hyperspot.models.radenex import preset
+        ff = width * 7 // 2
+        hybrid = preset(f"radenex-w{width}", width=width, vocab=vocab,
+                        heads=heads, kv_heads=heads // 4, dim=128,
+                        window=1024, keep_first=4, latent_heads=heads,
+                        latent_dim=128, rot_dim=64, kv_rank=512,
+                        ff=3 * ff // 2, layers=8)
+        return hybrid, ModelSpec(f"llama-w{width}", width, 8, heads,
+                                 heads // 4, 128, ff, vocab,
+                                 max_position=16384)
     # equal width, feed-forwards, vocabulary and number of feed-forwards
     from hyperspot.models.sumosun import preset
     ff = width * 7 // 2
@@ -733,9 +747,10 @@ def main():
                          "hybrid design beside the closest other model of "
                          "equal size, at these widths (default 2048 4096)")
     ap.add_argument("--compare-design", default="sumosun",
-                    choices=["sumosun", "tefezen", "mutusun"],
-                    help="with --compare: Sumosun beside a plain decoder, or "
-                         "Tefezen or Mutusun beside a Mixtral-like one")
+                    choices=["sumosun", "tefezen", "mutusun", "radenex"],
+                    help="with --compare: Sumosun or Radenex beside a plain "
+                         "decoder, or Tefezen or Mutusun beside a "
+                         "Mixtral-like one")
     ap.add_argument("--compare-model", default=None, metavar="PREFIX",
                     help="with --compare: only models of this name prefix")
     ap.add_argument("--compare-reps", type=int, default=3)

@@ -2,7 +2,7 @@
 """Isolated kernel microbenchmarks (GPU only) — us/call + achieved GB/s.
 
 Usage: python bench_kernels.py [--iters N]
-           [--which attn|gemm|fp8|hybrid|latent|sigmoid|all]
+           [--which attn|gemm|fp8|hybrid|latent|sigmoid|kept|all]
 
 Shapes mirror the flagship bench (Llama-3-8B bf16, bs=256 ctx=512 decode):
 the numbers here are the per-kernel budget lines behind bench.py's step
@@ -567,6 +567,127 @@ def bench_sigmoid(iters, W):
         common(m, B, B, tag)
 
 
+def bench_kept(iters, W):
+    """Kernels of the Radenex design at width W and the like kernels of a
+    plain decoder."""
+    import hyperspot.ops as ops
+    from hyperspot.engine.kv_cache import KVPages, LatentKV
+    from hyperspot.engine.layer_spec import UNBOUNDED
+    from hyperspot.engine.rotary import frequencies
+    from hyperspot.models.llama import (SPAN_TOKENS, LatentSpan,
+                                        prefill_tiles)
+    from hyperspot.ops import hybrid, latent
+    dev, bf, f32 = DEV, torch.bfloat16, torch.float32
+    n_ = ops._native()
+    report = lambda name, tag, fn, nbytes, flops=0: report_kernel(
+        iters, name, f"w{W}_{tag}", fn, nbytes, flops, timed_graph)
+    rnd = lambda *s, d=bf: (torch.randn(*s, device=dev) * 0.3).to(d)
+    i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=dev)
+    H, G, D, R, rank = W // 128, W // 512, 128, 64, 512
+    win, keep, ff, plain_ff = 1024, 4, W * 21 // 4, W * 7 // 2
+    fr, turn = (frequencies(n, 1e4).to(dev) for n in (R, D))
+    sink, nw = torch.zeros(H, device=dev), torch.ones(W, device=dev)
+    w2 = torch.ones(W, dtype=bf, device=dev)
+    uk, uv, kw = rnd(rank, H * D), rnd(H * D, rank), rnd(rank, d=f32)
+
+    def common(m, T, tag):
+        x, r, y = rnd(T, W), rnd(T, W, d=f32), rnd(T, W)
+        nxt = hybrid.NextInput(nw, 1e-5)
+        report("add_next", tag, lambda: hybrid.add_next(x, r, nxt, m),
+               T * W * 12)
+        report("fused_add_rmsnorm", tag, lambda: ops.fused_add_rmsnorm(
+            x, y, w2, 1e-5), T * W * 8)
+        gu = rnd(T, 2 * plain_ff)
+        report("silu_mul", tag, lambda: ops.silu_mul(gu), T * plain_ff * 6)
+
+    def plain_heads(T, ctx, nb, m, tag):
+        q, k, v = (x.view(T, -1, D) for x in rnd(
+            T, (H + 2 * G) * D).split([H * D, G * D, G * D], -1))
+        kc = rnd(2, nb, G, 16, D)
+        cs = torch.randn(ctx, D, device=dev)
+        report("rope_kv_append", tag, lambda: ops.rope_kv_append(
+            q, k, v, m.positions, cs, m.slot_mapping, kc[0], kc[1]),
+            2 * T * D * (2 * H + 4 * G))
+        return q, k, v, kc
+
+    def joined(T, parts):
+        """Column views of a merged projection and the side activation."""
+        x = rnd(T, sum(parts) + ff).split([*parts, ff], -1)
+        out = rnd(T, H * D + ff)
+        return x[:-1], out[:, :H * D], hybrid.SideRelu(x[-1],
+                                                       out[:, H * D:])
+
+    def appends(T, m, kvp, lat, tag):
+        (q, k, v), out, side = joined(T, [H * D, G * D, G * D])
+        (lq, kv, g), lout, lside = joined(T, [H * (D + R), rank + R, H])
+        for s, sl, what in ((None, None, ""), (side, lside, " (with side)")):
+            extra = 4 * T * ff * (s is not None)
+            report("rope_norm_append" + what, tag,
+                   lambda: hybrid.rope_norm_append(
+                       q, k, v, m, fr, turn, kvp, 1.0, 1e-5, s),
+                   2 * T * D * (2 * H + 4 * G) + extra)
+            report("latent_rope_append" + what, tag,
+                   lambda: latent.rope_append(
+                       lq, kv, kw, m, fr, lat, H, 1e-5, 1.2, sl),
+                   T * (4 * H * R + 4 * (rank + R)) + extra)
+        return q, out, lq, g, lout
+
+    for lens in ([2048], [8192], [1024] * 8):
+        m, nb = meta_for(lens)
+        T, tag = sum(lens), "x".join(map(str, (len(lens), lens[0])))
+        m.latent = {UNBOUNDED: LatentSpan(
+            m.slot_mapping, m.seq_start[:-1].contiguous(),
+            i32([0] * len(lens)), i32(prefill_tiles(lens, SPAN_TOKENS)[0]),
+            None)}
+        kvp = KVPages(torch.zeros(nb, G, 16, D, dtype=bf, device=dev),
+                      torch.zeros(nb, G, D, 16, dtype=bf, device=dev))
+        lat = LatentKV(torch.zeros(nb, 16, rank + R, dtype=bf, device=dev))
+        q, out, lq, g, lout = appends(T, m, kvp, lat, tag)
+        pairs = sum(min(p + 1, win) for x in lens for p in range(x))
+        causal = sum(x * (x + 1) // 2 for x in lens)
+        nbytes = 2 * T * D * (2 * H + 2 * G)
+        for w, name, n in ((win, "windowed", pairs),
+                           (UNBOUNDED, "all", causal)):
+            report(f"kept_attn_prefill ({name})", tag,
+                   lambda: hybrid.window_attention(
+                       out, q, kvp, m, turn, sink, w, keep, 0.09), nbytes,
+                   n * H * 4 * D)
+        sp, c = m.latent[UNBOUNDED], rnd(T, rank + R)
+        kn, vt = c[:, :rank] @ uk, uv @ c[:, :rank].t()
+        report("latent_attn_prefill", tag, lambda: n_.latent_attn_prefill(
+            lout, lq, kn, c, vt, m.positions, m.seq_start, sp.start, sp.first,
+            sp.tiles, H, UNBOUNDED, 0.07, sink, g),
+            2 * T * H * (2 * D + R + 2 * D), causal * H * 2 * (2 * D + R))
+        report("latent attention, with expansion", tag,
+               lambda: latent.attention(lq, lat, m, uk, uv, H, UNBOUNDED,
+                                        0.07, sink, g, lout),
+               2 * T * (H * (2 * D + R) + rank + R),
+               causal * H * 2 * (2 * D + R) + T * rank * H * 4 * D)
+        q2, k2, v2, kc = plain_heads(T, max(lens), nb, m, tag)
+        report("attn_prefill_mfma", tag, lambda: ops.attention(
+            q2, k2, v2, kc[0], kc[1], m, 0.088), nbytes, causal * H * 4 * D)
+        common(m, T, tag)
+    for B in (1, 32, 256):
+        ctx = 1024
+        m, nb = meta_for([1] * B, "decode", ctx)
+        tag = f"b{B}_ctx{ctx}"
+        kvp = KVPages(rnd(nb, G, 16, D), rnd(nb, G, D, 16))
+        lat = LatentKV(rnd(nb, 16, rank + R))
+        q, out, lq, g, lout = appends(B, m, kvp, lat, tag)
+        nbytes = 4 * B * (ctx + 1) * G * D
+        report("kept_attn_decode", tag, lambda: hybrid.window_attention(
+            out, q, kvp, m, turn, sink, win, keep, 0.09), nbytes)
+        nbytes_l = 2 * B * ((ctx + 1) * (rank + R) + H * (2 * rank + R))
+        report("latent attention, absorbed", tag, lambda: latent.attention(
+            lq, lat, m, uk, uv, H, UNBOUNDED, 0.07, sink, g, lout),
+            nbytes_l + 4 * H * rank * D,
+            2 * B * H * ((ctx + 1) * (2 * rank + R) + 2 * rank * D))
+        q2, k2, v2, kc = plain_heads(B, ctx + 1, nb, m, tag)
+        report("paged_attn_decode", tag, lambda: ops.paged_attn_decode(
+            q2, kc[0], kc[1], m.block_tables, m.seq_lens, 0.088), nbytes)
+        common(m, B, tag)
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--which", default="attn")
@@ -585,6 +706,9 @@ def main():
     if args.which in ("sigmoid", "all"):
         for width in (2048, 4096):
             bench_sigmoid(args.iters, width)
+    if args.which in ("kept", "all"):
+        for width in (2048, 4096):
+            bench_kept(args.iters, width)
     if args.which in ("fp8", "all"):
         bench_fp8_gemm(args.iters)
 
