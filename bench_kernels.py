@@ -650,7 +650,8 @@ def bench_kept(iters, W):
                            (UNBOUNDED, "all", causal)):
             report(f"kept_attn_prefill ({name})", tag,
                    lambda: hybrid.window_attention(
-                       out, q, kvp, m, turn, sink, w, keep, 0.09), nbytes,
+                       out, q, kvp, m, turn, sink, w, keep, 0.09, True),
+                   nbytes,
                    n * H * 4 * D)
         sp, c = m.latent[UNBOUNDED], rnd(T, rank + R)
         kn, vt = c[:, :rank] @ uk, uv @ c[:, :rank].t()
@@ -676,8 +677,24 @@ def bench_kept(iters, W):
         q, out, lq, g, lout = appends(B, m, kvp, lat, tag)
         nbytes = 4 * B * (ctx + 1) * G * D
         report("kept_attn_decode", tag, lambda: hybrid.window_attention(
-            out, q, kvp, m, turn, sink, win, keep, 0.09), nbytes)
+            out, q, kvp, m, turn, sink, win, keep, 0.09, True), nbytes)
         nbytes_l = 2 * B * ((ctx + 1) * (rank + R) + H * (2 * rank + R))
+        qa, split = rnd(B, H, rank), latent.absorbed_split(
+            B * -(-H // 32), m.block_tables.shape[1] * 16)
+        part = torch.empty(B, H, split, rank + 4, device=dev)
+        report("latent_absorb", tag, lambda: n_.latent_absorb(
+            qa, lq, uk, None, H), 2 * H * (D * rank + B * (D + rank)),
+            2 * B * H * D * rank)
+        report("latent_attn_decode", tag, lambda: n_.latent_attn_decode(
+            part if split > 1 else torch.empty_like(qa), qa, lq, lat.kv,
+            m.block_tables, m.positions, None, None, split, UNBOUNDED, 0.07,
+            sink), nbytes_l,
+            2 * B * H * (ctx + 1) * (2 * rank + R))
+        if split > 1:
+            report("latent_merge_values", tag, lambda: n_.latent_merge_values(
+                lout, part, uv, None, B, H, split, g),
+                2 * H * (D * rank + B * (D + 2 * split * rank)),
+                2 * B * H * D * rank)
         report("latent attention, absorbed", tag, lambda: latent.attention(
             lq, lat, m, uk, uv, H, UNBOUNDED, 0.07, sink, g, lout),
             nbytes_l + 4 * H * rank * D,

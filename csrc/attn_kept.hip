@@ -26,6 +26,10 @@
 // registers, and V^T comes straight from the transposed pages.  The weights
 // enter as a bf16 high and low part.  A pair of an output's dimensions is in
 // one lane.
+//
+// BOUNDED: the caller knows that scores and sinks are small enough for their
+// exponentials as they are (normed queries and keys: |score| <= D |scale|), so
+// no running maximum is kept.
 #include <float.h>
 
 #include <type_traits>
@@ -147,7 +151,7 @@ constexpr int VS = KV + 8;        // V^T row in LDS, padded against conflicts
 // HW heads a workgroup.  Waves: row group = wave >> 1 (32 query rows each),
 // and wave & 1 is the head (HW 2) or which 32 tokens of a step (HW 1).
 // a.scale is in units of log2(e).
-template <int DP, int EP, int HW>
+template <int DP, int EP, int HW, bool BOUNDED>
 __global__ __launch_bounds__(256, DP <= 128 && EP <= 128 ? 2 : 1)
 void kept_attn_prefill_kernel(Kept<bf16> a,
                               const int* __restrict__ seq_start,
@@ -159,8 +163,12 @@ void kept_attn_prefill_kernel(Kept<bf16> a,
   constexpr int NB = HW == 2 ? 2 : 1;            // 32-token blocks a wave
   constexpr int TILE_BYTES = (KV * KS + EP * VS) * 2;
   constexpr int OUT_BYTES = HW == 2 ? 0 : 2 * (EP + 2) * 32 * 4;
+  constexpr int TC = EP < 128 ? EP : 128;        // columns turned at a time
+  constexpr int TS = TC + 4;
+  constexpr int TURN_BYTES = KV * TS * 4;
+  constexpr int BYTES = TILE_BYTES > OUT_BYTES ? TILE_BYTES : OUT_BYTES;
   __shared__ __attribute__((aligned(16)))
-      char smem[TILE_BYTES > OUT_BYTES ? TILE_BYTES : OUT_BYTES];
+      char smem[BYTES > TURN_BYTES ? BYTES : TURN_BYTES];
   short* k_lds = reinterpret_cast<short*>(smem);
   short* v_lds = k_lds + KV * KS;
   const int D = a.D, E = a.E, G = a.G;
@@ -196,10 +204,11 @@ void kept_attn_prefill_kernel(Kept<bf16> a,
   #pragma unroll
   for (int e = 0; e < ET; ++e) acc[e] = f32x16_t(0.f);
   // the sink is counted once: by one half of the lanes, and of the tokens
-  float m = -FLT_MAX, l = 0.f;
+  float m = BOUNDED ? 0.f : -FLT_MAX, l = 0.f;
   if (a.sink) {
-    m = a.sink[h] * LOG2E;
-    l = hf == 0 && (HW == 2 || half == 0) ? 1.f : 0.f;
+    const float s = a.sink[h] * LOG2E;
+    if (!BOUNDED) m = s;
+    if (hf == 0 && (HW == 2 || half == 0)) l = exp2_fast(s - m);
   }
 
   const int last = p0 + n - 1;
@@ -292,22 +301,24 @@ void kept_attn_prefill_kernel(Kept<bf16> a,
           if (at > qp || (at <= qp - a.window && at >= a.keep)) x = -FLT_MAX;
         }
         sc[i][r] = x;
-        mx = fmaxf(mx, x);
+        if constexpr (!BOUNDED) mx = fmaxf(mx, x);
       }
     }
-    mx = fmaxf(mx, __shfl_xor(mx, 32));
-    if (!__all(mx == m)) {
-      const float alpha = m == -FLT_MAX ? 0.f : exp2_fast(m - mx);
-      #pragma unroll
-      for (int e = 0; e < ET; ++e)
+    if constexpr (!BOUNDED) {
+      mx = fmaxf(mx, __shfl_xor(mx, 32));
+      if (!__all(mx == m)) {
+        const float alpha = m == -FLT_MAX ? 0.f : exp2_fast(m - mx);
         #pragma unroll
-        for (int r = 0; r < 16; ++r) acc[e][r] *= alpha;
-      l *= alpha;
-      m = mx;
+        for (int e = 0; e < ET; ++e)
+          #pragma unroll
+          for (int r = 0; r < 16; ++r) acc[e][r] *= alpha;
+        l *= alpha;
+        m = mx;
+      }
     }
     // a column without a visible key yet has m = -FLT_MAX: with base 0 its
     // masked scores weigh exp2(-FLT_MAX) = 0
-    const float base = m == -FLT_MAX ? 0.f : m;
+    const float base = BOUNDED || m == -FLT_MAX ? 0.f : m;
     #pragma unroll
     for (int i = 0; i < NB; ++i) {
       short8_t ph[2], pl[2];
@@ -316,7 +327,8 @@ void kept_attn_prefill_kernel(Kept<bf16> a,
         float p[8];
         #pragma unroll
         for (int j = 0; j < 8; ++j) {
-          p[j] = exp2_fast(sc[i][c * 8 + j] - base);
+          p[j] = exp2_fast(BOUNDED ? sc[i][c * 8 + j]
+                                   : sc[i][c * 8 + j] - base);
           l += p[j];
         }
         split_bf16x8(p, &ph[c], &pl[c]);
@@ -369,38 +381,56 @@ void kept_attn_prefill_kernel(Kept<bf16> a,
       }
     }
     __syncthreads();
-    if (half == 1) return;
-    const float m1 = ml[(rg * 2) * 32 + col], l1 = ml[(rg * 2 + 1) * 32 + col];
-    const float top = fmaxf(m, m1);
-    const float w0 = m == -FLT_MAX ? 0.f : exp2_fast(m - top);
-    const float w1 = m1 == -FLT_MAX ? 0.f : exp2_fast(m1 - top);
-    l = l * w0 + l1 * w1;
-    #pragma unroll
-    for (int e = 0; e < ET; ++e)
+    if (half == 0) {
+      const float m1 = ml[(rg * 2) * 32 + col];
+      const float l1 = ml[(rg * 2 + 1) * 32 + col];
+      const float top = fmaxf(m, m1);
+      const float w0 = m == -FLT_MAX ? 0.f : exp2_fast(m - top);
+      const float w1 = m1 == -FLT_MAX ? 0.f : exp2_fast(m1 - top);
+      l = l * w0 + l1 * w1;
       #pragma unroll
-      for (int r = 0; r < 16; ++r)
-        acc[e][r] = acc[e][r] * w0 +
-                    o_lds[((rg * ET + e) * 16 + r) * 64 + lane] * w1;
+      for (int e = 0; e < ET; ++e)
+        #pragma unroll
+        for (int r = 0; r < 16; ++r)
+          acc[e][r] = acc[e][r] * w0 +
+                      o_lds[((rg * ET + e) * 16 + r) * 64 + lane] * w1;
+    }
   }
-  if (row >= n) return;
+  const bool writes = row < n && (HW == 2 || half == 0);
   const float inv = 1.f / l;
   bf16* orow = a.out + (long)(t0 + row) * a.os + (long)h * E;
+  float* cs_lds = reinterpret_cast<float*>(smem);    // [KV][TS] (cos, sin)
   #pragma unroll
-  for (int e = 0; e < ET; ++e)
-    #pragma unroll
-    for (int r = 0; r < 16; r += 4) {
-      const int c = e * 32 + 8 * (r >> 2) + 4 * hf;
-      if (c >= E) continue;
-      float x[4];
-      #pragma unroll
-      for (int i = 0; i < 4; ++i) x[i] = acc[e][r + i] * inv;
-      if (a.turn) {
-        turn_back(a, qp, c, x);
-        turn_back(a, qp, c + 2, x + 2);
+  for (int e0 = 0; e0 < ET; e0 += TC / 32) {
+    if (a.turn) {                     // the rows' angles, for all heads here
+      __syncthreads();
+      for (int u = tid; u < KV * (TC / 2); u += 256) {
+        const int r = u / (TC / 2), i = u % (TC / 2);
+        if (e0 * 32 + 2 * i < E)
+          angle<bf16>(-(long)(p0 + r), a.turn[e0 * 16 + i],
+                      &cs_lds[r * TS + 2 * i], &cs_lds[r * TS + 2 * i + 1]);
       }
-      *reinterpret_cast<uint2*>(orow + c) =
-          uint2{cvt_pk_bf16(x[0], x[1]), cvt_pk_bf16(x[2], x[3])};
+      __syncthreads();
     }
+    if (!writes) continue;
+    #pragma unroll
+    for (int e = e0; e < e0 + TC / 32; ++e)
+      #pragma unroll
+      for (int r = 0; r < 16; r += 4) {
+        const int c = e * 32 + 8 * (r >> 2) + 4 * hf;
+        if (c >= E) continue;
+        float x[4];
+        #pragma unroll
+        for (int i = 0; i < 4; ++i) x[i] = acc[e][r + i] * inv;
+        if (a.turn) {
+          float cs[4];
+          load_vec<float, 4>(cs_lds + row * TS + c - e0 * 32, cs);
+          turn_pairs<4>(x, cs);
+        }
+        *reinterpret_cast<uint2*>(orow + c) =
+            uint2{cvt_pk_bf16(x[0], x[1]), cvt_pk_bf16(x[2], x[3])};
+      }
+  }
 }
 
 // ============================ matrix-core decode ===========================
@@ -408,7 +438,7 @@ constexpr int NC = 16;            // query heads per workgroup, at most
 constexpr int PART = 4;           // floats past the values of a part: m, l
 
 // a.scale is in units of log2(e)
-template <int DP, int EP>
+template <int DP, int EP, bool BOUNDED>
 __global__ __launch_bounds__(256, DP <= 128 && EP <= 128 ? 2 : 1)
 void kept_attn_decode_kernel(Kept<bf16> a, float* __restrict__ partial) {
   constexpr int KC = (DP + 31) / 32, ET = EP / 16;
@@ -441,10 +471,11 @@ void kept_attn_decode_kernel(Kept<bf16> a, float* __restrict__ partial) {
   #pragma unroll
   for (int e = 0; e < ET; ++e) acc[e] = f32x4_t(0.f);
   // the sink is counted once: by one part, wave and quarter of the lanes
-  float m = -FLT_MAX, l = 0.f;
+  float m = BOUNDED ? 0.f : -FLT_MAX, l = 0.f;
   if (a.sink && z == 0 && wid == 0) {
-    m = a.sink[h0 + min(col, cols - 1)] * LOG2E;
-    l = gr == 0 ? 1.f : 0.f;
+    const float s = a.sink[h0 + min(col, cols - 1)] * LOG2E;
+    if (!BOUNDED) m = s;
+    if (gr == 0) l = exp2_fast(s - m);
   }
 
   // blocks of 32 tokens: kept ones ahead of the window's first, then those of
@@ -501,23 +532,25 @@ void kept_attn_decode_kernel(Kept<bf16> a, float* __restrict__ partial) {
       const int at = tp + j;
       p[j] = at <= pos && (at >= lo || at < a.keep)
           ? sc[j >> 2][j & 3] * a.scale : -FLT_MAX;
-      mx = fmaxf(mx, p[j]);
+      if constexpr (!BOUNDED) mx = fmaxf(mx, p[j]);
     }
-    mx = fmaxf(mx, __shfl_xor(mx, 16));
-    mx = fmaxf(mx, __shfl_xor(mx, 32));
-    if (!__all(mx == m)) {
-      const float alpha = m == -FLT_MAX ? 0.f : exp2_fast(m - mx);
-      #pragma unroll
-      for (int e = 0; e < ET; ++e)
+    if constexpr (!BOUNDED) {
+      mx = fmaxf(mx, __shfl_xor(mx, 16));
+      mx = fmaxf(mx, __shfl_xor(mx, 32));
+      if (!__all(mx == m)) {
+        const float alpha = m == -FLT_MAX ? 0.f : exp2_fast(m - mx);
         #pragma unroll
-        for (int r = 0; r < 4; ++r) acc[e][r] *= alpha;
-      l *= alpha;
-      m = mx;
+        for (int e = 0; e < ET; ++e)
+          #pragma unroll
+          for (int r = 0; r < 4; ++r) acc[e][r] *= alpha;
+        l *= alpha;
+        m = mx;
+      }
     }
-    const float base = m == -FLT_MAX ? 0.f : m;
+    const float base = BOUNDED || m == -FLT_MAX ? 0.f : m;
     #pragma unroll
     for (int j = 0; j < 8; ++j) {
-      p[j] = exp2_fast(p[j] - base);
+      p[j] = exp2_fast(BOUNDED ? p[j] : p[j] - base);
       l += p[j];
     }
     short8_t ph, pl;
@@ -645,8 +678,8 @@ void launch_kept_attn_prefill(bf16* out, const bf16* q, const bf16* k_cache,
                               const int* tiles, const double* turn,
                               const float* sink, int num_tiles,
                               int max_blocks, int H, int G, int D, int E,
-                              int window, int keep, float scale, long qs,
-                              long os, hipStream_t stream) {
+                              int window, int keep, float scale, bool bounded,
+                              long qs, long os, hipStream_t stream) {
   if (num_tiles == 0) return;
   const Kept<bf16> a{out, q, k_cache, v_cache, block_tables, positions, turn,
                      sink, max_blocks, H, G, D, E, window, keep,
@@ -654,18 +687,21 @@ void launch_kept_attn_prefill(bf16* out, const bf16* q, const bf16* k_cache,
   // two heads share a tile's keys where enough workgroups remain
   const int hw = H / G % 2 == 0 && (long)H / 2 * num_tiles >= 512 ? 2 : 1;
   const dim3 grid((unsigned)(H / hw), (unsigned)num_tiles);
+  #define RUN(DP, EP, HW, BOUNDED)                                          \
+    kept_attn_prefill_kernel<DP, EP, HW, BOUNDED>                           \
+        <<<grid, 256, 0, stream>>>(a, seq_start, tiles)
   #define CASE(DP, EP)                                                      \
     if (D <= DP && E <= EP) {                                               \
-      if (hw == 2)                                                          \
-        kept_attn_prefill_kernel<DP, EP, 2>                                 \
-            <<<grid, 256, 0, stream>>>(a, seq_start, tiles);                \
-      else                                                                  \
-        kept_attn_prefill_kernel<DP, EP, 1>                                 \
-            <<<grid, 256, 0, stream>>>(a, seq_start, tiles);                \
+      if (hw == 2) {                                                        \
+        if (bounded) RUN(DP, EP, 2, true); else RUN(DP, EP, 2, false);      \
+      } else {                                                              \
+        if (bounded) RUN(DP, EP, 1, true); else RUN(DP, EP, 1, false);      \
+      }                                                                     \
       return;                                                               \
     }
   KEPT_SIZES(CASE)
   #undef CASE
+  #undef RUN
   throw std::runtime_error("kept_attn_prefill: head sizes");
 }
 
@@ -674,8 +710,9 @@ void launch_kept_attn_decode(bf16* out, const bf16* q, const bf16* k_cache,
                              const long* positions, const double* turn,
                              const float* sink, float* partial, long rows,
                              int max_blocks, int H, int G, int D, int E,
-                             int window, int keep, float scale, long qs,
-                             long os, int split, hipStream_t stream) {
+                             int window, int keep, float scale, bool bounded,
+                             long qs, long os, int split,
+                             hipStream_t stream) {
   if (rows == 0) return;
   const Kept<bf16> a{out, q, k_cache, v_cache, block_tables, positions, turn,
                      sink, max_blocks, H, G, D, E, window, keep,
@@ -684,20 +721,21 @@ void launch_kept_attn_decode(bf16* out, const bf16* q, const bf16* k_cache,
   const int cols = group < NC ? group : NC;
   const int lds = (4 * cols * E + 8 * NC) * (int)sizeof(float);
   const dim3 grid((unsigned)rows, (unsigned)(G * hb), (unsigned)split);
+  auto run = [&](auto kernel) {
+    if (lds > 65536)
+      HIP_CHECK(hipFuncSetAttribute(
+          reinterpret_cast<const void*>(kernel),
+          hipFuncAttributeMaxDynamicSharedMemorySize, lds));
+    kernel<<<grid, 256, lds, stream>>>(a, partial);
+    if (split > 1)
+      kept_attn_merge_kernel<<<
+          dim3((unsigned)rows, (unsigned)((H * E + 1023) / 1024)), 256, 0,
+          stream>>>(a, partial, split);
+  };
   #define CASE(DP, EP)                                                      \
-    if (D <= DP && E <= EP) {                                               \
-      if (lds > 65536)                                                      \
-        HIP_CHECK(hipFuncSetAttribute(                                      \
-            reinterpret_cast<const void*>(&kept_attn_decode_kernel<DP, EP>),\
-            hipFuncAttributeMaxDynamicSharedMemorySize, lds));              \
-      kept_attn_decode_kernel<DP, EP><<<grid, 256, lds, stream>>>(a,        \
-                                                                  partial); \
-      if (split > 1)                                                        \
-        kept_attn_merge_kernel<<<                                           \
-            dim3((unsigned)rows, (unsigned)((H * E + 1023) / 1024)), 256,   \
-            0, stream>>>(a, partial, split);                                \
-      return;                                                               \
-    }
+    if (D <= DP && E <= EP)                                                 \
+      return bounded ? run(&kept_attn_decode_kernel<DP, EP, true>)          \
+                     : run(&kept_attn_decode_kernel<DP, EP, false>);
   KEPT_SIZES(CASE)
   #undef CASE
   throw std::runtime_error("kept_attn_decode: head sizes");

@@ -641,11 +641,13 @@ void latent_attn_prefill_kernel(
   short* k_lds = reinterpret_cast<short*>(smem);
   short* v_lds = k_lds + KV * KS;
 
-  const int s = tiles[2 * blockIdx.x];
-  const int t0 = seq_start[s] + tiles[2 * blockIdx.x + 1];
+  // later rows see more: they start first; a head stays on one die
+  const int tile = gridDim.y - 1 - blockIdx.y;
+  const int s = tiles[2 * tile];
+  const int t0 = seq_start[s] + tiles[2 * tile + 1];
   const int n = min(QT, seq_start[s + 1] - t0);
   if (n <= 0) return;
-  const int h = blockIdx.y;
+  const int h = blockIdx.x;
   const long kv0r = kv_start[s];                 // first kv row
   // positions relative to the first kv row's token
   const int p0 = (int)positions[t0] - kv_first[s];
@@ -943,7 +945,7 @@ void launch_latent_merge_values(bf16* out, const float* partial,
   if (R == 0) return;
   // few rows: fewer a workgroup, then fewer values a workgroup
   int rb = 16;
-  while (rb > 1 && (R + rb - 1) / rb * H < 512) rb /= 2;
+  while (rb > 1 && (R + rb - 1) / rb * H < 256) rb /= 2;
   const unsigned nz = R * H < 128 ? (unsigned)((E + 63) / 64) : 1;
   const dim3 grid((unsigned)((R + rb - 1) / rb), (unsigned)H, nz);
   #define CASE(RB)                                                          \
@@ -970,7 +972,7 @@ void launch_latent_attn_prefill(bf16* out, const bf16* q, const bf16* kn,
     if (D + rot <= DP && E <= EP) {                                         \
       allow_lds(&latent_attn_prefill_kernel<DP, EP>, prefill_lds(DP, EP));  \
       latent_attn_prefill_kernel<DP, EP>                                    \
-          <<<dim3((unsigned)num_tiles, (unsigned)H), 256,                   \
+          <<<dim3((unsigned)H, (unsigned)num_tiles), 256,                   \
              prefill_lds(DP, EP), stream>>>(                                \
               out, q, kn, lat, vt, positions, seq_start, kv_start,          \
               kv_first, tiles, sink, H, D, E, rank, rot, nkv, window,       \

@@ -246,12 +246,6 @@ DEV float dot2_bf16(unsigned a, unsigned b, float c) {
 // dot2 K path) or 2 float2 (for the PV path).  gfx950-native converts.
 typedef __attribute__((ext_vector_type(2))) float float2v;
 
-DEV unsigned pk_bf16(float a, float b) {
-  unsigned r;
-  asm("v_cvt_pk_bf16_f32 %0, %1, %2" : "=v"(r) : "v"(a), "v"(b));
-  return r;
-}
-
 // SPLIT > 1 (flash-decode): grid.z WGs share one (row, kvh), each owning
 // pages [4*z+wid :: 4*SPLIT]; per-WG partials (m, l, o) land in `partial`
 // [rows, kvh, SPLIT, GROUP, D+2] fp32 and a second kernel merges them.
@@ -360,8 +354,8 @@ __global__ __launch_bounds__(256) void paged_attn_v3_kernel(
         for (int i = 0; i < 4; ++i) {
           float2v lo = __builtin_amdgcn_cvt_pk_f32_fp8(kq[i], false);
           float2v hi = __builtin_amdgcn_cvt_pk_f32_fp8(kq[i], true);
-          kw[2 * i] = pk_bf16(lo.x, lo.y);
-          kw[2 * i + 1] = pk_bf16(hi.x, hi.y);
+          kw[2 * i] = cvt_pk_bf16(lo.x, lo.y);
+          kw[2 * i + 1] = cvt_pk_bf16(hi.x, hi.y);
         }
       } else {
         #pragma unroll

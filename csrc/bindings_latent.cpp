@@ -440,6 +440,7 @@ void latent_attn_prefill(Tensor out, Tensor q, Tensor kn, Tensor lat,
   TORCH_CHECK(positions.numel() == q.size(0), "latent_attn_prefill: rows");
   const long B = seq_start.numel() - 1;
   check_tiles(tiles, seq_start, B);
+  TORCH_CHECK(tiles.size(0) <= 65535, "latent_attn_prefill: tiles");
   check_ints(kv_start, B, "kv_start");
   check_ints(kv_first, B, "kv_first");
   launch_latent_attn_prefill(

@@ -47,12 +47,12 @@ void launch_kept_attn_general(T*, const T*, const T*, const T*, const int*,
 void launch_kept_attn_prefill(bf16*, const bf16*, const bf16*, const bf16*,
                               const int*, const long*, const int*, const int*,
                               const double*, const float*, int, int, int, int,
-                              int, int, int, int, float, long, long,
+                              int, int, int, int, float, bool, long, long,
                               hipStream_t);
 void launch_kept_attn_decode(bf16*, const bf16*, const bf16*, const bf16*,
                              const int*, const long*, const double*,
                              const float*, float*, long, int, int, int, int,
-                             int, int, int, float, long, long, int,
+                             int, int, int, float, bool, long, long, int,
                              hipStream_t);
 template <typename T>
 void launch_clamped_glu(T*, const T*, long, int, float, hipStream_t);
@@ -424,7 +424,8 @@ void kept_attn_general(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
 void kept_attn_prefill(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
                        Tensor block_tables, Tensor positions,
                        Tensor seq_start, Tensor tiles, Tensor turn,
-                       Maybe sink, long window, long keep, double scale) {
+                       Maybe sink, long window, long keep, double scale,
+                       bool bounded) {
   const auto a = check_kept(out, q, k_cache, v_cache, block_tables, positions,
                             turn, sink, window, keep);
   TORCH_CHECK(kept_attn_fits(out, q, k_cache, v_cache), "kept_attn: sizes");
@@ -435,7 +436,7 @@ void kept_attn_prefill(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
       block_tables.data_ptr<int>(), positions.data_ptr<long>(),
       seq_start.data_ptr<int>(), tiles.data_ptr<int>(), a.turn, a.sink,
       (int)tiles.size(0), (int)block_tables.size(1), a.d.H, a.d.G, a.d.D,
-      a.d.E, (int)window, (int)keep, (float)scale, q.stride(0),
+      a.d.E, (int)window, (int)keep, (float)scale, bounded, q.stride(0),
       out.stride(0), stream());
 }
 
@@ -443,7 +444,7 @@ void kept_attn_prefill(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
 void kept_attn_decode(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
                       Tensor block_tables, Tensor positions, Tensor turn,
                       Maybe sink, Maybe partial, long split, long window,
-                      long keep, double scale) {
+                      long keep, double scale, bool bounded) {
   const auto a = check_kept(out, q, k_cache, v_cache, block_tables, positions,
                             turn, sink, window, keep);
   const long rows = q.size(0);
@@ -459,8 +460,8 @@ void kept_attn_decode(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
       block_tables.data_ptr<int>(), positions.data_ptr<long>(), a.turn,
       a.sink, split > 1 ? ptr<float>(*partial) : nullptr, rows,
       (int)block_tables.size(1), a.d.H, a.d.G, a.d.D, a.d.E, (int)window,
-      (int)keep, (float)scale, q.stride(0), out.stride(0), (int)split,
-      stream());
+      (int)keep, (float)scale, bounded, q.stride(0), out.stride(0),
+      (int)split, stream());
 }
 
 }  // namespace

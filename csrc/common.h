@@ -139,11 +139,16 @@ typedef __attribute__((ext_vector_type(8))) short short8_t;
 typedef __attribute__((ext_vector_type(4))) float f32x4_t;
 typedef __attribute__((ext_vector_type(16))) float f32x16_t;
 
-// two floats -> packed bf16 (round to nearest even)
+// two floats -> packed bf16 (round to nearest even), one v_cvt_pk_bf16_f32.
+// Not as inline assembly: the compiler would not see that its operands may
+// come straight from a transcendental or matrix instruction, whose results
+// need a wait before they are read.
 DEV unsigned cvt_pk_bf16(float a, float b) {
-  unsigned r;
-  asm("v_cvt_pk_bf16_f32 %0, %1, %2" : "=v"(r) : "v"(a), "v"(b));
-  return r;
+  typedef __attribute__((ext_vector_type(2))) float float2_t;
+  typedef __attribute__((ext_vector_type(2))) __bf16 bf16x2_t;
+  union { bf16x2_t v; unsigned u; } r;
+  r.v = __builtin_convertvector(float2_t{a, b}, bf16x2_t);
+  return r.u;
 }
 
 // f = hi + lo to ~16 bits of mantissa: a float operand as two bf16 ones

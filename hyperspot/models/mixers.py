@@ -491,6 +491,9 @@ class KeptWindowAttention(JoinedMixer):
         tp, r = get_tp_size(), get_tp_rank()
         self.sink = None if m.sink is None else _rows(_param(
             torch.full((m.heads // tp,), float(m.sink))), tp, r, m.heads)
+        # normed queries and keys: a score is at most dim * |scale|
+        self.bounded = m.qk_norm and m.dim * abs(m.scale) <= 40 \
+            and abs(m.sink or 0.0) <= 40
 
     def forward(self, x, meta, cache) -> torch.Tensor:
         m = self.spec
@@ -499,7 +502,8 @@ class KeptWindowAttention(JoinedMixer):
                                 gain(m.stretch),
                                 self.eps if m.qk_norm else None, side)
         hybrid.window_attention(out, q, cache, meta, self.turn, self.sink,
-                                m.window, m.keep_first, m.scale)
+                                m.window, m.keep_first, m.scale,
+                                self.bounded)
         return self.o_proj(joined)
 
     def tensors(self, p: str):

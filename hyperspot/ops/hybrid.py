@@ -311,10 +311,12 @@ def rope_norm_append(q, k, v, meta, freqs, turn, cache, gain: float,
 
 
 def window_attention(out, q, cache, meta, turn, sink, window: int, keep: int,
-                     scale: float) -> None:
+                     scale: float, bounded: bool = False) -> None:
     """out [T, H * E] (a column view): softmax attention over the last
     `window` positions and the first `keep`, `sink` [H] float in the
-    denominators (None: nothing); outputs turned back by `turn`."""
+    denominators (None: nothing); outputs turned back by `turn`.  `bounded`:
+    scores and sinks lie within +-40, so their exponentials need no running
+    maximum."""
     row_seq = meta.row_seq if meta.mode == "prefill" else None
     if not q.is_cuda:
         torch_ref.window_attention(
@@ -330,7 +332,7 @@ def window_attention(out, q, cache, meta, turn, sink, window: int, keep: int,
                             scale)
     elif meta.mode == "prefill":
         n.kept_attn_prefill(out, q, *where, meta.seq_start, meta.tiles, turn,
-                            sink, window, keep, scale)
+                            sink, window, keep, scale, bounded)
     else:
         reach = min(window + keep,
                     meta.block_tables.shape[1] * cache.k.shape[2])
@@ -338,7 +340,7 @@ def window_attention(out, q, cache, meta, turn, sink, window: int, keep: int,
         partial = None if split == 1 else torch.empty(
             T * H * split * (E + 4), dtype=torch.float32, device=q.device)
         n.kept_attn_decode(out, q, *where, turn, sink, partial, split, window,
-                           keep, scale)
+                           keep, scale, bounded)
 
 
 def norm_append(q, k, v, qw, kw, meta, cache, eps: float) -> None:

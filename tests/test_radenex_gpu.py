@@ -175,11 +175,17 @@ def attention_case(H, G, D, E, window, keep, starts, lens, dtype,
     wide = torch.full((T, H * E + 16), 7.0, dtype=dtype, device=DEV)
     out = wide[:, 8:8 + H * E]
     freqs = frequencies(E if turn else 0, 50.0)
-    hybrid.window_attention(
-        out, buf.to(DEV)[:, :H * D], KVPages(kc.to(DEV), vc.to(DEV)), m,
+    run = lambda to, bounded: hybrid.window_attention(
+        to, buf.to(DEV)[:, :H * D], KVPages(kc.to(DEV), vc.to(DEV)), m,
         freqs.to(DEV), None if bias is None else bias.to(DEV), window, keep,
-        scale)
+        scale, bounded)
+    run(out, False)
     assert (wide[:, :8] == 7.0).all() and (wide[:, -8:] == 7.0).all()
+    if not loud:                       # small scores: without their maximum
+        again = torch.full_like(wide, 7.0)
+        run(again[:, 8:8 + H * E], True)
+        assert (again[:, :8] == 7.0).all() and (again[:, -8:] == 7.0).all()
+        assert rel(again, f64(wide)) < tol(dtype)
     want, row, x = [], 0, f64(buf)
     for i in range(n):
         ki, vi = f64(k[i]), f64(v[i])
