@@ -282,9 +282,7 @@ void kept_attn_prefill_kernel(Kept<bf16> a,
     constexpr bool FULL = decltype(full)::value;
     const int b0 = HW == 2 ? 0 : half;           // first block in LDS
     f32x16_t sc[NB];
-    float mx = m;
-    #pragma unroll
-    for (int i = 0; i < NB; ++i) {
+    auto scores = [&](int i) {
       sc[i] = f32x16_t(0.f);
       #pragma unroll
       for (int c = 0; c < KC; ++c)
@@ -301,26 +299,9 @@ void kept_attn_prefill_kernel(Kept<bf16> a,
           if (at > qp || (at <= qp - a.window && at >= a.keep)) x = -FLT_MAX;
         }
         sc[i][r] = x;
-        if constexpr (!BOUNDED) mx = fmaxf(mx, x);
       }
-    }
-    if constexpr (!BOUNDED) {
-      mx = fmaxf(mx, __shfl_xor(mx, 32));
-      if (!__all(mx == m)) {
-        const float alpha = m == -FLT_MAX ? 0.f : exp2_fast(m - mx);
-        #pragma unroll
-        for (int e = 0; e < ET; ++e)
-          #pragma unroll
-          for (int r = 0; r < 16; ++r) acc[e][r] *= alpha;
-        l *= alpha;
-        m = mx;
-      }
-    }
-    // a column without a visible key yet has m = -FLT_MAX: with base 0 its
-    // masked scores weigh exp2(-FLT_MAX) = 0
-    const float base = BOUNDED || m == -FLT_MAX ? 0.f : m;
-    #pragma unroll
-    for (int i = 0; i < NB; ++i) {
+    };
+    auto values = [&](int i, float base) {
       short8_t ph[2], pl[2];
       #pragma unroll
       for (int c = 0; c < 2; ++c) {
@@ -342,6 +323,36 @@ void kept_attn_prefill_kernel(Kept<bf16> a,
           acc[e] = mfma32(vf, ph[c], acc[e]);
           acc[e] = mfma32(vf, pl[c], acc[e]);
         }
+    };
+    if constexpr (BOUNDED) {
+      #pragma unroll
+      for (int i = 0; i < NB; ++i) {
+        scores(i);
+        values(i, 0.f);
+      }
+    } else {
+      float mx = m;
+      #pragma unroll
+      for (int i = 0; i < NB; ++i) {
+        scores(i);
+        #pragma unroll
+        for (int r = 0; r < 16; ++r) mx = fmaxf(mx, sc[i][r]);
+      }
+      mx = fmaxf(mx, __shfl_xor(mx, 32));
+      if (!__all(mx == m)) {
+        const float alpha = m == -FLT_MAX ? 0.f : exp2_fast(m - mx);
+        #pragma unroll
+        for (int e = 0; e < ET; ++e)
+          #pragma unroll
+          for (int r = 0; r < 16; ++r) acc[e][r] *= alpha;
+        l *= alpha;
+        m = mx;
+      }
+      // a column without a visible key yet has m = -FLT_MAX: with base 0 its
+      // masked scores weigh exp2(-FLT_MAX) = 0
+      const float base = m == -FLT_MAX ? 0.f : m;
+      #pragma unroll
+      for (int i = 0; i < NB; ++i) values(i, base);
     }
   };
   int kv0 = kept > 0 ? 0 : from;

@@ -107,8 +107,8 @@ PRESETS = {
     # CPU / CI size, and one with the layer sizes of a real model
     "tiny-radenex": lambda: preset("tiny-radenex", 96, 512, 4, 2, 24, 20, 3,
                                    3, 24, 16, 40, 160, 4, (1, 3, 2)),
-    "radenex-7b": lambda: preset("radenex-7b", 4096, 102400, 32, 8, 128, 4096,
-                                 4, 32, 128, 64, 512, 14336, 32),
+    "radenex-8b": lambda: preset("radenex-8b", 4096, 102400, 32, 8, 128, 4096,
+                                 4, 32, 128, 64, 512, 21504, 32),
 }
 
 

@@ -105,7 +105,8 @@ def _absorbed(out, q, cache, meta, row_seq, rows, uk, uv, heads, window,
 
 def absorbed_split(groups: int, reach: int) -> int:
     """How many workgroups share one row's window, each with at least 64
-    tokens: one for every compute unit where the batch alone gives fewer, two
-    otherwise.  Depends on shapes only, so a captured graph keeps it."""
-    fill = 256 if groups < 256 else 512
+    tokens: one for every compute unit where few rows would give each many
+    parts to combine, two otherwise.  Depends on shapes only, so a captured
+    graph keeps it."""
+    fill = 256 if groups < 128 else 512
     return max(1, min(16, fill // groups, reach // 64))

@@ -7,6 +7,11 @@ logits head) and writes profiles/tunableop_gfx950.csv, which ModelRunner
 loads read-only at engine init.
 
 Run on an MI355X box:  python tools/tune_gemms.py [--out FILE]
+
+With --design NAME the products of a design's layers that have a feed-forward
+beside the mixer are tuned instead, and FILE gains (or renews) the lines of
+those whose choice beats the library's own, timed in a replayed graph and
+checked against it over several replays.
 """
 
 from __future__ import annotations
@@ -14,22 +19,28 @@ from __future__ import annotations
 import argparse
 import os
 import sys
+import tempfile
 
 sys.path.insert(0, os.path.dirname(os.path.dirname(os.path.abspath(__file__))))
 
 ap = argparse.ArgumentParser()
 ap.add_argument("--out", default="profiles/tunableop_gfx950.csv")
 ap.add_argument("--include-70b", action="store_true")
+ap.add_argument("--design", default=None, metavar="NAME")
 args = ap.parse_args()
 
 # TunableOp reads its env at tuning-context construction — set everything
 # before torch loads.
-os.environ["PYTORCH_TUNABLEOP_ENABLED"] = "1"
-os.environ["PYTORCH_TUNABLEOP_TUNING"] = "1"
-os.environ["PYTORCH_TUNABLEOP_FILENAME"] = args.out
 os.environ["PYTORCH_TUNABLEOP_MAX_TUNING_DURATION_MS"] = "10"
 os.environ["PYTORCH_TUNABLEOP_MAX_TUNING_ITERATIONS"] = "30"
-os.environ["PYTORCH_TUNABLEOP_VERBOSE"] = "1"
+if args.design is None:
+    os.environ["PYTORCH_TUNABLEOP_ENABLED"] = "1"
+    os.environ["PYTORCH_TUNABLEOP_TUNING"] = "1"
+    os.environ["PYTORCH_TUNABLEOP_FILENAME"] = args.out
+    os.environ["PYTORCH_TUNABLEOP_VERBOSE"] = "1"
+else:            # switched on and off by the program, results merged by it
+    os.environ["PYTORCH_TUNABLEOP_FILENAME"] = os.path.join(
+        tempfile.mkdtemp(), "results.csv")
 
 import torch  # noqa: E402
 
@@ -57,8 +68,103 @@ def gemm_shapes(include_70b=False):
             yield m, h, spec["vocab"]   # logits head
 
 
+def joined_shapes(spec):
+    """(rows, k, n) of the merged projections and of the joined sum of every
+    kind of layer."""
+    from hyperspot.engine.layer_spec import LatentAttention
+    up8 = lambda n: (n + 7) // 8 * 8
+    w, out = spec.hidden_size, []
+    for m, ff in dict.fromkeys((x.mixer, x.ff) for x in spec.layers):
+        if isinstance(m, LatentAttention):
+            parts = [m.heads * (m.dim + m.rot_dim), m.kv_rank + m.rot_dim,
+                     m.heads]
+        else:
+            parts = [m.heads * m.dim, m.kv_heads * m.dim,
+                     m.kv_heads * m.vdim]
+        n = sum(map(up8, parts + [ff.ff]))
+        out += [(w, n), (m.heads * m.vdim + ff.ff, w)]
+    rows = (1, 2, 4, 8, 16, 24, 32, 48, 64, 96, 128, 192, 256, 384, 512, 768,
+            1024, 2048, 8192)
+    return [(m, k, n) for k, n in dict.fromkeys(out) for m in rows]
+
+
+def graph_time(fn, calls=5, replays=20):
+    """us a call within a replayed graph."""
+    fn()
+    torch.cuda.synchronize()
+    g = torch.cuda.CUDAGraph()
+    with torch.cuda.graph(g):
+        for _ in range(calls):
+            fn()
+    for _ in range(3):
+        g.replay()
+    a, b = (torch.cuda.Event(enable_timing=True) for _ in range(2))
+    a.record()
+    for _ in range(replays):
+        g.replay()
+    b.record()
+    torch.cuda.synchronize()
+    return a.elapsed_time(b) * 1e3 / (calls * replays)
+
+
+def same_in_graph(x, w):
+    """A replayed graph gives what the library's own choice gives, over and
+    over, with other work and other inputs between the replays."""
+    t, ok = torch.cuda.tunable, True
+    g = torch.cuda.CUDAGraph()
+    with torch.cuda.graph(g):
+        y = x @ w.t()
+    for _ in range(5):
+        x.normal_()
+        g.replay()
+        got = y.float()
+        t.enable(False)
+        want = (x @ w.t()).float()
+        t.enable(True)
+        torch.cuda.synchronize()
+        err = (got - want).pow(2).mean().sqrt() / want.pow(2).mean().sqrt()
+        ok = ok and float(err) < 1e-2
+    return ok
+
+
+def tune_design(name, out):
+    from hyperspot.engine.config import get_model_spec
+    t = torch.cuda.tunable
+    lines, keep, drop = open(out).read().splitlines(), {}, set()
+    for m, k, n in joined_shapes(get_model_spec(name)):
+        x = torch.randn(m, k, dtype=torch.bfloat16, device="cuda:0")
+        w = torch.randn(n, k, dtype=torch.bfloat16, device="cuda:0") * 0.02
+        fn = lambda: x @ w.t()
+        plain = graph_time(fn)
+        before = {r[:2] for r in t.get_results()}
+        t.enable(True)
+        t.tuning_enable(True)
+        fn()
+        t.tuning_enable(False)
+        new = [r for r in t.get_results() if r[:2] not in before]
+        tuned, good = graph_time(fn), same_in_graph(x, w)
+        t.enable(False)
+        plain = min(plain, graph_time(fn))
+        won = good and tuned < 0.97 * plain
+        for op, params, solution, ms in new:
+            if won:
+                keep[f"{op},{params}"] = f"{op},{params},{solution},{ms:g}"
+            else:
+                drop.add(f"{op},{params}")
+        print(f"{m}x{k}x{n}: {plain:.1f} us, tuned {tuned:.1f} us"
+              f"{'' if good else ', WRONG'}{' *' if won else ''}", flush=True)
+        del x, w
+    head = lambda line: ",".join(line.split(",")[:2])
+    lines = [x for x in lines if head(x) not in keep and head(x) not in drop]
+    with open(out, "w") as f:
+        f.write("\n".join(lines + list(keep.values())) + "\n")
+    print(f"{len(keep)} choices kept")
+
+
 def main():
     assert torch.cuda.is_available()
+    if args.design:
+        return tune_design(args.design, args.out)
     dev = "cuda:0"
     seen = set()
     shapes = [s for s in gemm_shapes(args.include_70b)
