@@ -518,22 +518,24 @@ __global__ __launch_bounds__(256, 2) void latent_attn_decode_kernel(
 
 // Partial results of RB <= 16 rows and one head combined, then W_uv of that
 // head: out[row, h] = W_uv[h] sum_p weight_p o_p.  split <= 16, rank <= 512.
-// A wave has 16 of every gridDim.z * 64 values; its first weights are on their
-// way while the results are combined.
-template <int RB>
-__global__ __launch_bounds__(256) void latent_merge_values_kernel(
+// NW waves, 4 or 8; a wave has 16 of every gridDim.z * NW * 16 values, its first
+// weights are on their way while the results are combined.
+template <int RB, int NW>
+__global__ __launch_bounds__(64 * NW) void latent_merge_values_kernel(
     bf16* __restrict__ out, const float* __restrict__ partial,
     const bf16* __restrict__ uv, const int* __restrict__ rows, long R,
     int split, int H, int E, int rank, long os, Gate<bf16> gate) {
   extern __shared__ __attribute__((aligned(16))) short merged[];
   __shared__ float weight[16][17];
-  constexpr int RK = RB < 4 ? RB : 4;        // rows combined together
+  constexpr int GROUPS = NW / 4;             // of waves, each has other rows
+  constexpr int RG = RB < GROUPS ? 1 : RB / GROUPS;
+  constexpr int RK = RG < 4 ? RG : 4;        // rows combined together
   const int h = blockIdx.y, tid = threadIdx.x;
   const long r0 = (long)blockIdx.x * RB;
   const int live = (int)min((long)RB, R - r0);
   const int XS = rank + 8;
   const int lane = tid & 63, wid = tid >> 6, col = lane & 15, gr = lane >> 4;
-  int n0 = (blockIdx.z * 4 + wid) * 16;
+  int n0 = (blockIdx.z * NW + wid) * 16;
   short8_t wf[16];
   auto weights = [&]() {
     const bool wn = n0 + col < E;
@@ -546,7 +548,7 @@ __global__ __launch_bounds__(256) void latent_merge_values_kernel(
   weights();
   const long r = rows && col < live ? rows[r0 + col] : r0 + col;
   const float f = col < live ? gate(r, h) : 0.f;
-  {
+  if (tid < 256) {
     const int i = tid >> 4, p = tid & 15;
     const bool in = i < live && p < split;
     const float* src = partial +
@@ -563,9 +565,9 @@ __global__ __launch_bounds__(256) void latent_merge_values_kernel(
   }
   __syncthreads();
   // a wave has a quarter of the columns
-  const int quarter = rank / 4;
-  for (int c = wid * quarter + lane * 2; c < (wid + 1) * quarter; c += 128)
-    for (int i0 = 0; i0 < live; i0 += RK) {
+  const int quarter = rank / 4, part = wid & 3;
+  for (int c = part * quarter + lane * 2; c < (part + 1) * quarter; c += 128)
+    for (int i0 = (wid >> 2) * RK; i0 < live; i0 += GROUPS * RK) {
       float2 o[RK] = {};
       const float* src[RK];
       #pragma unroll
@@ -605,7 +607,7 @@ __global__ __launch_bounds__(256) void latent_merge_values_kernel(
       *reinterpret_cast<uint2*>(out + r * os + (long)h * E + n) =
           uint2{cvt_pk_bf16(acc[0] * f, acc[1] * f),
                 cvt_pk_bf16(acc[2] * f, acc[3] * f)};
-    n0 += gridDim.z * 64;
+    n0 += gridDim.z * NW * 16;
     if (n0 < E) weights();
   }
 }
@@ -946,14 +948,18 @@ void launch_latent_merge_values(bf16* out, const float* partial,
   // few rows: fewer a workgroup, then fewer values a workgroup
   int rb = 16;
   while (rb > 1 && (R + rb - 1) / rb * H < 256) rb /= 2;
-  const unsigned nz = R * H < 128 ? (unsigned)((E + 63) / 64) : 1;
+  const long units = R * H;
+  const bool wide = units >= 128 && units <= 4096;
+  const unsigned nz = units < 128 ? (unsigned)((E + 63) / 64) : 1;
   const dim3 grid((unsigned)((R + rb - 1) / rb), (unsigned)H, nz);
+  auto run = [&](auto kernel, int threads) {
+    kernel<<<grid, threads, 16 * (rank + 8) * 2, stream>>>(
+        out, partial, uv, rows, R, split, H, E, rank, os, Gate<bf16>{g, gs});
+  };
   #define CASE(RB)                                                          \
     if (rb == RB)                                                           \
-      latent_merge_values_kernel<RB>                                        \
-          <<<grid, 256, 16 * (rank + 8) * 2, stream>>>(                     \
-              out, partial, uv, rows, R, split, H, E, rank, os,             \
-              Gate<bf16>{g, gs});
+      wide ? run(&latent_merge_values_kernel<RB, 8>, 512)                   \
+           : run(&latent_merge_values_kernel<RB, 4>, 256);
   CASE(1) CASE(2) CASE(4) CASE(8) CASE(16)
   #undef CASE
 }
