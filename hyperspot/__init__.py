@@ -6,7 +6,7 @@ data plane exists only as specification).  This package is the *serving plane*:
 
   - ``hyperspot.engine``   — paged-KV continuous-batching inference engine
   - ``hyperspot.models``   — model families (Llama-3, Mixtral MoE, Sumosun,
-    Tefezen, Mutusun)
+    Tefezen, Mutusun, Radenex)
   - ``hyperspot.ops``      — op layer: hand-written CDNA4 HIP kernels (gfx950)
                              with PyTorch fp32 reference implementations for CPU
   - ``hyperspot.parallel`` — TP/EP process groups over RCCL (xGMI)
