@@ -518,8 +518,8 @@ __global__ __launch_bounds__(256, 2) void latent_attn_decode_kernel(
 
 // Partial results of RB <= 16 rows and one head combined, then W_uv of that
 // head: out[row, h] = W_uv[h] sum_p weight_p o_p.  split <= 16, rank <= 512.
-// NW waves, 4 or 8; a wave has 16 of every gridDim.z * NW * 16 values, its first
-// weights are on their way while the results are combined.
+// NW waves, 4 or 8; a wave has 16 of every gridDim.z * NW * 16 values, its
+// first weights are on their way while the results are combined.
 template <int RB, int NW>
 __global__ __launch_bounds__(64 * NW) void latent_merge_values_kernel(
     bf16* __restrict__ out, const float* __restrict__ partial,
